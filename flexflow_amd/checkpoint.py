@@ -44,6 +44,14 @@ def convert_hf_model(model_or_state_dict, dst_folder: str, dtype=np.float16) -> 
     return written
 
 
+def load_config(folder: str) -> dict:
+    """A model folder's config.json as Model takes it: families of the
+    runtime's registry ("architecture") as they are, HF LLaMA as sizes."""
+    with open(os.path.join(folder, "config.json")) as f:
+        c = json.load(f)
+    return c if "architecture" in c else llama_config_from_hf(c)
+
+
 def llama_config_from_hf(src: Union[str, Mapping]) -> dict:
     """LLAMAConfig (llama.h:30-79) from an HF config.json path, a folder
     holding one, or an already-parsed dict."""

@@ -31,6 +31,15 @@ namespace ffmi {
 typedef _Float16 h8 __attribute__((ext_vector_type(8)));
 typedef _Float16 h4 __attribute__((ext_vector_type(4)));
 typedef float f4 __attribute__((ext_vector_type(4)));
+typedef __bf16 bf8 __attribute__((ext_vector_type(8)));
+
+// bf16 <-> fp32, round to nearest even
+__device__ __forceinline__ uint16_t f2bf(float v) {
+  return __builtin_bit_cast(uint16_t, (__bf16)v);
+}
+__device__ __forceinline__ float bf2f(uint16_t v) {
+  return __builtin_bit_cast(float, (uint32_t)v << 16);
+}
 
 // Weight fragment load.  NT (FFMI_W_STREAM launches: a model whose weights
 // exceed the Infinity Cache, each weight byte read by one workgroup) puts the
@@ -132,6 +141,7 @@ hipError_t launch_fill_weight(uint16_t *dst, size_t n, uint64_t key, int kind, h
 hipError_t launch_fill_weight_f32(float *dst, size_t n, uint64_t key, int kind, hipStream_t s,
                                   int cols = 0, uint64_t pa = 1, uint64_t pb = 0,
                                   float scale = 1.0f);
+hipError_t launch_fill_weight_bf16(uint16_t *dst, size_t n, uint64_t key, int kind, hipStream_t s);
 float weight_amp(int kind);
 // ---- full-precision path (kernels/f32.hip) ----
 hipError_t launch_gemm_f32(const float *X, const float *W, float *Y, int T, int N, int K,
@@ -148,7 +158,7 @@ hipError_t launch_attention_f32(const char *blob, int T, const float *qbuf, cons
                                 const float *vc, float *out, int heads, int d, int slots,
                                 float scale, hipStream_t s);
 hipError_t launch_softmax_topk_f32(const float *logits, int T, int V, int k, int32_t *ids,
-                                   float *probs, hipStream_t s);
+                                   float *probs, hipStream_t s, int ld = 0);  // (0: ld = V)
 ffmi_status attn_rope_fault(ffmi_attn *h, int from_pos);
 // Packed weights (weights.hip): 1 KiB block (tile t, k-step kt) at
 // t * w_tile_stride(KT) + kt * w_k_stride(P) halves, P = tiles per k-row of
@@ -191,6 +201,20 @@ hipError_t launch_gemm(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float
                        size_t ws_bytes, int T, int N, int K, int epilogue, hipStream_t s,
                        Partials *defer = nullptr, int wpitch = 0, const FuseArgs *fuse = nullptr);
 size_t gemm_workspace_bytes(int T, int N, int K, int epilogue);
+// The same GEMM on bf16 operands in packed activation tiles, one entry per
+// epilogue: Y bf16; Y bf16 = relu(x)^2; or fp32 slabs in `ws` (*defer, or one
+// unsplit [T][ceil16(N)] slab when defer is null).  flags: FFMI_X_PACKED |
+// FFMI_Y_PACKED | FFMI_W_STREAM
+size_t gemm_bf16_workspace_bytes(int T, int N, int K);
+hipError_t launch_gemm_bf16_plain(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
+                                  size_t ws_bytes, int T, int N, int K, int flags, hipStream_t s,
+                                  Partials *defer = nullptr);
+hipError_t launch_gemm_bf16_relu2(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
+                                  size_t ws_bytes, int T, int N, int K, int flags, hipStream_t s,
+                                  Partials *defer = nullptr);
+hipError_t launch_gemm_bf16_f32(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
+                                size_t ws_bytes, int T, int N, int K, int flags, hipStream_t s,
+                                Partials *defer = nullptr);
 // fp16 Y[T][N] (row-major) of deferred split-K slabs, summed in slab order and
 // rounded once: the value every consumer of the slabs computes (tensor capture)
 hipError_t launch_partials_reduce(const Partials &p, uint16_t *Y, int T, int N, hipStream_t s);

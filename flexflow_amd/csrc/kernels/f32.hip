@@ -406,7 +406,7 @@ hipError_t launch_attention_f32(const char *blob, int T, const float *qbuf, cons
 // previous pick in that order (arg_topk.cu:208-330 ties: lower index first).
 // ---------------------------------------------------------------------------
 __global__ __launch_bounds__(1024) void f32_softmax_topk_kernel(const float *__restrict__ logits,
-                                                               int V, int k,
+                                                               int V, int ld, int k,
                                                                int32_t *__restrict__ ids,
                                                                float *__restrict__ probs) {
   __shared__ float shf[16];
@@ -414,7 +414,7 @@ __global__ __launch_bounds__(1024) void f32_softmax_topk_kernel(const float *__r
   __shared__ float sp[16];
   __shared__ int si[16];
   const int t = blockIdx.x, tid = threadIdx.x, nw = blockDim.x >> 6;
-  const float *z = logits + (size_t)t * V;
+  const float *z = logits + (size_t)t * ld;
   float mx = -3.402823466e38f;
   for (int i = tid; i < V; i += blockDim.x) mx = fmaxf(mx, z[i]);
 #pragma unroll
@@ -463,10 +463,12 @@ __global__ __launch_bounds__(1024) void f32_softmax_topk_kernel(const float *__r
 }
 
 hipError_t launch_softmax_topk_f32(const float *logits, int T, int V, int k, int32_t *ids,
-                                   float *probs, hipStream_t s) {
+                                   float *probs, hipStream_t s, int ld) {
   if (T <= 0) return hipSuccess;
-  if (k < 1 || k > V) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(f32_softmax_topk_kernel, dim3(T), dim3(1024), 0, s, logits, V, k, ids, probs);
+  if (ld == 0) ld = V;
+  if (k < 1 || k > V || ld < V) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(f32_softmax_topk_kernel, dim3(T), dim3(1024), 0, s, logits, V, ld, k, ids,
+                     probs);
   return hipGetLastError();
 }
 

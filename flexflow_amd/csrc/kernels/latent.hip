@@ -1,0 +1,844 @@
+// latent.hip -- latent attention over a paged cache (latent.h), the 32-bit
+// residual stream's post-sublayer norms, and the loaders' packing kernels.
+#include <algorithm>
+
+#include "latent.h"
+
+namespace ffmi {
+
+// ---------------------------------------------------------------------------
+// residual stream (fp32 x, bf16 packed copy for the GEMMs)
+// ---------------------------------------------------------------------------
+__device__ __forceinline__ uint4 pack8_bf16(const f4 &a, const f4 &b) {
+  uint4 o;
+  o.x = f2bf(a[0]) | ((uint32_t)f2bf(a[1]) << 16);
+  o.y = f2bf(a[2]) | ((uint32_t)f2bf(a[3]) << 16);
+  o.z = f2bf(b[0]) | ((uint32_t)f2bf(b[1]) << 16);
+  o.w = f2bf(b[2]) | ((uint32_t)f2bf(b[3]) << 16);
+  return o;
+}
+__device__ __forceinline__ void unpack8_bf16(const uint4 &v, f4 &a, f4 &b) {
+  const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const float lo = __builtin_bit_cast(float, w[i] << 16);
+    const float hi = __builtin_bit_cast(float, w[i] & 0xffff0000u);
+    if (i < 2) a[2 * i] = lo, a[2 * i + 1] = hi;
+    else b[2 * i - 4] = lo, b[2 * i - 3] = hi;
+  }
+}
+
+__global__ __launch_bounds__(256) void embed_pos_kernel(
+    const char *__restrict__ blob_src, uint4 *__restrict__ blob_dst, int blob_n16,
+    const uint16_t *__restrict__ embed, const uint16_t *__restrict__ pos, float *__restrict__ x,
+    uint16_t *__restrict__ xb, int H) {
+  const int t = blockIdx.x;
+  const PagedToken tk = reinterpret_cast<const PagedToken *>(blob_src)[t];  // tokens come first
+  const uint4 *src = reinterpret_cast<const uint4 *>(blob_src);
+  for (int i = t * 256 + threadIdx.x; i < blob_n16; i += gridDim.x * 256) blob_dst[i] = src[i];
+  for (int c = threadIdx.x; c < H / 8; c += 256) {
+    f4 a, b, pa, pb;
+    unpack8_bf16(*reinterpret_cast<const uint4 *>(embed + (size_t)tk.token * H + c * 8), a, b);
+    unpack8_bf16(*reinterpret_cast<const uint4 *>(pos + (size_t)tk.pos * H + c * 8), pa, pb);
+    a += pa, b += pb;
+    *reinterpret_cast<f4 *>(x + (size_t)t * H + c * 8) = a;
+    *reinterpret_cast<f4 *>(x + (size_t)t * H + c * 8 + 4) = b;
+    if (xb) *reinterpret_cast<uint4 *>(xb + act_packed_off(t, c * 8, H)) = pack8_bf16(a, b);
+  }
+}
+
+hipError_t launch_embed_pos(const char *blob_src, char *blob_dst, size_t blob_bytes,
+                            const uint16_t *embed, const uint16_t *pos, float *x, uint16_t *xb,
+                            int T, int H, hipStream_t s) {
+  if (T <= 0) return hipSuccess;
+  if (H % 32) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(embed_pos_kernel, dim3(T), dim3(256), 0, s, blob_src,
+                     reinterpret_cast<uint4 *>(blob_dst), (int)((blob_bytes + 15) / 16), embed, pos,
+                     x, xb, H);
+  return hipGetLastError();
+}
+
+template <int NT>
+__device__ __forceinline__ float row_sum(float v, float *sh) {
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
+  if ((threadIdx.x & 63) == 0) sh[threadIdx.x >> 6] = v;
+  __syncthreads();
+  v = sh[0];
+#pragma unroll
+  for (int i = 1; i < NT / 64; ++i) v += sh[i];
+  return v;
+}
+__device__ __forceinline__ float inv_rms(float ss, int n, float eps) {
+  return __fdiv_rn(1.0f, sqrtf(__fdiv_rn(ss, (float)n) + eps));
+}
+
+// One workgroup per row; the slab, x and w loads of a chunk are all issued
+// before the reduction.
+template <int NT, int MAXC, int MAXS>
+__global__ __launch_bounds__(NT) void post_norm_kernel(const float *__restrict__ yp, int S, int NP,
+                                                       const float *__restrict__ w,
+                                                       float *__restrict__ x,
+                                                       uint16_t *__restrict__ xb, int H, int n,
+                                                       float eps) {
+  __shared__ float sh[NT / 64];
+  const int row = blockIdx.x, T = gridDim.x, nchunk = H >> 3;
+  f4 y[MAXC][2], xv[MAXC][2], wv[MAXC][2];
+  float ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = min((int)threadIdx.x + c * NT, nchunk - 1);
+    const float *q = yp + (size_t)row * NP + ch * 8;
+    f4 lo[MAXS], hi[MAXS];
+#pragma unroll
+    for (int sl = 0; sl < MAXS; ++sl) {
+      const float *qs = q + (size_t)min(sl, S - 1) * T * NP;
+      lo[sl] = *reinterpret_cast<const f4 *>(qs);
+      hi[sl] = *reinterpret_cast<const f4 *>(qs + 4);
+    }
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      xv[c][h] = *reinterpret_cast<const f4 *>(x + (size_t)row * H + ch * 8 + 4 * h);
+      wv[c][h] = *reinterpret_cast<const f4 *>(w + ch * 8 + 4 * h);
+    }
+    y[c][0] = lo[0], y[c][1] = hi[0];
+#pragma unroll
+    for (int sl = 1; sl < MAXS; ++sl)
+      if (sl < S) y[c][0] += lo[sl], y[c][1] += hi[sl];
+    if ((int)threadIdx.x + c * NT < nchunk)
+#pragma unroll
+      for (int h = 0; h < 2; ++h)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss = fmaf(y[c][h][e], y[c][h][e], ss);
+  }
+  const float r = inv_rms(row_sum<NT>(ss, sh), n, eps);
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = threadIdx.x + c * NT;
+    if (ch >= nchunk) continue;
+#pragma unroll
+    for (int h = 0; h < 2; ++h)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) xv[c][h][e] += y[c][h][e] * r * wv[c][h][e];
+    *reinterpret_cast<f4 *>(x + (size_t)row * H + ch * 8) = xv[c][0];
+    *reinterpret_cast<f4 *>(x + (size_t)row * H + ch * 8 + 4) = xv[c][1];
+    if (xb)
+      *reinterpret_cast<uint4 *>(xb + act_packed_off(row, ch * 8, H)) = pack8_bf16(xv[c][0], xv[c][1]);
+  }
+}
+
+hipError_t launch_post_norm(Partials y, const float *w, float *x, uint16_t *xb, int T, int H, int n,
+                            float eps, hipStream_t s) {
+  if (T <= 0) return hipSuccess;
+  if (H % 32 || y.NP < H || y.NP % 4 || y.S < 1 || y.S > 8 || !y.p) return hipErrorInvalidValue;
+  const int nchunk = H / 8;
+#define FFMI_PN(NT, MC, MS)                                                                     \
+  hipLaunchKernelGGL((post_norm_kernel<NT, MC, MS>), dim3(T), dim3(NT), 0, s, y.p, y.S, y.NP, w, \
+                     x, xb, H, n, eps)
+#define FFMI_PNS(NT, MC)               \
+  do {                                 \
+    if (y.S == 1) FFMI_PN(NT, MC, 1);  \
+    else if (y.S == 2) FFMI_PN(NT, MC, 2); \
+    else if (y.S <= 4) FFMI_PN(NT, MC, 4); \
+    else FFMI_PN(NT, MC, 8);           \
+  } while (0)
+  if (nchunk <= 128) FFMI_PNS(128, 1);
+  else if (nchunk <= 256) FFMI_PNS(256, 1);
+  else if (nchunk <= 512) FFMI_PNS(512, 1);
+  else if (nchunk <= 1024) FFMI_PNS(1024, 1);
+  else if (nchunk <= 2048) FFMI_PNS(1024, 2);
+  else return hipErrorInvalidValue;
+#undef FFMI_PNS
+#undef FFMI_PN
+  return hipGetLastError();
+}
+
+__global__ __launch_bounds__(256) void row_norm_kernel(const int32_t *__restrict__ rows,
+                                                       const float *__restrict__ x,
+                                                       const float *__restrict__ w,
+                                                       uint16_t *__restrict__ hb,
+                                                       float *__restrict__ hf, int H, int n,
+                                                       float eps) {
+  __shared__ float sh[4];
+  const int i = blockIdx.x;
+  const float *xr = x + (size_t)rows[i] * H;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < H / 4; c += 256) {
+    const f4 v = *reinterpret_cast<const f4 *>(xr + c * 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss = fmaf(v[e], v[e], ss);
+  }
+  const float r = inv_rms(row_sum<256>(ss, sh), n, eps);
+  for (int c = threadIdx.x; c < H / 8; c += 256) {
+    f4 v[2];
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      v[h] = *reinterpret_cast<const f4 *>(xr + c * 8 + 4 * h);
+      const f4 wv = *reinterpret_cast<const f4 *>(w + c * 8 + 4 * h);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[h][e] = v[h][e] * r * wv[e];
+      if (hf) *reinterpret_cast<f4 *>(hf + (size_t)i * H + c * 8 + 4 * h) = v[h];
+    }
+    if (hb) *reinterpret_cast<uint4 *>(hb + act_packed_off(i, c * 8, H)) = pack8_bf16(v[0], v[1]);
+  }
+}
+
+hipError_t launch_row_norm(const char *blob, int off_rows, const float *x, const float *w,
+                           uint16_t *hb, float *hf, int R, int H, int n, float eps, hipStream_t s) {
+  if (R <= 0) return hipSuccess;
+  if (H % 32) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(row_norm_kernel, dim3(R), dim3(256), 0, s,
+                     reinterpret_cast<const int32_t *>(blob + off_rows), x, w, hb, hf, H, n, eps);
+  return hipGetLastError();
+}
+
+__global__ void relu2_f32_kernel(float *u, size_t n) {
+  for (size_t i = blockIdx.x * (size_t)blockDim.x + threadIdx.x; i < n;
+       i += (size_t)gridDim.x * blockDim.x) {
+    const float v = fmaxf(u[i], 0.f);
+    u[i] = v * v;
+  }
+}
+hipError_t launch_relu2_f32(float *u, size_t n, hipStream_t s) {
+  if (n == 0) return hipSuccess;
+  hipLaunchKernelGGL(relu2_f32_kernel, dim3((unsigned)std::min<size_t>((n + 255) / 256, 16384)),
+                     dim3(256), 0, s, u, n);
+  return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// latent store: one wave per token
+// ---------------------------------------------------------------------------
+__device__ __forceinline__ float ld_elem(const uint16_t *p) { return bf2f(*p); }
+__device__ __forceinline__ float ld_elem(const float *p) { return *p; }
+__device__ __forceinline__ void st_elem(uint16_t *p, float v) { *p = f2bf(v); }
+__device__ __forceinline__ void st_elem(float *p, float v) { *p = v; }
+
+template <class E>
+__device__ __forceinline__ void latent_store_token(const PagedToken &tk, const E *d, const float *w,
+                                                   E *cache, int rank, int n, float eps) {
+  const int lane = threadIdx.x & 63;
+  float ss = 0.f;
+  for (int i = lane; i < rank; i += 64) {
+    const float v = ld_elem(d + i);
+    ss = fmaf(v, v, ss);
+  }
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
+  const float r = inv_rms(ss, n, eps);
+  E *dst = cache + (size_t)tk.row * rank;
+  for (int i = lane; i < rank; i += 64) st_elem(dst + i, ld_elem(d + i) * r * w[i]);
+}
+
+__global__ __launch_bounds__(256) void latent_store_f32_kernel(const PagedToken *__restrict__ tok,
+                                                               int T, LatentStore st) {
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (t >= T) return;
+  latent_store_token(tok[t], (const float *)st.d + (size_t)t * st.ldd, st.w, (float *)st.cache,
+                     st.rank, st.n, st.eps);
+}
+hipError_t launch_latent_store_f32(const char *blob, int off_tokens, int T, const LatentStore &st,
+                                   hipStream_t s) {
+  if (T <= 0) return hipSuccess;
+  hipLaunchKernelGGL(latent_store_f32_kernel, dim3((T + 3) / 4), dim3(256), 0, s,
+                     reinterpret_cast<const PagedToken *>(blob + off_tokens), T, st);
+  return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// per-head products (bf16 MFMA): Y[t][h][n] = sum_k X[t][h][k] W_h[n][k]
+// ---------------------------------------------------------------------------
+// W_h tile-major: block (h, nt, kt) of 16 x 32 at ((h * NTt + nt) * KT + kt) *
+// 512.  Four waves, WM of them over row groups of MT tiles, 4 / WM over groups
+// of NT weight tiles.  D = W . X^T: a lane holds four consecutive columns of
+// one row.
+struct HgDev {
+  const uint16_t *X, *W, *gate;
+  uint16_t *Y;
+  int T, heads, KT, NTt, ldx, ldg, packed;
+  int gx, gz;  // weight-tile groups, row groups of the launch
+};
+template <int MT, int NT, int WM>
+__device__ __forceinline__ void head_gemm_block(const HgDev &a, int b) {
+  constexpr int WN = 4 / WM;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, l15 = lane & 15;
+  const int bx = b % a.gx, h = (b / a.gx) % a.heads, bz = b / (a.gx * a.heads);
+  const int nt0 = (bx * WN + wave % WN) * NT;
+  const int m0 = (bz * WM + wave / WN) * MT * 16;
+  if (nt0 >= a.NTt || m0 >= a.T) return;
+  const int K = a.KT * 32;
+  const uint16_t *xr[MT], *wr[NT];
+#pragma unroll
+  for (int i = 0; i < MT; ++i)
+    xr[i] = a.X + (size_t)min(m0 + i * 16 + l15, a.T - 1) * a.ldx + (size_t)h * K + 8 * g;
+#pragma unroll
+  for (int j = 0; j < NT; ++j)
+    wr[j] = a.W + ((size_t)h * a.NTt + min(nt0 + j, a.NTt - 1)) * a.KT * 512 + lane * 8;
+  f4 acc[MT][NT];
+#pragma unroll
+  for (int i = 0; i < MT; ++i)
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[i][j] = f4{0.f, 0.f, 0.f, 0.f};
+  constexpr int U = MT * NT >= 8 ? 2 : 4;  // k-steps of loads issued ahead of their MFMAs
+  for (int k0 = 0; k0 < a.KT; k0 += U) {
+    bf8 x[U][MT], w[U][NT];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int k = min(k0 + u, a.KT - 1);
+#pragma unroll
+      for (int j = 0; j < NT; ++j) w[u][j] = *reinterpret_cast<const bf8 *>(wr[j] + (size_t)k * 512);
+#pragma unroll
+      for (int i = 0; i < MT; ++i) x[u][i] = *reinterpret_cast<const bf8 *>(xr[i] + k * 32);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (k0 + u < a.KT)
+#pragma unroll
+        for (int i = 0; i < MT; ++i)
+#pragma unroll
+          for (int j = 0; j < NT; ++j)
+            acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[u][j], x[u][i], acc[i][j], 0, 0, 0);
+  }
+  const int N = a.NTt * 16, Yw = a.heads * N;
+#pragma unroll
+  for (int i = 0; i < MT; ++i) {
+    const int m = m0 + i * 16 + l15;
+    if (m >= a.T) continue;
+    float sc = 1.f;
+    if (a.gate) sc = __fdiv_rn(1.0f, 1.0f + expf(-bf2f(a.gate[(size_t)m * a.ldg + h])));
+#pragma unroll
+    for (int j = 0; j < NT; ++j) {
+      if (nt0 + j >= a.NTt) continue;
+      const int n = h * N + (nt0 + j) * 16 + 4 * g;
+      const f4 v = acc[i][j];
+      const uint2 o = make_uint2(f2bf(v[0] * sc) | ((uint32_t)f2bf(v[1] * sc) << 16),
+                                 f2bf(v[2] * sc) | ((uint32_t)f2bf(v[3] * sc) << 16));
+      *reinterpret_cast<uint2 *>(a.Y + (a.packed ? act_packed_off(m, n, Yw) : (size_t)m * Yw + n)) = o;
+    }
+  }
+}
+
+template <int MT, int NT, int WM>
+__global__ __launch_bounds__(256) void latent_prep_kernel(const PagedToken *__restrict__ tok,
+                                                          HgDev a, int nprod, LatentStore st) {
+  if ((int)blockIdx.x < nprod) {
+    head_gemm_block<MT, NT, WM>(a, blockIdx.x);
+    return;
+  }
+  const int t = (blockIdx.x - nprod) * 4 + (threadIdx.x >> 6);
+  if (t >= a.T) return;
+  latent_store_token(tok[t], (const uint16_t *)st.d + (size_t)t * st.ldd, st.w,
+                     (uint16_t *)st.cache, st.rank, st.n, st.eps);
+}
+
+static hipError_t run_prep(const PagedToken *tok, const LatentStore &st, const HeadGemm &hg,
+                           hipStream_t s) {
+  if (hg.T <= 0) return hipSuccess;
+  if (hg.K % 32 || hg.N % 32 || hg.ldx % 8) return hipErrorInvalidValue;
+  HgDev a;
+  a.X = (const uint16_t *)hg.X, a.W = (const uint16_t *)hg.W, a.gate = (const uint16_t *)hg.gate;
+  a.Y = (uint16_t *)hg.Y;
+  a.T = hg.T, a.heads = hg.heads, a.KT = hg.K / 32, a.NTt = hg.N / 16, a.ldx = hg.ldx;
+  a.ldg = hg.ldg, a.packed = hg.packed ? 1 : 0;
+  const int nst = st.cache ? (hg.T + 3) / 4 : 0;
+#define FFMI_PREP(MT, NT, WM)                                                                   \
+  do {                                                                                          \
+    a.gx = (a.NTt + (4 / WM) * NT - 1) / ((4 / WM) * NT);                                       \
+    a.gz = (hg.T + WM * MT * 16 - 1) / (WM * MT * 16);                                          \
+    const int np = a.gx * a.heads * a.gz;                                                       \
+    hipLaunchKernelGGL((latent_prep_kernel<MT, NT, WM>), dim3(np + nst), dim3(256), 0, s, tok, a, \
+                       np, st);                                                                 \
+  } while (0)
+  if (hg.T <= 16) FFMI_PREP(1, 1, 1);
+  else if (hg.T <= 32) FFMI_PREP(2, 1, 1);
+  else if (hg.T <= 128) FFMI_PREP(2, 2, 1);
+  else FFMI_PREP(4, 4, 2);
+#undef FFMI_PREP
+  return hipGetLastError();
+}
+hipError_t launch_latent_prep(const char *blob, int off_tokens, const LatentStore &st,
+                              const HeadGemm &hg, hipStream_t s) {
+  return run_prep(reinterpret_cast<const PagedToken *>(blob + off_tokens), st, hg, s);
+}
+hipError_t launch_head_gemm(const HeadGemm &hg, hipStream_t s) {
+  return run_prep(nullptr, LatentStore(), hg, s);
+}
+
+// fp32: W_h as [K][N] row-major, one workgroup per (token, head)
+__global__ __launch_bounds__(256) void head_gemm_f32_kernel(const float *__restrict__ X,
+                                                            const float *__restrict__ W,
+                                                            const float *__restrict__ gate,
+                                                            float *__restrict__ Y, int heads, int K,
+                                                            int N, int ldx, int ldg) {
+  const int t = blockIdx.x, h = blockIdx.y;
+  const float *x = X + (size_t)t * ldx + (size_t)h * K, *w = W + (size_t)h * K * N;
+  const float sc =
+      gate ? __fdiv_rn(1.0f, 1.0f + expf(-gate[(size_t)t * ldg + h])) : 1.0f;
+  for (int n = threadIdx.x; n < N; n += 256) {
+    float acc = 0.f;
+    for (int k = 0; k < K; ++k) acc = fmaf(x[k], w[(size_t)k * N + n], acc);
+    Y[((size_t)t * heads + h) * N + n] = acc * sc;
+  }
+}
+hipError_t launch_head_gemm_f32(const HeadGemm &hg, hipStream_t s) {
+  if (hg.T <= 0) return hipSuccess;
+  hipLaunchKernelGGL(head_gemm_f32_kernel, dim3(hg.T, hg.heads), dim3(256), 0, s,
+                     (const float *)hg.X, (const float *)hg.W, (const float *)hg.gate,
+                     (float *)hg.Y, hg.heads, hg.K, hg.N, hg.ldx, hg.ldg);
+  return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// attention over the pages, MFMA form
+// ---------------------------------------------------------------------------
+// One workgroup: up to RT * 16 rows against a range of 64-token pages.  Scores
+// S^T = C . Q'^T (lane: 4 keys of one row), outputs O^T = C^T . P^T with C^T
+// read from the row-major page in LDS by the transposing LDS load; the k order
+// of the second product is the key order the scores already have in the
+// lanes (16-lane group g: keys 4g..4g+3 and 16+4g..).
+//   scores:  RT == 4: waves 2 (row pairs) x 2 (key halves); RT <= 2: each wave
+//            one 16-key tile, all rows
+//   outputs: each wave a quarter of the latent's columns, all rows
+// Softmax state in fp32, base-2 exponents; weights meet the second product in
+// bf16, the sums take them unrounded.
+typedef short s4 __attribute__((ext_vector_type(4)));
+typedef short s8 __attribute__((ext_vector_type(8)));
+typedef uint32_t u4 __attribute__((ext_vector_type(4)));
+constexpr int kRankPad = 8;  // LDS row padding (elements)
+
+template <int RC, int RT>
+__global__ __launch_bounds__(256, 1) void latent_attn_kernel(
+    const char *__restrict__ blob, int off_blocks, const uint16_t *__restrict__ Q,
+    const uint16_t *__restrict__ cache, uint16_t *__restrict__ O, float *__restrict__ slabs,
+    float *__restrict__ ml, int heads, float scale_log2) {
+  constexpr int R = RC * 64, KS = RC * 2, DT = RC, LDC = R + kRankPad;
+  constexpr int SR = RT == 4 ? 2 : RT;      // row tiles of a wave's scores
+  constexpr int KW = RT == 4 ? 2 : 1;       // key tiles of a wave's scores
+  constexpr int NK = 4 / KW;                // waves over the keys
+  constexpr int CPT = 64 * R / 8 / 256;     // 16-B page chunks per thread
+  constexpr int LDP = kPageTokens + 8;
+  __shared__ __attribute__((aligned(16))) uint16_t sC[2][64 * LDC];
+  __shared__ __attribute__((aligned(16))) uint16_t sP[RT * 16 * LDP];
+  __shared__ float sM[NK][RT * 16], sL[NK][RT * 16];
+  const LatentBlock bk = reinterpret_cast<const LatentBlock *>(blob + off_blocks)[blockIdx.x];
+  if (bk.nrows <= 0) return;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, l15 = lane & 15;
+  const int wk = RT == 4 ? (wave & 1) : wave, wr = RT == 4 ? (wave >> 1) : 0;
+  const int32_t *table = reinterpret_cast<const int32_t *>(blob) + bk.table;
+
+  // the next page: through registers, or (R == 512: a row is one 1 KiB wave
+  // access) straight into LDS, where 64 more registers would not fit
+  constexpr bool DMA = R == 512;
+  auto dma = [&](int tile, int buf) {
+    const uint16_t *page = cache + (size_t)table[tile] * (64 * R);
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const int row = wave * 16 + i;
+      __builtin_amdgcn_global_load_lds(
+          (const __attribute__((address_space(1))) void *)(page + (size_t)row * R + lane * 8),
+          (__attribute__((address_space(3))) void *)(&sC[buf][row * LDC]), 16, 0, 0);
+    }
+  };
+  u4 pre[DMA ? 1 : CPT];
+  auto fetch = [&](int tile) {
+    const uint16_t *page = cache + (size_t)table[tile] * (64 * R);
+#pragma unroll
+    for (int i = 0; i < (DMA ? 0 : CPT); ++i) pre[i] = *reinterpret_cast<const u4 *>(page + (tid + i * 256) * 8);
+  };
+  auto stage = [&](int buf) {
+#pragma unroll
+    for (int i = 0; i < (DMA ? 0 : CPT); ++i) {
+      const int c = tid + i * 256;
+      *reinterpret_cast<u4 *>(&sC[buf][(c / (R / 8)) * LDC + (c % (R / 8)) * 8]) = pre[i];
+    }
+  };
+  if constexpr (DMA) dma(bk.tile0, 0);
+  else fetch(bk.tile0);
+  // this wave's rows of Q' as B operands (rows past the block re-read its last)
+  bf8 q[SR][KS];
+  int qpos[SR];
+#pragma unroll
+  for (int i = 0; i < SR; ++i) {
+    const int r = min((wr * SR + i) * 16 + l15, bk.nrows - 1);
+    const uint16_t *qr = Q + (size_t)(bk.row0 + r) * R + 8 * g;
+#pragma unroll
+    for (int k = 0; k < KS; ++k) q[i][k] = *reinterpret_cast<const bf8 *>(qr + k * 32);
+    qpos[i] = bk.pos0 + (bk.row0 + r - bk.seg_row) / heads;
+  }
+  f4 acc[RT][DT];
+#pragma unroll
+  for (int i = 0; i < RT; ++i)
+#pragma unroll
+    for (int d = 0; d < DT; ++d) acc[i][d] = f4{0.f, 0.f, 0.f, 0.f};
+  float m[RT], l[SR];
+#pragma unroll
+  for (int i = 0; i < RT; ++i) m[i] = -1e30f;
+#pragma unroll
+  for (int i = 0; i < SR; ++i) l[i] = 0.f;
+  if constexpr (DMA) {
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  } else {
+    stage(0);
+    if (bk.ntiles > 1) fetch(bk.tile0 + 1);
+  }
+  __syncthreads();
+  for (int it = 0; it < bk.ntiles; ++it) {
+    if constexpr (DMA)  // (its buffer was last read before the previous round's last barrier)
+      if (it + 1 < bk.ntiles) dma(bk.tile0 + it + 1, (it + 1) & 1);
+    const uint16_t *C = sC[it & 1];
+    f4 s[SR][KW];
+#pragma unroll
+    for (int i = 0; i < SR; ++i)
+#pragma unroll
+      for (int k = 0; k < KW; ++k) s[i][k] = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      bf8 c[KW];
+#pragma unroll
+      for (int k = 0; k < KW; ++k)
+        c[k] = *reinterpret_cast<const bf8 *>(&C[((wk * KW + k) * 16 + l15) * LDC + ks * 32 + 8 * g]);
+#pragma unroll
+      for (int k = 0; k < KW; ++k)
+#pragma unroll
+        for (int i = 0; i < SR; ++i)
+          s[i][k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c[k], q[i][ks], s[i][k], 0, 0, 0);
+    }
+    // scale, mask, this wave's maximum of every row
+    const int key0 = (bk.tile0 + it) * 64 + wk * KW * 16 + 4 * g;
+#pragma unroll
+    for (int i = 0; i < SR; ++i) {
+      float mx = -1e30f;
+#pragma unroll
+      for (int k = 0; k < KW; ++k)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float v = key0 + k * 16 + e <= qpos[i] ? s[i][k][e] * scale_log2 : -INFINITY;
+          s[i][k][e] = v;
+          mx = fmaxf(mx, v);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16));
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      if (g == 0) sM[wk][(wr * SR + i) * 16 + l15] = mx;
+    }
+    __syncthreads();
+    float alpha[RT];
+    bool moved = false;
+#pragma unroll
+    for (int i = 0; i < RT; ++i) {
+      float mn = m[i];
+#pragma unroll
+      for (int k = 0; k < NK; ++k) mn = fmaxf(mn, sM[k][i * 16 + l15]);
+      alpha[i] = __builtin_amdgcn_exp2f(m[i] - mn);
+      moved |= mn != m[i];
+      m[i] = mn;
+    }
+#pragma unroll
+    for (int i = 0; i < SR; ++i) {
+      float mi = m[i], ai = alpha[i];
+      if (RT == 4 && wr) mi = m[RT == 4 ? 2 + i : i], ai = alpha[RT == 4 ? 2 + i : i];
+      float sum = 0.f;
+#pragma unroll
+      for (int k = 0; k < KW; ++k) {
+        float p[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          p[e] = __builtin_amdgcn_exp2f(s[i][k][e] - mi);
+          sum += p[e];
+        }
+        *reinterpret_cast<uint2 *>(&sP[((wr * SR + i) * 16 + l15) * LDP + (wk * KW + k) * 16 + 4 * g]) =
+            make_uint2(f2bf(p[0]) | ((uint32_t)f2bf(p[1]) << 16),
+                       f2bf(p[2]) | ((uint32_t)f2bf(p[3]) << 16));
+      }
+      l[i] = l[i] * ai + sum;
+    }
+    if (!DMA && it + 1 < bk.ntiles) {
+      stage((it + 1) & 1);  // (last read by the outputs of tile it - 1)
+      if (it + 2 < bk.ntiles) fetch(bk.tile0 + it + 2);
+    }
+    __syncthreads();
+    if (__any(moved))
+#pragma unroll
+      for (int i = 0; i < RT; ++i)
+#pragma unroll
+        for (int d = 0; d < DT; ++d) acc[i][d] *= alpha[i];
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb) {
+      s8 p[RT];
+#pragma unroll
+      for (int i = 0; i < RT; ++i) {
+        const uint16_t *pr = &sP[(i * 16 + l15) * LDP + kb * 32 + 4 * g];
+        const s4 lo = *reinterpret_cast<const s4 *>(pr), hi = *reinterpret_cast<const s4 *>(pr + 16);
+        p[i] = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
+      }
+#pragma unroll
+      for (int d = 0; d < DT; ++d) {
+        const uint16_t *cr =
+            &C[(kb * 32 + 4 * g + (l15 >> 2)) * LDC + (wave * DT + d) * 16 + 4 * (l15 & 3)];
+        const s4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (__attribute__((address_space(3))) s4 *)(cr));
+        const s4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (__attribute__((address_space(3))) s4 *)(cr + 16 * LDC));
+        const bf8 a = __builtin_bit_cast(
+            bf8, __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+#pragma unroll
+        for (int i = 0; i < RT; ++i)
+          acc[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, __builtin_bit_cast(bf8, p[i]),
+                                                              acc[i][d], 0, 0, 0);
+      }
+    }
+    if constexpr (DMA) {
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      __syncthreads();
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < SR; ++i) {
+    float v = l[i];
+    v += __shfl_xor(v, 16);
+    v += __shfl_xor(v, 32);
+    if (g == 0) sL[wk][(wr * SR + i) * 16 + l15] = v;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < RT; ++i) {
+    float sum = sL[0][i * 16 + l15];
+#pragma unroll
+    for (int k = 1; k < NK; ++k) sum += sL[k][i * 16 + l15];
+    const int r = i * 16 + l15;
+    if (r >= bk.nrows) continue;
+    if (bk.slot >= 0) {
+      const size_t pr = (size_t)bk.slot * (RT * 16) + r;
+#pragma unroll
+      for (int d = 0; d < DT; ++d)
+        *reinterpret_cast<f4 *>(slabs + pr * R + (wave * DT + d) * 16 + 4 * g) = acc[i][d];
+      if (wave == 0 && g == 0) ml[pr * 2] = m[i], ml[pr * 2 + 1] = sum;
+    } else {
+      const float inv = __fdiv_rn(1.0f, sum);
+      uint16_t *o = O + (size_t)(bk.row0 + r) * R + wave * DT * 16 + 4 * g;
+#pragma unroll
+      for (int d = 0; d < DT; ++d) {
+        const f4 v = acc[i][d] * inv;
+        *reinterpret_cast<uint2 *>(o + d * 16) =
+            make_uint2(f2bf(v[0]) | ((uint32_t)f2bf(v[1]) << 16),
+                       f2bf(v[2]) | ((uint32_t)f2bf(v[3]) << 16));
+      }
+    }
+  }
+}
+
+// partials of split blocks, in slot order
+template <int RC>
+__global__ __launch_bounds__(RC * 16) void latent_merge_kernel(
+    const char *__restrict__ blob, int off_merges, const float *__restrict__ slabs,
+    const float *__restrict__ ml, uint16_t *__restrict__ O, int block_rows) {
+  constexpr int R = RC * 64;
+  const LatentMerge mg = reinterpret_cast<const LatentMerge *>(blob + off_merges)[blockIdx.x];
+  const int r = blockIdx.y;
+  if (r >= mg.nrows) return;
+  float M = -1e30f;
+  for (int i = 0; i < mg.nslots; ++i)
+    M = fmaxf(M, ml[((size_t)(mg.slot0 + i) * block_rows + r) * 2]);
+  f4 acc = f4{0.f, 0.f, 0.f, 0.f};
+  float sum = 0.f;
+#pragma unroll 4
+  for (int i = 0; i < mg.nslots; ++i) {
+    const size_t pr = (size_t)(mg.slot0 + i) * block_rows + r;
+    const float w = __builtin_amdgcn_exp2f(ml[pr * 2] - M);
+    sum = fmaf(w, ml[pr * 2 + 1], sum);
+    const f4 v = *reinterpret_cast<const f4 *>(slabs + pr * R + threadIdx.x * 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) acc[e] = fmaf(w, v[e], acc[e]);
+  }
+  const float inv = __fdiv_rn(1.0f, sum);
+  *reinterpret_cast<uint2 *>(O + (size_t)(mg.row0 + r) * R + threadIdx.x * 4) =
+      make_uint2(f2bf(acc[0] * inv) | ((uint32_t)f2bf(acc[1] * inv) << 16),
+                 f2bf(acc[2] * inv) | ((uint32_t)f2bf(acc[3] * inv) << 16));
+}
+
+bool latent_rank_supported(int rank) {
+  const int rc = rank / 64;
+  return rank % 64 == 0 && (rc == 1 || rc == 2 || rc == 3 || rc == 4 || rc == 6 || rc == 8);
+}
+
+hipError_t launch_latent_attention(const char *blob, const PagedLists &pl, const uint16_t *q,
+                                   const uint16_t *cache, uint16_t *o, float *slabs, float *ml,
+                                   int rank, float scale, hipStream_t s) {
+  if (pl.num_blocks <= 0) return hipSuccess;
+  const float sl = scale * 1.4426950408889634f;
+#define FFMI_LA2(RC, RT)                                                                        \
+  hipLaunchKernelGGL((latent_attn_kernel<RC, RT>), dim3(pl.num_blocks), dim3(256), 0, s, blob,  \
+                     pl.off_blocks, q, cache, o, slabs, ml, pl.heads, sl)
+#define FFMI_LA(RC)                                                                             \
+  case RC:                                                                                      \
+    if (pl.row_tiles == 1) FFMI_LA2(RC, 1);                                                     \
+    else if (pl.row_tiles == 2) FFMI_LA2(RC, 2);                                                \
+    else if (pl.row_tiles == 4) FFMI_LA2(RC, 4);                                                \
+    else return hipErrorInvalidValue;                                                           \
+    if (pl.num_merges > 0)                                                                      \
+      hipLaunchKernelGGL((latent_merge_kernel<RC>), dim3(pl.num_merges, pl.row_tiles * 16),     \
+                         dim3(RC * 16), 0, s, blob, pl.off_merges, slabs, ml, o,                \
+                         pl.row_tiles * 16);                                                    \
+    break
+  if (rank % 64) return hipErrorInvalidValue;
+  switch (rank / 64) {
+    FFMI_LA(1);
+    FFMI_LA(2);
+    FFMI_LA(3);
+    FFMI_LA(4);
+    FFMI_LA(6);
+    FFMI_LA(8);
+    default: return hipErrorInvalidValue;
+  }
+#undef FFMI_LA
+#undef FFMI_LA2
+  return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// attention, one workgroup per row (fp32, and bf16 ranks without an MFMA form)
+// ---------------------------------------------------------------------------
+constexpr int kRowsMaxRank = 2048;
+template <class E>
+__global__ __launch_bounds__(256) void latent_rows_kernel(const char *__restrict__ blob,
+                                                          int off_blocks, const E *__restrict__ Q,
+                                                          const E *__restrict__ cache,
+                                                          E *__restrict__ O, int heads, int rank,
+                                                          float scale) {
+  __shared__ float sq[kRowsMaxRank], sp[256], red[4];
+  __shared__ int srow[256];
+  const LatentBlock bk = reinterpret_cast<const LatentBlock *>(blob + off_blocks)[blockIdx.x];
+  const int r = blockIdx.y, tid = threadIdx.x;
+  if (r >= bk.nrows) return;
+  const int32_t *table = reinterpret_cast<const int32_t *>(blob) + bk.table;
+  const size_t row = (size_t)bk.row0 + r;
+  const int n = bk.pos0 + (int)(row - bk.seg_row) / heads + 1;  // visible positions
+  for (int i = tid; i < rank; i += 256) sq[i] = ld_elem(Q + row * rank + i);
+  float acc[kRowsMaxRank / 256];
+#pragma unroll
+  for (int i = 0; i < kRowsMaxRank / 256; ++i) acc[i] = 0.f;
+  float m = -1e30f, l = 0.f;
+  for (int j0 = 0; j0 < n; j0 += 256) {
+    __syncthreads();
+    const int j = j0 + tid;
+    float sv = -INFINITY;
+    if (j < n) {
+      const int cr = table[j >> 6] * kPageTokens + (j & 63);
+      srow[tid] = cr;
+      const E *c = cache + (size_t)cr * rank;
+      float a = 0.f;
+      for (int i = 0; i < rank; ++i) a = fmaf(sq[i], ld_elem(c + i), a);
+      sv = a * scale;
+    }
+    float mx = sv;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
+    if ((tid & 63) == 0) red[tid >> 6] = mx;
+    __syncthreads();
+    const float mn = fmaxf(m, fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])));
+    const float p = j < n ? expf(sv - mn) : 0.f;
+    sp[tid] = p;
+    float sum = p;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) sum += __shfl_xor(sum, o);
+    __syncthreads();
+    if ((tid & 63) == 0) red[tid >> 6] = sum;
+    __syncthreads();
+    const float al = expf(m - mn);
+    l = l * al + (red[0] + red[1] + red[2] + red[3]);
+    m = mn;
+    const int cnt = min(256, n - j0);
+#pragma unroll
+    for (int i = 0; i < kRowsMaxRank / 256; ++i) {
+      const int d = tid + i * 256;
+      if (d >= rank) break;
+      float a = acc[i] * al;
+      for (int k = 0; k < cnt; ++k) a = fmaf(sp[k], ld_elem(cache + (size_t)srow[k] * rank + d), a);
+      acc[i] = a;
+    }
+  }
+  const float inv = __fdiv_rn(1.0f, l);
+#pragma unroll
+  for (int i = 0; i < kRowsMaxRank / 256; ++i) {
+    const int d = tid + i * 256;
+    if (d < rank) st_elem(O + row * rank + d, acc[i] * inv);
+  }
+}
+
+hipError_t launch_latent_attention_rows(const char *blob, const PagedLists &pl, const void *q,
+                                        const void *cache, void *o, int rank, float scale,
+                                        bool bf16, hipStream_t s) {
+  if (pl.num_blocks <= 0) return hipSuccess;
+  if (rank > kRowsMaxRank || pl.num_merges > 0) return hipErrorInvalidValue;
+  const dim3 grid(pl.num_blocks, pl.row_tiles * 16);
+  if (bf16)
+    hipLaunchKernelGGL(latent_rows_kernel<uint16_t>, grid, dim3(256), 0, s, blob, pl.off_blocks,
+                       (const uint16_t *)q, (const uint16_t *)cache, (uint16_t *)o, pl.heads, rank,
+                       scale);
+  else
+    hipLaunchKernelGGL(latent_rows_kernel<float>, grid, dim3(256), 0, s, blob, pl.off_blocks,
+                       (const float *)q, (const float *)cache, (float *)o, pl.heads, rank, scale);
+  return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// loading
+// ---------------------------------------------------------------------------
+__device__ __forceinline__ uint16_t pack_elem(const uint16_t *src, int ld, const PackSpec &p, int n,
+                                              int k) {
+  const int hn = n / p.np, jn = n % p.np, hk = k / p.kp, jk = k % p.kp;
+  if (hn >= p.rows || jn >= p.nb || hk >= p.cols || jk >= p.kb) return 0;
+  if (p.transpose) return src[((size_t)hn * p.kb + jk) * ld + jn];
+  return src[(size_t)(hn * p.nb + jn) * ld + hk * p.kb + jk];
+}
+__global__ void pack_bf16_kernel(const uint16_t *__restrict__ src, int ld, PackSpec p,
+                                 uint16_t *__restrict__ dst, int NT, int KT, size_t ts, size_t ks) {
+  const long gid = blockIdx.x * (long)blockDim.x + threadIdx.x;
+  if (gid >= (long)NT * KT * 64) return;
+  const int lane = (int)(gid & 63), kt = (int)((gid >> 6) % KT), nt = (int)((gid >> 6) / KT);
+  const int n = nt * 16 + (lane & 15), k = kt * 32 + 8 * (lane >> 4);
+  uint32_t v[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    v[j] = pack_elem(src, ld, p, n, k + 2 * j) |
+           ((uint32_t)pack_elem(src, ld, p, n, k + 2 * j + 1) << 16);
+  *reinterpret_cast<uint4 *>(dst + nt * ts + kt * ks + lane * 8) = make_uint4(v[0], v[1], v[2], v[3]);
+}
+hipError_t launch_pack_bf16(const uint16_t *src, int ld, const PackSpec &p, uint16_t *dst,
+                            int tile_offset, int pitch, bool perhead, hipStream_t s) {
+  const int N = p.rows * p.np, K = p.cols * p.kp;
+  if (N % 16 || K % 32) return hipErrorInvalidValue;
+  const int NT = N / 16, KT = K / 32;
+  const size_t ts = perhead ? (size_t)KT * 512 : w_tile_stride(KT);
+  const size_t ks = perhead ? 512 : w_k_stride(pitch);
+  hipLaunchKernelGGL(pack_bf16_kernel, dim3((unsigned)(((long)NT * KT * 64 + 255) / 256)),
+                     dim3(256), 0, s, src, ld, p, dst + tile_offset * ts, NT, KT, ts, ks);
+  return hipGetLastError();
+}
+__global__ void pack_f32_kernel(const uint16_t *__restrict__ src, int ld, PackSpec p,
+                                float *__restrict__ dst, int N, int K) {
+  const long i = blockIdx.x * (long)blockDim.x + threadIdx.x;
+  if (i >= (long)N * K) return;
+  dst[i] = bf2f(pack_elem(src, ld, p, (int)(i / K), (int)(i % K)));
+}
+hipError_t launch_pack_f32(const uint16_t *src, int ld, const PackSpec &p, float *dst,
+                           hipStream_t s) {
+  const int N = p.rows * p.np, K = p.cols * p.kp;
+  hipLaunchKernelGGL(pack_f32_kernel, dim3((unsigned)(((long)N * K + 255) / 256)), dim3(256), 0, s,
+                     src, ld, p, dst, N, K);
+  return hipGetLastError();
+}
+
+__global__ void pack_act_bf16_kernel(const uint16_t *__restrict__ X, uint16_t *__restrict__ Xp,
+                                     int T, int K) {
+  const int kt = blockIdx.x, mt = blockIdx.y, l = threadIdx.x, r = mt * 16 + (l & 15);
+  uint4 v = make_uint4(0, 0, 0, 0);
+  if (r < T) v = *reinterpret_cast<const uint4 *>(X + (size_t)r * K + kt * 32 + 8 * (l >> 4));
+  *reinterpret_cast<uint4 *>(Xp + act_packed_off(r, kt * 32 + 8 * (l >> 4), K)) = v;
+}
+hipError_t launch_pack_act_bf16(const uint16_t *X, uint16_t *Xp, int T, int K, hipStream_t s) {
+  if (T <= 0 || K % 32) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(pack_act_bf16_kernel, dim3(K / 32, (T + 15) / 16), dim3(64), 0, s, X, Xp, T, K);
+  return hipGetLastError();
+}
+
+}  // namespace ffmi

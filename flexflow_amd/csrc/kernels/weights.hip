@@ -16,6 +16,9 @@
 // contiguous band of k-row kt instead of ~230 streams 128 KiB apart: the
 // T = 168 gate/up loop went 57 -> 44 us in scripts/probe/xl2_probe.hip (the
 // old tile-major order, FFMI_W_TILE_MAJOR=1, stays for A/B runs).
+#include <algorithm>
+#include <type_traits>
+
 #include "../ffmi_internal.h"
 
 namespace ffmi {
@@ -31,6 +34,9 @@ __device__ __forceinline__ uint64_t splitmix64(uint64_t z) {
 // mod rows (the token-chain init's tied lm_head, oracle.h orc_gen_weight_rows)
 // (OUT = float: the full-precision model's fp32 weights, the same values
 // before the fp16 rounding -- the oracle's fp32 mode)
+struct Bf16Bits {  // (OUT = Bf16Bits: rounded to bf16)
+  uint16_t v;
+};
 template <class OUT>
 __global__ void fill_weight_kernel(OUT *dst, size_t n, uint64_t key, float center, float amp,
                                    int cols, uint64_t pa, uint64_t pb) {
@@ -44,6 +50,7 @@ __global__ void fill_weight_kernel(OUT *dst, size_t n, uint64_t key, float cente
     float t = __fsub_rn(__fmul_rn(2.0f, u), 1.0f);
     float w = __fadd_rn(center, __fmul_rn(t, amp));
     if constexpr (sizeof(OUT) == 4) dst[i] = w;
+    else if constexpr (std::is_same_v<OUT, Bf16Bits>) dst[i].v = f2bf(w);
     else dst[i] = __half_as_ushort(__float2half_rn(w));
   }
 }
@@ -73,6 +80,15 @@ hipError_t launch_fill_weight_f32(float *dst, size_t n, uint64_t key, int kind, 
   if (blocks > 65536) blocks = 65536;
   hipLaunchKernelGGL(fill_weight_kernel<float>, dim3((unsigned)blocks), dim3(256), 0, s, dst, n,
                      key, kind == 1 ? 1.0f : 0.0f, weight_amp(kind) * scale, cols, pa, pb);
+  return hipGetLastError();
+}
+
+hipError_t launch_fill_weight_bf16(uint16_t *dst, size_t n, uint64_t key, int kind, hipStream_t s) {
+  if (n == 0) return hipSuccess;
+  const size_t blocks = std::min<size_t>((n + 255) / 256, 65536);
+  hipLaunchKernelGGL(fill_weight_kernel<Bf16Bits>, dim3((unsigned)blocks), dim3(256), 0, s,
+                     reinterpret_cast<Bf16Bits *>(dst), n, key, kind == 1 ? 1.0f : 0.0f,
+                     weight_amp(kind), 0, 1, 0);
   return hipGetLastError();
 }
 

@@ -7,17 +7,15 @@
 
 #include "request_manager.h"
 
-struct ffmi_rm {
-  ffmi::RequestManager rm;
-};
-
-extern "C" ffmi_status ffmi_model_create(const ffmi_llama_config *cfg, const ffmi_model_opts *o,
-                                         ffmi_model **out) {
-  if (o && o->full_precision) return ffmi::create_llama_f32(cfg, o, out);
-  return ffmi::create_llama_gpu(cfg, o, out);
+extern "C" ffmi_status ffmi_model_create_json(const char *config_json, const ffmi_model_opts *o,
+                                              ffmi_model **out) {
+  FFMI_CHECK(config_json && o && out, FFMI_ERR_INVALID);
+  return ffmi::create_model_from_json(config_json, o, out);
 }
 
 extern "C" void ffmi_model_destroy(ffmi_model *m) { delete m; }
+
+extern "C" int ffmi_model_vocab_size(ffmi_model *m) { return m ? m->vocab_size() : -1; }
 
 extern "C" ffmi_status ffmi_model_set_profiling(ffmi_model *m, int level) {
   if (!m || level < 0 || level > 2) return FFMI_ERR_INVALID;
@@ -125,16 +123,6 @@ extern "C" ffmi_status ffmi_rm_set_ssm_exchange(ffmi_rm *rm, int nranks, int ran
   return FFMI_OK;
 }
 
-static int comm_allgather_cb(void *ctx, const void *mine, size_t bytes, void *all) {
-  return ffmi_comm_allgather(static_cast<ffmi_comm *>(ctx), mine, bytes, all) == FFMI_OK ? 0 : 1;
-}
-
-extern "C" ffmi_status ffmi_rm_set_ssm_exchange_comm(ffmi_rm *rm, ffmi_comm *comm) {
-  if (!rm || !comm) return FFMI_ERR_INVALID;
-  rm->rm.set_ssm_exchange(ffmi::comm_size(comm), ffmi::comm_rank(comm), comm_allgather_cb, comm);
-  return FFMI_OK;
-}
-
 extern "C" ffmi_status ffmi_rm_register_output_filepath(ffmi_rm *rm, const char *path) {
   if (!rm) return FFMI_ERR_INVALID;
   rm->rm.register_output_filepath(path ? path : "");
@@ -170,6 +158,19 @@ extern "C" ffmi_status ffmi_rm_serve_incr_decoding(ffmi_rm *rm, ffmi_model *llm)
 extern "C" ffmi_status ffmi_rm_serve_spec_infer(ffmi_rm *rm, ffmi_model *llm) {
   if (!rm || !llm || llm->mode != FFMI_MODEL_TREE) return FFMI_ERR_INVALID;
   return rm->rm.serve_spec_infer(llm);
+}
+
+extern "C" ffmi_status ffmi_rm_replay_step(ffmi_rm *rm, ffmi_model *llm,
+                                           const ffmi_replay_entry *entries, int num_entries,
+                                           float *logits, long cap_rows) {
+  if (!rm || !llm || llm->mode != FFMI_MODEL_INC || num_entries < 0 || (num_entries && !entries))
+    return FFMI_ERR_INVALID;
+  return rm->rm.replay_step(llm, entries, num_entries, logits, cap_rows);
+}
+
+extern "C" ffmi_status ffmi_rm_replay_end(ffmi_rm *rm, ffmi_model *llm, int64_t id) {
+  if (!rm || !llm) return FFMI_ERR_INVALID;
+  return rm->rm.replay_end(llm, id);
 }
 
 extern "C" int ffmi_rm_get_output(ffmi_rm *rm, int64_t guid, int *tokens, int cap) {

@@ -68,7 +68,28 @@ struct HashModel : public ffmi_model {
     return FFMI_OK;
   }
 
-  int slot_of(int r, int s) const { return r * slots + s; }
+  // a paged cache (set_pool): `cache` is then [pages][page tokens]
+  PagePool pool;
+  bool paged = false;
+  PagePool *page_pool() override { return paged ? &pool : nullptr; }
+  int vocab_size() const override { return vocab; }
+  int slot_of(int r, int s) const {
+    if (!paged) return r * slots + s;
+    return pool.table(r)[s / pool.page_tokens()] * pool.page_tokens() + s % pool.page_tokens();
+  }
+  // the pages an INC batch's tokens need, as a GPU model's step takes them
+  bool take_pages(const BatchConfig &bc) {
+    for (int t = 0; t < bc.num_tokens; ++t) {
+      const int r = bc.tokensInfo[t].request_index, d = bc.tokensInfo[t].abs_depth_in_request;
+      const int64_t guid = bc.requestsInfo[r].request_guid;
+      if (pool.owner(r) != guid) {
+        pool.release(r);
+        pool.set_owner(r, guid);
+      }
+      if (!pool.ensure(r, d + 1)) return false;
+    }
+    return true;
+  }
 
   // returns context hash for each token; -1 entries poison the hash
   void contexts(const PackedStep &ps, std::vector<uint64_t> *hs) {
@@ -107,11 +128,21 @@ struct HashModel : public ffmi_model {
     for (int t = 0; t < bc.num_tokens; ++t)
       if (bc.tokensInfo[t].token_id < 0 || bc.tokensInfo[t].token_id >= vocab)
         return FFMI_ERR_INVALID;
+    if (paged && !take_pages(bc)) return FFMI_ERR_OOM;
     PackedStep ps;
     pack_inc(bc, max_requests, slots, &ps);
     std::vector<uint64_t> hs;
     contexts(ps, &hs);
     for (size_t t = 0; t < hs.size(); ++t) ir->token_ids[t] = next_token(hs[t]);
+    return FFMI_OK;
+  }
+  // "logits": 1 at the next token
+  ffmi_status run_inc_logits(const BatchConfig &bc, const int *rows, int n, float *out) override {
+    std::unique_ptr<InferenceResult> r(new InferenceResult());
+    const ffmi_status st = run_inc(bc, r.get());
+    if (st != FFMI_OK) return st;
+    std::fill(out, out + (size_t)n * vocab, 0.f);
+    for (int i = 0; i < n; ++i) out[(size_t)i * vocab + r->token_ids[rows[i]]] = 1.f;
     return FFMI_OK;
   }
   ffmi_status run_tree(const TreeVerifyBatchConfig &bc, InferenceResult *ir) override {
@@ -196,6 +227,20 @@ extern "C" ffmi_status ffmi_test_hash_model_create(int vocab, int mode, int max_
   if (!out) return FFMI_ERR_INVALID;
   return ffmi::create_hash_model(vocab, mode, max_requests, max_seq, max_tree, salt,
                                  disagree_pct, out);
+}
+
+extern "C" ffmi_status ffmi_test_hash_model_set_pool(ffmi_model *m, int pages, int page_tokens) {
+  ffmi::HashModel *h = dynamic_cast<ffmi::HashModel *>(m);
+  if (!h || pages <= 0 || page_tokens <= 0) return FFMI_ERR_INVALID;
+  h->paged = true;
+  h->pool.init(pages, page_tokens, h->max_requests);
+  h->cache.assign((size_t)pages * page_tokens, -1);
+  return FFMI_OK;
+}
+
+extern "C" int ffmi_test_hash_model_free_pages(ffmi_model *m) {
+  ffmi::HashModel *h = dynamic_cast<ffmi::HashModel *>(m);
+  return h && h->paged ? h->pool.free_pages() : -1;
 }
 
 extern "C" ffmi_status ffmi_test_hash_model_set_capacity(ffmi_model *m, int max_tokens) {

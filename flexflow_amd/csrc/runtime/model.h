@@ -10,6 +10,7 @@
 
 #include "../ffmi_internal.h"
 #include "batch_config.h"
+#include "page_pool.h"
 
 namespace ffmi {
 
@@ -90,6 +91,17 @@ struct ffmi_model {
     (void)ir;
     return FFMI_ERR_UNSUPPORTED;
   }
+  // an INC step whose caller wants the logits of batch tokens rows[0, n):
+  // fp32 [n][vocab] to `out` (host)
+  virtual ffmi_status run_inc_logits(const ffmi::BatchConfig &bc, const int *rows, int n,
+                                     float *out) {
+    (void)bc, (void)rows, (void)n, (void)out;
+    return FFMI_ERR_UNSUPPORTED;
+  }
+  virtual int vocab_size() const { return -1; }
+  // the page pool of a model with a paged cache (null: fixed cache slots per
+  // request); the scheduler admits requests against it
+  virtual ffmi::PagePool *page_pool() { return nullptr; }
   // tokens one step can hold (-1: unknown), checked by serve_spec_infer
   // against the largest batch the scheduler can build for an SSM
   virtual int token_capacity() const { return -1; }
@@ -130,6 +142,15 @@ struct ffmi_model {
 };
 
 namespace ffmi {
+// Model classes by config.json's "architecture" (or HF "architectures"[0]):
+// each family's source file registers its factory (model_registry.cpp).
+class Json;
+typedef ffmi_status (*ModelFactory)(const Json &config, const ffmi_model_opts *o, ffmi_model **out);
+struct ModelRegistrar {
+  ModelRegistrar(const char *architecture, ModelFactory f);
+};
+ffmi_status create_model_from_json(const char *config_json, const ffmi_model_opts *o,
+                                   ffmi_model **out);
 ffmi_status create_llama_gpu(const ffmi_llama_config *cfg, const ffmi_model_opts *o,
                              ffmi_model **out);
 // full precision (--use-full-precision): runtime/llama_f32.cpp

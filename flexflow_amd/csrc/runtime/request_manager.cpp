@@ -226,6 +226,7 @@ BatchConfig RequestManager::prepare_next_batch(const BatchConfig &old_bc,
     if (check_inf_req_completion(old_bc, i)) {
       if (is_eos_token(request.tokens.back())) request.tokens.pop_back();
       complete_request(request);
+      if (pool) pool->release(i);
       continue;
     }
     auto &R = new_bc.requestsInfo[i];
@@ -267,6 +268,10 @@ BatchConfig RequestManager::prepare_next_batch(const BatchConfig &old_bc,
     if (!new_bc.request_completed[i]) continue;
     if (pending_infr_request_queue.empty() || new_bc.num_tokens >= max_tokens_per_batch) continue;
     Request new_request = pending_infr_request_queue.front();
+    // a paged cache: in order, as soon as the request's longest length fits
+    if (pool && !pool->reserve(i, new_request.guid,
+                               std::max(new_request.max_length, (int)new_request.tokens.size())))
+      break;
     pending_infr_request_queue.pop_front();
     auto &R = new_bc.requestsInfo[i];
     R.first_token_depth_in_request = 0;
@@ -1049,6 +1054,12 @@ ffmi_status RequestManager::serve_incr_decoding(ffmi_model *llm) {
   apply_limits();
   stats = Stats();
   const double t0 = now_us();
+  if (!replays.empty()) return FFMI_ERR_INVALID;  // (replayed requests hold slots)
+  pool = llm->page_pool();
+  if (pool) {
+    FFMI_CHECK(max_requests_per_batch <= pool->num_slots(), FFMI_ERR_INVALID);
+    for (int i = 0; i < pool->num_slots(); ++i) pool->release(i);
+  }
   BatchConfig *bc = new BatchConfig();
   InferenceResult *ir = new InferenceResult();
   ffmi_status st = FFMI_OK;
@@ -1071,6 +1082,89 @@ ffmi_status RequestManager::serve_incr_decoding(ffmi_model *llm) {
   delete ir;
   stats.wall_us = now_us() - t0;
   return st;
+}
+
+// One replay step: the entries' tokens in order, cut into batches of at most
+// max_tokens_per_batch; each batch through the model's INC step.
+ffmi_status RequestManager::replay_step(ffmi_model *llm, const ffmi_replay_entry *entries, int n,
+                                        float *logits, long cap_rows) {
+  apply_limits();
+  const int V = llm->vocab_size();
+  FFMI_CHECK(V > 0, FFMI_ERR_UNSUPPORTED);
+  pool = llm->page_pool();
+  if (pool) FFMI_CHECK(max_requests_per_batch <= pool->num_slots(), FFMI_ERR_INVALID);
+  long rows_total = 0;
+  for (int e = 0; e < n; ++e) {
+    FFMI_CHECK(entries[e].num_tokens >= 0 && entries[e].num_want >= 0, FFMI_ERR_INVALID);
+    for (int f = 0; f < e; ++f) FFMI_CHECK(entries[f].id != entries[e].id, FFMI_ERR_INVALID);
+    for (int w = 0; w < entries[e].num_want; ++w) {
+      const int p = entries[e].want[w];
+      FFMI_CHECK(p >= 0 && p < entries[e].num_tokens && (w == 0 || p > entries[e].want[w - 1]),
+                 FFMI_ERR_INVALID);
+    }
+    rows_total += entries[e].num_want;
+  }
+  FFMI_CHECK(rows_total <= cap_rows && (rows_total == 0 || logits), FFMI_ERR_INVALID);
+  // admit
+  for (int e = 0; e < n; ++e) {
+    if (replays.count(entries[e].id)) continue;
+    std::vector<bool> used(max_requests_per_batch, false);
+    for (const auto &kv : replays) used[kv.second.slot] = true;
+    int slot = 0;
+    while (slot < max_requests_per_batch && used[slot]) ++slot;
+    FFMI_CHECK(slot < max_requests_per_batch, FFMI_ERR_INVALID);  // no request slot free
+    if (pool) pool->reserve(slot, entries[e].id, 0);
+    replays[entries[e].id].slot = slot;
+  }
+  const int cap = std::min(max_tokens_per_batch, (int)BatchConfig::MAX_NUM_TOKENS);
+  std::unique_ptr<BatchConfig> bc(new BatchConfig());
+  std::vector<int> rows;
+  long done_rows = 0;
+  int e = 0, at = 0, w = 0;
+  while (e < n) {
+    *bc = BatchConfig();
+    rows.clear();
+    while (e < n && bc->num_tokens < cap) {
+      const ffmi_replay_entry &E = entries[e];
+      Replay &rp = replays[E.id];
+      const int take = std::min(cap - bc->num_tokens, E.num_tokens - at);
+      if (take > 0) {
+        auto &R = bc->requestsInfo[rp.slot];
+        bc->request_completed[rp.slot] = false;
+        R.first_token_depth_in_request = rp.depth;
+        R.first_token_offset_in_batch = bc->num_tokens;
+        R.num_tokens_in_batch = take;
+        R.max_length = max_sequence_length;
+        R.request_guid = E.id;
+        R.prompt_phase = take > 1;
+        for (int j = 0; j < take; ++j) {
+          auto &tk = bc->tokensInfo[bc->num_tokens];
+          tk.request_index = rp.slot;
+          tk.abs_depth_in_request = rp.depth + j;
+          tk.token_id = E.tokens[at + j];
+          if (w < E.num_want && E.want[w] == at + j) rows.push_back(bc->num_tokens), ++w;
+          bc->num_tokens++;
+        }
+        rp.depth += take;
+        at += take;
+      }
+      if (at == E.num_tokens) ++e, at = 0, w = 0;
+    }
+    if (bc->num_tokens == 0) break;
+    const ffmi_status st = llm->run_inc_logits(*bc, rows.data(), (int)rows.size(),
+                                               logits + (size_t)done_rows * V);
+    if (st != FFMI_OK) return st;
+    done_rows += (long)rows.size();
+  }
+  return FFMI_OK;
+}
+
+ffmi_status RequestManager::replay_end(ffmi_model *llm, int64_t id) {
+  auto it = replays.find(id);
+  FFMI_CHECK(it != replays.end(), FFMI_ERR_INVALID);
+  if (PagePool *p = llm->page_pool()) p->release(it->second.slot);
+  replays.erase(it);
+  return FFMI_OK;
 }
 
 // Does a beam batch staged from placeholder results (`spec`: the previous

@@ -153,6 +153,10 @@ class RequestManager {
 
   ffmi_status serve_incr_decoding(ffmi_model *llm);
   ffmi_status serve_spec_infer(ffmi_model *llm);
+  // replay of given tokens (include/ffmi.h ffmi_rm_replay_step)
+  ffmi_status replay_step(ffmi_model *llm, const ffmi_replay_entry *entries, int n, float *logits,
+                          long cap_rows);
+  ffmi_status replay_end(ffmi_model *llm, int64_t id);
   // the speculation phase as chained beam steps (model.h): every SSM's
   // MAX_BEAM_DEPTH steps staged and launched up front, the bookkeeping
   // replayed on the results (identical batches and trees)
@@ -214,6 +218,11 @@ class RequestManager {
   // parent index of each node of dfs_tree_inputs[guid] (-1 for the root)
   std::unordered_map<RequestGuid, std::vector<int>> dfs_tree_parents;
   int spec_extensions = 0;
+  PagePool *pool = nullptr;  // of the model being served (null: fixed slots)
+  struct Replay {
+    int slot = 0, depth = 0;  // tokens in the cache
+  };
+  std::map<int64_t, Replay> replays;
   std::unordered_map<RequestGuid, std::vector<std::pair<int, int>>> committed_tokens;
   std::vector<ffmi_model *> ssm_models;
   std::map<RequestGuid, ProfileInfo> profiling_requests;
@@ -236,3 +245,7 @@ class RequestManager {
 double now_us();
 
 }  // namespace ffmi
+
+struct ffmi_rm {  // the C handle
+  ffmi::RequestManager rm;
+};

@@ -8,7 +8,8 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 # FFMI_LIB_VARIANT=<suffix> loads libffmi_<suffix>.so from the same directory
-# (build-flag A/B runs, e.g. scripts/gpu_ab.sh "" FFMI_LIB_VARIANT=x); the default is libffmi.so
+# (build-flag A/B runs, e.g. scripts/gpu_ab.sh "" FFMI_LIB_VARIANT=x, or a library with one
+# model family only, e.g. vapipel); the default is libffmi.so
 _VARIANT = os.environ.get("FFMI_LIB_VARIANT", "")
 LIB_PATH = os.path.join(_HERE, f"libffmi_{_VARIANT}.so" if _VARIANT else "libffmi.so")
 
@@ -26,6 +27,7 @@ DBG_KINDS = {"hidden": 0, "logits": 1, "attn_norm": 2, "qkv": 3, "attn_out": 4, 
              "ffn_norm": 6, "mlp_act": 7, "down": 8, "embed": 9}
 DBG_HIDDEN, DBG_LOGITS = DBG_KINDS["hidden"], DBG_KINDS["logits"]
 EPI_NONE, EPI_SILU_MUL = 0, 1
+BF16_PLAIN, BF16_RELU2, BF16_SUM = 0, 1, 2  # ffmi_linear_bf16
 X_PACKED = 0x10  # FFMI_X_PACKED flag for the epilogue argument
 Y_PACKED = 0x20  # FFMI_Y_PACKED
 W_STREAM = 0x40  # FFMI_W_STREAM: non-temporal weight loads (speed only)
@@ -92,7 +94,16 @@ class ModelOpts(ctypes.Structure):
                 ("max_requests", c_int), ("max_tokens", c_int), ("max_seq_len", c_int),
                 ("max_tree_tokens", c_int), ("weight_seed", c_uint64), ("use_graphs", c_int),
                 ("weights_folder", ctypes.c_char_p), ("weight_init", c_int),
-                ("full_precision", c_int)]
+                ("full_precision", c_int), ("kv_pool_tokens", c_int)]
+
+
+class ReplayEntry(ctypes.Structure):
+    _fields_ = [("id", c_int64), ("tokens", ctypes.POINTER(ctypes.c_int32)), ("num_tokens", c_int),
+                ("want", ctypes.POINTER(ctypes.c_int32)), ("num_want", c_int)]
+
+
+class PagedSeq(ctypes.Structure):
+    _fields_ = [("num_tokens", c_int), ("pos0", c_int), ("pages", ctypes.POINTER(ctypes.c_int32))]
 
 
 class RMConfig(ctypes.Structure):
@@ -177,7 +188,18 @@ SIGNATURES = {
     "ffmi_fill_weight": (c_int, [c_void_p, c_size_t, ctypes.c_char_p, c_uint64, c_int, c_void_p]),
     "ffmi_model_create": (c_int, [ctypes.POINTER(LlamaConfig), ctypes.POINTER(ModelOpts),
                                   ctypes.POINTER(c_void_p)]),
+    "ffmi_model_create_json": (c_int, [ctypes.c_char_p, ctypes.POINTER(ModelOpts),
+                                       ctypes.POINTER(c_void_p)]),
     "ffmi_model_destroy": (None, [c_void_p]),
+    "ffmi_model_vocab_size": (c_int, [c_void_p]),
+    "ffmi_linear_bf16": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p]),
+    "ffmi_post_rmsnorm": (c_int, [c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_float,
+                                  c_void_p]),
+    "ffmi_latent_attention": (c_int, [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float,
+                                      ctypes.POINTER(PagedSeq), c_int, c_int]),
+    "ffmi_rm_replay_step": (c_int, [c_void_p, c_void_p, ctypes.POINTER(ReplayEntry), c_int,
+                                    c_void_p, c_long]),
+    "ffmi_rm_replay_end": (c_int, [c_void_p, c_void_p, c_int64]),
     "ffmi_model_set_profiling": (c_int, [c_void_p, c_int]),
     "ffmi_model_op_stats": (c_int, [c_void_p, ctypes.POINTER(OpStat), c_int]),
     "ffmi_model_set_debug": (c_int, [c_void_p, c_int]),
@@ -223,6 +245,8 @@ TEST_SIGNATURES = {
     "ffmi_test_hash_model_create": (c_int, [c_int, c_int, c_int, c_int, c_int, c_uint64, c_int,
                                             ctypes.POINTER(c_void_p)]),
     "ffmi_test_hash_model_set_capacity": (c_int, [c_void_p, c_int]),
+    "ffmi_test_hash_model_set_pool": (c_int, [c_void_p, c_int, c_int]),
+    "ffmi_test_hash_model_free_pages": (c_int, [c_void_p]),
 }
 TEST_LIB_PATH = os.path.join(os.path.dirname(LIB_PATH), "libffmi_testmodel.so")
 
@@ -254,6 +278,8 @@ def lib():
                               "`python -c 'import __graft_entry__ as g; g.build()'`")
         L = ctypes.CDLL(LIB_PATH, mode=ctypes.RTLD_GLOBAL)
         for name, (res, args) in SIGNATURES.items():
+            if _VARIANT and not hasattr(L, name):
+                continue  # another family's entry point
             fn = getattr(L, name)
             fn.restype = res
             fn.argtypes = args

@@ -4,6 +4,7 @@ python/flexflow/serve/serve.py LLM/SSM).  All work happens in the C++
 runtime and HIP kernels; this file only marshals arguments.
 """
 import ctypes
+import json
 import os
 from dataclasses import dataclass
 from typing import List, Optional, Union
@@ -12,7 +13,8 @@ from . import ffmi as F
 
 
 class Model:
-    """A LLaMA model on one GPU (one TP shard).  mode: "inc" (incremental
+    """A model on one GPU (one TP shard).  config: a LLaMA size dict (ffmi.LlamaConfig), or the
+    config.json of a family that the runtime's registry names ("architecture").  mode: "inc" (incremental
     decoding LLM), "tree" (SpecInfer verify LLM) or "beam" (SSM)."""
 
     MODES = {"inc": F.MODEL_INC, "beam": F.MODEL_BEAM, "tree": F.MODEL_TREE}
@@ -20,25 +22,37 @@ class Model:
     def __init__(self, config: dict, mode: str = "inc", *, max_requests=8, max_tokens=128,
                  max_seq_len=512, max_tree_tokens=23, weight_seed=20250117, tp_rank=0,
                  tp_size=1, comm=None, weights_folder: Optional[str] = None,
-                 weight_init: Union[int, str] = 0, full_precision: bool = False):
+                 weight_init: Union[int, str] = 0, full_precision: bool = False,
+                 kv_pool_tokens: int = 0):
         """weights_folder: a checkpoint in the reference's per-tensor format
-        (see checkpoint.convert_hf_model); None: seeded synthetic weights,
+        (see checkpoint.convert_hf_model) or the family's own (Vapipel:
+        model.safetensors); None: seeded synthetic weights,
         `weight_init` "uniform" (0, the bench's), "depth_scaled" (1) or
         "token_chain" (2) -- include/ffmi.h ffmi_model_opts.  full_precision:
         the reference's --use-full-precision (every tensor fp32,
-        runtime/llama_f32.cpp); default the fp16 model."""
+        runtime/llama_f32.cpp); default the 16-bit model.  kv_pool_tokens:
+        size of a paged cache's pool (0: max_requests * max_seq_len)."""
         L = F.lib()
         self.config = dict(config)
         self.mode = mode
-        cfg = F.LlamaConfig.from_dict(config)
         opts = F.ModelOpts(self.MODES[mode], tp_rank, tp_size, comm.handle if comm else None,
                            max_requests, max_tokens, max_seq_len, max_tree_tokens, weight_seed, 0,
                            weights_folder.encode() if weights_folder else None,
-                           F.WEIGHT_INITS.get(weight_init, weight_init), int(full_precision))
+                           F.WEIGHT_INITS.get(weight_init, weight_init), int(full_precision),
+                           kv_pool_tokens)
         h = ctypes.c_void_p()
-        F.check(L.ffmi_model_create(ctypes.byref(cfg), ctypes.byref(opts), ctypes.byref(h)),
-                "ffmi_model_create")
+        if "architecture" in config or "architectures" in config:
+            st = L.ffmi_model_create_json(json.dumps(config).encode(), ctypes.byref(opts),
+                                          ctypes.byref(h))
+        else:
+            cfg = F.LlamaConfig.from_dict(config)
+            st = L.ffmi_model_create(ctypes.byref(cfg), ctypes.byref(opts), ctypes.byref(h))
+        F.check(st, "ffmi_model_create")
         self.handle = h
+
+    @property
+    def vocab_size(self) -> int:
+        return F.lib().ffmi_model_vocab_size(self.handle)
 
     def set_profiling(self, level: int):
         F.check(F.lib().ffmi_model_set_profiling(self.handle, level), "set_profiling")
@@ -67,7 +81,7 @@ class Model:
         width = F.lib().ffmi_model_debug_width(self.handle, kind)
         if width <= 0:
             raise F.FFMIError(f"debug_tensor({which}): no such tensor")
-        buf = np.empty(1024 * width, np.float32)
+        buf = np.empty(2048 * width, np.float32)
         T = F.lib().ffmi_model_debug_tensor(self.handle, kind, layer,
                                             buf.ctypes.data_as(ctypes.c_void_p), buf.size)
         if T < 0:
@@ -97,7 +111,7 @@ class HashModel(Model):
     """Scheduler test double (CPU only, see ffmi_test_hash_model_create)."""
 
     def __init__(self, vocab=1000, mode="inc", *, max_requests=8, max_seq_len=512,
-                 max_tree_tokens=23, salt=0, disagree_pct=0, max_tokens=None):
+                 max_tree_tokens=23, salt=0, disagree_pct=0, max_tokens=None, pool=None):
         self.mode = mode
         h = ctypes.c_void_p()
         F.check(F.test_lib().ffmi_test_hash_model_create(vocab, self.MODES[mode], max_requests,
@@ -107,6 +121,11 @@ class HashModel(Model):
         self.handle = h
         if max_tokens is not None:  # a GPU model's token capacity per step
             F.check(F.test_lib().ffmi_test_hash_model_set_capacity(h, max_tokens), "capacity")
+        if pool is not None:  # a paged cache: (pages, tokens per page)
+            F.check(F.test_lib().ffmi_test_hash_model_set_pool(h, *pool), "pool")
+
+    def free_pages(self) -> int:
+        return F.test_lib().ffmi_test_hash_model_free_pages(self.handle)
 
 
 class Comm:
@@ -335,6 +354,31 @@ class RequestManager:
 
     def serve_spec_infer(self, llm: Model):
         F.check(F.lib().ffmi_rm_serve_spec_infer(self.handle, llm.handle), "serve spec")
+
+    def replay_step(self, llm: Model, entries):
+        """One step of given tokens: entries is a list of (id, tokens, want);
+        returns the wanted logits [rows, vocab] fp32, in order (include/ffmi.h
+        ffmi_rm_replay_step)."""
+        import numpy as np
+        arr = (F.ReplayEntry * max(1, len(entries)))()
+        keep, rows = [], 0
+        for a, (rid, tokens, want) in zip(arr, entries):
+            t = np.ascontiguousarray(tokens, np.int32)
+            w = np.ascontiguousarray(want, np.int32)
+            keep += [t, w]
+            a.id, a.num_tokens, a.num_want = rid, len(t), len(w)
+            a.tokens = t.ctypes.data_as(ctypes.POINTER(ctypes.c_int32))
+            a.want = w.ctypes.data_as(ctypes.POINTER(ctypes.c_int32))
+            rows += len(w)
+        out = np.empty((rows, llm.vocab_size), np.float32)
+        F.check(F.lib().ffmi_rm_replay_step(self.handle, llm.handle, arr, len(entries),
+                                            out.ctypes.data_as(ctypes.c_void_p), rows),
+                "replay step")
+        return out
+
+    def replay_end(self, llm: Model, rid: int):
+        """The replayed request is finished: its slot and pages are free."""
+        F.check(F.lib().ffmi_rm_replay_end(self.handle, llm.handle, rid), "replay end")
 
     def get_generation_result(self, guid: int) -> GenerationResult:
         L = F.lib()

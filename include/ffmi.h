@@ -335,6 +335,37 @@ ffmi_status ffmi_silu_mul_f32(const float *a, const float *b, float *out, size_t
                               ffmi_stream stream);
 ffmi_status ffmi_arg_topk_f32(const float *logits, int T, int V, int k, int32_t *ids,
                               float *probs, ffmi_stream stream);
+/* ------------------------------------------------------------------------ */
+/* bf16 products and latent attention (the Vapipel family's operators)       */
+/* ------------------------------------------------------------------------ */
+typedef enum {
+  FFMI_BF16_PLAIN = 0, /* Y bf16 = X W^T                                      */
+  FFMI_BF16_RELU2 = 1, /* Y bf16 = relu(X W^T)^2                              */
+  FFMI_BF16_SUM = 2    /* Y fp32 = X W^T, the unrounded sums                  */
+} ffmi_bf16_epilogue;
+/* X [T][in], W [out][in] row-major bf16, Y [T][out] row-major; in and out
+ * multiples of 32.  Packs both operands on every call: the models keep theirs
+ * packed. */
+ffmi_status ffmi_linear_bf16(const void *X, const void *W, void *Y, int T, int out_dim, int in_dim,
+                             int epilogue, ffmi_stream stream);
+/* x[T][H] += y / rms(y) * w in fp32, y the sum of `slabs` [T][H] matrices, the
+ * mean over the first n columns (the rest zero); H % 32 == 0, slabs <= 8 */
+ffmi_status ffmi_post_rmsnorm(const float *y, int slabs, const float *w, float *x, int T, int H,
+                              int n, float eps, ffmi_stream stream);
+/* Latent attention over a paged cache.  seqs: per request its tokens in this
+ * batch, at positions [pos0, pos0 + num_tokens), and its page table; cache
+ * [pages][64][rank], the batch's own latents already stored.  Row t * heads +
+ * h of q and o [T * heads][rank] is head h of batch token t:
+ *   o = sum_j softmax_j(q . c_j * scale) c_j  over j <= the token's position.
+ * full_precision: fp32 elements; else bf16.  Blocking. */
+typedef struct {
+  int num_tokens, pos0;
+  const int32_t *pages; /* host, ceil((pos0 + num_tokens) / 64) entries       */
+} ffmi_paged_seq;
+ffmi_status ffmi_latent_attention(const void *q, const void *cache, int pages, void *o, int heads,
+                                  int rank, float scale, const ffmi_paged_seq *seqs, int num_seqs,
+                                  int full_precision);
+
 /* seeded synthetic weights, identical to oracle/orc_gen_weight then fp16.
  * kind 0: matrix (uniform, std 0.02); 1: norm weight (1 +- 0.1);
  * FFMI_WKIND_DEPTH | L: o_proj / down_proj of an L-layer model under the
@@ -398,11 +429,21 @@ typedef struct {
    * and softmax in fp32 (runtime/llama_f32.cpp, kernels/f32.hip); lm_head
    * replicated under TP.  0: the fp16 model (the measured path). */
   int full_precision;
+  /* Models with a paged cache (ffmi_model_create_json): tokens the pool holds
+   * for all requests together, in whole pages of 64 (0: max_requests *
+   * max_seq_len).  The scheduler admits requests while their longest length
+   * fits what is left. */
+  int kv_pool_tokens;
 } ffmi_model_opts;
 
 typedef struct ffmi_model ffmi_model;
 ffmi_status ffmi_model_create(const ffmi_llama_config *cfg, const ffmi_model_opts *o,
                               ffmi_model **out);
+/* The model class config.json names ("architecture", or HF "architectures"),
+ * from the text of that file.  weights_folder: the checkpoint (safetensors, or
+ * the family's own format), NULL: seeded synthetic weights. */
+ffmi_status ffmi_model_create_json(const char *config_json, const ffmi_model_opts *o,
+                                   ffmi_model **out);
 void ffmi_model_destroy(ffmi_model *m);
 /* Per-op device timing with HIP events on the model's stream (the
  * reference's --profiling, model.cc:4548-4550).  level 0: off; 1: sampled
@@ -555,6 +596,25 @@ int64_t ffmi_rm_register_request(ffmi_rm *rm, const int *prompt, int n_prompt,
  * (serve_incr_decoding / serve_spec_infer, request_manager.cc:3012-3173). */
 ffmi_status ffmi_rm_serve_incr_decoding(ffmi_rm *rm, ffmi_model *llm);
 ffmi_status ffmi_rm_serve_spec_infer(ffmi_rm *rm, ffmi_model *llm);
+/* Replay of given tokens through the engine (an INC model): one step runs the
+ * next tokens of every entry's request as one batch -- portions of prompts
+ * beside single tokens -- from what earlier steps left in the cache, and
+ * returns the logits asked for.  A request is admitted at its first entry and
+ * holds a request slot until ffmi_rm_replay_end gives it back.  A step of more
+ * than max_tokens_per_batch tokens runs as several batches.  logits: host,
+ * fp32 [wanted][vocab], in the order of the entries and of `want` (places
+ * among the entry's tokens, ascending); cap_rows: its rows. */
+typedef struct {
+  int64_t id;
+  const int32_t *tokens;
+  int num_tokens;
+  const int32_t *want;
+  int num_want;
+} ffmi_replay_entry;
+ffmi_status ffmi_rm_replay_step(ffmi_rm *rm, ffmi_model *llm, const ffmi_replay_entry *entries,
+                                int num_entries, float *logits, long cap_rows);
+ffmi_status ffmi_rm_replay_end(ffmi_rm *rm, ffmi_model *llm, int64_t id);
+int ffmi_model_vocab_size(ffmi_model *m);
 /* GenerationResult.output_tokens; returns count (or needed size) */
 int ffmi_rm_get_output(ffmi_rm *rm, int64_t guid, int *tokens, int cap);
 typedef struct {
@@ -609,9 +669,10 @@ long ffmi_debug_markers(long long *dst, long n);
 const char *ffmi_status_str(ffmi_status s);
 /* message + file:line of the last failing check on this process */
 const char *ffmi_last_error(void);
-/* "ffmi 0.3 (gfx950)": 0.2 appended full_precision to ffmi_attn_cfg and
+/* "ffmi 0.4 (gfx950)": 0.2 appended full_precision to ffmi_attn_cfg and
  * ffmi_model_opts (struct sizes changed) and added the *_f32 entry points;
- * 0.3 appended spec_extensions to ffmi_rm_config */
+ * 0.3 appended spec_extensions to ffmi_rm_config; 0.4 appended kv_pool_tokens
+ * to ffmi_model_opts and added models by config.json and replay steps */
 const char *ffmi_version(void);
 
 #ifdef __cplusplus

@@ -18,6 +18,10 @@ ffmi_status ffmi_test_hash_model_create(int vocab, int mode, int max_requests,
  * max_tokens: larger steps fail with FFMI_ERR_INVALID, and the scheduler's
  * up-front SSM capacity check sees it.  TEST USE ONLY. */
 ffmi_status ffmi_test_hash_model_set_capacity(ffmi_model *m, int max_tokens);
+/* A paged cache of `pages` pages for an INC hash model (contexts read through
+ * the page tables), and its free pages (-1: no pool).  TEST USE ONLY. */
+ffmi_status ffmi_test_hash_model_set_pool(ffmi_model *m, int pages, int page_tokens);
+int ffmi_test_hash_model_free_pages(ffmi_model *m);
 
 #ifdef __cplusplus
 }

@@ -1,0 +1,271 @@
+"""The Vapipel model through the engine against the plain implementation
+(vapipel_ref.py): layers, schedules (whole prompts, portions, token by token,
+mixed batches, reused slots and pages), generation, and bin/trace_run."""
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+
+import flexflow_amd as fa
+import vapipel_models as VM
+import vapipel_ref as R
+
+pytestmark = pytest.mark.gpu
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+# sizes that are no multiples of the kernels' tiles, layers that differ, shared
+# latents, layers without a feed-forward, scales that are not 1/sqrt(dim)
+ODD = VM.model_config(77, 72, 700, [
+    VM.layer(3, 24, 40, 20, 0.11, 50), VM.layer(1, 64, 8, 96, 0.3, None),
+    VM.layer(5, 12, 20, 20, 0.2, 33, kv_from=0), VM.layer(2, 40, 24, 96, 0.25, 130, kv_from=1),
+    VM.layer(20, 8, 8, 130, 0.4, 64)])
+WIDE = VM.model_config(300, 256, 400, [
+    VM.layer(8, 32, 64, 512, 0.2, 320), VM.layer(8, 32, 64, 512, 0.2, 320, kv_from=0),
+    VM.layer(1, 160, 1, 600, 0.05, 64)], eps=1e-3)
+ONE = VM.model_config(64, 32, 300, [VM.layer(1, 32, 32, 64, 0.17, 32)])
+CONFIGS = {"odd": ODD, "wide": WIDE, "one": ONE}
+WEIGHTS = {k: VM.random_weights(c, 11, sharp=3.0) for k, c in CONFIGS.items()}
+
+
+def tokens(cfg, n, seed):
+    return [int(t) for t in np.random.default_rng(seed).integers(0, cfg["vocab"], n)]
+
+
+@pytest.fixture(scope="module")
+def folders(tmp_path_factory):
+    d = tmp_path_factory.mktemp("vapipel")
+    return {k: VM.write_checkpoint(d / k, c, WEIGHTS[k]) for k, c in CONFIGS.items()}
+
+
+@pytest.fixture(scope="module")
+def engine(folders):
+    """engine(name, full): (rm, model) over a pool of 12 pages, kept per module"""
+    made = {}
+
+    def get(name, full):
+        if (name, full) not in made:
+            cfg = fa.load_config(folders[name])
+            m = fa.Model(cfg, "inc", max_requests=4, max_tokens=256, max_seq_len=cfg["max_positions"],
+                         weights_folder=folders[name], full_precision=full, kv_pool_tokens=12 * 64)
+            rm = fa.RequestManager(max_requests_per_batch=4, max_tokens_per_batch=256,
+                                   max_spec_tree_token_num=0,
+                                   max_sequence_length=cfg["max_positions"])
+            made[name, full] = (rm, m)
+        return made[name, full]
+    return get
+
+
+_ref = {}
+
+
+def reference(name, toks):
+    key = (name, tuple(toks))
+    if key not in _ref:
+        layers = []
+        _ref[key] = R.forward(CONFIGS[name], WEIGHTS[name], toks, layers), layers
+    return _ref[key]
+
+
+def close(got, want, full):
+    """rows' rms error, the mean taken off, relative to the logits' rms"""
+    d = got - want
+    d = d - d.mean(1, keepdims=True)
+    err = np.sqrt((d * d).mean(1)).max() / np.sqrt((want * want).mean())
+    limit = 3e-5 if full else 6e-2
+    assert err < limit, err
+
+
+_next = [0]
+
+
+def run(eng, toks, cuts):
+    """one request alone, cut into portions; every position's logits"""
+    rm, m = eng
+    _next[0] += 1
+    rid, out, at = _next[0], [], 0
+    for n in cuts:
+        part = toks[at:at + n]
+        if part:
+            out.append(rm.replay_step(m, [(rid, part, range(len(part)))]))
+        at += n
+    assert at >= len(toks)
+    rm.replay_end(m, rid)
+    return np.concatenate(out)
+
+
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_residual_stream_after_every_layer(engine, name, full):
+    rm, m = engine(name, full)
+    toks = tokens(CONFIGS[name], 90, 3)
+    want, layers = reference(name, toks)
+    m.set_debug(True)
+    try:
+        got = run((rm, m), toks, [90])
+        for i, ref in enumerate(layers):
+            h = m.debug_tensor("hidden", i)
+            rms = np.sqrt((ref * ref).mean())
+            assert np.sqrt(((h - ref) ** 2).mean()) < (1e-5 if full else 2e-2) * rms, i
+    finally:
+        m.set_debug(False)
+    close(got, want, full)
+
+
+CUTS = {"whole": [1000], "token by token": [1] * 150, "twos": [2] * 75, "threes": [3] * 50,
+        "below a page": [63] * 3, "a page": [64] * 3, "past a page": [65] * 3,
+        "prompt then tokens": [100] + [1] * 50, "changing": [1, 2, 61, 2, 17, 3, 40, 1, 1, 22]}
+
+
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_portions(engine, name, full):
+    toks = tokens(CONFIGS[name], 150, 4)
+    want, _ = reference(name, toks)
+    for how, cuts in CUTS.items():
+        print(name, full, how, flush=True)
+        close(run(engine(name, full), toks, cuts), want, full)
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_first_tokens_and_single_token_prompts(engine, full):
+    for t in range(5):
+        toks = [t] + tokens(ONE, 3, t)
+        want, _ = reference("one", toks)
+        close(run(engine("one", full), toks, [1] * 4), want, full)
+        close(run(engine("one", full), toks, [2, 2]), want, full)
+
+
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("name", ["odd", "wide"])
+def test_mixed_batches_on_reused_slots_and_pages(engine, name, full):
+    """Requests of unequal length, portions beside single tokens, one left out
+    of steps, ended and replaced while others run: each against itself alone."""
+    rm, m = engine(name, full)
+    cfg = CONFIGS[name]
+    rng = np.random.default_rng(8)
+    live, left, done = {}, [(n, 20 + i) for i, n in enumerate((1, 150, 33, 64, 129, 2, 90, 65))], 0
+    while left or live:
+        while left and len(live) < 4 and (len(live) < 2 or rng.random() < 0.5):
+            n, seed = left.pop(0)
+            _next[0] += 1
+            live[_next[0]] = [tokens(cfg, n, seed), 0, []]
+        entries = []
+        for rid, (toks, at, _) in live.items():
+            if len(live) > 1 and rng.random() < 0.2:
+                continue  # left out of this step
+            k = int(rng.choice([1, 1, 2, 3, 17, 40]))
+            part = toks[at:at + k]
+            entries.append((rid, part, range(len(part))))
+        if not entries:
+            continue
+        out, r = rm.replay_step(m, entries), 0
+        for rid, part, _ in entries:
+            live[rid][1] += len(part)
+            live[rid][2].append(out[r:r + len(part)])
+            r += len(part)
+        for rid in [k for k, v in live.items() if v[1] == len(v[0])]:
+            toks, _, got = live.pop(rid)
+            close(np.concatenate(got), reference(name, toks)[0], full)
+            rm.replay_end(m, rid)
+            done += 1
+    assert done == 8
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_long_decoding(engine, full):
+    toks = tokens(ODD, 600, 5)
+    got = run(engine("odd", full), toks, [70] + [1] * 530)
+    close(got, reference("odd", toks)[0], full)
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_far_key_decides(folders, tmp_path, full):
+    """Weights under which every query wants one marked token's latent: the
+    marker is seen from any distance, by prompts and by decoded tokens, and a
+    sequence without it differs."""
+    cfg = ONE
+    w = {k: v.copy() for k, v in WEIGHTS["one"].items()}
+    marker, W = 9, cfg["width"]
+    rng = np.random.default_rng(1)
+    w["pos"] *= 0
+    w["embed"][:] = VM.bf16(rng.standard_normal(w["embed"].shape) * 0.5)
+    w["embed"][:, 0], w["embed"][:, 1] = 1.0, 0.0
+    w["embed"][marker, 1] = 8.0
+    q, dkv, uk = (np.zeros_like(w["l0.mix." + n]) for n in ("q", "dkv", "uk"))
+    q[0, 0] = 8.0            # every query: a constant
+    dkv[0, 1] = 1.0          # latent 0: the marker
+    dkv[1:, 2:] = VM.bf16(rng.standard_normal((len(dkv) - 1, W - 2)) * 0.1)
+    uk[0, 0] = 4.0
+    w.update({"l0.mix.q": q, "l0.mix.dkv": dkv, "l0.mix.uk": uk})
+    folder = VM.write_checkpoint(tmp_path / "far", cfg, w)
+    m = fa.Model(cfg, "inc", max_requests=4, max_tokens=256, max_seq_len=300,
+                 weights_folder=folder, full_precision=full)
+    rm = fa.RequestManager(max_requests_per_batch=4, max_tokens_per_batch=256,
+                           max_spec_tree_token_num=0, max_sequence_length=300)
+    base = [t for t in tokens(cfg, 400, 2) if t != marker][:200]
+    plain = R.forward(cfg, w, base)
+    for at in (0, 1, 63, 64, 65, 127, 128, 190):
+        toks = base[:at] + [marker] + base[at + 1:]
+        want = R.forward(cfg, w, toks)
+        assert np.abs(want[-1] - plain[-1]).max() > 0.3
+        for cuts in ([200], [at or 1, 200], [150] + [1] * 50):
+            close(run((rm, m), toks, cuts), want, full)
+
+
+def test_refused_steps(engine):
+    rm, m = engine("one", True)
+    ok = tokens(ONE, 299, 1)
+    for bad in ([64], [-1], ok + [1, 1]):
+        _next[0] += 1
+        with pytest.raises(fa.ffmi.FFMIError):
+            rm.replay_step(m, [(_next[0], bad, [])])
+        rm.replay_end(m, _next[0])
+    close(run((rm, m), ok[:40], [40]), reference("one", ok[:40])[0], True)
+
+
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("pool", [0, 3 * 64])
+def test_greedy_generation(folders, full, pool):
+    """generate() through the scheduler: continuous batching over two slots,
+    and over a pool that holds one request at a time."""
+    cfg = fa.load_config(folders["odd"])
+    m = fa.Model(cfg, "inc", max_requests=2, max_tokens=48, max_seq_len=160,
+                 weights_folder=folders["odd"], full_precision=full, kv_pool_tokens=pool)
+    rm = fa.RequestManager(max_requests_per_batch=2, max_tokens_per_batch=48,
+                           max_spec_tree_token_num=0, max_sequence_length=160, bos_token_id=1)
+    prompts = [tokens(ODD, n, 60 + n) for n in (3, 90, 40, 1)]
+    res = fa.generate(rm, m, prompts, max_length=132)
+    for p, r in zip(prompts, res):
+        seq = r.output_tokens
+        assert seq[:len(p) + 1] == [1] + p and len(seq) == 132
+        # every pick: the plain implementation's, or a tie within rounding
+        logits = R.forward(ODD, WEIGHTS["odd"], seq[:-1])[len(p):]
+        lead = logits.max(1) - logits[np.arange(len(logits)), seq[len(p) + 1:]]
+        assert lead.max() < (1e-4 if full else 0.12 * logits.std()), lead.max()
+        assert (lead == 0).mean() > (0.99 if full else 0.9)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_trace_run(folders, tmp_path, dtype):
+    """bin/trace_run over a small trace, compared with the plain model."""
+    a, b = tokens(ODD, 140, 31), tokens(ODD, 70, 32)
+    steps = [dict(step=0, entries=[dict(id="a", tokens=a[:100], want=[0, 63, 64, 99])], end=[]),
+             dict(step=1, entries=[dict(id="a", tokens=a[100:102], want=[]),
+                                   dict(id="b", tokens=b[:69], want=[68])], end=[]),
+             dict(step=2, entries=[dict(id="b", tokens=b[69:], want=[0]),
+                                   dict(id="a", tokens=a[102:103], want=[0])], end=["b"]),
+             dict(step=3, entries=[dict(id="a", tokens=a[103:], want=[36]),
+                                   dict(id="c", tokens=b[:5], want=[4])], end=["a", "c"])]
+    want = {0: [a[:1], a[:64], a[:65], a[:100]], 2: [b, a[:103]], 1: [b[:69]], 3: [a, b[:5]]}
+    p = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", folders["odd"],
+                        "--dtype", dtype, "--out", str(tmp_path), "--max-tokens", "320"],
+                       input="".join(json.dumps(s) + "\n" for s in steps), text=True,
+                       capture_output=True, timeout=110)
+    assert p.returncode == 0, p.stderr[-2000:]
+    assert [l for l in p.stdout.splitlines() if l.startswith("done")] == ["done %d" % i for i in range(4)]
+    for i, seqs in want.items():
+        got = np.fromfile(tmp_path / ("%d.f32" % i), "<f4").reshape(len(seqs), -1)
+        close(got, np.stack([reference("odd", s)[0][-1] for s in seqs]), dtype == "float32")
