@@ -276,6 +276,78 @@ def run_leg(llm_cfg, ssm_cfg, prompts, max_len, B, mtb, rm_kw, args, widths, tre
             "p50_token_latency_ms": round(statistics.median(lat) / 1000.0, 3)}
 
 
+# --model vapipel: (name, width, heads, head size, latent, ff, layers), LLaMA beside
+# it at the same width, heads, ff and layers
+VAPIPEL_SIZES = [("width2048", 2048, 16, 128, 256, 5632, 8), ("width4096", 4096, 32, 128, 512, 11008, 8)]
+
+
+def vapipel_config(width, heads, dim, rank, ff, layers, vocab=32000, positions=4096):
+    mix = dict(heads=heads, dim=dim, vdim=dim, kv_rank=rank, scale=dim ** -0.5)
+    return dict(architecture="Vapipel", vocab=vocab, width=width, max_positions=positions,
+                norm=dict(eps=1e-6),
+                layers=[dict(type="latent_attention", mixer=mix, mlp=dict(kind="dense", ff=ff))
+                        for _ in range(layers)])
+
+
+def bench_decoder(cfg, B, prompt_len, decode, mtb, repeats):
+    """Prefill and decode throughput of incremental decoding: generates of one
+    new token (the prompts' steps alone) and of `decode`, best of `repeats`."""
+    seq = prompt_len + decode + 8
+    llm = fa.Model(cfg, "inc", max_requests=B, max_tokens=mtb, max_seq_len=seq, max_tree_tokens=0,
+                   weight_seed=20250117)
+    prompts = make_prompts(B, prompt_len - 1, 32000)
+
+    def once(new):
+        rm = fa.RequestManager(max_requests_per_batch=B, max_tokens_per_batch=mtb,
+                               max_spec_tree_token_num=0, max_sequence_length=seq)
+        device_sync()
+        t = time.time()
+        res = fa.generate(rm, llm, prompts, max_length=prompt_len + new)
+        device_sync()
+        assert all(len(r.output_tokens) == prompt_len + new for r in res)
+        return time.time() - t, rm.stats().llm_steps
+
+    once(decode)  # warm (graphs captured)
+    pre = min(once(1) for _ in range(repeats))
+    full = min(once(decode) for _ in range(repeats))
+    llm.close()
+    steps = full[1] - pre[1]
+    return {"prefill_tokens_per_s": round(B * prompt_len / pre[0], 1),
+            "decode_tokens_per_s": round(B * (decode - 1) / (full[0] - pre[0]), 1),
+            "decode_step_us": round((full[0] - pre[0]) / max(1, steps) * 1e6, 1),
+            "prefill_ms": round(pre[0] * 1e3, 2), "prefill_steps": pre[1]}
+
+
+def bench_vapipel(args):
+    """--model vapipel: the latent-attention decoder (random weights) and LLaMA
+    at equal sizes, incremental decoding, one GPU.  One JSON line."""
+    legs = []
+    for name, width, heads, dim, rank, ff, layers in VAPIPEL_SIZES:
+        cfgs = {"vapipel": vapipel_config(width, heads, dim, rank, ff, layers),
+                "llama": dict(num_layers=layers, vocab_size=32000, num_heads=heads,
+                              num_kv_heads=heads, hidden=width, intermediate=ff, rms_eps=1e-6,
+                              rope_theta=10000.0)}
+        for prompt in (args.prefill, 1024):
+            leg = {"size": name, "kv_rank": rank, "layers": layers, "batch": args.batch,
+                   "prompt": prompt, "decode": args.decode}
+            for fam, cfg in cfgs.items():
+                if args.only_family and fam != args.only_family:
+                    continue
+                leg[fam] = bench_decoder(cfg, args.batch, prompt, args.decode,
+                                         args.max_tokens_per_batch, args.steps)
+            legs.append(leg)
+            print(f"[bench] {json.dumps(leg)}", file=sys.stderr, flush=True)
+    head = legs[-1].get("vapipel") or legs[-1]["llama"]
+    print(json.dumps({
+        "metric": "decode tokens/s, latent-attention decoder beside LLaMA at equal size",
+        "value": head["decode_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
+        "warmup": 1, "ms_per_step": round(head["decode_step_us"] / 1e3, 4),
+        "higher_is_better": True, "scaling": "strong", "vs_baseline": None, "dtype": "bf16",
+        "data": "synthetic", "config": {"model": "Vapipel", "global_batch": args.batch,
+                                        "seq_len": 1024 + args.decode, "parallelism": "tp1"},
+        "legs": legs}), flush=True)
+
+
 def pmc_traffic(kernel):
     """HBM bytes per launch of the roofline kernel, measured with rocprofv3
     --pmc FETCH_SIZE in a separate run (scripts/round_gpu.sh ->
@@ -356,6 +428,11 @@ def main():
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
     ap.add_argument("--mode", choices=["spec", "incr"], default="spec")
+    ap.add_argument("--model", choices=["llama", "vapipel"], default="llama",
+                    help="llama: the headline workload; vapipel: prefill and decode throughput "
+                         "of the latent-attention decoder beside LLaMA at equal sizes (one GPU)")
+    ap.add_argument("--only-family", choices=["llama", "vapipel"], default=None,
+                    help="--model vapipel: run one of the two (profiling)")
     ap.add_argument("--batch", type=int, default=8)
     ap.add_argument("--prefill", type=int, default=128)
     ap.add_argument("--decode", type=int, default=128)
@@ -411,6 +488,11 @@ def main():
     # N-rank path on a one-GPU box (with FFMI_TP_TRANSPORT=xgmi-only, since
     # RCCL refuses two ranks on one GPU); timings are then not a scaling result
     fa.set_device(int(os.environ.get("FFMI_BENCH_DEVICE", local)))
+    if args.model == "vapipel":
+        if world > 1:
+            raise SystemExit("--model vapipel runs on one GPU")
+        bench_vapipel(args)
+        return
     comm = None
     transport = "rccl"
     transport_reason = "FFMI_TP_TRANSPORT=rccl"

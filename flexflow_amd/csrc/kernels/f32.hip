@@ -405,6 +405,9 @@ hipError_t launch_attention_f32(const char *blob, int T, const float *qbuf, cons
 // (p desc, index asc), each round taking the first element after the
 // previous pick in that order (arg_topk.cu:208-330 ties: lower index first).
 // ---------------------------------------------------------------------------
+// NV > 0: the row (V <= NV * 1024) is read once, all loads in flight together,
+// and kept in registers; NV == 0: any V, read per pass.
+template <int NV>
 __global__ __launch_bounds__(1024) void f32_softmax_topk_kernel(const float *__restrict__ logits,
                                                                int V, int ld, int k,
                                                                int32_t *__restrict__ ids,
@@ -415,8 +418,21 @@ __global__ __launch_bounds__(1024) void f32_softmax_topk_kernel(const float *__r
   __shared__ int si[16];
   const int t = blockIdx.x, tid = threadIdx.x, nw = blockDim.x >> 6;
   const float *z = logits + (size_t)t * ld;
+  float zr[NV ? NV : 1];
+#pragma unroll
+  for (int j = 0; j < NV; ++j) zr[j] = z[min(tid + j * 1024, V - 1)];
+  // f(i, z_i) for this thread's elements, ascending
+  auto each = [&](auto f) {
+    if constexpr (NV > 0) {
+#pragma unroll
+      for (int j = 0; j < NV; ++j)
+        if (tid + j * 1024 < V) f(tid + j * 1024, zr[j]);
+    } else {
+      for (int i = tid; i < V; i += 1024) f(i, z[i]);
+    }
+  };
   float mx = -3.402823466e38f;
-  for (int i = tid; i < V; i += blockDim.x) mx = fmaxf(mx, z[i]);
+  each([&](int, float v) { mx = fmaxf(mx, v); });
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off));
   if ((tid & 63) == 0) shf[tid >> 6] = mx;
@@ -424,7 +440,7 @@ __global__ __launch_bounds__(1024) void f32_softmax_topk_kernel(const float *__r
   mx = shf[0];
   for (int w = 1; w < nw; ++w) mx = fmaxf(mx, shf[w]);
   double sum = 0.0;
-  for (int i = tid; i < V; i += blockDim.x) sum += (double)expf(__fsub_rn(z[i], mx));
+  each([&](int, float v) { sum += (double)expf(__fsub_rn(v, mx)); });
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) sum += __shfl_xor(sum, off);
   if ((tid & 63) == 0) shd[tid >> 6] = sum;
@@ -435,13 +451,16 @@ __global__ __launch_bounds__(1024) void f32_softmax_topk_kernel(const float *__r
   float pprev = 3.402823466e38f;
   int iprev = -1;
   for (int r = 0; r < k; ++r) {
-    float bp = -1.f;
+    float bp = -1.f, bz = -3.402823466e38f;
     int bi = V;
-    for (int i = tid; i < V; i += blockDim.x) {
-      const float p = __fdiv_rn(expf(__fsub_rn(z[i], mx)), s);
+    each([&](int i, float v) {
+      // a logit this far below the row's best (first round) or the thread's has
+      // a smaller probability (exp is monotone to a few ulps): not evaluated
+      if (v < (r == 0 ? mx : bz) - 1e-3f) return;
+      const float p = __fdiv_rn(expf(__fsub_rn(v, mx)), s);
       const bool after = p < pprev || (p == pprev && i > iprev);
-      if (after && (p > bp || (p == bp && i < bi))) bp = p, bi = i;
-    }
+      if (after && (p > bp || (p == bp && i < bi))) bp = p, bi = i, bz = v;
+    });
 #pragma unroll
     for (int off = 32; off > 0; off >>= 1) {
       const float op = __shfl_xor(bp, off);
@@ -467,8 +486,12 @@ hipError_t launch_softmax_topk_f32(const float *logits, int T, int V, int k, int
   if (T <= 0) return hipSuccess;
   if (ld == 0) ld = V;
   if (k < 1 || k > V || ld < V) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(f32_softmax_topk_kernel, dim3(T), dim3(1024), 0, s, logits, V, ld, k, ids,
-                     probs);
+  if (V <= 32 * 1024)
+    hipLaunchKernelGGL(f32_softmax_topk_kernel<32>, dim3(T), dim3(1024), 0, s, logits, V, ld, k,
+                       ids, probs);
+  else
+    hipLaunchKernelGGL(f32_softmax_topk_kernel<0>, dim3(T), dim3(1024), 0, s, logits, V, ld, k, ids,
+                       probs);
   return hipGetLastError();
 }
 

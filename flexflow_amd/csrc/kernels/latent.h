@@ -29,6 +29,8 @@ struct LatentBlock {
   int32_t table;          // offset of the request's page table (int32 units)
   int32_t tile0, ntiles;
   int32_t slot;
+  int32_t page0;          // the page of tile0: one dependent load less at the start
+  int32_t pad[3];
 };
 struct LatentMerge {
   int32_t row0, nrows, slot0, nslots;

@@ -391,14 +391,13 @@ hipError_t launch_head_gemm_f32(const HeadGemm &hg, hipStream_t s) {
 // ---------------------------------------------------------------------------
 // attention over the pages, MFMA form
 // ---------------------------------------------------------------------------
-// One workgroup: up to RT * 16 rows against a range of 64-token pages.  Scores
-// S^T = C . Q'^T (lane: 4 keys of one row), outputs O^T = C^T . P^T with C^T
-// read from the row-major page in LDS by the transposing LDS load; the k order
-// of the second product is the key order the scores already have in the
-// lanes (16-lane group g: keys 4g..4g+3 and 16+4g..).
-//   scores:  RT == 4: waves 2 (row pairs) x 2 (key halves); RT <= 2: each wave
-//            one 16-key tile, all rows
-//   outputs: each wave a quarter of the latent's columns, all rows
+// One workgroup of eight waves: up to RT * 16 rows against a range of 64-token
+// pages.  Scores S^T = C . Q'^T (lane: 4 keys of one row), outputs O^T = C^T .
+// P^T with C^T read from the row-major page in LDS by the transposing LDS load;
+// the k order of the second product is the key order the scores already have
+// in the lanes (16-lane group g: keys 4g..4g+3 and 16+4g..).
+//   scores:  wave = (16-key tile, half of the rows); RT == 1: four waves only
+//   outputs: each wave an eighth of the latent's columns, all rows
 // Softmax state in fp32, base-2 exponents; weights meet the second product in
 // bf16, the sums take them unrounded.
 typedef short s4 __attribute__((ext_vector_type(4)));
@@ -407,53 +406,57 @@ typedef uint32_t u4 __attribute__((ext_vector_type(4)));
 constexpr int kRankPad = 8;  // LDS row padding (elements)
 
 template <int RC, int RT>
-__global__ __launch_bounds__(256, 1) void latent_attn_kernel(
+__global__ __launch_bounds__(512) void latent_attn_kernel(
     const char *__restrict__ blob, int off_blocks, const uint16_t *__restrict__ Q,
     const uint16_t *__restrict__ cache, uint16_t *__restrict__ O, float *__restrict__ slabs,
     float *__restrict__ ml, int heads, float scale_log2) {
-  constexpr int R = RC * 64, KS = RC * 2, DT = RC, LDC = R + kRankPad;
-  constexpr int SR = RT == 4 ? 2 : RT;      // row tiles of a wave's scores
-  constexpr int KW = RT == 4 ? 2 : 1;       // key tiles of a wave's scores
-  constexpr int NK = 4 / KW;                // waves over the keys
-  constexpr int CPT = 64 * R / 8 / 256;     // 16-B page chunks per thread
+  constexpr int R = RC * 64, KS = RC * 2, LDC = R + kRankPad;
+  constexpr int SR = RT == 4 ? 2 : 1;           // row tiles of a wave's scores
+  constexpr int NT = RC * 4, DT = (NT + 7) / 8;  // column tiles: all, of a wave's outputs
   constexpr int LDP = kPageTokens + 8;
   __shared__ __attribute__((aligned(16))) uint16_t sC[2][64 * LDC];
   __shared__ __attribute__((aligned(16))) uint16_t sP[RT * 16 * LDP];
-  __shared__ float sM[NK][RT * 16], sL[NK][RT * 16];
+  __shared__ float sM[4][RT * 16], sL[4][RT * 16];
   const LatentBlock bk = reinterpret_cast<const LatentBlock *>(blob + off_blocks)[blockIdx.x];
   if (bk.nrows <= 0) return;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, l15 = lane & 15;
-  const int wk = RT == 4 ? (wave & 1) : wave, wr = RT == 4 ? (wave >> 1) : 0;
+  const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int wk = wave & 3, wr = wave >> 2;
+  const bool scoring = RT > 1 || wr == 0;
   const int32_t *table = reinterpret_cast<const int32_t *>(blob) + bk.table;
 
-  // the next page: through registers, or (R == 512: a row is one 1 KiB wave
-  // access) straight into LDS, where 64 more registers would not fit
-  constexpr bool DMA = R == 512;
-  auto dma = [&](int tile, int buf) {
-    const uint16_t *page = cache + (size_t)table[tile] * (64 * R);
+  // the next page: through registers, RC 16-byte chunks per thread, or (R ==
+  // 512: a row is one 1 KiB wave access) straight into LDS where those
+  // registers would not fit
+  constexpr bool DMA = RC == 8 && RT == 4;
+  auto page_at = [&](int i0) {
+    return cache + (size_t)(i0 == 0 ? bk.page0 : table[bk.tile0 + i0]) * (64 * R);
+  };
+  auto dma = [&](int i0, int buf) {
+    const uint16_t *page = page_at(i0);
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int row = wave * 16 + i;
+    for (int i = 0; i < 8; ++i) {
+      const int row = wave * 8 + i;
       __builtin_amdgcn_global_load_lds(
           (const __attribute__((address_space(1))) void *)(page + (size_t)row * R + lane * 8),
           (__attribute__((address_space(3))) void *)(&sC[buf][row * LDC]), 16, 0, 0);
     }
   };
-  u4 pre[DMA ? 1 : CPT];
-  auto fetch = [&](int tile) {
-    const uint16_t *page = cache + (size_t)table[tile] * (64 * R);
+  u4 pre[RC];
+  auto fetch = [&](int i0) {
+    const uint16_t *page = page_at(i0);
 #pragma unroll
-    for (int i = 0; i < (DMA ? 0 : CPT); ++i) pre[i] = *reinterpret_cast<const u4 *>(page + (tid + i * 256) * 8);
+    for (int i = 0; i < RC; ++i) pre[i] = *reinterpret_cast<const u4 *>(page + (tid + i * 512) * 8);
   };
   auto stage = [&](int buf) {
 #pragma unroll
-    for (int i = 0; i < (DMA ? 0 : CPT); ++i) {
-      const int c = tid + i * 256;
+    for (int i = 0; i < RC; ++i) {
+      const int c = tid + i * 512;
       *reinterpret_cast<u4 *>(&sC[buf][(c / (R / 8)) * LDC + (c % (R / 8)) * 8]) = pre[i];
     }
   };
-  if constexpr (DMA) dma(bk.tile0, 0);
-  else fetch(bk.tile0);
+  if constexpr (DMA) dma(0, 0);
+  else fetch(0);
   // this wave's rows of Q' as B operands (rows past the block re-read its last)
   bf8 q[SR][KS];
   int qpos[SR];
@@ -479,46 +482,44 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
   } else {
     stage(0);
-    if (bk.ntiles > 1) fetch(bk.tile0 + 1);
+    if (bk.ntiles > 1) fetch(1);
   }
   __syncthreads();
   for (int it = 0; it < bk.ntiles; ++it) {
     if constexpr (DMA)  // (its buffer was last read before the previous round's last barrier)
-      if (it + 1 < bk.ntiles) dma(bk.tile0 + it + 1, (it + 1) & 1);
+      if (it + 1 < bk.ntiles) dma(it + 1, (it + 1) & 1);
     const uint16_t *C = sC[it & 1];
-    f4 s[SR][KW];
+    f4 s[SR];
+    if (scoring) {
+      // two chains per row tile (even / odd k-steps)
+      f4 s2[SR];
 #pragma unroll
-    for (int i = 0; i < SR; ++i)
+      for (int i = 0; i < SR; ++i) s[i] = s2[i] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int k = 0; k < KW; ++k) s[i][k] = f4{0.f, 0.f, 0.f, 0.f};
+      for (int ks = 0; ks < KS; ks += 2) {
+        const uint16_t *cr = &C[(wk * 16 + l15) * LDC + ks * 32 + 8 * g];
+        const bf8 c0 = *reinterpret_cast<const bf8 *>(cr), c1 = *reinterpret_cast<const bf8 *>(cr + 32);
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      bf8 c[KW];
+        for (int i = 0; i < SR; ++i) {
+          s[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c0, q[i][ks], s[i], 0, 0, 0);
+          s2[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c1, q[i][ks + 1], s2[i], 0, 0, 0);
+        }
+      }
+      // scale, mask, this wave's maximum of every row
+      const int key0 = (bk.tile0 + it) * 64 + wk * 16 + 4 * g;
 #pragma unroll
-      for (int k = 0; k < KW; ++k)
-        c[k] = *reinterpret_cast<const bf8 *>(&C[((wk * KW + k) * 16 + l15) * LDC + ks * 32 + 8 * g]);
-#pragma unroll
-      for (int k = 0; k < KW; ++k)
-#pragma unroll
-        for (int i = 0; i < SR; ++i)
-          s[i][k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(c[k], q[i][ks], s[i][k], 0, 0, 0);
-    }
-    // scale, mask, this wave's maximum of every row
-    const int key0 = (bk.tile0 + it) * 64 + wk * KW * 16 + 4 * g;
-#pragma unroll
-    for (int i = 0; i < SR; ++i) {
-      float mx = -1e30f;
-#pragma unroll
-      for (int k = 0; k < KW; ++k)
+      for (int i = 0; i < SR; ++i) {
+        float mx = -1e30f;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          const float v = key0 + k * 16 + e <= qpos[i] ? s[i][k][e] * scale_log2 : -INFINITY;
-          s[i][k][e] = v;
+          const float v = key0 + e <= qpos[i] ? (s[i][e] + s2[i][e]) * scale_log2 : -INFINITY;
+          s[i][e] = v;
           mx = fmaxf(mx, v);
         }
-      mx = fmaxf(mx, __shfl_xor(mx, 16));
-      mx = fmaxf(mx, __shfl_xor(mx, 32));
-      if (g == 0) sM[wk][(wr * SR + i) * 16 + l15] = mx;
+        mx = fmaxf(mx, __shfl_xor(mx, 16));
+        mx = fmaxf(mx, __shfl_xor(mx, 32));
+        if (g == 0) sM[wk][(wr * SR + i) * 16 + l15] = mx;
+      }
     }
     __syncthreads();
     float alpha[RT];
@@ -527,33 +528,31 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
     for (int i = 0; i < RT; ++i) {
       float mn = m[i];
 #pragma unroll
-      for (int k = 0; k < NK; ++k) mn = fmaxf(mn, sM[k][i * 16 + l15]);
+      for (int k = 0; k < 4; ++k) mn = fmaxf(mn, sM[k][i * 16 + l15]);
       alpha[i] = __builtin_amdgcn_exp2f(m[i] - mn);
       moved |= mn != m[i];
       m[i] = mn;
     }
+    if (scoring) {
 #pragma unroll
-    for (int i = 0; i < SR; ++i) {
-      float mi = m[i], ai = alpha[i];
-      if (RT == 4 && wr) mi = m[RT == 4 ? 2 + i : i], ai = alpha[RT == 4 ? 2 + i : i];
-      float sum = 0.f;
-#pragma unroll
-      for (int k = 0; k < KW; ++k) {
-        float p[4];
+      for (int i = 0; i < SR; ++i) {
+        const float mi = RT > 1 && wr ? m[RT > 1 ? SR + i : i] : m[i];
+        const float ai = RT > 1 && wr ? alpha[RT > 1 ? SR + i : i] : alpha[i];
+        float p[4], sum = 0.f;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          p[e] = __builtin_amdgcn_exp2f(s[i][k][e] - mi);
+          p[e] = __builtin_amdgcn_exp2f(s[i][e] - mi);
           sum += p[e];
         }
-        *reinterpret_cast<uint2 *>(&sP[((wr * SR + i) * 16 + l15) * LDP + (wk * KW + k) * 16 + 4 * g]) =
+        *reinterpret_cast<uint2 *>(&sP[((wr * SR + i) * 16 + l15) * LDP + wk * 16 + 4 * g]) =
             make_uint2(f2bf(p[0]) | ((uint32_t)f2bf(p[1]) << 16),
                        f2bf(p[2]) | ((uint32_t)f2bf(p[3]) << 16));
+        l[i] = l[i] * ai + sum;
       }
-      l[i] = l[i] * ai + sum;
     }
     if (!DMA && it + 1 < bk.ntiles) {
       stage((it + 1) & 1);  // (last read by the outputs of tile it - 1)
-      if (it + 2 < bk.ntiles) fetch(bk.tile0 + it + 2);
+      if (it + 2 < bk.ntiles) fetch(it + 2);
     }
     __syncthreads();
     if (__any(moved))
@@ -572,6 +571,7 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
       }
 #pragma unroll
       for (int d = 0; d < DT; ++d) {
+        if (NT % 8 && wave * DT + d >= NT) continue;
         const uint16_t *cr =
             &C[(kb * 32 + 4 * g + (l15 >> 2)) * LDC + (wave * DT + d) * 16 + 4 * (l15 & 3)];
         const s4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
@@ -591,32 +591,36 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
       __syncthreads();
     }
   }
+  if (scoring) {
 #pragma unroll
-  for (int i = 0; i < SR; ++i) {
-    float v = l[i];
-    v += __shfl_xor(v, 16);
-    v += __shfl_xor(v, 32);
-    if (g == 0) sL[wk][(wr * SR + i) * 16 + l15] = v;
+    for (int i = 0; i < SR; ++i) {
+      float v = l[i];
+      v += __shfl_xor(v, 16);
+      v += __shfl_xor(v, 32);
+      if (g == 0) sL[wk][(wr * SR + i) * 16 + l15] = v;
+    }
   }
   __syncthreads();
 #pragma unroll
   for (int i = 0; i < RT; ++i) {
     float sum = sL[0][i * 16 + l15];
 #pragma unroll
-    for (int k = 1; k < NK; ++k) sum += sL[k][i * 16 + l15];
+    for (int k = 1; k < 4; ++k) sum += sL[k][i * 16 + l15];
     const int r = i * 16 + l15;
     if (r >= bk.nrows) continue;
     if (bk.slot >= 0) {
       const size_t pr = (size_t)bk.slot * (RT * 16) + r;
 #pragma unroll
       for (int d = 0; d < DT; ++d)
-        *reinterpret_cast<f4 *>(slabs + pr * R + (wave * DT + d) * 16 + 4 * g) = acc[i][d];
+        if (NT % 8 == 0 || wave * DT + d < NT)
+          *reinterpret_cast<f4 *>(slabs + pr * R + (wave * DT + d) * 16 + 4 * g) = acc[i][d];
       if (wave == 0 && g == 0) ml[pr * 2] = m[i], ml[pr * 2 + 1] = sum;
     } else {
       const float inv = __fdiv_rn(1.0f, sum);
       uint16_t *o = O + (size_t)(bk.row0 + r) * R + wave * DT * 16 + 4 * g;
 #pragma unroll
       for (int d = 0; d < DT; ++d) {
+        if (NT % 8 && wave * DT + d >= NT) continue;
         const f4 v = acc[i][d] * inv;
         *reinterpret_cast<uint2 *>(o + d * 16) =
             make_uint2(f2bf(v[0]) | ((uint32_t)f2bf(v[1]) << 16),
@@ -626,31 +630,55 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
   }
 }
 
-// partials of split blocks, in slot order
+// partials of split blocks, in slot order: one workgroup per row, the slots'
+// weights first (one lane each), then the slabs in groups of independent loads
 template <int RC>
-__global__ __launch_bounds__(RC * 16) void latent_merge_kernel(
+constexpr int kMergeThreads = RC <= 4 ? 64 : 128;
+template <int RC>
+__global__ __launch_bounds__(kMergeThreads<RC>) void latent_merge_kernel(
     const char *__restrict__ blob, int off_merges, const float *__restrict__ slabs,
     const float *__restrict__ ml, uint16_t *__restrict__ O, int block_rows) {
-  constexpr int R = RC * 64;
+  constexpr int R = RC * 64, G = 8;
   const LatentMerge mg = reinterpret_cast<const LatentMerge *>(blob + off_merges)[blockIdx.x];
-  const int r = blockIdx.y;
+  const int r = blockIdx.y, lane = threadIdx.x & 63;
   if (r >= mg.nrows) return;
-  float M = -1e30f;
-  for (int i = 0; i < mg.nslots; ++i)
-    M = fmaxf(M, ml[((size_t)(mg.slot0 + i) * block_rows + r) * 2]);
+  const size_t row0 = (size_t)mg.slot0 * block_rows + r;
+  const int col = threadIdx.x * 4;
+  const float *sl = slabs + row0 * R + min(col, R - 4);
   f4 acc = f4{0.f, 0.f, 0.f, 0.f};
-  float sum = 0.f;
-#pragma unroll 4
-  for (int i = 0; i < mg.nslots; ++i) {
-    const size_t pr = (size_t)(mg.slot0 + i) * block_rows + r;
-    const float w = __builtin_amdgcn_exp2f(ml[pr * 2] - M);
-    sum = fmaf(w, ml[pr * 2 + 1], sum);
-    const f4 v = *reinterpret_cast<const f4 *>(slabs + pr * R + threadIdx.x * 4);
+  float M = -1e30f, sum = 0.f;
+  constexpr int L = 64;  // slots at a time (every wave works out the same weights)
+  for (int s0 = 0; s0 < mg.nslots; s0 += L) {
+    const int n = min(L, mg.nslots - s0);
+    const size_t mi = (row0 + (size_t)(s0 + min(lane, n - 1)) * block_rows) * 2;
+    const float m = lane < n ? ml[mi] : -1e30f, l = lane < n ? ml[mi + 1] : 0.f;
+    float mx = m;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) acc[e] = fmaf(w, v[e], acc[e]);
+    for (int o = L / 2; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
+    mx = fmaxf(mx, M);
+    const float a = __builtin_amdgcn_exp2f(M - mx), w = __builtin_amdgcn_exp2f(m - mx);
+    float ls = w * l;
+#pragma unroll
+    for (int o = L / 2; o > 0; o >>= 1) ls += __shfl_xor(ls, o);
+    sum = sum * a + ls;
+    acc *= a;
+    M = mx;
+    for (int i0 = 0; i0 < n; i0 += G) {
+      f4 v[G];
+#pragma unroll
+      for (int i = 0; i < G; ++i)
+        v[i] = *reinterpret_cast<const f4 *>(sl + (size_t)(s0 + min(i0 + i, n - 1)) * block_rows * R);
+#pragma unroll
+      for (int i = 0; i < G; ++i) {
+        const float wi = i0 + i < n ? __shfl(w, i0 + i) : 0.f;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[e] = fmaf(wi, v[i][e], acc[e]);
+      }
+    }
   }
   const float inv = __fdiv_rn(1.0f, sum);
-  *reinterpret_cast<uint2 *>(O + (size_t)(mg.row0 + r) * R + threadIdx.x * 4) =
+  if (col >= R) return;
+  *reinterpret_cast<uint2 *>(O + (size_t)(mg.row0 + r) * R + col) =
       make_uint2(f2bf(acc[0] * inv) | ((uint32_t)f2bf(acc[1] * inv) << 16),
                  f2bf(acc[2] * inv) | ((uint32_t)f2bf(acc[3] * inv) << 16));
 }
@@ -666,7 +694,7 @@ hipError_t launch_latent_attention(const char *blob, const PagedLists &pl, const
   if (pl.num_blocks <= 0) return hipSuccess;
   const float sl = scale * 1.4426950408889634f;
 #define FFMI_LA2(RC, RT)                                                                        \
-  hipLaunchKernelGGL((latent_attn_kernel<RC, RT>), dim3(pl.num_blocks), dim3(256), 0, s, blob,  \
+  hipLaunchKernelGGL((latent_attn_kernel<RC, RT>), dim3(pl.num_blocks), dim3(512), 0, s, blob,  \
                      pl.off_blocks, q, cache, o, slabs, ml, pl.heads, sl)
 #define FFMI_LA(RC)                                                                             \
   case RC:                                                                                      \
@@ -676,7 +704,7 @@ hipError_t launch_latent_attention(const char *blob, const PagedLists &pl, const
     else return hipErrorInvalidValue;                                                           \
     if (pl.num_merges > 0)                                                                      \
       hipLaunchKernelGGL((latent_merge_kernel<RC>), dim3(pl.num_merges, pl.row_tiles * 16),     \
-                         dim3(RC * 16), 0, s, blob, pl.off_merges, slabs, ml, o,                \
+                         dim3(kMergeThreads<RC>), 0, s, blob, pl.off_merges, slabs, ml, o,                \
                          pl.row_tiles * 16);                                                    \
     break
   if (rank % 64) return hipErrorInvalidValue;

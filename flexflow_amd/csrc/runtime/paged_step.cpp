@@ -8,8 +8,10 @@
 namespace ffmi {
 
 static size_t up16(size_t v) { return (v + 15) & ~(size_t)15; }
-// workgroups that fill the chip; fewer blocks than this are split over keys
-constexpr int kTargetBlocks = 256;
+// workgroups that fill the chip; fewer blocks than this are split over keys --
+// from kSplitTiles pages on (a page costs a workgroup ~1.6 us, the merge of the
+// partials ~5 us)
+constexpr int kTargetBlocks = 256, kSplitTiles = 5;
 
 ffmi_status PagedStep::init(int max_tokens, int max_requests, int max_positions,
                             const std::vector<int> &head_counts, int max_slots) {
@@ -128,12 +130,12 @@ ffmi_status PagedStep::stage(const int32_t *token_ids, const std::vector<Seg> &i
     for (const Placed &s : segs) {
       const int nrows = s.n * l.heads, row0 = s.t0 * l.heads;
       for (int r = 0; r < nrows; r += br) {
-        LatentBlock b;
+        LatentBlock b{};
         b.row0 = row0 + r, b.nrows = std::min(br, nrows - r);
         b.seg_row = row0, b.pos0 = s.pos0, b.table = s.table;
         const int last = s.pos0 + (r + b.nrows - 1) / l.heads;  // last visible position
         const int tiles = last / kPageTokens + 1;
-        int ns = std::min(want, tiles);
+        int ns = tiles < kSplitTiles ? 1 : std::min(want, tiles);
         if (slots + ns > max_slots_) ns = 1;
         const int per = (tiles + ns - 1) / ns;
         ns = (tiles + per - 1) / per;
@@ -141,6 +143,7 @@ ffmi_status PagedStep::stage(const int32_t *token_ids, const std::vector<Seg> &i
         for (int i = 0; i < ns; ++i) {
           b.tile0 = i * per, b.ntiles = std::min(per, tiles - i * per);
           b.slot = ns > 1 ? slots++ : -1;
+          b.page0 = reinterpret_cast<const int32_t *>(host)[s.table + b.tile0];
           blocks_.push_back(b);
         }
       }
