@@ -398,6 +398,20 @@ struct LlamaF32 : public ffmi_model {
     memcpy(ir->token_ids, res_h, bc.num_tokens * sizeof(int32_t));
     return FFMI_OK;
   }
+  int vocab_size() const override { return V; }
+  ffmi_status run_inc_logits(const BatchConfig &bc, const int *rows, int n, float *out) override {
+    if (mode != FFMI_MODEL_INC) return FFMI_ERR_INVALID;
+    FFMI_CHECK(bc.num_tokens <= o.max_tokens, FFMI_ERR_INVALID);
+    pack_inc(bc, o.max_requests, slots, &ps);
+    ffmi_status st = forward(1);
+    if (st != FFMI_OK) return st;
+    for (int i = 0; i < n; ++i) {
+      FFMI_CHECK(rows[i] >= 0 && rows[i] < bc.num_tokens, FFMI_ERR_INVALID);
+      FFMI_HIP(hipMemcpy(out + (size_t)i * V, logits + (size_t)rows[i] * V, (size_t)V * 4,
+                         hipMemcpyDeviceToHost));
+    }
+    return FFMI_OK;
+  }
   ffmi_status run_tree(const TreeVerifyBatchConfig &bc, InferenceResult *ir) override {
     if (mode != FFMI_MODEL_TREE) return FFMI_ERR_INVALID;
     FFMI_CHECK(bc.num_tokens <= o.max_tokens, FFMI_ERR_INVALID);

@@ -1305,6 +1305,24 @@ struct LlamaGPU : public ffmi_model {
     memcpy(ir->token_ids, ids_h, bc.num_tokens * sizeof(int32_t));
     return FFMI_OK;
   }
+  int vocab_size() const override { return c.vocab_size; }
+  ffmi_status run_inc_logits(const BatchConfig &bc, const int *rows, int n, float *out) override {
+    if (mode != FFMI_MODEL_INC) return FFMI_ERR_INVALID;
+    FFMI_CHECK(Vl == c.vocab_size, FFMI_ERR_UNSUPPORTED);  // (a vocab shard has its columns only)
+    FFMI_CHECK(bc.num_tokens <= o.max_tokens, FFMI_ERR_INVALID);
+    pack_inc(bc, o.max_requests, slots, &ps);
+    cur_slot = 0;
+    ffmi_status st = forward(1);
+    if (st != FFMI_OK) return st;
+    std::vector<_Float16> row(Vl);
+    for (int i = 0; i < n; ++i) {
+      FFMI_CHECK(rows[i] >= 0 && rows[i] < bc.num_tokens, FFMI_ERR_INVALID);
+      FFMI_HIP(hipMemcpy(row.data(), logits + (size_t)rows[i] * Vl, (size_t)Vl * 2,
+                         hipMemcpyDeviceToHost));
+      for (int v = 0; v < Vl; ++v) out[(size_t)i * Vl + v] = (float)row[v];
+    }
+    return FFMI_OK;
+  }
   ffmi_status run_tree(const TreeVerifyBatchConfig &bc, InferenceResult *ir) override {
     if (mode != FFMI_MODEL_TREE) return FFMI_ERR_INVALID;
     FFMI_CHECK(bc.num_tokens <= o.max_tokens, FFMI_ERR_INVALID);

@@ -255,6 +255,17 @@ def test_greedy_generation(folders, full, pool):
         assert (lead == 0).mean() > (0.99 if full else 0.9)
 
 
+def test_command_line(folders):
+    prompt = tokens(ODD, 12, 77)
+    p = subprocess.run([sys.executable, "-m", "flexflow_amd", "--model", folders["odd"],
+                        "--prompt", " ".join(map(str, prompt)), "--max-length", "20",
+                        "--use-full-precision"], cwd=ROOT, text=True, capture_output=True, timeout=110)
+    assert p.returncode == 0, p.stderr[-2000:]
+    got = json.loads(p.stdout.splitlines()[-1])["tokens"]
+    want, lead = R.greedy(ODD, WEIGHTS["odd"], prompt, 20)
+    assert lead > 1e-4 and got == want
+
+
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_trace_run(folders, tmp_path, dtype):
     """bin/trace_run over a small trace, compared with the plain model."""
