@@ -357,15 +357,17 @@ class RequestManager:
 
     def replay_step(self, llm: Model, entries):
         """One step of given tokens: entries is a list of (id, tokens, want);
-        returns the wanted logits [rows, vocab] fp32, in order (include/ffmi.h
-        ffmi_rm_replay_step)."""
+        returns the wanted logits [rows, vocab] fp32, in the order of the
+        entries and of `want` (include/ffmi.h ffmi_rm_replay_step)."""
         import numpy as np
         arr = (F.ReplayEntry * max(1, len(entries)))()
-        keep, rows = [], 0
+        keep, rows, order = [], 0, []
         for a, (rid, tokens, want) in zip(arr, entries):
             t = np.ascontiguousarray(tokens, np.int32)
-            w = np.ascontiguousarray(want, np.int32)
+            w, back = np.unique(np.asarray(want, np.int32), return_inverse=True)  # ascending
+            w = np.ascontiguousarray(w, np.int32)
             keep += [t, w]
+            order.append(rows + back.reshape(-1))
             a.id, a.num_tokens, a.num_want = rid, len(t), len(w)
             a.tokens = t.ctypes.data_as(ctypes.POINTER(ctypes.c_int32))
             a.want = w.ctypes.data_as(ctypes.POINTER(ctypes.c_int32))
@@ -374,7 +376,7 @@ class RequestManager:
         F.check(F.lib().ffmi_rm_replay_step(self.handle, llm.handle, arr, len(entries),
                                             out.ctypes.data_as(ctypes.c_void_p), rows),
                 "replay step")
-        return out
+        return out[np.concatenate(order)] if order else out
 
     def replay_end(self, llm: Model, rid: int):
         """The replayed request is finished: its slot and pages are free."""

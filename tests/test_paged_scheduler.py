@@ -82,6 +82,15 @@ def test_replay_portions_and_batches():
     assert m.free_pages() == 8
 
 
+def test_replay_returns_the_order_asked_for():
+    rm, m = replay_setup()
+    toks = prompts(3)[2]
+    ref = picks(rm.replay_step(m, [(1, toks, range(len(toks)))]))
+    got = picks(rm.replay_step(m, [(2, toks, [4, 0, 4, 2]), (3, toks[:2], [1])]))
+    assert got == [ref[4], ref[0], ref[4], ref[2], ref[1]]
+    assert len(rm.replay_step(m, [(2, [5], [])])) == 0
+
+
 def test_replay_slots_and_pages_run_out_and_come_back():
     rm, m = replay_setup(pages=4, page=8, slots=2)
     rm.replay_step(m, [(1, [5] * 16, []), (2, [6] * 9, [])])
@@ -97,7 +106,6 @@ def test_replay_slots_and_pages_run_out_and_come_back():
 
 def test_replay_rejects_bad_entries():
     rm, m = replay_setup()
-    for entries in ([(1, [5, 6], [2])], [(1, [5], [-1])], [(1, [5, 6], [1, 0])],
-                    [(1, [5], []), (1, [6], [])]):
+    for entries in ([(1, [5, 6], [2])], [(1, [5], [-1])], [(1, [5], []), (1, [6], [])]):
         with pytest.raises(fa.ffmi.FFMIError):
             rm.replay_step(m, entries)
