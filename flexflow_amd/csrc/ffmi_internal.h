@@ -196,7 +196,13 @@ struct FuseArgs {
   int nss = 0;                      // consumer: partials per row (= K/16)
   const uint16_t *wnorm = nullptr;  // consumer: norm weight [K]
   float eps = 0.f;
+  float limit = 0.f;                // clamped gated unit (bf16 paired tiles)
 };
+// g = min(gate, limit), u = up within +-limit: g sigmoid(1.702 g) (u + 1)
+__device__ __forceinline__ float clamped_glu(float gate, float up, float limit) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g * __fdiv_rn(1.0f, 1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
 hipError_t launch_gemm(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
                        size_t ws_bytes, int T, int N, int K, int epilogue, hipStream_t s,
                        Partials *defer = nullptr, int wpitch = 0, const FuseArgs *fuse = nullptr);
@@ -215,6 +221,11 @@ hipError_t launch_gemm_bf16_relu2(const uint16_t *X, const uint16_t *Wp, uint16_
 hipError_t launch_gemm_bf16_f32(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
                                 size_t ws_bytes, int T, int N, int K, int flags, hipStream_t s,
                                 Partials *defer = nullptr);
+// Wp: gate and up tiles interleaved (2 N columns); Y bf16 = clamped_glu
+size_t gemm_bf16_glu_workspace_bytes(int T, int N, int K);
+hipError_t launch_gemm_bf16_glu(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
+                                size_t ws_bytes, int T, int N, int K, int flags, float limit,
+                                hipStream_t s);
 // fp16 Y[T][N] (row-major) of deferred split-K slabs, summed in slab order and
 // rounded once: the value every consumer of the slabs computes (tensor capture)
 hipError_t launch_partials_reduce(const Partials &p, uint16_t *Y, int T, int N, hipStream_t s);

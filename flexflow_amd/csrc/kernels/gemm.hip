@@ -15,7 +15,7 @@ hipError_t launch_partials_reduce(const Partials &p, uint16_t *Y, int T, int N, 
   const unsigned blocks = (unsigned)((total + 255) / 256);
 #define FFMI_PRED(MS)                                                                          \
   hipLaunchKernelGGL((gemm_reduce_kernel<0, MS>), dim3(blocks), dim3(256), 0, s, p.p, Y, T, N, \
-                     p.NP / 16, p.S, 0)
+                     p.NP / 16, p.S, 0, 0.f)
   if (p.S <= 2) FFMI_PRED(2);
   else if (p.S <= 4) FFMI_PRED(4);
   else if (p.S <= 8) FFMI_PRED(8);

@@ -3,6 +3,10 @@
 
 namespace ffmi {
 
+size_t gemm_bf16_workspace_bytes(int T, int N, int K) {
+  return std::max(gemm_slab_bytes(T, N, K, 0), (size_t)T * ((N + 15) / 16) * 16 * sizeof(float));
+}
+
 hipError_t launch_gemm_bf16_f32(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
                                size_t ws_bytes, int T, int N, int K, int flags, hipStream_t s,
                                Partials *defer) {

@@ -63,10 +63,13 @@ __device__ __forceinline__ uint16_t silu_mul_h(float gacc, float uacc) {
 //   2 bf16, plain     3 bf16, squared ReLU     4 bf16 operands, fp32 slabs out
 //   (4 always writes the split-K slab layout, S = 1 included: its consumer
 //   takes the fp32 sums unrounded)
+//   5 bf16, clamped gated unit of paired [gate|up] tiles (`lim`: its limit)
 template <int EPI>
 constexpr bool epi_bf16 = EPI >= 2;
 template <int EPI>
 constexpr bool epi_f32 = EPI == 4;
+template <int EPI>
+constexpr bool epi_paired = EPI == 1 || EPI == 5;
 // (fragments are 16 raw bytes per lane in either format)
 template <int EPI>
 __device__ __forceinline__ f4 mma16(h8 a, h8 b, f4 c) {
@@ -84,6 +87,13 @@ __device__ __forceinline__ uint16_t out16(float v) {
   }
   if constexpr (epi_bf16<EPI>) return f2bf(v);
   else return __half_as_ushort(__float2half_rn(v));
+}
+
+// output of a (gate, up) pair of sums
+template <int EPI>
+__device__ __forceinline__ uint16_t pair16(float g, float u, float lim) {
+  if constexpr (EPI == 5) return f2bf(clamped_glu(g, u, lim));
+  else return silu_mul_h(g, u);
 }
 
 // Split-K over workgroups (grid.y = S > 1, small-N layers only): each
@@ -453,7 +463,7 @@ __global__ __launch_bounds__(KW * 64) void gemm_skinny_kernel(
     }
     return;
   }
-  if (EPI != 1) {
+  if constexpr (!epi_paired<EPI>) {
 #pragma unroll
     for (int j = 0; j < NT; ++j) {
       int n = (tile0 + j) * 16 + (lane & 15);
@@ -478,7 +488,7 @@ __global__ __launch_bounds__(KW * 64) void gemm_skinny_kernel(
           int m = m0 + i * 16 + (lane >> 4) * 4 + r;
           if (m >= T) continue;
           Y[yp ? act_packed_off(m, n, N) : (size_t)m * N + n] =
-              silu_mul_h(acc[i][0][r], acc[i][1][r]);
+              pair16<EPI>(acc[i][0][r], acc[i][1][r], fz.limit);
         }
     }
   }
@@ -654,11 +664,11 @@ static hipError_t dispatch_fused(const uint16_t *X, const uint16_t *Wp, uint16_t
 template <int E, int MT, int U>
 static hipError_t dispatch_nt(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
                               int T, int N, int K, int KT, int S, hipStream_t s,
-                              int xp, int yp, bool nt, int wpitch) {
+                              int xp, int yp, bool nt, int wpitch, const FuseArgs &fz) {
   int ntiles = (N + 15) / 16;
-  if (!wpitch) wpitch = E == 1 ? 2 * ntiles : ntiles;
-  if constexpr (E == 1)
-    return run<MT, 2, 4, U, 1>(X, Wp, Y, ws, T, N, K, KT, 2 * ntiles, 1, s, xp, yp, nt, wpitch);
+  if (!wpitch) wpitch = epi_paired<E> ? 2 * ntiles : ntiles;
+  if constexpr (epi_paired<E>)
+    return run<MT, 2, 4, U, E>(X, Wp, Y, ws, T, N, K, KT, 2 * ntiles, 1, s, xp, yp, nt, wpitch, fz);
   else {
   // diagnostics: FFMI_SKINNY="NT,KW" forces the tile count and K-split waves
   // of every unsplit skinny launch (A/B runs, scripts/gemm_bench.py)
@@ -763,7 +773,8 @@ static hipError_t dispatch_nt(const uint16_t *X, const uint16_t *Wp, uint16_t *Y
 template <int MTW, int NTW, int EPI>
 __device__ __forceinline__ void mid_store(const f4 (&acc)[MTW][NTW], uint16_t *__restrict__ Y,
                                           float *__restrict__ Ypart, int T, int N, int NTILES,
-                                          int S, int ks, int tile0, int m0, int lane, int yp) {
+                                          int S, int ks, int tile0, int m0, int lane, int yp,
+                                          float lim) {
   const int mr = lane & 15, nq = (lane >> 4) * 4;
   if (S > 1 || epi_f32<EPI>) {
     const int NP = NTILES * 16;
@@ -783,10 +794,10 @@ __device__ __forceinline__ void mid_store(const f4 (&acc)[MTW][NTW], uint16_t *_
     return;
   }
 #pragma unroll
-  for (int j = 0; j < NTW; j += (EPI == 1 ? 2 : 1)) {
+  for (int j = 0; j < NTW; j += (epi_paired<EPI> ? 2 : 1)) {
     const int tile = tile0 + j;
     if (tile >= NTILES) continue;
-    const int n = (EPI == 1 ? (tile >> 1) : tile) * 16 + nq;
+    const int n = (epi_paired<EPI> ? (tile >> 1) : tile) * 16 + nq;
     if (n >= N) continue;
 #pragma unroll
     for (int i = 0; i < MTW; ++i) {
@@ -795,7 +806,7 @@ __device__ __forceinline__ void mid_store(const f4 (&acc)[MTW][NTW], uint16_t *_
       uint16_t o[4];
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        if constexpr (EPI == 1) o[r] = silu_mul_h(acc[i][j][r], acc[i][j + 1][r]);
+        if constexpr (epi_paired<EPI>) o[r] = pair16<EPI>(acc[i][j][r], acc[i][j + 1][r], lim);
         else o[r] = out16<EPI>(acc[i][j][r]);
       uint16_t *dst = yp ? Y + act_packed_off(m, n, N) : Y + (size_t)m * N + n;
       if (n + 4 <= N && (((uintptr_t)dst & 7) == 0)) {
@@ -824,7 +835,7 @@ template <int MTW, int NTW, int PF, int EPI, bool STAMP = false, bool XP = false
 __global__ __launch_bounds__(256, NTW <= 8 && MTW * NTW <= 24 ? 2 : 1) void gemm_mid_kernel(
     const uint16_t *__restrict__ X, const uint16_t *__restrict__ Wp,
     uint16_t *__restrict__ Y, float *__restrict__ Ypart, int T, int N, int K, int KT,
-    int NTILES, int S, int yp, size_t wts, size_t wks) {
+    int NTILES, int S, int yp, size_t wts, size_t wks, float lim) {
   long long st0 = 0, st1 = 0, st2 = 0, ck1 = 0, ck2 = 0;
   if (STAMP) st0 = rt_now();
   static_assert(NTW % 2 == 0, "gate/up tiles come in pairs");
@@ -934,7 +945,7 @@ __global__ __launch_bounds__(256, NTW <= 8 && MTW * NTW <= 24 ? 2 : 1) void gemm
   if (kb < ke) kloop(std::integral_constant<int, MTW>{});
   if (STAMP) st2 = rt_now(), ck2 = __builtin_amdgcn_s_memtime();
 
-  mid_store<MTW, NTW, EPI>(acc, Y, Ypart, T, N, NTILES, S, ks, tile0, m0, lane, yp);
+  mid_store<MTW, NTW, EPI>(acc, Y, Ypart, T, N, NTILES, S, ks, tile0, m0, lane, yp, lim);
   if (STAMP) {
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     const long long st3 = rt_now();
@@ -969,7 +980,7 @@ template <int EPI, int NB>
 __global__ __launch_bounds__(512, 1) void gemm_tile_kernel(
     const uint16_t *__restrict__ X, const uint16_t *__restrict__ Wp, uint16_t *__restrict__ Y,
     float *__restrict__ Yf, int T, int N, int KT, int NTILES, int MT, int nbm, int yp, size_t wts,
-    size_t wks) {
+    size_t wks, float lim) {
   __shared__ __attribute__((aligned(1024))) h8 lds[NB][32][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int nwg = gridDim.x, b = blockIdx.x;
@@ -1041,7 +1052,7 @@ __global__ __launch_bounds__(512, 1) void gemm_tile_kernel(
     }
   }
   mid_store<8, 4, EPI>(acc, Y, Yf, T, N, NTILES, 1, 0, bn * 16 + wn * 4,
-                       (bm * 16 + wm * 8) * 16, lane, yp);
+                       (bm * 16 + wm * 8) * 16, lane, yp, lim);
 }
 
 static inline long long *stamp_buf() {
@@ -1059,7 +1070,7 @@ static long g_stamp_entries = 0;
 // per 4 consecutive output columns (16-B slab loads, 8-B fp16 store).
 template <int EPI, int MAXS>
 __global__ void gemm_reduce_kernel(const float *__restrict__ Ypart, uint16_t *__restrict__ Y,
-                                   int T, int N, int NTILES, int S, int yp) {
+                                   int T, int N, int NTILES, int S, int yp, float lim) {
   const int NP = NTILES * 16;
   const int nq = (N + 3) / 4;
   const long idx = blockIdx.x * (long)blockDim.x + threadIdx.x;
@@ -1070,26 +1081,26 @@ __global__ void gemm_reduce_kernel(const float *__restrict__ Ypart, uint16_t *__
   // all MAXS >= S slab loads go out before the first add (one memory round
   // trip, not S); indices past S re-read the last slab and are not added
   f4 pa[MAXS], pu[MAXS];
-  const float *src = EPI != 1 ? Ypart + (size_t)m * NP + n
+  const float *src = !epi_paired<EPI> ? Ypart + (size_t)m * NP + n
                               : Ypart + (size_t)m * NP + (n >> 4) * 32 + (n & 15);
 #pragma unroll
   for (int s = 0; s < MAXS; ++s) {
     const float *q = src + (size_t)min(s, S - 1) * slab;
     pa[s] = *reinterpret_cast<const f4 *>(q);
-    if (EPI == 1) pu[s] = *reinterpret_cast<const f4 *>(q + 16);
+    if (epi_paired<EPI>) pu[s] = *reinterpret_cast<const f4 *>(q + 16);
   }
   acc = pa[0];
-  if (EPI == 1) up = pu[0];
+  if (epi_paired<EPI>) up = pu[0];
 #pragma unroll
   for (int s = 1; s < MAXS; ++s)
     if (s < S) {
       acc += pa[s];
-      if (EPI == 1) up += pu[s];
+      if (epi_paired<EPI>) up += pu[s];
     }
   uint16_t o[4];
 #pragma unroll
   for (int r = 0; r < 4; ++r)
-    o[r] = EPI == 1 ? silu_mul_h(acc[r], up[r]) : out16<EPI>(acc[r]);
+    o[r] = epi_paired<EPI> ? pair16<EPI>(acc[r], up[r], lim) : out16<EPI>(acc[r]);
   uint16_t *dst = yp ? Y + act_packed_off(m, n, N) : Y + (size_t)m * N + n;
   if (n + 4 <= N && (((uintptr_t)dst & 7) == 0)) {
     *reinterpret_cast<uint2 *>(dst) =
@@ -1215,9 +1226,10 @@ static inline size_t gemm_slab_bytes(int T, int N, int K, int epilogue) {
 template <int E, int MTW, int NTW, int PF>
 static hipError_t run_mid(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
                           size_t ws_bytes, int T, int N, int K, hipStream_t s,
-                          bool xpacked, int yp, int S, Partials *defer, bool nt, int wpitch) {
+                          bool xpacked, int yp, int S, Partials *defer, bool nt, int wpitch,
+                          float lim) {
   const int KT = K / 32;
-  constexpr bool epi = E == 1;  // paired tiles
+  constexpr bool epi = epi_paired<E>;
   const int ntiles = (N + 15) / 16 * (epi ? 2 : 1);
   const size_t wts = w_tile_stride(KT), wks = w_k_stride(wpitch ? wpitch : ntiles);
   const int mtiles = (T + 15) / 16;
@@ -1236,7 +1248,7 @@ static hipError_t run_mid(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, fl
   const bool ntl = nt && mblocks == 1;
 #define FFMI_MID2(ST, XPK, U, NL)                                                                  \
   hipLaunchKernelGGL((gemm_mid_kernel<MTW, NTW, PF, E, ST, XPK, U, NL>), grid, dim3(256), 0, s, X, \
-                     Wp, Y, ws, T, N, K, KT, ntiles, S, yp, wts, wks)
+                     Wp, Y, ws, T, N, K, KT, ntiles, S, yp, wts, wks, lim)
 #define FFMI_MID(ST, XPK)                                     \
   do {                                                        \
     const bool u_ = uld && NTW % 4;                           \
@@ -1278,7 +1290,7 @@ static hipError_t run_mid(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, fl
     const unsigned blocks = (unsigned)((total + 255) / 256);
 #define FFMI_RED(MS)                                                                          \
   hipLaunchKernelGGL((gemm_reduce_kernel<E, MS>), dim3(blocks), dim3(256), 0, s, ws, Y, T, N, \
-                     ntiles, S, yp)
+                     ntiles, S, yp, lim)
     if (S <= 2) FFMI_RED(2);
     else if (S <= 4) FFMI_RED(4);
     else FFMI_RED(8);
@@ -1301,7 +1313,8 @@ static hipError_t launch_gemm_kind(const uint16_t *X, const uint16_t *Wp, uint16
   const bool xp = (epilogue & FFMI_X_PACKED) != 0;
   const int yp = (epilogue & FFMI_Y_PACKED) ? 1 : 0;
   const bool nt = (epilogue & FFMI_W_STREAM) != 0;
-  constexpr int paired = E == 1 ? 1 : 0;
+  constexpr int paired = epi_paired<E> ? 1 : 0;
+  const float lim = fuse ? fuse->limit : 0.f;
   if (epi_f32<E> && (!ws || ws_bytes < (size_t)T * ((N + 15) / 16) * 16 * sizeof(float)))
     return hipErrorInvalidValue;
   if ((xp && K % 32) || (yp && N % 32)) return hipErrorInvalidValue;
@@ -1342,7 +1355,7 @@ static hipError_t launch_gemm_kind(const uint16_t *X, const uint16_t *Wp, uint16
       if (defer) defer->S = 0;
       const size_t wts = w_tile_stride(KT), wks = w_k_stride(wpitch ? wpitch : ntiles);
       hipLaunchKernelGGL((gemm_tile_kernel<E, 4>), dim3(nbn * nbm), dim3(512), 0, s, X, Wp, Y, ws, T,
-                         N, KT, ntiles, mtiles, nbm, yp, wts, wks);
+                         N, KT, ntiles, mtiles, nbm, yp, wts, wks, lim);
       if (epi_f32<E> && defer) defer->p = ws, defer->S = 1, defer->NP = ntiles * 16;
       return hipGetLastError();
     }
@@ -1350,7 +1363,7 @@ static hipError_t launch_gemm_kind(const uint16_t *X, const uint16_t *Wp, uint16
   if (mtiles > 4) {
     const MidPlan p = mid_plan(T, N, K, paired, defer != nullptr && !paired);
 #define FFMI_RUN(M, NW) \
-  return run_mid<E, M, NW, 4>(X, Wp, Y, ws, ws_bytes, T, N, K, s, xp, yp, SM, defer, nt, wpitch)
+  return run_mid<E, M, NW, 4>(X, Wp, Y, ws, ws_bytes, T, N, K, s, xp, yp, SM, defer, nt, wpitch, lim)
     const int SM = epi_f32<E> && !defer ? 1 : p.S;
     if (p.MTW == 4) {
       if (p.NTW == 2) FFMI_RUN(4, 2);
@@ -1375,13 +1388,14 @@ static hipError_t launch_gemm_kind(const uint16_t *X, const uint16_t *Wp, uint16
 #undef FFMI_RUN
   }
   const int xi = xp ? 1 : 0;
+  const FuseArgs fz = fuse ? *fuse : FuseArgs();
   int S = skinny_split(T, N, K, paired, defer != nullptr);
   const size_t need = (size_t)S * T * ((N + 15) / 16) * 16 * sizeof(float);
   if (S > 1 && (!ws || ws_bytes < need)) S = 1;
   hipError_t e;
-  if (mtiles <= 1) e = dispatch_nt<E, 1, 8>(X, Wp, Y, ws, T, N, K, KT, S, s, xi, yp, nt, wpitch);
-  else if (mtiles <= 2) e = dispatch_nt<E, 2, 8>(X, Wp, Y, ws, T, N, K, KT, S, s, xi, yp, nt, wpitch);
-  else e = dispatch_nt<E, 4, 4>(X, Wp, Y, ws, T, N, K, KT, S, s, xi, yp, nt, wpitch);
+  if (mtiles <= 1) e = dispatch_nt<E, 1, 8>(X, Wp, Y, ws, T, N, K, KT, S, s, xi, yp, nt, wpitch, fz);
+  else if (mtiles <= 2) e = dispatch_nt<E, 2, 8>(X, Wp, Y, ws, T, N, K, KT, S, s, xi, yp, nt, wpitch, fz);
+  else e = dispatch_nt<E, 4, 4>(X, Wp, Y, ws, T, N, K, KT, S, s, xi, yp, nt, wpitch, fz);
   if ((S > 1 || epi_f32<E>) && defer && e == hipSuccess) defer->p = ws, defer->S = S, defer->NP = (N + 15) / 16 * 16;
   return e;
 }

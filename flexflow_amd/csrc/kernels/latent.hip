@@ -1,219 +1,14 @@
-// latent.hip -- latent attention over a paged cache (latent.h), the 32-bit
-// residual stream's post-sublayer norms, and the loaders' packing kernels.
+// latent.hip -- latent attention over a paged cache (latent.h).
 #include <algorithm>
 
+#include "device_util.h"
 #include "latent.h"
 
 namespace ffmi {
 
 // ---------------------------------------------------------------------------
-// residual stream (fp32 x, bf16 packed copy for the GEMMs)
-// ---------------------------------------------------------------------------
-__device__ __forceinline__ uint4 pack8_bf16(const f4 &a, const f4 &b) {
-  uint4 o;
-  o.x = f2bf(a[0]) | ((uint32_t)f2bf(a[1]) << 16);
-  o.y = f2bf(a[2]) | ((uint32_t)f2bf(a[3]) << 16);
-  o.z = f2bf(b[0]) | ((uint32_t)f2bf(b[1]) << 16);
-  o.w = f2bf(b[2]) | ((uint32_t)f2bf(b[3]) << 16);
-  return o;
-}
-__device__ __forceinline__ void unpack8_bf16(const uint4 &v, f4 &a, f4 &b) {
-  const uint32_t w[4] = {v.x, v.y, v.z, v.w};
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const float lo = __builtin_bit_cast(float, w[i] << 16);
-    const float hi = __builtin_bit_cast(float, w[i] & 0xffff0000u);
-    if (i < 2) a[2 * i] = lo, a[2 * i + 1] = hi;
-    else b[2 * i - 4] = lo, b[2 * i - 3] = hi;
-  }
-}
-
-__global__ __launch_bounds__(256) void embed_pos_kernel(
-    const char *__restrict__ blob_src, uint4 *__restrict__ blob_dst, int blob_n16,
-    const uint16_t *__restrict__ embed, const uint16_t *__restrict__ pos, float *__restrict__ x,
-    uint16_t *__restrict__ xb, int H) {
-  const int t = blockIdx.x;
-  const PagedToken tk = reinterpret_cast<const PagedToken *>(blob_src)[t];  // tokens come first
-  const uint4 *src = reinterpret_cast<const uint4 *>(blob_src);
-  for (int i = t * 256 + threadIdx.x; i < blob_n16; i += gridDim.x * 256) blob_dst[i] = src[i];
-  for (int c = threadIdx.x; c < H / 8; c += 256) {
-    f4 a, b, pa, pb;
-    unpack8_bf16(*reinterpret_cast<const uint4 *>(embed + (size_t)tk.token * H + c * 8), a, b);
-    unpack8_bf16(*reinterpret_cast<const uint4 *>(pos + (size_t)tk.pos * H + c * 8), pa, pb);
-    a += pa, b += pb;
-    *reinterpret_cast<f4 *>(x + (size_t)t * H + c * 8) = a;
-    *reinterpret_cast<f4 *>(x + (size_t)t * H + c * 8 + 4) = b;
-    if (xb) *reinterpret_cast<uint4 *>(xb + act_packed_off(t, c * 8, H)) = pack8_bf16(a, b);
-  }
-}
-
-hipError_t launch_embed_pos(const char *blob_src, char *blob_dst, size_t blob_bytes,
-                            const uint16_t *embed, const uint16_t *pos, float *x, uint16_t *xb,
-                            int T, int H, hipStream_t s) {
-  if (T <= 0) return hipSuccess;
-  if (H % 32) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(embed_pos_kernel, dim3(T), dim3(256), 0, s, blob_src,
-                     reinterpret_cast<uint4 *>(blob_dst), (int)((blob_bytes + 15) / 16), embed, pos,
-                     x, xb, H);
-  return hipGetLastError();
-}
-
-template <int NT>
-__device__ __forceinline__ float row_sum(float v, float *sh) {
-#pragma unroll
-  for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
-  if ((threadIdx.x & 63) == 0) sh[threadIdx.x >> 6] = v;
-  __syncthreads();
-  v = sh[0];
-#pragma unroll
-  for (int i = 1; i < NT / 64; ++i) v += sh[i];
-  return v;
-}
-__device__ __forceinline__ float inv_rms(float ss, int n, float eps) {
-  return __fdiv_rn(1.0f, sqrtf(__fdiv_rn(ss, (float)n) + eps));
-}
-
-// One workgroup per row; the slab, x and w loads of a chunk are all issued
-// before the reduction.
-template <int NT, int MAXC, int MAXS>
-__global__ __launch_bounds__(NT) void post_norm_kernel(const float *__restrict__ yp, int S, int NP,
-                                                       const float *__restrict__ w,
-                                                       float *__restrict__ x,
-                                                       uint16_t *__restrict__ xb, int H, int n,
-                                                       float eps) {
-  __shared__ float sh[NT / 64];
-  const int row = blockIdx.x, T = gridDim.x, nchunk = H >> 3;
-  f4 y[MAXC][2], xv[MAXC][2], wv[MAXC][2];
-  float ss = 0.f;
-#pragma unroll
-  for (int c = 0; c < MAXC; ++c) {
-    const int ch = min((int)threadIdx.x + c * NT, nchunk - 1);
-    const float *q = yp + (size_t)row * NP + ch * 8;
-    f4 lo[MAXS], hi[MAXS];
-#pragma unroll
-    for (int sl = 0; sl < MAXS; ++sl) {
-      const float *qs = q + (size_t)min(sl, S - 1) * T * NP;
-      lo[sl] = *reinterpret_cast<const f4 *>(qs);
-      hi[sl] = *reinterpret_cast<const f4 *>(qs + 4);
-    }
-#pragma unroll
-    for (int h = 0; h < 2; ++h) {
-      xv[c][h] = *reinterpret_cast<const f4 *>(x + (size_t)row * H + ch * 8 + 4 * h);
-      wv[c][h] = *reinterpret_cast<const f4 *>(w + ch * 8 + 4 * h);
-    }
-    y[c][0] = lo[0], y[c][1] = hi[0];
-#pragma unroll
-    for (int sl = 1; sl < MAXS; ++sl)
-      if (sl < S) y[c][0] += lo[sl], y[c][1] += hi[sl];
-    if ((int)threadIdx.x + c * NT < nchunk)
-#pragma unroll
-      for (int h = 0; h < 2; ++h)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) ss = fmaf(y[c][h][e], y[c][h][e], ss);
-  }
-  const float r = inv_rms(row_sum<NT>(ss, sh), n, eps);
-#pragma unroll
-  for (int c = 0; c < MAXC; ++c) {
-    const int ch = threadIdx.x + c * NT;
-    if (ch >= nchunk) continue;
-#pragma unroll
-    for (int h = 0; h < 2; ++h)
-#pragma unroll
-      for (int e = 0; e < 4; ++e) xv[c][h][e] += y[c][h][e] * r * wv[c][h][e];
-    *reinterpret_cast<f4 *>(x + (size_t)row * H + ch * 8) = xv[c][0];
-    *reinterpret_cast<f4 *>(x + (size_t)row * H + ch * 8 + 4) = xv[c][1];
-    if (xb)
-      *reinterpret_cast<uint4 *>(xb + act_packed_off(row, ch * 8, H)) = pack8_bf16(xv[c][0], xv[c][1]);
-  }
-}
-
-hipError_t launch_post_norm(Partials y, const float *w, float *x, uint16_t *xb, int T, int H, int n,
-                            float eps, hipStream_t s) {
-  if (T <= 0) return hipSuccess;
-  if (H % 32 || y.NP < H || y.NP % 4 || y.S < 1 || y.S > 8 || !y.p) return hipErrorInvalidValue;
-  const int nchunk = H / 8;
-#define FFMI_PN(NT, MC, MS)                                                                     \
-  hipLaunchKernelGGL((post_norm_kernel<NT, MC, MS>), dim3(T), dim3(NT), 0, s, y.p, y.S, y.NP, w, \
-                     x, xb, H, n, eps)
-#define FFMI_PNS(NT, MC)               \
-  do {                                 \
-    if (y.S == 1) FFMI_PN(NT, MC, 1);  \
-    else if (y.S == 2) FFMI_PN(NT, MC, 2); \
-    else if (y.S <= 4) FFMI_PN(NT, MC, 4); \
-    else FFMI_PN(NT, MC, 8);           \
-  } while (0)
-  if (nchunk <= 128) FFMI_PNS(128, 1);
-  else if (nchunk <= 256) FFMI_PNS(256, 1);
-  else if (nchunk <= 512) FFMI_PNS(512, 1);
-  else if (nchunk <= 1024) FFMI_PNS(1024, 1);
-  else if (nchunk <= 2048) FFMI_PNS(1024, 2);
-  else return hipErrorInvalidValue;
-#undef FFMI_PNS
-#undef FFMI_PN
-  return hipGetLastError();
-}
-
-__global__ __launch_bounds__(256) void row_norm_kernel(const int32_t *__restrict__ rows,
-                                                       const float *__restrict__ x,
-                                                       const float *__restrict__ w,
-                                                       uint16_t *__restrict__ hb,
-                                                       float *__restrict__ hf, int H, int n,
-                                                       float eps) {
-  __shared__ float sh[4];
-  const int i = blockIdx.x;
-  const float *xr = x + (size_t)rows[i] * H;
-  float ss = 0.f;
-  for (int c = threadIdx.x; c < H / 4; c += 256) {
-    const f4 v = *reinterpret_cast<const f4 *>(xr + c * 4);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) ss = fmaf(v[e], v[e], ss);
-  }
-  const float r = inv_rms(row_sum<256>(ss, sh), n, eps);
-  for (int c = threadIdx.x; c < H / 8; c += 256) {
-    f4 v[2];
-#pragma unroll
-    for (int h = 0; h < 2; ++h) {
-      v[h] = *reinterpret_cast<const f4 *>(xr + c * 8 + 4 * h);
-      const f4 wv = *reinterpret_cast<const f4 *>(w + c * 8 + 4 * h);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) v[h][e] = v[h][e] * r * wv[e];
-      if (hf) *reinterpret_cast<f4 *>(hf + (size_t)i * H + c * 8 + 4 * h) = v[h];
-    }
-    if (hb) *reinterpret_cast<uint4 *>(hb + act_packed_off(i, c * 8, H)) = pack8_bf16(v[0], v[1]);
-  }
-}
-
-hipError_t launch_row_norm(const char *blob, int off_rows, const float *x, const float *w,
-                           uint16_t *hb, float *hf, int R, int H, int n, float eps, hipStream_t s) {
-  if (R <= 0) return hipSuccess;
-  if (H % 32) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(row_norm_kernel, dim3(R), dim3(256), 0, s,
-                     reinterpret_cast<const int32_t *>(blob + off_rows), x, w, hb, hf, H, n, eps);
-  return hipGetLastError();
-}
-
-__global__ void relu2_f32_kernel(float *u, size_t n) {
-  for (size_t i = blockIdx.x * (size_t)blockDim.x + threadIdx.x; i < n;
-       i += (size_t)gridDim.x * blockDim.x) {
-    const float v = fmaxf(u[i], 0.f);
-    u[i] = v * v;
-  }
-}
-hipError_t launch_relu2_f32(float *u, size_t n, hipStream_t s) {
-  if (n == 0) return hipSuccess;
-  hipLaunchKernelGGL(relu2_f32_kernel, dim3((unsigned)std::min<size_t>((n + 255) / 256, 16384)),
-                     dim3(256), 0, s, u, n);
-  return hipGetLastError();
-}
-
-// ---------------------------------------------------------------------------
 // latent store: one wave per token
 // ---------------------------------------------------------------------------
-__device__ __forceinline__ float ld_elem(const uint16_t *p) { return bf2f(*p); }
-__device__ __forceinline__ float ld_elem(const float *p) { return *p; }
-__device__ __forceinline__ void st_elem(uint16_t *p, float v) { *p = f2bf(v); }
-__device__ __forceinline__ void st_elem(float *p, float v) { *p = v; }
-
 template <class E>
 __device__ __forceinline__ void latent_store_token(const PagedToken &tk, const E *d, const float *w,
                                                    E *cache, int rank, int n, float eps) {
@@ -417,7 +212,7 @@ __global__ __launch_bounds__(512) void latent_attn_kernel(
   __shared__ __attribute__((aligned(16))) uint16_t sC[2][64 * LDC];
   __shared__ __attribute__((aligned(16))) uint16_t sP[RT * 16 * LDP];
   __shared__ float sM[4][RT * 16], sL[4][RT * 16];
-  const LatentBlock bk = reinterpret_cast<const LatentBlock *>(blob + off_blocks)[blockIdx.x];
+  const PagedBlock bk = reinterpret_cast<const PagedBlock *>(blob + off_blocks)[blockIdx.x];
   if (bk.nrows <= 0) return;
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -639,7 +434,7 @@ __global__ __launch_bounds__(kMergeThreads<RC>) void latent_merge_kernel(
     const char *__restrict__ blob, int off_merges, const float *__restrict__ slabs,
     const float *__restrict__ ml, uint16_t *__restrict__ O, int block_rows) {
   constexpr int R = RC * 64, G = 8;
-  const LatentMerge mg = reinterpret_cast<const LatentMerge *>(blob + off_merges)[blockIdx.x];
+  const PagedMerge mg = reinterpret_cast<const PagedMerge *>(blob + off_merges)[blockIdx.x];
   const int r = blockIdx.y, lane = threadIdx.x & 63;
   if (r >= mg.nrows) return;
   const size_t row0 = (size_t)mg.slot0 * block_rows + r;
@@ -734,7 +529,7 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const char *__restrict
                                                           float scale) {
   __shared__ float sq[kRowsMaxRank], sp[256], red[4];
   __shared__ int srow[256];
-  const LatentBlock bk = reinterpret_cast<const LatentBlock *>(blob + off_blocks)[blockIdx.x];
+  const PagedBlock bk = reinterpret_cast<const PagedBlock *>(blob + off_blocks)[blockIdx.x];
   const int r = blockIdx.y, tid = threadIdx.x;
   if (r >= bk.nrows) return;
   const int32_t *table = reinterpret_cast<const int32_t *>(blob) + bk.table;
@@ -805,67 +600,6 @@ hipError_t launch_latent_attention_rows(const char *blob, const PagedLists &pl, 
   else
     hipLaunchKernelGGL(latent_rows_kernel<float>, grid, dim3(256), 0, s, blob, pl.off_blocks,
                        (const float *)q, (const float *)cache, (float *)o, pl.heads, rank, scale);
-  return hipGetLastError();
-}
-
-// ---------------------------------------------------------------------------
-// loading
-// ---------------------------------------------------------------------------
-__device__ __forceinline__ uint16_t pack_elem(const uint16_t *src, int ld, const PackSpec &p, int n,
-                                              int k) {
-  const int hn = n / p.np, jn = n % p.np, hk = k / p.kp, jk = k % p.kp;
-  if (hn >= p.rows || jn >= p.nb || hk >= p.cols || jk >= p.kb) return 0;
-  if (p.transpose) return src[((size_t)hn * p.kb + jk) * ld + jn];
-  return src[(size_t)(hn * p.nb + jn) * ld + hk * p.kb + jk];
-}
-__global__ void pack_bf16_kernel(const uint16_t *__restrict__ src, int ld, PackSpec p,
-                                 uint16_t *__restrict__ dst, int NT, int KT, size_t ts, size_t ks) {
-  const long gid = blockIdx.x * (long)blockDim.x + threadIdx.x;
-  if (gid >= (long)NT * KT * 64) return;
-  const int lane = (int)(gid & 63), kt = (int)((gid >> 6) % KT), nt = (int)((gid >> 6) / KT);
-  const int n = nt * 16 + (lane & 15), k = kt * 32 + 8 * (lane >> 4);
-  uint32_t v[4];
-#pragma unroll
-  for (int j = 0; j < 4; ++j)
-    v[j] = pack_elem(src, ld, p, n, k + 2 * j) |
-           ((uint32_t)pack_elem(src, ld, p, n, k + 2 * j + 1) << 16);
-  *reinterpret_cast<uint4 *>(dst + nt * ts + kt * ks + lane * 8) = make_uint4(v[0], v[1], v[2], v[3]);
-}
-hipError_t launch_pack_bf16(const uint16_t *src, int ld, const PackSpec &p, uint16_t *dst,
-                            int tile_offset, int pitch, bool perhead, hipStream_t s) {
-  const int N = p.rows * p.np, K = p.cols * p.kp;
-  if (N % 16 || K % 32) return hipErrorInvalidValue;
-  const int NT = N / 16, KT = K / 32;
-  const size_t ts = perhead ? (size_t)KT * 512 : w_tile_stride(KT);
-  const size_t ks = perhead ? 512 : w_k_stride(pitch);
-  hipLaunchKernelGGL(pack_bf16_kernel, dim3((unsigned)(((long)NT * KT * 64 + 255) / 256)),
-                     dim3(256), 0, s, src, ld, p, dst + tile_offset * ts, NT, KT, ts, ks);
-  return hipGetLastError();
-}
-__global__ void pack_f32_kernel(const uint16_t *__restrict__ src, int ld, PackSpec p,
-                                float *__restrict__ dst, int N, int K) {
-  const long i = blockIdx.x * (long)blockDim.x + threadIdx.x;
-  if (i >= (long)N * K) return;
-  dst[i] = bf2f(pack_elem(src, ld, p, (int)(i / K), (int)(i % K)));
-}
-hipError_t launch_pack_f32(const uint16_t *src, int ld, const PackSpec &p, float *dst,
-                           hipStream_t s) {
-  const int N = p.rows * p.np, K = p.cols * p.kp;
-  hipLaunchKernelGGL(pack_f32_kernel, dim3((unsigned)(((long)N * K + 255) / 256)), dim3(256), 0, s,
-                     src, ld, p, dst, N, K);
-  return hipGetLastError();
-}
-
-__global__ void pack_act_bf16_kernel(const uint16_t *__restrict__ X, uint16_t *__restrict__ Xp,
-                                     int T, int K) {
-  const int kt = blockIdx.x, mt = blockIdx.y, l = threadIdx.x, r = mt * 16 + (l & 15);
-  uint4 v = make_uint4(0, 0, 0, 0);
-  if (r < T) v = *reinterpret_cast<const uint4 *>(X + (size_t)r * K + kt * 32 + 8 * (l >> 4));
-  *reinterpret_cast<uint4 *>(Xp + act_packed_off(r, kt * 32 + 8 * (l >> 4), K)) = v;
-}
-hipError_t launch_pack_act_bf16(const uint16_t *X, uint16_t *Xp, int T, int K, hipStream_t s) {
-  if (T <= 0 || K % 32) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(pack_act_bf16_kernel, dim3(K / 32, (T + 15) / 16), dim3(64), 0, s, X, Xp, T, K);
   return hipGetLastError();
 }
 

@@ -1,0 +1,385 @@
+// lightning.hip -- linear attention with a fixed decay per head (lightning.h).
+#include "lightning.h"
+
+#include <algorithm>
+
+#include "device_util.h"
+
+namespace ffmi {
+
+typedef short s4 __attribute__((ext_vector_type(4)));
+typedef uint32_t u4 __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ float sigmoid_f(float v) { return __fdiv_rn(1.0f, 1.0f + expf(-v)); }
+__device__ __forceinline__ float silu_f(float v) { return v * sigmoid_f(v); }
+__device__ __forceinline__ float sum_at(const Partials &y, size_t slab, size_t at) {
+  float v = y.p[at];
+  for (int s = 1; s < y.S; ++s) v += y.p[at + s * slab];
+  return v;
+}
+
+// ---------------------------------------------------------------------------
+// token by token: a workgroup per (32 value columns, head, span), the state in
+// registers: thread = (row ri of every 32 rows, 4 columns)
+// ---------------------------------------------------------------------------
+template <int P>
+__global__ __launch_bounds__(256) void lightning_recurrent_kernel(const char *__restrict__ blob,
+                                                                  int off_spans, Lightning a,
+                                                                  int limit) {
+  __shared__ float sq[2][P * 32], sk[2][P * 32], sv[2][32], red[2][4][32];
+  const PagedSpan sp = reinterpret_cast<const PagedSpan *>(blob + off_spans)[blockIdx.z];
+  if (sp.n > limit) return;
+  const int tid = threadIdx.x, h = blockIdx.y, c0 = blockIdx.x * 32;
+  const int cl = (tid & 7) * 4, ri = tid >> 3;
+  float *S = a.state + (((size_t)sp.slot * a.H + h) * a.dg) * a.vg + c0 + cl;
+  const float decay = a.powers[(size_t)h * (kLightningChunk + 1) + 1];
+  f4 st[P];
+#pragma unroll
+  for (int p = 0; p < P; ++p) {
+    const int row = p * 32 + ri;
+    st[p] = f4{0.f, 0.f, 0.f, 0.f};
+    if (sp.pos0 > 0 && row < a.dg) st[p] = *reinterpret_cast<const f4 *>(S + (size_t)row * a.vg);
+  }
+  const size_t slab = (size_t)a.T * a.y.NP;
+  const size_t colk = (size_t)a.H * a.dg, colv = 2 * colk;
+  auto load = [&](int t, int b) {
+    const size_t row = (size_t)(sp.t0 + t) * a.y.NP;
+    for (int i = tid; i < 2 * a.dg + 32; i += 256) {
+      if (i < a.dg) sq[b][i] = silu_f(sum_at(a.y, slab, row + (size_t)h * a.dg + i));
+      else if (i < 2 * a.dg) sk[b][i - a.dg] = silu_f(sum_at(a.y, slab, row + colk + (size_t)h * a.dg + i - a.dg));
+      else sv[b][i - 2 * a.dg] = silu_f(sum_at(a.y, slab, row + colv + (size_t)h * a.vg + c0 + i - 2 * a.dg));
+    }
+  };
+  load(0, 0);
+  for (int t = 0; t < sp.n; ++t) {
+    const int b = t & 1;
+    __syncthreads();
+    const f4 v = *reinterpret_cast<const f4 *>(&sv[b][cl]);
+    f4 o = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int p = 0; p < P; ++p) {
+      const int row = p * 32 + ri;
+      if (row >= a.dg) continue;
+      const float k = sk[b][row], q = sq[b][row];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        st[p][e] = fmaf(decay, st[p][e], k * v[e]);
+        o[e] = fmaf(q, st[p][e], o[e]);
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      o[e] += __shfl_xor(o[e], 8);
+      o[e] += __shfl_xor(o[e], 16);
+      o[e] += __shfl_xor(o[e], 32);
+    }
+    if ((tid & 63) < 8) *reinterpret_cast<f4 *>(&red[b][tid >> 6][cl]) = o;
+    if (t + 1 < sp.n) load(t + 1, b ^ 1);
+    __syncthreads();
+    if (tid < 32)
+      a.o[(size_t)(sp.t0 + t) * a.H * a.vg + (size_t)h * a.vg + c0 + tid] =
+          red[b][0][tid] + red[b][1][tid] + red[b][2][tid] + red[b][3][tid];
+  }
+#pragma unroll
+  for (int p = 0; p < P; ++p) {
+    const int row = p * 32 + ri;
+    if (row < a.dg) *reinterpret_cast<f4 *>(S + (size_t)row * a.vg) = st[p];
+  }
+}
+
+static bool bad_shape(const Lightning &a, int max_dim) {
+  return a.H < 1 || a.dg % 32 || a.vg % 32 || a.dg < 32 || a.vg < 32 || a.dg > max_dim || a.y.S < 1 ||
+         a.y.NP < 2 * a.H * (a.dg + a.vg);
+}
+
+hipError_t launch_lightning_recurrent(const char *blob, int off_spans, int num_spans,
+                                      const Lightning &a, int limit, hipStream_t s) {
+  if (num_spans <= 0) return hipSuccess;
+  if (bad_shape(a, kLightningMaxDim)) return hipErrorInvalidValue;
+  const dim3 grid(a.vg / 32, a.H, num_spans);
+#define FFMI_LR(P)                                                                                 \
+  hipLaunchKernelGGL((lightning_recurrent_kernel<P>), grid, dim3(256), 0, s, blob, off_spans, a, limit)
+  if (a.dg <= 32) FFMI_LR(1);
+  else if (a.dg <= 64) FFMI_LR(2);
+  else if (a.dg <= 128) FFMI_LR(4);
+  else if (a.dg <= 256) FFMI_LR(8);
+  else FFMI_LR(16);
+#undef FFMI_LR
+  return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// chunks
+// ---------------------------------------------------------------------------
+// silu of the q | k | v columns, 8 a thread
+__global__ __launch_bounds__(256) void lightning_qkv_kernel(Lightning a, int cols) {
+  const int n8 = cols / 8;
+  const long id = blockIdx.x * 256L + threadIdx.x;
+  if (id >= (long)a.T * n8) return;
+  const int t = (int)(id / n8), c = (int)(id % n8) * 8;
+  const float *p = a.y.p + (size_t)t * a.y.NP + c;
+  f4 lo = *reinterpret_cast<const f4 *>(p), hi = *reinterpret_cast<const f4 *>(p + 4);
+  for (int s = 1; s < a.y.S; ++s) {
+    const float *ps = p + (size_t)s * a.T * a.y.NP;
+    lo += *reinterpret_cast<const f4 *>(ps), hi += *reinterpret_cast<const f4 *>(ps + 4);
+  }
+#pragma unroll
+  for (int e = 0; e < 4; ++e) lo[e] = silu_f(lo[e]), hi[e] = silu_f(hi[e]);
+  *reinterpret_cast<uint4 *>(a.qkv + (size_t)t * cols + c) = pack8_bf16(lo, hi);
+}
+
+// value and remainder in bf16
+__device__ __forceinline__ void split2(float v, __bf16 &hi, __bf16 &lo) {
+  hi = (__bf16)v;
+  lo = (__bf16)(v - (float)hi);
+}
+// operand of 8 k-values from row-major LDS rows: column c0 + (lane & 15), rows
+// kb * 32 + {4g .. 4g + 3, 16 + 4g ..}
+template <int LD>
+__device__ __forceinline__ bf8 read_columns(const uint16_t *tile, int kb, int c0) {
+  const int lane = threadIdx.x & 63, g = lane >> 4, l15 = lane & 15;
+  const uint16_t *p = tile + (kb * 32 + 4 * g + (l15 >> 2)) * LD + c0 + 4 * (l15 & 3);
+  const s4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4 *)(p));
+  const s4 hi =
+      __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4 *)(p + 16 * LD));
+  return __builtin_bit_cast(bf8, __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+}
+
+// A workgroup per (64 value columns, head, span).  Per chunk of 64 tokens
+//   O^T = S_prev^T Q^T, row i times d^(i + 1),  + V^T . P^T with
+//   P = (q_i . k_j) d^(i - j) for j <= i;
+//   S   = d^n S_prev + K^T . (v_j d^(n - 1 - j))
+// Wave w: rows 16 w .. of the outputs, value columns 16 w .. of the state, which
+// stays in its registers (lane: 4 rows dt * 16 + 4g .. of one column) and goes to
+// LDS once a chunk as the operand [column][row] of every wave's outputs.
+template <int KS>
+__global__ __launch_bounds__(256) void lightning_chunk_kernel(const char *__restrict__ blob,
+                                                              int off_spans, Lightning a, int limit) {
+  constexpr int DK = KS * 32, LDK = DK + 8, LDV = 64 + 8, C = kLightningChunk;
+  __shared__ __attribute__((aligned(16))) uint16_t sK[C * LDK], sV[C * LDV], sHi[64 * LDK], sLo[64 * LDK];
+  __shared__ float pw[C + 1];
+  const PagedSpan sp = reinterpret_cast<const PagedSpan *>(blob + off_spans)[blockIdx.z];
+  if (sp.n <= limit) return;
+  const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int h = blockIdx.y, c0 = blockIdx.x * 64, cols = a.H * (2 * a.dg + a.vg);
+  const uint16_t *Q = a.qkv + (size_t)sp.t0 * cols + (size_t)h * a.dg;
+  const uint16_t *K = Q + (size_t)a.H * a.dg;
+  const uint16_t *V = a.qkv + (size_t)sp.t0 * cols + (size_t)2 * a.H * a.dg + (size_t)h * a.vg + c0;
+  if (tid <= C) pw[tid] = a.powers[(size_t)h * (C + 1) + tid];
+  const int vw = min(64, a.vg - c0);  // value columns of this workgroup
+
+  const u4 zero = {0, 0, 0, 0};
+  u4 pk[KS], pv[2];
+  auto fetch = [&](int t0) {  // rows past the span and columns past the widths: zeros
+#pragma unroll
+    for (int i = 0; i < KS; ++i) {
+      const int ch = tid + i * 256, r = ch / (DK / 8), c = ch % (DK / 8) * 8;
+      pk[i] = zero;
+      if (t0 + r < sp.n && c < a.dg) pk[i] = *reinterpret_cast<const u4 *>(K + (size_t)(t0 + r) * cols + c);
+    }
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int ch = tid + i * 256, r = ch >> 3, c = (ch & 7) * 8;
+      pv[i] = zero;
+      if (t0 + r < sp.n && c < vw) pv[i] = *reinterpret_cast<const u4 *>(V + (size_t)(t0 + r) * cols + c);
+    }
+  };
+  auto stage = [&]() {
+#pragma unroll
+    for (int i = 0; i < KS; ++i) {
+      const int ch = tid + i * 256;
+      *reinterpret_cast<u4 *>(&sK[(ch / (DK / 8)) * LDK + ch % (DK / 8) * 8]) = pk[i];
+    }
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int ch = tid + i * 256;
+      *reinterpret_cast<u4 *>(&sV[(ch >> 3) * LDV + (ch & 7) * 8]) = pv[i];
+    }
+  };
+  fetch(0);
+  // the state: rows dt * 16 + 4g + e, column wave * 16 + l15
+  f4 st[2 * KS];
+  const int vcol = wave * 16 + l15;
+  float *S = a.state + (((size_t)sp.slot * a.H + h) * a.dg) * a.vg + c0 + vcol;
+#pragma unroll
+  for (int dt = 0; dt < 2 * KS; ++dt) {
+    st[dt] = f4{0.f, 0.f, 0.f, 0.f};
+    if (sp.pos0 > 0 && dt * 16 < a.dg && vcol < vw)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) st[dt][e] = S[(size_t)(dt * 16 + 4 * g + e) * a.vg];
+  }
+  auto publish = [&]() {
+#pragma unroll
+    for (int dt = 0; dt < 2 * KS; ++dt) {
+      __bf16 hi[4], lo[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) split2(st[dt][e], hi[e], lo[e]);
+      const int at = vcol * LDK + dt * 16 + 4 * g;
+      auto two = [](const __bf16 *v) {
+        return make_uint2(__builtin_bit_cast(uint16_t, v[0]) | ((uint32_t)__builtin_bit_cast(uint16_t, v[1]) << 16),
+                          __builtin_bit_cast(uint16_t, v[2]) | ((uint32_t)__builtin_bit_cast(uint16_t, v[3]) << 16));
+      };
+      *reinterpret_cast<uint2 *>(&sHi[at]) = two(hi);
+      *reinterpret_cast<uint2 *>(&sLo[at]) = two(lo);
+    }
+  };
+  publish();
+  const int i = wave * 16 + l15;  // this lane's row of the chunk
+  for (int t0 = 0; t0 < sp.n; t0 += C) {
+    const int n = min(C, sp.n - t0);
+    stage();
+    bf8 q[KS];
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      u4 v = zero;
+      if (i < n && ks * 32 < a.dg)
+        v = *reinterpret_cast<const u4 *>(Q + (size_t)(t0 + i) * cols + ks * 32 + 8 * g);
+      q[ks] = __builtin_bit_cast(bf8, v);
+    }
+    __syncthreads();
+    if (t0 + C < sp.n) fetch(t0 + C);
+    // from the state before the chunk
+    f4 o[4];
+#pragma unroll
+    for (int vt = 0; vt < 4; ++vt) {
+      o[vt] = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const int at = (vt * 16 + l15) * LDK + ks * 32 + 8 * g;
+        o[vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf8 *>(&sHi[at]), q[ks],
+                                                        o[vt], 0, 0, 0);
+        o[vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf8 *>(&sLo[at]), q[ks],
+                                                        o[vt], 0, 0, 0);
+      }
+      o[vt] *= pw[i + 1];
+    }
+    // within the chunk: keys of 32 at a time
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb) {
+      if (kb * 32 > wave * 16 + 15) continue;  // (all after this wave's rows)
+      bf8 ph, plo;
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        f4 s = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks)
+          s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              *reinterpret_cast<const bf8 *>(&sK[(kb * 32 + j * 16 + l15) * LDK + ks * 32 + 8 * g]), q[ks],
+              s, 0, 0, 0);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int key = kb * 32 + j * 16 + 4 * g + e;
+          const float w = key <= i ? s[e] * pw[max(i - key, 0)] : 0.f;
+          __bf16 hi, lo;
+          split2(w, hi, lo);
+          ph[j * 4 + e] = hi, plo[j * 4 + e] = lo;
+        }
+      }
+#pragma unroll
+      for (int vt = 0; vt < 4; ++vt) {
+        const bf8 v = read_columns<LDV>(sV, kb, vt * 16);
+        o[vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, ph, o[vt], 0, 0, 0);
+        o[vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, plo, o[vt], 0, 0, 0);
+      }
+    }
+    // the state after the chunk
+    const float dn = pw[n];
+#pragma unroll
+    for (int dt = 0; dt < 2 * KS; ++dt) st[dt] *= dn;
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb) {
+      const bf8 v = read_columns<LDV>(sV, kb, wave * 16);
+      bf8 vh, vl;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int key = kb * 32 + 4 * g + (e & 3) + 16 * (e >> 2);
+        __bf16 hi, lo;
+        split2((float)v[e] * pw[max(n - 1 - key, 0)], hi, lo);  // (rows past the span are zeros)
+        vh[e] = hi, vl[e] = lo;
+      }
+#pragma unroll
+      for (int dt = 0; dt < 2 * KS; ++dt) {
+        const bf8 k = read_columns<LDK>(sK, kb, dt * 16);
+        st[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, vh, st[dt], 0, 0, 0);
+        st[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, vl, st[dt], 0, 0, 0);
+      }
+    }
+    if (i < n) {
+      float *dst = a.o + (size_t)(sp.t0 + t0 + i) * a.H * a.vg + (size_t)h * a.vg + c0 + 4 * g;
+#pragma unroll
+      for (int vt = 0; vt < 4; ++vt)
+        if (vt * 16 < vw) *reinterpret_cast<f4 *>(dst + vt * 16) = o[vt];
+    }
+    __syncthreads();
+    if (t0 + C < sp.n) publish();
+  }
+#pragma unroll
+  for (int dt = 0; dt < 2 * KS; ++dt)
+    if (dt * 16 < a.dg && vcol < vw)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) S[(size_t)(dt * 16 + 4 * g + e) * a.vg] = st[dt][e];
+}
+
+hipError_t launch_lightning_chunks(const char *blob, int off_spans, int num_spans, const Lightning &a,
+                                   int limit, hipStream_t s) {
+  if (num_spans <= 0) return hipSuccess;
+  if (bad_shape(a, kLightningMaxChunkDim) || !a.qkv) return hipErrorInvalidValue;
+  const int cols = a.H * (2 * a.dg + a.vg);
+  const long n = (long)a.T * (cols / 8);
+  hipLaunchKernelGGL(lightning_qkv_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, a, cols);
+  const dim3 grid((a.vg + 63) / 64, a.H, num_spans);
+#define FFMI_LC(KS)                                                                                   \
+  hipLaunchKernelGGL((lightning_chunk_kernel<KS>), grid, dim3(256), 0, s, blob, off_spans, a, limit)
+  if (a.dg <= 32) FFMI_LC(1);
+  else if (a.dg <= 64) FFMI_LC(2);
+  else if (a.dg <= 128) FFMI_LC(4);
+  else FFMI_LC(8);
+#undef FFMI_LC
+  return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// norm over all heads, gate
+// ---------------------------------------------------------------------------
+__global__ __launch_bounds__(256) void gated_norm_kernel(const float *__restrict__ o, Partials y,
+                                                         int gate_col, const float *__restrict__ w,
+                                                         uint16_t *__restrict__ hb,
+                                                         float *__restrict__ hf, int H, int n,
+                                                         float eps) {
+  __shared__ float sh[4];
+  const int t = blockIdx.x, T = gridDim.x;
+  const float *row = o + (size_t)t * H;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < H / 4; c += 256) {
+    const f4 v = *reinterpret_cast<const f4 *>(row + c * 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss = fmaf(v[e], v[e], ss);
+  }
+  const float r = inv_rms(row_sum<256>(ss, sh), n, eps);
+  for (int c = threadIdx.x; c < H / 8; c += 256) {
+    f4 v[2];
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const int at = c * 8 + 4 * k;
+      const float *gp = y.p + (size_t)t * y.NP + gate_col + at;
+      f4 gt = *reinterpret_cast<const f4 *>(gp);
+      for (int s = 1; s < y.S; ++s) gt += *reinterpret_cast<const f4 *>(gp + (size_t)s * T * y.NP);
+      v[k] = *reinterpret_cast<const f4 *>(row + at);
+      const f4 wv = *reinterpret_cast<const f4 *>(w + at);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[k][e] = v[k][e] * r * wv[e] * sigmoid_f(gt[e]);
+      if (hf) *reinterpret_cast<f4 *>(hf + (size_t)t * H + at) = v[k];
+    }
+    if (hb) *reinterpret_cast<uint4 *>(hb + act_packed_off(t, c * 8, H)) = pack8_bf16(v[0], v[1]);
+  }
+}
+hipError_t launch_gated_norm(const float *o, const Partials &y, int gate_col, const float *w,
+                             uint16_t *hb, float *hf, int T, int H, int n, float eps, hipStream_t s) {
+  if (T <= 0) return hipSuccess;
+  if (H % 32 || gate_col % 4 || y.S < 1) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(gated_norm_kernel, dim3(T), dim3(256), 0, s, o, y, gate_col, w, hb, hf, H, n, eps);
+  return hipGetLastError();
+}
+
+}  // namespace ffmi

@@ -1,0 +1,622 @@
+// paged_attn.hip -- attention over paged keys and values (paged_attn.h).
+#include "paged_attn.h"
+
+#include <algorithm>
+
+#include "device_util.h"
+
+namespace ffmi {
+
+typedef uint32_t u4 __attribute__((ext_vector_type(4)));
+
+int attn_width(int dim) { return dim <= 64 ? 64 : dim <= 128 ? 128 : dim <= 256 ? 256 : 0; }
+
+// ---------------------------------------------------------------------------
+// queries, keys, values: one wave per (token, head)
+// ---------------------------------------------------------------------------
+// column n of a row of deferred sums; several slabs: their loads together
+__device__ __forceinline__ float slab_sum(const Partials &y, size_t slab, size_t at) {
+  float v = y.p[at];
+  if (y.S > 1) {
+    float p[7];
+#pragma unroll
+    for (int s = 1; s < 8; ++s) p[s - 1] = y.p[at + (size_t)min(s, y.S - 1) * slab];
+#pragma unroll
+    for (int s = 1; s < 8; ++s)
+      if (s < y.S) v += p[s - 1];
+  }
+  return v;
+}
+
+template <class E, int NE>
+__global__ __launch_bounds__(256) void attn_prep_kernel(const PagedToken *__restrict__ tok, int T,
+                                                        AttnPrep a) {
+  const int heads = a.H + 2 * a.G, lane = threadIdx.x & 63;
+  const long id = blockIdx.x * 4L + (threadIdx.x >> 6);
+  const int hd = (int)(id % heads);
+  const long t = id / heads;
+  if (t >= T) return;
+  const bool isv = hd >= a.H + a.G, isq = hd < a.H;
+  const int g = isq ? 0 : (hd - a.H) % a.G;
+  const int wd = isv ? a.vg : a.dg;  // columns of this head
+  const int col = isv ? (a.H + a.G) * a.dg + g * a.vg : hd * a.dg;
+  const PagedToken tk = tok[t];
+  const size_t slab = (size_t)T * a.y.NP, row = (size_t)t * a.y.NP + col;
+  float v[NE], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int c = lane + i * 64;
+    v[i] = 0.f;
+    if (c < wd) v[i] = slab_sum(a.y, slab, row + c) + a.bias[col + c];
+    ss = fmaf(v[i], v[i], ss);
+  }
+  const size_t page = (size_t)(tk.row / kPageTokens), key = tk.row % kPageTokens;
+  if (isv) {
+    E *dst = (E *)a.vc + (page * a.G + g) * kPageTokens * a.vp;
+    const float lam = a.vmix ? *a.vmix : 0.f;
+    float *first = a.first ? a.first + ((size_t)t * a.G + g) * a.vg : nullptr;
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int c = lane + i * 64;
+      if (c < wd && first) {
+        if (a.vmix) v[i] = (1.0f - lam) * v[i] + lam * first[c];
+        else first[c] = v[i];
+      }
+      if (c < a.vp) st_elem(dst + val_off((int)key, c, a.vp), v[i]);
+    }
+    return;
+  }
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
+  float r = inv_rms(ss, a.dim, a.eps);
+  if (isq && a.coef != 0.f) r *= 1.0f + a.coef * logf((float)((tk.pos + 1) / a.every + 1));
+  const float *w = isq ? a.qnorm : a.knorm;
+  E *dst = isq ? (E *)a.q + ((size_t)t * a.H + hd) * a.dp
+               : (E *)a.kc + (page * a.G + g) * kPageTokens * a.dp;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int c = lane + i * 64;
+    if (c < a.dp) st_elem(dst + (isq ? c : key_off((int)key, c, a.dp)), c < wd ? v[i] * r * w[c] : 0.f);
+  }
+}
+
+hipError_t launch_attn_prep(const char *blob, int off_tokens, int T, const AttnPrep &a, bool f32,
+                            hipStream_t s) {
+  if (T <= 0) return hipSuccess;
+  const int wide = std::max(std::max(a.dp, a.vp), std::max(a.dg, a.vg));
+  if (wide > 1024 || a.y.S < 1 || a.y.S > 8 || a.every < 1) return hipErrorInvalidValue;
+  const PagedToken *tok = reinterpret_cast<const PagedToken *>(blob + off_tokens);
+  const dim3 grid((unsigned)(((long)T * (a.H + 2 * a.G) + 3) / 4));
+#define FFMI_AP(E, NE) hipLaunchKernelGGL((attn_prep_kernel<E, NE>), grid, dim3(256), 0, s, tok, T, a)
+  if (f32) {
+    if (wide <= 256) FFMI_AP(float, 4);
+    else FFMI_AP(float, 16);
+  } else {
+    if (wide <= 64) FFMI_AP(uint16_t, 1);
+    else if (wide <= 128) FFMI_AP(uint16_t, 2);
+    else if (wide <= 256) FFMI_AP(uint16_t, 4);
+    else FFMI_AP(uint16_t, 16);
+  }
+#undef FFMI_AP
+  return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// attention, MFMA form
+// ---------------------------------------------------------------------------
+// Scores S^T = K . Q^T (a lane: 4 keys of one row), outputs O^T = V^T . P^T; the
+// values' key order in the cache makes a lane's score registers the second
+// product's operand as they stand, so weights never leave their lane.  Softmax
+// state in fp32, base-2 exponents; weights meet the second product in bf16, the
+// sums take them unrounded.
+//
+// Up to 16 rows (decoding, short portions): operands straight from memory, the
+// workgroup's four waves over half-pages, their results merged through LDS.
+// More rows (prompts): four waves of two row tiles each over pages staged in
+// LDS, double-buffered, the next page's loads in flight through registers.
+template <int KS, int NK>
+__device__ __forceinline__ void score_bias(const float *bh, int D, bool far, bool whole, int qpos,
+                                           int key0, float scale, f4 (&s)[NK], float &mx) {
+#pragma unroll
+  for (int i = 0; i < NK; ++i) {
+    const int k0 = key0 + i * 16;
+    f4 b;
+    if (far) {
+      const float f = bh[0];
+      b = f4{f, f, f, f};
+    } else {
+      const float *p = bh + (D - min(max(qpos - k0 - 3, -4), D));
+      b = f4{p[0], p[1], p[2], p[3]};
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      float v = fmaf(s[i][e], scale, b[e]);
+      if (!whole && k0 + e > qpos) v = -INFINITY;
+      s[i][e] = v;
+      mx = fmaxf(mx, v);
+    }
+  }
+}
+__device__ __forceinline__ bf8 pack_weights(const f4 &lo, const f4 &hi) {
+  bf8 p;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) p[e] = (__bf16)lo[e], p[4 + e] = (__bf16)hi[e];
+  return p;
+}
+
+template <int DP, int VP>
+constexpr int attn_lds_bytes() {
+  constexpr int prompt = 2 * 64 * (DP + VP) * 2, merge = 4 * 16 * (VP + 4) * 4 + 4 * 16 * 2 * 4;
+  return prompt > merge ? prompt : merge;
+}
+
+template <int DP, int VP>
+__device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, const PagedBlock &bk,
+                                              const AttnArgs &a, float *__restrict__ slabs,
+                                              float *__restrict__ ml, char *lds) {
+  constexpr int KS = DP / 32, VT = VP / 16, LDO = VP + 4;
+  float *sO = reinterpret_cast<float *>(lds), *sM = sO + 4 * 16 * LDO, *sL = sM + 64;
+  const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int grp = blockIdx.y, R = a.H / a.G;
+  const int32_t *table = reinterpret_cast<const int32_t *>(blob) + bk.table;
+  const int row = bk.row0 + min(l15, bk.nrows - 1), token = row / R, head = grp * R + row % R;
+  const int qpos = bk.pos0 + token - bk.seg_row / R;
+  const int qmin = bk.pos0 + (bk.row0 - bk.seg_row) / R;  // the block's first row
+  const float *bh = a.bias + (size_t)head * (a.D + 8);
+  const uint16_t *Kc = (const uint16_t *)a.kc, *Vc = (const uint16_t *)a.vc;
+  const int units = 2 * bk.ntiles;
+
+  bf8 k[2][KS], v[VT];
+  auto fetch = [&](int u) {
+    const size_t page = (size_t)(u < 2 ? bk.page0 : table[bk.tile0 + (u >> 1)]) * a.G + grp;
+    const uint16_t *kp = Kc + page * (64 * DP) + (size_t)(u & 1) * (2 * KS * 512) + lane * 8;
+    const uint16_t *vp = Vc + page * (64 * VP) + (size_t)(u & 1) * (VP * 32) + l15 * 32 + g * 8;
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks)
+        k[i][ks] = *reinterpret_cast<const bf8 *>(kp + (i * KS + ks) * 512);
+#pragma unroll
+    for (int d = 0; d < VT; ++d) v[d] = *reinterpret_cast<const bf8 *>(vp + d * 512);
+  };
+  if (wave < units) fetch(wave);
+  bf8 q[KS];
+  {
+    const uint16_t *qr = (const uint16_t *)a.q + ((size_t)token * a.H + head) * DP + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) q[ks] = *reinterpret_cast<const bf8 *>(qr + ks * 32);
+  }
+  f4 acc[VT];
+#pragma unroll
+  for (int d = 0; d < VT; ++d) acc[d] = f4{0.f, 0.f, 0.f, 0.f};
+  float m = -1e30f, l = 0.f;
+  for (int u = wave; u < units; u += 4) {
+    f4 s[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      s[i] = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks)
+        s[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k[i][ks], q[ks], s[i], 0, 0, 0);
+    }
+    bf8 vv[VT];
+#pragma unroll
+    for (int d = 0; d < VT; ++d) vv[d] = v[d];
+    if (u + 4 < units) fetch(u + 4);
+    const int base = bk.tile0 * 64 + u * 32;
+    float mx = -1e30f;
+    score_bias<KS, 2>(bh, a.D, qmin - (base + 31) >= a.D, base + 31 <= qmin, qpos, base + 4 * g,
+                      a.scale, s, mx);
+    mx = fmaxf(mx, __shfl_xor(mx, 16));
+    mx = fmaxf(mx, __shfl_xor(mx, 32));
+    const float mn = fmaxf(m, mx), alpha = __builtin_amdgcn_exp2f(m - mn);
+    m = mn;
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        s[i][e] = __builtin_amdgcn_exp2f(s[i][e] - mn);
+        sum += s[i][e];
+      }
+    l = l * alpha + sum;
+    const bf8 p = pack_weights(s[0], s[1]);
+    const bool same = __all(alpha == 1.0f);
+#pragma unroll
+    for (int d = 0; d < VT; ++d) {
+      if (!same) acc[d] *= alpha;
+      acc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv[d], p, acc[d], 0, 0, 0);
+    }
+  }
+  l += __shfl_xor(l, 16);
+  l += __shfl_xor(l, 32);
+  if (g == 0) sM[wave * 16 + l15] = m, sL[wave * 16 + l15] = l;
+  __syncthreads();
+  {
+    float M = sM[l15];
+#pragma unroll
+    for (int w = 1; w < 4; ++w) M = fmaxf(M, sM[w * 16 + l15]);
+    const float f = __builtin_amdgcn_exp2f(m - M);
+#pragma unroll
+    for (int d = 0; d < VT; ++d)
+      *reinterpret_cast<f4 *>(&sO[(wave * 16 + l15) * LDO + d * 16 + 4 * g]) = acc[d] * f;
+  }
+  __syncthreads();
+  // the four waves' sums: 16 threads a row, VP / 16 columns each
+  constexpr int NC = VP / 16;
+  const int r = tid >> 4, c0 = (tid & 15) * NC;
+  if (r >= bk.nrows) return;
+  float M = sM[r], L = 0.f;
+#pragma unroll
+  for (int w = 1; w < 4; ++w) M = fmaxf(M, sM[w * 16 + r]);
+#pragma unroll
+  for (int w = 0; w < 4; ++w) L += sL[w * 16 + r] * __builtin_amdgcn_exp2f(sM[w * 16 + r] - M);
+  f4 o[NC / 4];
+#pragma unroll
+  for (int c = 0; c < NC / 4; ++c) {
+    o[c] = *reinterpret_cast<const f4 *>(&sO[r * LDO + c0 + c * 4]);
+#pragma unroll
+    for (int w = 1; w < 4; ++w)
+      o[c] += *reinterpret_cast<const f4 *>(&sO[(w * 16 + r) * LDO + c0 + c * 4]);
+  }
+  if (bk.slot >= 0) {
+    const size_t pr = ((size_t)bk.slot * a.G + grp) * 16 + r;
+#pragma unroll
+    for (int c = 0; c < NC / 4; ++c) *reinterpret_cast<f4 *>(slabs + pr * VP + c0 + c * 4) = o[c];
+    if ((tid & 15) == 0) ml[pr * 2] = M, ml[pr * 2 + 1] = L;
+    return;
+  }
+  const float inv = __fdiv_rn(1.0f, L);
+  const int gr = bk.row0 + r, tk = gr / R, hc = (grp * R + gr % R) * a.vg;
+#pragma unroll
+  for (int c = 0; c < NC / 4; ++c) {
+    if (c0 + c * 4 >= a.vg) continue;
+    const f4 v4 = o[c] * inv;
+    *reinterpret_cast<uint2 *>((uint16_t *)a.o + act_packed_off(tk, hc + c0 + c * 4, a.H * a.vg)) =
+        make_uint2(f2bf(v4[0]) | ((uint32_t)f2bf(v4[1]) << 16),
+                   f2bf(v4[2]) | ((uint32_t)f2bf(v4[3]) << 16));
+  }
+}
+
+template <int DP, int VP>
+__device__ __forceinline__ void attn_many_rows(const char *__restrict__ blob, const PagedBlock &bk,
+                                               const AttnArgs &a, float *__restrict__ slabs,
+                                               float *__restrict__ ml, char *lds) {
+  constexpr int KS = DP / 32, VT = VP / 16, MR = 2;
+  uint16_t *sK = reinterpret_cast<uint16_t *>(lds), *sV = sK + 2 * 64 * DP;
+  const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int grp = blockIdx.y, R = a.H / a.G;
+  const int32_t *table = reinterpret_cast<const int32_t *>(blob) + bk.table;
+  const uint16_t *Kc = (const uint16_t *)a.kc, *Vc = (const uint16_t *)a.vc;
+
+  // pages are stored as their operands: staging is a straight copy
+  constexpr int NKC = DP / 32, NVC = VP / 32;  // 16-byte chunks per thread
+  u4 pk[NKC], pv[NVC];
+  auto fetch = [&](int it) {
+    const size_t page = (size_t)(it == 0 ? bk.page0 : table[bk.tile0 + it]) * a.G + grp;
+    const u4 *kp = reinterpret_cast<const u4 *>(Kc + page * (64 * DP)) + tid;
+    const u4 *vp = reinterpret_cast<const u4 *>(Vc + page * (64 * VP)) + tid;
+#pragma unroll
+    for (int i = 0; i < NKC; ++i) pk[i] = kp[i * 256];
+#pragma unroll
+    for (int i = 0; i < NVC; ++i) pv[i] = vp[i * 256];
+  };
+  auto stage = [&](int buf) {
+    u4 *kd = reinterpret_cast<u4 *>(sK + buf * 64 * DP) + tid;
+    u4 *vd = reinterpret_cast<u4 *>(sV + buf * 64 * VP) + tid;
+#pragma unroll
+    for (int i = 0; i < NKC; ++i) kd[i * 256] = pk[i];
+#pragma unroll
+    for (int i = 0; i < NVC; ++i) vd[i * 256] = pv[i];
+  };
+  fetch(0);
+  // this wave's rows (past the block: its last row again)
+  bf8 q[MR][KS];
+  int qpos[MR];
+  const float *bh[MR];
+  const int wrow0 = min(wave * MR * 16, bk.nrows - 1), wrow1 = min(wave * MR * 16 + MR * 16, bk.nrows) - 1;
+  const int qmin = bk.pos0 + (bk.row0 + wrow0 - bk.seg_row) / R;
+  const int qmax = bk.pos0 + (bk.row0 + wrow1 - bk.seg_row) / R;
+  const bool idle = wave * MR * 16 >= bk.nrows;
+#pragma unroll
+  for (int i = 0; i < MR; ++i) {
+    const int row = bk.row0 + min((wave * MR + i) * 16 + l15, bk.nrows - 1);
+    const int token = row / R, head = grp * R + row % R;
+    qpos[i] = bk.pos0 + token - bk.seg_row / R;
+    bh[i] = a.bias + (size_t)head * (a.D + 8);
+    const uint16_t *qr = (const uint16_t *)a.q + ((size_t)token * a.H + head) * DP + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) q[i][ks] = *reinterpret_cast<const bf8 *>(qr + ks * 32);
+  }
+  f4 acc[MR][VT];
+  float m[MR], l[MR];
+#pragma unroll
+  for (int i = 0; i < MR; ++i) {
+    m[i] = -1e30f, l[i] = 0.f;
+#pragma unroll
+    for (int d = 0; d < VT; ++d) acc[i][d] = f4{0.f, 0.f, 0.f, 0.f};
+  }
+  stage(0);
+  if (bk.ntiles > 1) fetch(1);
+  __syncthreads();
+  for (int it = 0; it < bk.ntiles; ++it) {
+    if (it + 1 < bk.ntiles) {
+      stage((it + 1) & 1);  // (its buffer was last read before the previous barrier)
+      if (it + 2 < bk.ntiles) fetch(it + 2);
+    }
+    const int base = (bk.tile0 + it) * 64;
+    if (!idle && base <= qmax) {
+      const uint16_t *kt = sK + (it & 1) * 64 * DP + lane * 8;
+      const uint16_t *vt = sV + (it & 1) * 64 * VP + l15 * 32 + g * 8;
+      f4 s[MR][4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+#pragma unroll
+        for (int i = 0; i < MR; ++i) s[i][j] = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+          const bf8 kf = *reinterpret_cast<const bf8 *>(kt + (j * KS + ks) * 512);
+#pragma unroll
+          for (int i = 0; i < MR; ++i)
+            s[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, q[i][ks], s[i][j], 0, 0, 0);
+        }
+      }
+      const bool far = qmin - (base + 63) >= a.D, whole = base + 63 <= qmin;
+      bf8 p[MR][2];
+#pragma unroll
+      for (int i = 0; i < MR; ++i) {
+        float mx = -1e30f;
+        score_bias<KS, 4>(bh[i], a.D, far, whole, qpos[i], base + 4 * g, a.scale, s[i], mx);
+        mx = fmaxf(mx, __shfl_xor(mx, 16));
+        mx = fmaxf(mx, __shfl_xor(mx, 32));
+        const float mn = fmaxf(m[i], mx), alpha = __builtin_amdgcn_exp2f(m[i] - mn);
+        m[i] = mn;
+        float sum = 0.f;
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            s[i][j][e] = __builtin_amdgcn_exp2f(s[i][j][e] - mn);
+            sum += s[i][j][e];
+          }
+        l[i] = l[i] * alpha + sum;
+        if (!__all(alpha == 1.0f))
+#pragma unroll
+          for (int d = 0; d < VT; ++d) acc[i][d] *= alpha;
+#pragma unroll
+        for (int h = 0; h < 2; ++h) p[i][h] = pack_weights(s[i][2 * h], s[i][2 * h + 1]);
+      }
+#pragma unroll
+      for (int h = 0; h < 2; ++h)
+#pragma unroll
+        for (int d = 0; d < VT; ++d) {
+          const bf8 vf = *reinterpret_cast<const bf8 *>(vt + h * VP * 32 + d * 512);
+#pragma unroll
+          for (int i = 0; i < MR; ++i)
+            acc[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, p[i][h], acc[i][d], 0, 0, 0);
+        }
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < MR; ++i) {
+    float L = l[i];
+    L += __shfl_xor(L, 16);
+    L += __shfl_xor(L, 32);
+    const int r = (wave * MR + i) * 16 + l15;
+    if (r >= bk.nrows) continue;
+    if (bk.slot >= 0) {
+      const size_t pr = ((size_t)(bk.slot + wave * MR + i) * a.G + grp) * 16 + l15;
+#pragma unroll
+      for (int d = 0; d < VT; ++d) *reinterpret_cast<f4 *>(slabs + pr * VP + d * 16 + 4 * g) = acc[i][d];
+      if (g == 0) ml[pr * 2] = m[i], ml[pr * 2 + 1] = L;
+      continue;
+    }
+    const float inv = __fdiv_rn(1.0f, L);
+    const int gr = bk.row0 + r, tk = gr / R, hc = (grp * R + gr % R) * a.vg + 4 * g;
+#pragma unroll
+    for (int d = 0; d < VT; ++d) {
+      if (d * 16 >= a.vg) continue;
+      const f4 v4 = acc[i][d] * inv;
+      *reinterpret_cast<uint2 *>((uint16_t *)a.o + act_packed_off(tk, hc + d * 16, a.H * a.vg)) =
+          make_uint2(f2bf(v4[0]) | ((uint32_t)f2bf(v4[1]) << 16),
+                     f2bf(v4[2]) | ((uint32_t)f2bf(v4[3]) << 16));
+    }
+  }
+}
+
+// MANY: the step has blocks of more than 16 rows (and maybe others)
+template <int DP, int VP, bool MANY>
+__global__ __launch_bounds__(256) void paged_attn_kernel(const char *__restrict__ blob, int off_blocks,
+                                                         AttnArgs a, float *__restrict__ slabs,
+                                                         float *__restrict__ ml) {
+  __shared__ __attribute__((aligned(16))) char
+      lds[MANY ? attn_lds_bytes<DP, VP>() : 4 * 16 * (VP + 4) * 4 + 512];
+  const PagedBlock bk = reinterpret_cast<const PagedBlock *>(blob + off_blocks)[blockIdx.x];
+  if (bk.nrows <= 0) return;
+  if constexpr (MANY) {
+    if (bk.nrows > 16) {
+      attn_many_rows<DP, VP>(blob, bk, a, slabs, ml, lds);
+      return;
+    }
+  }
+  attn_few_rows<DP, VP>(blob, bk, a, slabs, ml, lds);
+}
+
+// partials of split blocks, in slot order: a workgroup per 16 rows of a block
+template <int VP>
+__global__ __launch_bounds__(256) void paged_attn_merge_kernel(const char *__restrict__ blob,
+                                                               int off_merges, AttnArgs a,
+                                                               const float *__restrict__ slabs,
+                                                               const float *__restrict__ ml) {
+  constexpr int NC = VP / 16, U = 4;
+  const PagedMerge mg = reinterpret_cast<const PagedMerge *>(blob + off_merges)[blockIdx.x];
+  const int r = blockIdx.y * 16 + (threadIdx.x >> 4), c0 = (threadIdx.x & 15) * NC;
+  if (r >= mg.nrows) return;
+  const int grp = blockIdx.z, R = a.H / a.G, units = mg.nrows > 16 ? kAttnTiles : 1;
+  const size_t pr0 = ((size_t)(mg.slot0 + blockIdx.y) * a.G + grp) * 16 + (r & 15);
+  const size_t step = (size_t)units * a.G * 16;
+  float M = -1e30f;
+  for (int i = 0; i < mg.nslots; ++i) M = fmaxf(M, ml[(pr0 + i * step) * 2]);
+  float L = 0.f;
+  f4 o[NC / 4];
+#pragma unroll
+  for (int c = 0; c < NC / 4; ++c) o[c] = f4{0.f, 0.f, 0.f, 0.f};
+  for (int i0 = 0; i0 < mg.nslots; i0 += U) {
+    f4 v[U][NC / 4];
+    float w[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const size_t pr = pr0 + min(i0 + u, mg.nslots - 1) * step;
+      w[u] = i0 + u < mg.nslots ? __builtin_amdgcn_exp2f(ml[pr * 2] - M) : 0.f;
+      L = fmaf(w[u], ml[pr * 2 + 1], L);
+#pragma unroll
+      for (int c = 0; c < NC / 4; ++c) v[u][c] = *reinterpret_cast<const f4 *>(slabs + pr * VP + c0 + c * 4);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int c = 0; c < NC / 4; ++c) o[c] += v[u][c] * w[u];
+  }
+  const float inv = __fdiv_rn(1.0f, L);
+  const int gr = mg.row0 + r, tk = gr / R, hc = (grp * R + gr % R) * a.vg;
+#pragma unroll
+  for (int c = 0; c < NC / 4; ++c) {
+    if (c0 + c * 4 >= a.vg) continue;
+    const f4 v4 = o[c] * inv;
+    *reinterpret_cast<uint2 *>((uint16_t *)a.o + act_packed_off(tk, hc + c0 + c * 4, a.H * a.vg)) =
+        make_uint2(f2bf(v4[0]) | ((uint32_t)f2bf(v4[1]) << 16),
+                   f2bf(v4[2]) | ((uint32_t)f2bf(v4[3]) << 16));
+  }
+}
+
+template <int DP, int VP>
+static hipError_t run_paged_attn(const char *blob, const PagedLists &pl, const AttnArgs &a,
+                                 float *slabs, float *ml, hipStream_t s) {
+  const dim3 grid(pl.num_blocks, a.G);
+  if (pl.row_tiles > 1)
+    hipLaunchKernelGGL((paged_attn_kernel<DP, VP, true>), grid, dim3(256), 0, s, blob, pl.off_blocks, a,
+                       slabs, ml);
+  else
+    hipLaunchKernelGGL((paged_attn_kernel<DP, VP, false>), grid, dim3(256), 0, s, blob, pl.off_blocks, a,
+                       slabs, ml);
+  if (pl.num_merges > 0)
+    hipLaunchKernelGGL((paged_attn_merge_kernel<VP>), dim3(pl.num_merges, pl.row_tiles, a.G), dim3(256),
+                       0, s, blob, pl.off_merges, a, slabs, ml);
+  return hipGetLastError();
+}
+
+hipError_t launch_paged_attn(const char *blob, const PagedLists &pl, const AttnArgs &a, float *slabs,
+                             float *ml, hipStream_t s) {
+  if (pl.num_blocks <= 0) return hipSuccess;
+  if (a.G < 1 || a.H % a.G || pl.heads != a.H / a.G || pl.groups != a.G || a.vg > a.vp || a.D < 0 ||
+      (pl.row_tiles != 1 && pl.row_tiles != kAttnTiles))
+    return hipErrorInvalidValue;
+#define FFMI_PA(DP, VP) \
+  if (a.dp == DP && a.vp == VP) return run_paged_attn<DP, VP>(blob, pl, a, slabs, ml, s)
+  FFMI_PA(64, 64);
+  FFMI_PA(64, 128);
+  FFMI_PA(64, 256);
+  FFMI_PA(128, 64);
+  FFMI_PA(128, 128);
+  FFMI_PA(128, 256);
+  FFMI_PA(256, 64);
+  FFMI_PA(256, 128);
+  FFMI_PA(256, 256);
+#undef FFMI_PA
+  return hipErrorInvalidValue;
+}
+
+// ---------------------------------------------------------------------------
+// attention, one workgroup per row (fp32, and bf16 widths without an MFMA form)
+// ---------------------------------------------------------------------------
+template <class E>
+__global__ __launch_bounds__(256) void paged_attn_rows_kernel(const char *__restrict__ blob,
+                                                              int off_blocks, AttnArgs a) {
+  __shared__ float sq[kAttnRowsMax], sp[256], red[4];
+  __shared__ int spage[256];
+  const PagedBlock bk = reinterpret_cast<const PagedBlock *>(blob + off_blocks)[blockIdx.x];
+  const int r = blockIdx.y, tid = threadIdx.x, grp = blockIdx.z, R = a.H / a.G;
+  if (r >= bk.nrows) return;
+  const int32_t *table = reinterpret_cast<const int32_t *>(blob) + bk.table;
+  const int row = bk.row0 + r, token = row / R, head = grp * R + row % R;
+  const int qpos = bk.pos0 + token - bk.seg_row / R, n = qpos + 1;
+  const float *bh = a.bias + (size_t)head * (a.D + 8);
+  const E *q = (const E *)a.q + ((size_t)token * a.H + head) * a.dp;
+  for (int i = tid; i < a.dp; i += 256) sq[i] = ld_elem(q + i);
+  float acc[kAttnRowsMax / 256];
+#pragma unroll
+  for (int i = 0; i < kAttnRowsMax / 256; ++i) acc[i] = 0.f;
+  constexpr bool base2 = sizeof(E) == 2;
+  float m = -1e30f, l = 0.f;
+  for (int j0 = 0; j0 < n; j0 += 256) {
+    __syncthreads();
+    const int j = j0 + tid;
+    float sv = -INFINITY;
+    if (j < n) {
+      const int page = table[j >> 6] * a.G + grp;
+      spage[tid] = page;
+      const E *k = (const E *)a.kc + (size_t)page * (64 * a.dp);
+      float d = 0.f;
+      for (int c = 0; c < a.dp; c += 8) {
+        const E *kc = k + key_off(j & 63, c, a.dp);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) d = fmaf(sq[c + e], ld_elem(kc + e), d);
+      }
+      sv = fmaf(d, a.scale, bh[a.D + 3 - min(qpos - j, a.D)]);
+    }
+    float mx = sv;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
+    if ((tid & 63) == 0) red[tid >> 6] = mx;
+    __syncthreads();
+    const float mn = fmaxf(m, fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])));
+    const float p = j < n ? (base2 ? exp2f(sv - mn) : expf(sv - mn)) : 0.f;
+    sp[tid] = p;
+    float sum = p;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) sum += __shfl_xor(sum, o);
+    __syncthreads();
+    if ((tid & 63) == 0) red[tid >> 6] = sum;
+    __syncthreads();
+    const float al = base2 ? exp2f(m - mn) : expf(m - mn);
+    l = l * al + (red[0] + red[1] + red[2] + red[3]);
+    m = mn;
+    const int cnt = min(256, n - j0);
+#pragma unroll
+    for (int i = 0; i < kAttnRowsMax / 256; ++i) {
+      const int c = tid + i * 256;
+      if (c >= a.vg) break;
+      float s = acc[i] * al;
+      for (int k = 0; k < cnt; ++k)
+        s = fmaf(sp[k], ld_elem((const E *)a.vc + (size_t)spage[k] * (64 * a.vp) +
+                                val_off((j0 + k) & 63, c, a.vp)), s);
+      acc[i] = s;
+    }
+  }
+  const float inv = __fdiv_rn(1.0f, l);
+#pragma unroll
+  for (int i = 0; i < kAttnRowsMax / 256; ++i) {
+    const int c = tid + i * 256, col = head * a.vg + c, Kw = a.H * a.vg;
+    if (c >= a.vg) break;
+    st_elem((E *)a.o + (base2 ? act_packed_off(token, col, Kw) : (size_t)token * Kw + col), acc[i] * inv);
+  }
+}
+
+hipError_t launch_paged_attn_rows(const char *blob, const PagedLists &pl, const AttnArgs &a, bool f32,
+                                  hipStream_t s) {
+  if (pl.num_blocks <= 0) return hipSuccess;
+  if (a.G < 1 || a.H % a.G || pl.heads != a.H / a.G || pl.groups != a.G || a.dp > kAttnRowsMax ||
+      a.vp > kAttnRowsMax || a.dp % 32 || a.vg > a.vp || a.D < 0 || pl.num_merges > 0)
+    return hipErrorInvalidValue;
+  const dim3 grid(pl.num_blocks, pl.row_tiles * 16, a.G);
+  if (f32)
+    hipLaunchKernelGGL(paged_attn_rows_kernel<float>, grid, dim3(256), 0, s, blob, pl.off_blocks, a);
+  else
+    hipLaunchKernelGGL(paged_attn_rows_kernel<uint16_t>, grid, dim3(256), 0, s, blob, pl.off_blocks, a);
+  return hipGetLastError();
+}
+
+}  // namespace ffmi

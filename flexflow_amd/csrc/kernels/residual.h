@@ -1,0 +1,28 @@
+// residual.h -- the 32-bit residual stream: launchers (residual.hip).
+#pragma once
+#include "paged.h"
+
+namespace ffmi {
+
+// x = embed[token] * scale + pos[p] in fp32 (pos null: no positions); xb
+// (optional) the bf16 packed tiles.  blob_src: the step's staging in mapped
+// host memory, copied to blob_dst by this first kernel of the step.
+hipError_t launch_embed_pos(const char *blob_src, char *blob_dst, size_t blob_bytes,
+                            const uint16_t *embed, float scale, const uint16_t *pos, float *x,
+                            uint16_t *xb, int T, int H, hipStream_t s);
+// x += y / rms(y) * w on n columns (row stride H); y = sum of the fp32 slabs;
+// xb (optional): the new x in bf16 packed tiles
+hipError_t launch_post_norm(Partials y, const float *w, float *x, uint16_t *xb, int T, int H, int n,
+                            float eps, hipStream_t s);
+// x += y (y.S == 0: nothing to add), h = x / rms(x) * w: bf16 packed tiles (hb)
+// or fp32 rows (hf); w null: the sum only
+hipError_t launch_add_norm(Partials y, const float *w, float *x, uint16_t *hb, float *hf, int T,
+                           int H, int n, float eps, hipStream_t s);
+// h[i] = x[rows[i]] / rms * w: bf16 packed tiles (hb) or fp32 rows (hf)
+hipError_t launch_row_norm(const char *blob, int off_rows, const float *x, const float *w,
+                           uint16_t *hb, float *hf, int R, int H, int n, float eps, hipStream_t s);
+hipError_t launch_relu2_f32(float *u, size_t n, hipStream_t s);
+// Y[T][F] = clamped_glu of gu [T][gate F | up F]
+hipError_t launch_glu_f32(const float *gu, float *Y, int T, int F, float limit, hipStream_t s);
+
+}  // namespace ffmi

@@ -1,0 +1,224 @@
+// residual.hip -- the 32-bit residual stream (residual.h): input rows, sums of
+// sublayer outputs, norms.
+#include "residual.h"
+
+#include <algorithm>
+
+#include "device_util.h"
+
+namespace ffmi {
+
+__global__ __launch_bounds__(256) void embed_pos_kernel(
+    const char *__restrict__ blob_src, uint4 *__restrict__ blob_dst, int blob_n16,
+    const uint16_t *__restrict__ embed, float scale, const uint16_t *__restrict__ pos,
+    float *__restrict__ x, uint16_t *__restrict__ xb, int H) {
+  const int t = blockIdx.x;
+  const PagedToken tk = reinterpret_cast<const PagedToken *>(blob_src)[t];  // tokens come first
+  const uint4 *src = reinterpret_cast<const uint4 *>(blob_src);
+  for (int i = t * 256 + threadIdx.x; i < blob_n16; i += gridDim.x * 256) blob_dst[i] = src[i];
+  for (int c = threadIdx.x; c < H / 8; c += 256) {
+    f4 a, b;
+    unpack8_bf16(*reinterpret_cast<const uint4 *>(embed + (size_t)tk.token * H + c * 8), a, b);
+    a *= scale, b *= scale;
+    if (pos) {
+      f4 pa, pb;
+      unpack8_bf16(*reinterpret_cast<const uint4 *>(pos + (size_t)tk.pos * H + c * 8), pa, pb);
+      a += pa, b += pb;
+    }
+    *reinterpret_cast<f4 *>(x + (size_t)t * H + c * 8) = a;
+    *reinterpret_cast<f4 *>(x + (size_t)t * H + c * 8 + 4) = b;
+    if (xb) *reinterpret_cast<uint4 *>(xb + act_packed_off(t, c * 8, H)) = pack8_bf16(a, b);
+  }
+}
+
+hipError_t launch_embed_pos(const char *blob_src, char *blob_dst, size_t blob_bytes,
+                            const uint16_t *embed, float scale, const uint16_t *pos, float *x,
+                            uint16_t *xb, int T, int H, hipStream_t s) {
+  if (T <= 0) return hipSuccess;
+  if (H % 32) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(embed_pos_kernel, dim3(T), dim3(256), 0, s, blob_src,
+                     reinterpret_cast<uint4 *>(blob_dst), (int)((blob_bytes + 15) / 16), embed, scale,
+                     pos, x, xb, H);
+  return hipGetLastError();
+}
+
+// One workgroup per row; the slab, x and w loads of a chunk are all issued
+// before the reduction.
+//   PRE == false: x += y / rms(y) * w, hb the new x
+//   PRE == true:  x += y, h = x / rms(x) * w to hb or hf (w null: the sum only)
+template <int NT, int MAXC, int MAXS, bool PRE>
+__global__ __launch_bounds__(NT) void stream_norm_kernel(const float *__restrict__ yp, int S, int NP,
+                                                         const float *__restrict__ w,
+                                                         float *__restrict__ x,
+                                                         uint16_t *__restrict__ hb,
+                                                         float *__restrict__ hf, int H, int n,
+                                                         float eps) {
+  __shared__ float sh[NT / 64];
+  const int row = blockIdx.x, T = gridDim.x, nchunk = H >> 3;
+  f4 y[MAXC][2], xv[MAXC][2], wv[MAXC][2];
+  float ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = min((int)threadIdx.x + c * NT, nchunk - 1);
+    f4 lo[MAXS ? MAXS : 1], hi[MAXS ? MAXS : 1];
+    lo[0] = hi[0] = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int sl = 0; sl < MAXS; ++sl) {
+      const float *qs = yp + (size_t)row * NP + ch * 8 + (size_t)min(sl, S - 1) * T * NP;
+      lo[sl] = *reinterpret_cast<const f4 *>(qs);
+      hi[sl] = *reinterpret_cast<const f4 *>(qs + 4);
+    }
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      xv[c][h] = *reinterpret_cast<const f4 *>(x + (size_t)row * H + ch * 8 + 4 * h);
+      wv[c][h] = f4{0.f, 0.f, 0.f, 0.f};
+      if (!PRE || w) wv[c][h] = *reinterpret_cast<const f4 *>(w + ch * 8 + 4 * h);
+    }
+    y[c][0] = lo[0], y[c][1] = hi[0];
+#pragma unroll
+    for (int sl = 1; sl < MAXS; ++sl)
+      if (sl < S) y[c][0] += lo[sl], y[c][1] += hi[sl];
+    if constexpr (PRE) {
+#pragma unroll
+      for (int h = 0; h < 2; ++h) y[c][h] = xv[c][h] += y[c][h];
+    }
+    if ((int)threadIdx.x + c * NT < nchunk)
+#pragma unroll
+      for (int h = 0; h < 2; ++h)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss = fmaf(y[c][h][e], y[c][h][e], ss);
+  }
+  const float r = inv_rms(row_sum<NT>(ss, sh), n, eps);
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = threadIdx.x + c * NT;
+    if (ch >= nchunk) continue;
+#pragma unroll
+    for (int h = 0; h < 2; ++h)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float v = y[c][h][e] * r * wv[c][h][e];
+        if constexpr (PRE) y[c][h][e] = v;
+        else y[c][h][e] = xv[c][h][e] += v;
+      }
+    if (!PRE || MAXS) {
+      *reinterpret_cast<f4 *>(x + (size_t)row * H + ch * 8) = xv[c][0];
+      *reinterpret_cast<f4 *>(x + (size_t)row * H + ch * 8 + 4) = xv[c][1];
+    }
+    if (PRE && !w) continue;
+    if (hb)
+      *reinterpret_cast<uint4 *>(hb + act_packed_off(row, ch * 8, H)) = pack8_bf16(y[c][0], y[c][1]);
+    if (PRE && hf) {
+      *reinterpret_cast<f4 *>(hf + (size_t)row * H + ch * 8) = y[c][0];
+      *reinterpret_cast<f4 *>(hf + (size_t)row * H + ch * 8 + 4) = y[c][1];
+    }
+  }
+}
+
+template <bool PRE>
+static hipError_t run_stream_norm(Partials y, const float *w, float *x, uint16_t *hb, float *hf,
+                                  int T, int H, int n, float eps, hipStream_t s) {
+  if (T <= 0) return hipSuccess;
+  if (H % 32 || y.S < (PRE ? 0 : 1) || y.S > 8) return hipErrorInvalidValue;
+  if (y.S > 0 && (y.NP < H || y.NP % 4 || !y.p)) return hipErrorInvalidValue;
+  const int nchunk = H / 8;
+#define FFMI_SN(NT, MC, MS)                                                                       \
+  hipLaunchKernelGGL((stream_norm_kernel<NT, MC, MS, PRE>), dim3(T), dim3(NT), 0, s, y.p, y.S, \
+                     y.NP, w, x, hb, hf, H, n, eps)
+#define FFMI_SNS(NT, MC)                   \
+  do {                                     \
+    if (PRE && y.S == 0) FFMI_SN(NT, MC, (PRE ? 0 : 1)); \
+    else if (y.S == 1) FFMI_SN(NT, MC, 1); \
+    else if (y.S == 2) FFMI_SN(NT, MC, 2); \
+    else if (y.S <= 4) FFMI_SN(NT, MC, 4); \
+    else FFMI_SN(NT, MC, 8);               \
+  } while (0)
+  if (nchunk <= 128) FFMI_SNS(128, 1);
+  else if (nchunk <= 256) FFMI_SNS(256, 1);
+  else if (nchunk <= 512) FFMI_SNS(512, 1);
+  else if (nchunk <= 1024) FFMI_SNS(1024, 1);
+  else if (nchunk <= 2048) FFMI_SNS(1024, 2);
+  else return hipErrorInvalidValue;
+#undef FFMI_SNS
+#undef FFMI_SN
+  return hipGetLastError();
+}
+hipError_t launch_post_norm(Partials y, const float *w, float *x, uint16_t *xb, int T, int H, int n,
+                            float eps, hipStream_t s) {
+  return run_stream_norm<false>(y, w, x, xb, nullptr, T, H, n, eps, s);
+}
+hipError_t launch_add_norm(Partials y, const float *w, float *x, uint16_t *hb, float *hf, int T,
+                           int H, int n, float eps, hipStream_t s) {
+  return run_stream_norm<true>(y, w, x, hb, hf, T, H, n, eps, s);
+}
+
+__global__ __launch_bounds__(256) void row_norm_kernel(const int32_t *__restrict__ rows,
+                                                       const float *__restrict__ x,
+                                                       const float *__restrict__ w,
+                                                       uint16_t *__restrict__ hb,
+                                                       float *__restrict__ hf, int H, int n,
+                                                       float eps) {
+  __shared__ float sh[4];
+  const int i = blockIdx.x;
+  const float *xr = x + (size_t)rows[i] * H;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < H / 4; c += 256) {
+    const f4 v = *reinterpret_cast<const f4 *>(xr + c * 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss = fmaf(v[e], v[e], ss);
+  }
+  const float r = inv_rms(row_sum<256>(ss, sh), n, eps);
+  for (int c = threadIdx.x; c < H / 8; c += 256) {
+    f4 v[2];
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      v[h] = *reinterpret_cast<const f4 *>(xr + c * 8 + 4 * h);
+      const f4 wv = *reinterpret_cast<const f4 *>(w + c * 8 + 4 * h);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[h][e] = v[h][e] * r * wv[e];
+      if (hf) *reinterpret_cast<f4 *>(hf + (size_t)i * H + c * 8 + 4 * h) = v[h];
+    }
+    if (hb) *reinterpret_cast<uint4 *>(hb + act_packed_off(i, c * 8, H)) = pack8_bf16(v[0], v[1]);
+  }
+}
+
+hipError_t launch_row_norm(const char *blob, int off_rows, const float *x, const float *w,
+                           uint16_t *hb, float *hf, int R, int H, int n, float eps, hipStream_t s) {
+  if (R <= 0) return hipSuccess;
+  if (H % 32) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(row_norm_kernel, dim3(R), dim3(256), 0, s,
+                     reinterpret_cast<const int32_t *>(blob + off_rows), x, w, hb, hf, H, n, eps);
+  return hipGetLastError();
+}
+
+__global__ void relu2_f32_kernel(float *u, size_t n) {
+  for (size_t i = blockIdx.x * (size_t)blockDim.x + threadIdx.x; i < n;
+       i += (size_t)gridDim.x * blockDim.x) {
+    const float v = fmaxf(u[i], 0.f);
+    u[i] = v * v;
+  }
+}
+hipError_t launch_relu2_f32(float *u, size_t n, hipStream_t s) {
+  if (n == 0) return hipSuccess;
+  hipLaunchKernelGGL(relu2_f32_kernel, dim3((unsigned)std::min<size_t>((n + 255) / 256, 16384)),
+                     dim3(256), 0, s, u, n);
+  return hipGetLastError();
+}
+
+__global__ void glu_f32_kernel(const float *__restrict__ gu, float *__restrict__ Y, int F, size_t n,
+                               float limit) {
+  for (size_t i = blockIdx.x * (size_t)blockDim.x + threadIdx.x; i < n;
+       i += (size_t)gridDim.x * blockDim.x) {
+    const size_t t = i / F, c = i % F;
+    Y[i] = clamped_glu(gu[t * 2 * F + c], gu[t * 2 * F + F + c], limit);
+  }
+}
+hipError_t launch_glu_f32(const float *gu, float *Y, int T, int F, float limit, hipStream_t s) {
+  const size_t n = (size_t)T * F;
+  if (n == 0) return hipSuccess;
+  hipLaunchKernelGGL(glu_f32_kernel, dim3((unsigned)std::min<size_t>((n + 255) / 256, 16384)),
+                     dim3(256), 0, s, gu, Y, F, n, limit);
+  return hipGetLastError();
+}
+
+}  // namespace ffmi

@@ -4,6 +4,8 @@
 #include <vector>
 
 #include "../kernels/latent.h"
+#include "../kernels/packing.h"
+#include "../kernels/residual.h"
 #include "paged_step.h"
 
 namespace {
@@ -78,7 +80,7 @@ extern "C" ffmi_status ffmi_latent_attention(const void *q, const void *cache, i
   }
   constexpr int kSlots = 512;
   PagedStep step;
-  ffmi_status st = step.init(T, num_seqs, maxpos, {heads}, mfma ? kSlots : 0);
+  ffmi_status st = step.init(T, num_seqs, maxpos, {RowShape{heads}}, mfma ? kSlots : 0);
   if (st != FFMI_OK) return st;
   std::vector<int32_t> ids(T, 0);
   st = step.stage(ids.data(), segs, nullptr, 0);

@@ -10,21 +10,26 @@ namespace ffmi {
 static size_t up16(size_t v) { return (v + 15) & ~(size_t)15; }
 // workgroups that fill the chip; fewer blocks than this are split over keys --
 // from kSplitTiles pages on (a page costs a workgroup ~1.6 us, the merge of the
-// partials ~5 us)
+// partials ~5 us).  The per-block form runs two workgroups per CU, and its waves
+// share out half-pages: pairs of pages keep them even.
 constexpr int kTargetBlocks = 256, kSplitTiles = 5;
 
 ffmi_status PagedStep::init(int max_tokens, int max_requests, int max_positions,
-                            const std::vector<int> &head_counts, int max_slots) {
+                            const std::vector<RowShape> &shapes, int max_slots) {
   max_tokens_ = max_tokens, max_requests_ = max_requests, max_slots_ = max_slots;
   max_pages_ = (max_positions + kPageTokens - 1) / kPageTokens;
   cap_ = up16((size_t)max_tokens * sizeof(PagedToken)) + up16((size_t)max_tokens * 4) +
-         (size_t)max_requests * (max_pages_ + 16) * 4 + 256;
-  for (int h : head_counts) {
+         (size_t)max_requests * ((max_pages_ + 16) * 4 + sizeof(PagedSpan)) + 256;
+  for (const RowShape &h : shapes) {
+    bool known = false;
+    for (const RowShape &k : shapes_) known |= k.heads == h.heads && k.groups == h.groups;
+    if (known) continue;
     PagedLists l;
-    l.heads = h;
+    l.heads = h.heads, l.groups = h.groups;
     lists_.push_back(l);
-    const size_t nb = ((size_t)max_tokens * h + 15) / 16 + max_requests + max_slots + 128;
-    cap_ += nb * sizeof(LatentBlock) + (size_t)(max_slots + 64) * sizeof(LatentMerge) + 64;
+    shapes_.push_back(h);
+    const size_t nb = ((size_t)max_tokens * h.heads + 15) / 16 + max_requests + max_slots + 128;
+    cap_ += nb * sizeof(PagedBlock) + (size_t)(max_slots + 64) * sizeof(PagedMerge) + 64;
   }
   // mapped: the step's first kernel copies it into device memory
   if (hipHostMalloc((void **)&host, cap_, hipHostMallocCoherent | hipHostMallocMapped) !=
@@ -42,9 +47,9 @@ PagedStep::~PagedStep() {
   if (dev) (void)hipFree(dev);
 }
 
-const PagedLists &PagedStep::lists(int heads) const {
+const PagedLists &PagedStep::lists(int heads, int groups) const {
   for (const auto &l : lists_)
-    if (l.heads == heads) return l;
+    if (l.heads == heads && l.groups == groups) return l;
   return lists_.front();
 }
 
@@ -63,7 +68,7 @@ ffmi_status PagedStep::stage(const BatchConfig &bc, PagePool &pool, const int *r
       pool.release(slot);
       pool.set_owner(slot, guid);
     }
-    Seg s{0, bc.tokensInfo[t].abs_depth_in_request, nullptr};
+    Seg s{0, bc.tokensInfo[t].abs_depth_in_request, nullptr, slot};
     for (; t < n && bc.tokensInfo[t].request_index == slot; ++t, ++s.n) {
       FFMI_CHECK(bc.tokensInfo[t].abs_depth_in_request == s.pos0 + s.n, FFMI_ERR_INVALID);
       ids_[t] = bc.tokensInfo[t].token_id;
@@ -115,34 +120,55 @@ ffmi_status PagedStep::stage(const int32_t *token_ids, const std::vector<Seg> &i
            (size_t)((in[i].pos0 + in[i].n + kPageTokens - 1) / kPageTokens) * 4);
     off += (size_t)stride * 4;
   }
-  shape.assign({T, R, (int)segs.size(), stride});
-  for (PagedLists &l : lists_) {
+  off_spans = (int)(off = up16(off));
+  num_spans = (int)segs.size();
+  short_spans = long_spans = false;
+  for (size_t i = 0; i < segs.size(); ++i, off += sizeof(PagedSpan)) {
+    const PagedSpan sp{segs[i].t0, segs[i].n, segs[i].pos0, in[i].slot};
+    memcpy(host + off, &sp, sizeof(sp));
+    (sp.n <= kShortSpan ? short_spans : long_spans) = true;
+  }
+  off = up16(off);
+  shape.assign({T, R, num_spans, stride, short_spans, long_spans});
+  for (size_t li = 0; li < lists_.size(); ++li) {
+    PagedLists &l = lists_[li];
+    const RowShape &rs = shapes_[li];
     blocks_.clear();
     merges_.clear();
     int max_rows = 0;
     for (const Placed &s : segs) max_rows = std::max(max_rows, s.n * l.heads);
-    l.row_tiles = max_rows <= 16 ? 1 : max_rows <= 32 ? 2 : 4;
-    const int br = l.row_tiles * 16;
+    const auto tiles_for = [&](int rows) {
+      if (rs.per_block) return rows <= 16 ? 1 : rs.max_tiles;
+      return rows <= 16 ? 1 : rows <= 32 ? 2 : rs.max_tiles;
+    };
+    l.row_tiles = tiles_for(max_rows);
+    const auto block_rows = [&](const Placed &s) {
+      return 16 * (rs.per_block ? tiles_for(s.n * l.heads) : l.row_tiles);
+    };
     long base = 0;
-    for (const Placed &s : segs) base += ((long)s.n * l.heads + br - 1) / br;
-    const int want = base > 0 ? std::max(1L, kTargetBlocks / base) : 1;
+    for (const Placed &s : segs)
+      base += ((long)s.n * l.heads + block_rows(s) - 1) / block_rows(s) * rs.groups;
+    const int want = std::max(1L, kTargetBlocks * (rs.per_block ? 2 : 1) / std::max(1L, base));
     int slots = 0;
     for (const Placed &s : segs) {
-      const int nrows = s.n * l.heads, row0 = s.t0 * l.heads;
+      const int nrows = s.n * l.heads, row0 = s.t0 * l.heads, br = block_rows(s);
       for (int r = 0; r < nrows; r += br) {
-        LatentBlock b{};
+        PagedBlock b{};
         b.row0 = row0 + r, b.nrows = std::min(br, nrows - r);
         b.seg_row = row0, b.pos0 = s.pos0, b.table = s.table;
         const int last = s.pos0 + (r + b.nrows - 1) / l.heads;  // last visible position
         const int tiles = last / kPageTokens + 1;
+        const int units = rs.per_block && b.nrows > 16 ? rs.max_tiles : 1;  // slots of a partial
         int ns = tiles < kSplitTiles ? 1 : std::min(want, tiles);
-        if (slots + ns > max_slots_) ns = 1;
-        const int per = (tiles + ns - 1) / ns;
+        int per = (tiles + ns - 1) / ns;
+        if (rs.per_block && ns > 1) per = (per + 1) & ~1;
         ns = (tiles + per - 1) / per;
+        if (slots + ns * units > max_slots_) ns = 1, per = tiles;
         if (ns > 1) merges_.push_back({b.row0, b.nrows, slots, ns});
         for (int i = 0; i < ns; ++i) {
           b.tile0 = i * per, b.ntiles = std::min(per, tiles - i * per);
-          b.slot = ns > 1 ? slots++ : -1;
+          b.slot = ns > 1 ? slots : -1;
+          if (ns > 1) slots += units;
           b.page0 = reinterpret_cast<const int32_t *>(host)[s.table + b.tile0];
           blocks_.push_back(b);
         }
@@ -150,19 +176,19 @@ ffmi_status PagedStep::stage(const int32_t *token_ids, const std::vector<Seg> &i
     }
     // longest first: the causal triangle's short blocks fill the end
     std::stable_sort(blocks_.begin(), blocks_.end(),
-                     [](const LatentBlock &a, const LatentBlock &b) { return a.ntiles > b.ntiles; });
+                     [](const PagedBlock &a, const PagedBlock &b) { return a.ntiles > b.ntiles; });
     // padded counts: a decode step's launch shape changes every 32 blocks
-    blocks_.resize((blocks_.size() + 31) & ~(size_t)31, LatentBlock{});
-    if (!merges_.empty()) merges_.resize((merges_.size() + 7) & ~(size_t)7, LatentMerge{});
+    blocks_.resize((blocks_.size() + 31) & ~(size_t)31, PagedBlock{});
+    if (!merges_.empty()) merges_.resize((merges_.size() + 7) & ~(size_t)7, PagedMerge{});
     l.num_blocks = (int)blocks_.size(), l.num_merges = (int)merges_.size();
     l.off_blocks = (int)off;
-    off += blocks_.size() * sizeof(LatentBlock);
+    off += blocks_.size() * sizeof(PagedBlock);
     l.off_merges = (int)(off = up16(off));
-    off = up16(off + merges_.size() * sizeof(LatentMerge));
+    off = up16(off + merges_.size() * sizeof(PagedMerge));
     FFMI_CHECK(off <= cap_, FFMI_ERR_INVALID);
-    memcpy(host + l.off_blocks, blocks_.data(), blocks_.size() * sizeof(LatentBlock));
+    memcpy(host + l.off_blocks, blocks_.data(), blocks_.size() * sizeof(PagedBlock));
     if (!merges_.empty())
-      memcpy(host + l.off_merges, merges_.data(), merges_.size() * sizeof(LatentMerge));
+      memcpy(host + l.off_merges, merges_.data(), merges_.size() * sizeof(PagedMerge));
     shape.insert(shape.end(), {l.row_tiles, l.num_blocks, l.num_merges});
   }
   bytes = off;
