@@ -1,0 +1,428 @@
+"""The Fesenex model through the engine against the plain implementation
+(fesenex_ref.py): mechanisms, layers, schedules (whole prompts, portions, token
+by token, mixed batches, reused slots and pages), generation, bin/trace_run."""
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+
+import fesenex_models as FM
+import fesenex_ref as R
+import flexflow_amd as fa
+
+pytestmark = pytest.mark.gpu
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+# sizes that are no multiples of the kernels' tiles, layers that all differ
+ODD = FM.model_config(77, 72, [
+    FM.lightning(3, 24, 40, [0.5, 0.93, 0.9995]),
+    FM.attention(6, 3, 24, 12, 0.3, bias_max=40, q_temp=(0.4, 5), ff=50, limit=0.7, rel_rows=6),
+    FM.attention(4, 1, 40, 20, 0.11, bias_max=150, v_mix=True, rel_rows=24),
+    FM.lightning(1, 72, 8, [0.98], ff=33, limit=2.5),
+    FM.attention(2, 1, 88, 20, 0.2, bias_max=333, q_temp=(-0.2, 64), v_mix=True, ff=130),
+    FM.attention(1, 1, 12, 20, 0.4, bias_max=7, v_mix=True, rel_rows=8)], scale=0.5)
+# full heads of the widths large models have, groups of one and of many rows
+WIDE = FM.model_config(300, 256, [
+    FM.attention(8, 8, 128, 128, 0.09, bias_max=128, q_temp=(0.1, 32), v_mix=True, ff=320, rel_rows=32),
+    FM.lightning(2, 128, 160, [0.9, 0.999], ff=96),
+    FM.attention(16, 1, 64, 256, 0.125, bias_max=90, ff=64),
+    FM.attention(16, 8, 256, 128, 0.06, bias_max=1000, v_mix=True),
+    FM.lightning(2, 256, 64, [0.99, 1.0])], scale=16.0, eps=1e-3)
+# everything 1, and the smallest of each
+ONE = FM.model_config(64, 32, [FM.attention(1, 1, 32, 32, 1.0, bias_max=2, q_temp=(1.0, 1), v_mix=True, ff=32,
+                                            limit=1.0, rel_rows=2), FM.lightning(1, 32, 32, [1.0])])
+# widths beyond the MFMA forms
+HUGE = FM.model_config(50, 64, [FM.attention(2, 1, 300, 264, 0.05, ff=40), FM.lightning(1, 280, 24, [0.97]),
+                                FM.attention(2, 2, 20, 24, 0.2)])
+MODELS = {"odd": ODD, "wide": WIDE, "one": ONE, "huge": HUGE}
+WEIGHTS = {k: FM.random_weights(m, 11, sharp=1.5) for k, m in MODELS.items()}
+POSITIONS = 768
+
+
+def tokens(model, n, seed):
+    return [int(t) for t in np.random.default_rng(seed).integers(0, model[0]["vocab"], n)]
+
+
+def make_engine(folder, full, pool=12 * 64, batch=256):
+    cfg = fa.load_config(folder)
+    m = fa.Model(cfg, "inc", max_requests=4, max_tokens=batch, max_seq_len=POSITIONS, weights_folder=folder,
+                 full_precision=full, kv_pool_tokens=pool)
+    return fa.RequestManager(max_requests_per_batch=4, max_tokens_per_batch=batch, max_spec_tree_token_num=0,
+                             max_sequence_length=POSITIONS), m
+
+
+@pytest.fixture(scope="module")
+def folders(tmp_path_factory):
+    d = tmp_path_factory.mktemp("fesenex")
+    return {k: FM.write_checkpoint(d / k, m[0], WEIGHTS[k]) for k, m in MODELS.items()}
+
+
+@pytest.fixture(scope="module")
+def engine(folders):
+    """engine(name, full): (manager, model) over a pool of 12 pages, kept per module"""
+    made = {}
+
+    def get(name, full):
+        if (name, full) not in made:
+            made[name, full] = make_engine(folders[name], full)
+        return made[name, full]
+    return get
+
+
+_ref = {}
+
+
+def reference(name, toks):
+    key = (name, tuple(toks))
+    if key not in _ref:
+        layers = []
+        _ref[key] = R.forward(MODELS[name][0], WEIGHTS[name], toks, layers), layers
+    return _ref[key]
+
+
+def errors(got, want):
+    """rows' rms error, the mean taken off, relative to the logits' rms"""
+    d = got - want
+    d = d - d.mean(1, keepdims=True)
+    return np.sqrt((d * d).mean(1)) / np.sqrt((want * want).mean())
+
+
+def close(got, want, full):
+    """In bf16 a few rows sit where two attention weights nearly tie and
+    rounding alone moves them further, so their number is bounded, not only
+    their size."""
+    err = errors(got, want)
+    print("relative error %.3g median %.3g" % (err.max(), np.median(err)))
+    if full:
+        assert err.max() < 3e-5, err.max()
+    else:
+        over = (err > 4e-2).sum()
+        assert np.median(err) < 1e-2 and over <= max(1, 0.02 * len(err)) and err.max() < 0.15, \
+            (np.median(err), over, err.max())
+
+
+_next = [0]
+
+
+def run(eng, toks, cuts):
+    """one request alone, cut into portions; every position's logits"""
+    rm, m = eng
+    _next[0] += 1
+    rid, out, at = _next[0], [], 0
+    for n in cuts:
+        part = toks[at:at + n]
+        if part:
+            out.append(rm.replay_step(m, [(rid, part, range(len(part)))]))
+        at += n
+    assert at >= len(toks)
+    rm.replay_end(m, rid)
+    return np.concatenate(out)
+
+
+# ---- mechanisms ----
+ATT = dict(heads=4, kv_heads=2, dim=24, vdim=20, scale=0.2)
+MECHANISMS = {
+    "grouped attention": [FM.attention(**ATT)],
+    "distance bias": [FM.attention(**ATT, bias_max=90, rel_rows=10)],
+    "query temperature": [FM.attention(**ATT, q_temp=(0.8, 3))],
+    "value mixing": [FM.attention(**ATT, v_mix=True), FM.attention(**ATT, v_mix=True),
+                     FM.attention(2, 2, 40, 20, 0.2, v_mix=True)],
+    "mixing from a later layer on": [FM.attention(**ATT), FM.attention(**ATT, v_mix=True),
+                                     FM.lightning(1, 16, 16, [0.9]), FM.attention(**ATT, v_mix=True)],
+    "lightning": [FM.lightning(3, 40, 24, [0.0, 0.8, 0.999])],
+    "lightning without decay": [FM.lightning(2, 16, 100, [1.0, 1.0])],
+    "feed-forward": [FM.lightning(1, 16, 16, [0.5], ff=70, limit=0.3)],
+    "feed-forward, wide limit": [FM.lightning(1, 16, 16, [0.5], ff=70, limit=7.0)],
+}
+
+
+def wrong_temperature(n, coef, every):
+    p = np.arange(n)
+    return 1.0 + coef * np.log(p // every + 1.0)
+
+
+# a mistake planted in the plain implementation: (function, its wrong form)
+MISTAKES = {
+    "grouped attention": ("projection", lambda w, n, h, heads: (h @ w[n].T).reshape(len(h), heads, -1)),
+    "distance bias": ("distance_bucket", lambda n, rows, far, f=R.distance_bucket: f(max(n - 1, 0), rows, far)),
+    "query temperature": ("query_temperature", wrong_temperature),
+    "value mixing": ("mix_values", lambda v, first, lam: lam * v + (1.0 - lam) * first),
+    "mixing from a later layer on": ("mix_values", lambda v, first, lam: v),
+    "lightning": ("lightning_states", lambda q, k, v, d, f=R.lightning_states: f(q, k, v, d ** 2)),
+    "lightning without decay": ("lightning_states",
+                                lambda q, k, v, d, f=R.lightning_states: f(q, k, v, 0.99 * d)),
+    "feed-forward": ("sigmoid", lambda z, f=R.sigmoid: f(z / 1.702)),
+    "feed-forward, wide limit": ("sigmoid", lambda z, f=R.sigmoid: f(z / 1.702)),
+}
+
+
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("name", list(MECHANISMS))
+def test_mechanism_alone(tmp_path, monkeypatch, name, full):
+    """One mechanism at a time, as a prompt and in portions; the engine agrees
+    with the plain implementation and not with one that gets it wrong."""
+    model = FM.model_config(61, 48, MECHANISMS[name])
+    w = FM.random_weights(model, 5, sharp=2.0)
+    eng = make_engine(FM.write_checkpoint(tmp_path / "m", model[0], w), full)
+    toks = tokens(model, 140, 9)
+    want = R.forward(model[0], w, toks)
+    for cuts in ([140], [1] * 140, [63, 2, 17, 16, 42]):
+        got = run(eng, toks, cuts)
+        close(got, want, full)
+    own = errors(got, want).max()
+    monkeypatch.setattr(R, *MISTAKES[name])
+    assert errors(got, R.forward(model[0], w, toks)).max() > max(0.02, 4 * own)
+
+
+def test_distance_buckets():
+    """exact below half of the rows, the ends of the logarithmic ones, the rest"""
+    b = [R.distance_bucket(n, 16, 128) for n in range(300)]
+    assert b[:8] == list(range(8)) and b[8] == 8 and b[127] == 15 and set(b[128:]) == {15}
+    assert all(y - x in (0, 1) for x, y in zip(b, b[1:]))
+    # 8 rows from distance 8 to 128: a row per factor of sqrt(2)
+    assert [b.index(8 + 2 * i) for i in range(4)] == [8, 16, 32, 64]
+
+
+# ---- layers ----
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("name", list(MODELS))
+def test_residual_stream_after_every_layer(engine, name, full):
+    rm, m = engine(name, full)
+    toks = tokens(MODELS[name], 90, 3)
+    want, layers = reference(name, toks)
+    m.set_debug(True)
+    try:
+        got = run((rm, m), toks, [90])
+        for i, ref in enumerate(layers):
+            h = m.debug_tensor("hidden", i)
+            rms = np.sqrt((ref * ref).mean())
+            err = np.sqrt(((h - ref) ** 2).mean()) / rms
+            assert err < (5e-6 if full else 2e-2), (i, err)
+    finally:
+        m.set_debug(False)
+    close(got, want, full)
+
+
+# ---- schedules ----
+CUTS = {"whole": [1000], "token by token": [1] * 150, "twos": [2] * 75, "threes": [3] * 50,
+        "last short span": [16] * 10, "first long span": [17] * 9, "below a page": [63] * 3, "a page": [64] * 3,
+        "past a page": [65] * 3, "prompt then tokens": [100] + [1] * 50,
+        "changing": [1, 2, 61, 2, 17, 3, 40, 1, 1, 22]}
+
+
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("name", list(MODELS))
+def test_portions(engine, name, full):
+    toks = tokens(MODELS[name], 150, 4)
+    want, _ = reference(name, toks)
+    for how, cuts in CUTS.items():
+        print(name, full, how, flush=True)
+        close(run(engine(name, full), toks, cuts), want, full)
+
+
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("name", ["odd", "wide"])
+def test_long_contexts(engine, name, full):
+    """Contexts whose blocks are split over their pages: single tokens, short
+    portions and portions of several blocks, far into the sequence."""
+    toks = tokens(MODELS[name], 740, 6)
+    want, _ = reference(name, toks)
+    for cuts in ([740], [640, 40, 2, 18, 1, 1, 1, 37], [319, 1, 1, 130, 3, 65, 200, 21]):
+        close(run(engine(name, full), toks, cuts), want, full)
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_first_tokens_and_single_token_prompts(engine, full):
+    for t in range(5):
+        toks = [t] + tokens(ONE, 3, t)
+        want, _ = reference("one", toks)
+        close(run(engine("one", full), toks, [1] * 4), want, full)
+        close(run(engine("one", full), toks, [2, 2]), want, full)
+
+
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("name", ["odd", "wide"])
+def test_mixed_batches_on_reused_slots_and_pages(engine, name, full):
+    """Requests of unequal length, portions beside single tokens, one left out
+    of steps, ended and replaced while others run: each against itself alone."""
+    rm, m = engine(name, full)
+    model = MODELS[name]
+    rng = np.random.default_rng(8)
+    live, left, done = {}, [(n, 20 + i) for i, n in enumerate((1, 150, 33, 64, 129, 2, 90, 65, 300))], 0
+    while left or live:
+        while left and len(live) < 4 and (len(live) < 2 or rng.random() < 0.5):
+            n, seed = left.pop(0)
+            _next[0] += 1
+            live[_next[0]] = [tokens(model, n, seed), 0, []]
+        entries = []
+        for rid, (toks, at, _) in live.items():
+            if len(live) > 1 and rng.random() < 0.2:
+                continue  # left out of this step
+            k = int(rng.choice([1, 1, 2, 3, 17, 40, 70]))
+            part = toks[at:at + k]
+            entries.append((rid, part, range(len(part))))
+        if not entries:
+            continue
+        out, r = rm.replay_step(m, entries), 0
+        for rid, part, _ in entries:
+            live[rid][1] += len(part)
+            live[rid][2].append(out[r:r + len(part)])
+            r += len(part)
+        for rid in [k for k, v in live.items() if v[1] == len(v[0])]:
+            toks, _, got = live.pop(rid)
+            close(np.concatenate(got), reference(name, toks)[0], full)
+            rm.replay_end(m, rid)
+            done += 1
+    assert done == 9
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_long_decoding(engine, full):
+    toks = tokens(ODD, 600, 5)
+    got = run(engine("odd", full), toks, [70] + [1] * 530)
+    close(got, reference("odd", toks)[0], full)
+
+
+# ---- keys and states that decide ----
+@pytest.mark.parametrize("full", [True, False])
+def test_far_key_decides(tmp_path, full):
+    """Weights under which every query wants one marked token's key: the marker
+    is seen from any distance, by prompts and by decoded tokens, and a sequence
+    without it differs."""
+    model = FM.model_config(64, 40, [FM.attention(2, 1, 24, 32, 0.9, bias_max=64)])
+    w = FM.random_weights(model, 4)
+    marker, rng = 9, np.random.default_rng(1)
+    w["embed"][:, 0] = 0.0
+    w["embed"][marker, 0] = 6.0
+    q, k = np.zeros_like(w["l0.mix.q"]), np.zeros_like(w["l0.mix.k"])
+    qb, kb = np.zeros_like(w["l0.mix.q.b"]), np.zeros_like(w["l0.mix.k.b"])
+    qb[[0, 24]] = 1.0            # both heads' queries: the first axis
+    k[0, 0], kb[1] = 8.0, 1.0    # the marker's key lies on it, others' on the second
+    k[2:, 1:] = FM.bf16(rng.standard_normal((22, 39)) * 0.02)
+    for n, v in (("q", q), ("k", k), ("q.b", qb), ("k.b", kb)):
+        w["l0.mix." + n] = v
+    w["l0.mix.q.norm"][:] = w["l0.mix.k.norm"][:] = 1.0
+    eng = make_engine(FM.write_checkpoint(tmp_path / "far", model[0], w), full)
+    base = [t for t in tokens(model, 400, 2) if t != marker][:200]
+    plain = R.forward(model[0], w, base)
+    for at in (0, 1, 63, 64, 65, 127, 128, 190):
+        toks = base[:at] + [marker] + base[at + 1:]
+        want = R.forward(model[0], w, toks)
+        assert np.abs(want[-1] - plain[-1]).max() > 0.3
+        for cuts in ([200], [at or 1, 200], [150] + [1] * 50):
+            close(run(eng, toks, cuts), want, full)
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_each_bucket_of_the_distance_bias_decides(tmp_path, full):
+    """A table with one row far above the others: attention goes to the keys of
+    that bucket alone (their edges decide), before and past the last distance,
+    across pages, in prompts and in decoding."""
+    rows, far = 10, 70
+    model = FM.model_config(64, 40, [FM.attention(2, 1, 24, 32, 0.2, bias_max=far)])
+    model = model[0], [rows]
+    w = FM.random_weights(model, 4)
+    toks = tokens(model, 210, 3)
+    for row in range(rows):
+        rel = np.zeros_like(w["l0.mix.rel"])
+        rel[row] = 12.0
+        w["l0.mix.rel"] = rel
+        want = R.forward(model[0], w, toks)
+        eng = make_engine(FM.write_checkpoint(tmp_path / str(row), model[0], w), full)
+        for cuts in ([210], [130] + [1] * 80, [70, 2, 60, 78]):
+            close(run(eng, toks, cuts), want, full)
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_state_remembers_a_marked_token(tmp_path, full):
+    """Without decay a marked token's value stays in the state: it shows at any
+    later position, whatever portions carried it there, and not in the request
+    that takes the slot afterwards."""
+    model = FM.model_config(64, 40, [FM.lightning(2, 16, 24, [1.0, 1.0])])
+    w = FM.random_weights(model, 4)
+    marker = 9
+    w["embed"][:, 0] = 0.0
+    w["embed"][marker] = 0.0
+    w["embed"][marker, 0] = 8.0
+    w["l0.mix.k"][:, 0], w["l0.mix.v"][:, 0] = 3.0, 3.0  # far above other tokens' products
+    eng = make_engine(FM.write_checkpoint(tmp_path / "s", model[0], w), full)
+    base = [t for t in tokens(model, 400, 2) if t != marker][:200]
+    plain = R.forward(model[0], w, base)
+    for at in (0, 1, 15, 16, 63, 64, 127, 190):
+        toks = base[:at] + [marker] + base[at + 1:]
+        want = R.forward(model[0], w, toks)
+        assert np.abs(want[-1] - plain[-1]).max() > 0.3
+        for cuts in ([200], [at + 1, 200], [at or 1, 2, 17, 200], [150] + [1] * 50):
+            close(run(eng, toks, cuts), want, full)
+        close(run(eng, base, [200]), plain, full)
+
+
+def test_refused_steps(engine):
+    rm, m = engine("one", True)
+    ok = tokens(ONE, POSITIONS, 1)
+    for bad in ([64], [-1], ok + [1]):
+        _next[0] += 1
+        with pytest.raises(fa.ffmi.FFMIError):
+            rm.replay_step(m, [(_next[0], bad, [])])
+        rm.replay_end(m, _next[0])
+    close(run((rm, m), ok[:40], [40]), reference("one", ok[:40])[0], True)
+
+
+# ---- entry points ----
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("pool", [0, 3 * 64])
+def test_greedy_generation(folders, full, pool):
+    """generate() through the scheduler: continuous batching over two slots,
+    and over a pool that holds one request at a time."""
+    cfg = fa.load_config(folders["odd"])
+    m = fa.Model(cfg, "inc", max_requests=2, max_tokens=48, max_seq_len=160,
+                 weights_folder=folders["odd"], full_precision=full, kv_pool_tokens=pool)
+    rm = fa.RequestManager(max_requests_per_batch=2, max_tokens_per_batch=48,
+                           max_spec_tree_token_num=0, max_sequence_length=160, bos_token_id=1)
+    prompts = [tokens(ODD, n, 60 + n) for n in (3, 90, 40, 1)]
+    res = fa.generate(rm, m, prompts, max_length=132)
+    for p, r in zip(prompts, res):
+        seq = r.output_tokens
+        assert seq[:len(p) + 1] == [1] + p and len(seq) == 132
+        # every pick: the plain implementation's, or a tie within rounding
+        logits = R.forward(ODD[0], WEIGHTS["odd"], seq[:-1])[len(p):]
+        lead = logits.max(1) - logits[np.arange(len(logits)), seq[len(p) + 1:]]
+        assert lead.max() < (1e-4 if full else 0.12 * logits.std()), lead.max()
+        assert (lead == 0).mean() > (0.99 if full else 0.9)
+
+
+def test_command_line(folders):
+    prompt = tokens(ODD, 12, 77)
+    p = subprocess.run([sys.executable, "-m", "flexflow_amd", "--model", folders["odd"],
+                        "--prompt", " ".join(map(str, prompt)), "--max-length", "20",
+                        "--use-full-precision"], cwd=ROOT, text=True, capture_output=True, timeout=110)
+    assert p.returncode == 0, p.stderr[-2000:]
+    got = json.loads(p.stdout.splitlines()[-1])["tokens"]
+    want, lead = R.greedy(ODD[0], WEIGHTS["odd"], prompt, 20)
+    assert lead > 1e-4 and got == want
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_trace_run(folders, tmp_path, dtype):
+    """bin/trace_run over a small trace, compared with the plain model."""
+    a, b = tokens(ODD, 140, 31), tokens(ODD, 70, 32)
+    steps = [dict(step=0, entries=[dict(id="a", tokens=a[:100], want=[0, 63, 64, 99])], end=[]),
+             dict(step=1, entries=[dict(id="a", tokens=a[100:102], want=[]),
+                                   dict(id="b", tokens=b[:69], want=[68])], end=[]),
+             dict(step=2, entries=[dict(id="b", tokens=b[69:], want=[0]),
+                                   dict(id="a", tokens=a[102:103], want=[0])], end=["b"]),
+             dict(step=3, entries=[dict(id="a", tokens=a[103:], want=[36]),
+                                   dict(id="c", tokens=b[:5], want=[4])], end=["a", "c"])]
+    want = {0: [a[:1], a[:64], a[:65], a[:100]], 2: [b, a[:103]], 1: [b[:69]], 3: [a, b[:5]]}
+    p = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", folders["odd"],
+                        "--dtype", dtype, "--out", str(tmp_path), "--max-tokens", "320"],
+                       input="".join(json.dumps(s) + "\n" for s in steps), text=True,
+                       capture_output=True, timeout=110)
+    assert p.returncode == 0, p.stderr[-2000:]
+    assert [l for l in p.stdout.splitlines() if l.startswith("done")] == ["done %d" % i for i in range(4)]
+    for i, seqs in want.items():
+        got = np.fromfile(tmp_path / ("%d.f32" % i), "<f4").reshape(len(seqs), -1)
+        close(got, np.stack([reference("odd", s)[0][-1] for s in seqs]), dtype == "float32")
