@@ -289,6 +289,21 @@ def vapipel_config(width, heads, dim, rank, ff, layers, vocab=32000, positions=4
                         for _ in range(layers)])
 
 
+# --model fesenex: (name, width, heads, key/value heads, head size, ff, layers)
+FESENEX_SIZES = [("width2048", 2048, 16, 4, 128, 5632, 8), ("width4096", 4096, 32, 8, 128, 11008, 8)]
+
+
+def fesenex_config(width, heads, kv_heads, dim, ff, layers, vocab=32000):
+    """Three attention layers to one of linear attention, all with a feed-forward."""
+    att = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** -0.5, bias_max=1024,
+               q_temp=dict(coef=0.1, every=1024), v_mix=True)
+    lin = dict(heads=heads, dim=dim, vdim=dim, decay=[1.0 - 2.0 ** -(3 + 7.0 * h / heads) for h in range(heads)])
+    mlp = dict(kind="dense", ff=ff, limit=7.0)
+    return dict(architecture="Fesenex", vocab=vocab, width=width, embedding=dict(scale=1.0), norm=dict(eps=1e-6),
+                layers=[dict(type="lightning" if i % 4 == 2 else "attention", mixer=lin if i % 4 == 2 else att,
+                             mlp=mlp) for i in range(layers)])
+
+
 def bench_decoder(cfg, B, prompt_len, decode, mtb, repeats):
     """Prefill and decode throughput of incremental decoding: generates of one
     new token (the prompts' steps alone) and of `decode`, best of `repeats`."""
@@ -318,32 +333,43 @@ def bench_decoder(cfg, B, prompt_len, decode, mtb, repeats):
             "prefill_ms": round(pre[0] * 1e3, 2), "prefill_steps": pre[1]}
 
 
-def bench_vapipel(args):
-    """--model vapipel: the latent-attention decoder (random weights) and LLaMA
+def bench_family(args):
+    """--model vapipel | fesenex: the family's decoder (random weights) and LLaMA
     at equal sizes, incremental decoding, one GPU.  One JSON line."""
     legs = []
-    for name, width, heads, dim, rank, ff, layers in VAPIPEL_SIZES:
-        cfgs = {"vapipel": vapipel_config(width, heads, dim, rank, ff, layers),
+    sizes = VAPIPEL_SIZES if args.model == "vapipel" else FESENEX_SIZES
+    for name, width, heads, *more, ff, layers in sizes:
+        if args.only_size and name != args.only_size:
+            continue
+        if args.model == "vapipel":
+            dim, rank = more
+            leg0, own = {"kv_rank": rank}, vapipel_config(width, heads, dim, rank, ff, layers)
+        else:
+            kv_heads, dim = more
+            leg0, own = {"kv_heads": kv_heads}, fesenex_config(width, heads, kv_heads, dim, ff, layers)
+        cfgs = {args.model: own,
                 "llama": dict(num_layers=layers, vocab_size=32000, num_heads=heads,
                               num_kv_heads=heads, hidden=width, intermediate=ff, rms_eps=1e-6,
                               rope_theta=10000.0)}
         for prompt in (args.prefill, 1024):
-            leg = {"size": name, "kv_rank": rank, "layers": layers, "batch": args.batch,
+            leg = {"size": name, **leg0, "layers": layers, "batch": args.batch,
                    "prompt": prompt, "decode": args.decode}
             for fam, cfg in cfgs.items():
-                if args.only_family and fam != args.only_family:
+                if args.only_family and (fam == "llama") != (args.only_family == "llama"):
                     continue
                 leg[fam] = bench_decoder(cfg, args.batch, prompt, args.decode,
                                          args.max_tokens_per_batch, args.steps)
             legs.append(leg)
             print(f"[bench] {json.dumps(leg)}", file=sys.stderr, flush=True)
-    head = legs[-1].get("vapipel") or legs[-1]["llama"]
+    head = legs[-1].get(args.model) or legs[-1]["llama"]
+    what = {"vapipel": "latent-attention decoder",
+            "fesenex": "softmax- and linear-attention decoder"}[args.model]
     print(json.dumps({
-        "metric": "decode tokens/s, latent-attention decoder beside LLaMA at equal size",
+        "metric": f"decode tokens/s, {what} beside LLaMA at equal size",
         "value": head["decode_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
         "warmup": 1, "ms_per_step": round(head["decode_step_us"] / 1e3, 4),
         "higher_is_better": True, "scaling": "strong", "vs_baseline": None, "dtype": "bf16",
-        "data": "synthetic", "config": {"model": "Vapipel", "global_batch": args.batch,
+        "data": "synthetic", "config": {"model": args.model.capitalize(), "global_batch": args.batch,
                                         "seq_len": 1024 + args.decode, "parallelism": "tp1"},
         "legs": legs}), flush=True)
 
@@ -428,11 +454,12 @@ def main():
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
     ap.add_argument("--mode", choices=["spec", "incr"], default="spec")
-    ap.add_argument("--model", choices=["llama", "vapipel"], default="llama",
-                    help="llama: the headline workload; vapipel: prefill and decode throughput "
-                         "of the latent-attention decoder beside LLaMA at equal sizes (one GPU)")
-    ap.add_argument("--only-family", choices=["llama", "vapipel"], default=None,
-                    help="--model vapipel: run one of the two (profiling)")
+    ap.add_argument("--model", choices=["llama", "vapipel", "fesenex"], default="llama",
+                    help="llama: the headline workload; vapipel, fesenex: prefill and decode throughput "
+                         "of that family's decoder beside LLaMA at equal sizes (one GPU)")
+    ap.add_argument("--only-family", choices=["llama", "vapipel", "fesenex"], default=None,
+                    help="--model vapipel | fesenex: run one of the two (profiling)")
+    ap.add_argument("--only-size", default=None, help="--model vapipel | fesenex: run one size (profiling)")
     ap.add_argument("--batch", type=int, default=8)
     ap.add_argument("--prefill", type=int, default=128)
     ap.add_argument("--decode", type=int, default=128)
@@ -488,10 +515,10 @@ def main():
     # N-rank path on a one-GPU box (with FFMI_TP_TRANSPORT=xgmi-only, since
     # RCCL refuses two ranks on one GPU); timings are then not a scaling result
     fa.set_device(int(os.environ.get("FFMI_BENCH_DEVICE", local)))
-    if args.model == "vapipel":
+    if args.model != "llama":
         if world > 1:
-            raise SystemExit("--model vapipel runs on one GPU")
-        bench_vapipel(args)
+            raise SystemExit(f"--model {args.model} runs on one GPU")
+        bench_family(args)
         return
     comm = None
     transport = "rccl"

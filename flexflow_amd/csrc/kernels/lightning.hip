@@ -145,77 +145,90 @@ __device__ __forceinline__ bf8 read_columns(const uint16_t *tile, int kb, int c0
   return __builtin_bit_cast(bf8, __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
 }
 
-// A workgroup per (64 value columns, head, span).  Per chunk of 64 tokens
+// A workgroup per (VS value columns, head, span).  Per chunk of 64 tokens
 //   O^T = S_prev^T Q^T, row i times d^(i + 1),  + V^T . P^T with
 //   P = (q_i . k_j) d^(i - j) for j <= i;
 //   S   = d^n S_prev + K^T . (v_j d^(n - 1 - j))
-// Wave w: rows 16 w .. of the outputs, value columns 16 w .. of the state, which
-// stays in its registers (lane: 4 rows dt * 16 + 4g .. of one column) and goes to
-// LDS once a chunk as the operand [column][row] of every wave's outputs.
-template <int KS>
-__global__ __launch_bounds__(256) void lightning_chunk_kernel(const char *__restrict__ blob,
+// Wave w: rows 16 w .. of the outputs, and of the state 16 value columns and
+// an even share of the rows.  Its part of the state stays in its registers
+// (lane: 4 rows of one column) and goes to LDS once a chunk as the operand
+// [column][row] of every wave's outputs.
+template <int KS, int VS>
+__global__ __launch_bounds__(256, KS <= 4 || VS == 16 ? 2 : 1) void lightning_chunk_kernel(const char *__restrict__ blob,
                                                               int off_spans, Lightning a, int limit) {
-  constexpr int DK = KS * 32, LDK = DK + 8, LDV = 64 + 8, C = kLightningChunk;
-  __shared__ __attribute__((aligned(16))) uint16_t sK[C * LDK], sV[C * LDV], sHi[64 * LDK], sLo[64 * LDK];
+  constexpr int DK = KS * 32, LDK = DK + 8, LDV = VS + 8, C = kLightningChunk;
+  constexpr int VT = VS / 16, WD = 4 / VT;        // value tiles; waves that share one
+  constexpr int ND = (2 * KS + WD - 1) / WD;      // a wave's row tiles of the state
+  constexpr int NV = (C * VS / 8 + 255) / 256;    // 16-byte chunks of V per thread
+  __shared__ __attribute__((aligned(16))) uint16_t sK[C * LDK], sV[C * LDV], sHi[VS * LDK], sLo[VS * LDK];
   __shared__ float pw[C + 1];
   const PagedSpan sp = reinterpret_cast<const PagedSpan *>(blob + off_spans)[blockIdx.z];
   if (sp.n <= limit) return;
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int h = blockIdx.y, c0 = blockIdx.x * 64, cols = a.H * (2 * a.dg + a.vg);
+  const int h = blockIdx.y, c0 = blockIdx.x * VS, cols = a.H * (2 * a.dg + a.vg);
   const uint16_t *Q = a.qkv + (size_t)sp.t0 * cols + (size_t)h * a.dg;
   const uint16_t *K = Q + (size_t)a.H * a.dg;
   const uint16_t *V = a.qkv + (size_t)sp.t0 * cols + (size_t)2 * a.H * a.dg + (size_t)h * a.vg + c0;
   if (tid <= C) pw[tid] = a.powers[(size_t)h * (C + 1) + tid];
-  const int vw = min(64, a.vg - c0);  // value columns of this workgroup
+  const int vw = min(VS, a.vg - c0);  // value columns of this workgroup
+  const int i = wave * 16 + l15;      // this lane's row of the chunk
 
   const u4 zero = {0, 0, 0, 0};
-  u4 pk[KS], pv[2];
+  u4 pk[KS], pv[NV], pq[KS];
   auto fetch = [&](int t0) {  // rows past the span and columns past the widths: zeros
 #pragma unroll
-    for (int i = 0; i < KS; ++i) {
-      const int ch = tid + i * 256, r = ch / (DK / 8), c = ch % (DK / 8) * 8;
-      pk[i] = zero;
-      if (t0 + r < sp.n && c < a.dg) pk[i] = *reinterpret_cast<const u4 *>(K + (size_t)(t0 + r) * cols + c);
+    for (int j = 0; j < KS; ++j) {
+      const int ch = tid + j * 256, r = ch / (DK / 8), c = ch % (DK / 8) * 8;
+      pk[j] = zero;
+      if (t0 + r < sp.n && c < a.dg) pk[j] = *reinterpret_cast<const u4 *>(K + (size_t)(t0 + r) * cols + c);
     }
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const int ch = tid + i * 256, r = ch >> 3, c = (ch & 7) * 8;
-      pv[i] = zero;
-      if (t0 + r < sp.n && c < vw) pv[i] = *reinterpret_cast<const u4 *>(V + (size_t)(t0 + r) * cols + c);
+    for (int j = 0; j < NV; ++j) {
+      const int ch = tid + j * 256, r = ch / (VS / 8), c = ch % (VS / 8) * 8;
+      pv[j] = zero;
+      if (r < C && t0 + r < sp.n && c < vw)
+        pv[j] = *reinterpret_cast<const u4 *>(V + (size_t)(t0 + r) * cols + c);
+    }
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      pq[ks] = zero;
+      if (t0 + i < sp.n && ks * 32 < a.dg)
+        pq[ks] = *reinterpret_cast<const u4 *>(Q + (size_t)(t0 + i) * cols + ks * 32 + 8 * g);
     }
   };
   auto stage = [&]() {
 #pragma unroll
-    for (int i = 0; i < KS; ++i) {
-      const int ch = tid + i * 256;
-      *reinterpret_cast<u4 *>(&sK[(ch / (DK / 8)) * LDK + ch % (DK / 8) * 8]) = pk[i];
+    for (int j = 0; j < KS; ++j) {
+      const int ch = tid + j * 256;
+      *reinterpret_cast<u4 *>(&sK[(ch / (DK / 8)) * LDK + ch % (DK / 8) * 8]) = pk[j];
     }
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const int ch = tid + i * 256;
-      *reinterpret_cast<u4 *>(&sV[(ch >> 3) * LDV + (ch & 7) * 8]) = pv[i];
+    for (int j = 0; j < NV; ++j) {
+      const int ch = tid + j * 256, r = ch / (VS / 8);
+      if (r < C) *reinterpret_cast<u4 *>(&sV[r * LDV + ch % (VS / 8) * 8]) = pv[j];
     }
   };
   fetch(0);
-  // the state: rows dt * 16 + 4g + e, column wave * 16 + l15
-  f4 st[2 * KS];
-  const int vcol = wave * 16 + l15;
+  // the state: rows (d0 + dt) * 16 + 4g + e, column vcol
+  f4 st[ND];
+  const int vcol = wave % VT * 16 + l15, d0 = wave / VT * ND;
   float *S = a.state + (((size_t)sp.slot * a.H + h) * a.dg) * a.vg + c0 + vcol;
 #pragma unroll
-  for (int dt = 0; dt < 2 * KS; ++dt) {
+  for (int dt = 0; dt < ND; ++dt) {
     st[dt] = f4{0.f, 0.f, 0.f, 0.f};
-    if (sp.pos0 > 0 && dt * 16 < a.dg && vcol < vw)
+    if (sp.pos0 > 0 && (d0 + dt) * 16 < a.dg && vcol < vw)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) st[dt][e] = S[(size_t)(dt * 16 + 4 * g + e) * a.vg];
+      for (int e = 0; e < 4; ++e) st[dt][e] = S[(size_t)((d0 + dt) * 16 + 4 * g + e) * a.vg];
   }
   auto publish = [&]() {
 #pragma unroll
-    for (int dt = 0; dt < 2 * KS; ++dt) {
+    for (int dt = 0; dt < ND; ++dt) {
+      if (2 * KS % WD && d0 + dt >= 2 * KS) continue;
       __bf16 hi[4], lo[4];
 #pragma unroll
       for (int e = 0; e < 4; ++e) split2(st[dt][e], hi[e], lo[e]);
-      const int at = vcol * LDK + dt * 16 + 4 * g;
+      const int at = vcol * LDK + (d0 + dt) * 16 + 4 * g;
       auto two = [](const __bf16 *v) {
         return make_uint2(__builtin_bit_cast(uint16_t, v[0]) | ((uint32_t)__builtin_bit_cast(uint16_t, v[1]) << 16),
                           __builtin_bit_cast(uint16_t, v[2]) | ((uint32_t)__builtin_bit_cast(uint16_t, v[3]) << 16));
@@ -225,59 +238,72 @@ __global__ __launch_bounds__(256) void lightning_chunk_kernel(const char *__rest
     }
   };
   publish();
-  const int i = wave * 16 + l15;  // this lane's row of the chunk
+  __syncthreads();  // (pw)
+  // this lane's decays: of its weights (key <= row), of its row, of its values
+  const auto key_of = [&](int kb, int e) { return kb * 32 + 4 * g + (e & 3) + 16 * (e >> 2); };
+  float fp[2][8], fv[2][8];
+#pragma unroll
+  for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int key = key_of(kb, e);
+      fp[kb][e] = key <= i ? pw[max(i - key, 0)] : 0.f;
+      fv[kb][e] = pw[C - 1 - key];
+    }
+  const float fi = pw[i + 1];
   for (int t0 = 0; t0 < sp.n; t0 += C) {
     const int n = min(C, sp.n - t0);
+    if (n < C)  // (rows past the span are zeros)
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) fv[kb][e] = pw[max(n - 1 - key_of(kb, e), 0)];
     stage();
     bf8 q[KS];
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      u4 v = zero;
-      if (i < n && ks * 32 < a.dg)
-        v = *reinterpret_cast<const u4 *>(Q + (size_t)(t0 + i) * cols + ks * 32 + 8 * g);
-      q[ks] = __builtin_bit_cast(bf8, v);
-    }
+    for (int ks = 0; ks < KS; ++ks) q[ks] = __builtin_bit_cast(bf8, pq[ks]);
     __syncthreads();
     if (t0 + C < sp.n) fetch(t0 + C);
-    // from the state before the chunk
-    f4 o[4];
+    // from the state before the chunk: value and remainder, a chain each
+    f4 o[VT], olo[VT];
 #pragma unroll
-    for (int vt = 0; vt < 4; ++vt) {
-      o[vt] = f4{0.f, 0.f, 0.f, 0.f};
+    for (int vt = 0; vt < VT; ++vt) o[vt] = olo[vt] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
+    for (int ks = 0; ks < KS; ++ks)
+#pragma unroll
+      for (int vt = 0; vt < VT; ++vt) {
         const int at = (vt * 16 + l15) * LDK + ks * 32 + 8 * g;
         o[vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf8 *>(&sHi[at]), q[ks],
                                                         o[vt], 0, 0, 0);
-        o[vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf8 *>(&sLo[at]), q[ks],
-                                                        o[vt], 0, 0, 0);
+        olo[vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf8 *>(&sLo[at]), q[ks],
+                                                          olo[vt], 0, 0, 0);
       }
-      o[vt] *= pw[i + 1];
-    }
+#pragma unroll
+    for (int vt = 0; vt < VT; ++vt) o[vt] = (o[vt] + olo[vt]) * fi;
     // within the chunk: keys of 32 at a time
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb) {
       if (kb * 32 > wave * 16 + 15) continue;  // (all after this wave's rows)
       bf8 ph, plo;
+      f4 s[2];
+      s[0] = s[1] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        f4 s = f4{0.f, 0.f, 0.f, 0.f};
+      for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
-        for (int ks = 0; ks < KS; ++ks)
-          s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+        for (int j = 0; j < 2; ++j)
+          s[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
               *reinterpret_cast<const bf8 *>(&sK[(kb * 32 + j * 16 + l15) * LDK + ks * 32 + 8 * g]), q[ks],
-              s, 0, 0, 0);
+              s[j], 0, 0, 0);
+#pragma unroll
+      for (int j = 0; j < 2; ++j)
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          const int key = kb * 32 + j * 16 + 4 * g + e;
-          const float w = key <= i ? s[e] * pw[max(i - key, 0)] : 0.f;
           __bf16 hi, lo;
-          split2(w, hi, lo);
+          split2(s[j][e] * fp[kb][j * 4 + e], hi, lo);
           ph[j * 4 + e] = hi, plo[j * 4 + e] = lo;
         }
-      }
 #pragma unroll
-      for (int vt = 0; vt < 4; ++vt) {
+      for (int vt = 0; vt < VT; ++vt) {
         const bf8 v = read_columns<LDV>(sV, kb, vt * 16);
         o[vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, ph, o[vt], 0, 0, 0);
         o[vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, plo, o[vt], 0, 0, 0);
@@ -286,21 +312,21 @@ __global__ __launch_bounds__(256) void lightning_chunk_kernel(const char *__rest
     // the state after the chunk
     const float dn = pw[n];
 #pragma unroll
-    for (int dt = 0; dt < 2 * KS; ++dt) st[dt] *= dn;
+    for (int dt = 0; dt < ND; ++dt) st[dt] *= dn;
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb) {
-      const bf8 v = read_columns<LDV>(sV, kb, wave * 16);
+      const bf8 v = read_columns<LDV>(sV, kb, wave % VT * 16);
       bf8 vh, vl;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
-        const int key = kb * 32 + 4 * g + (e & 3) + 16 * (e >> 2);
         __bf16 hi, lo;
-        split2((float)v[e] * pw[max(n - 1 - key, 0)], hi, lo);  // (rows past the span are zeros)
+        split2((float)v[e] * fv[kb][e], hi, lo);
         vh[e] = hi, vl[e] = lo;
       }
 #pragma unroll
-      for (int dt = 0; dt < 2 * KS; ++dt) {
-        const bf8 k = read_columns<LDK>(sK, kb, dt * 16);
+      for (int dt = 0; dt < ND; ++dt) {
+        if (2 * KS % WD && d0 + dt >= 2 * KS) continue;
+        const bf8 k = read_columns<LDK>(sK, kb, (d0 + dt) * 16);
         st[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, vh, st[dt], 0, 0, 0);
         st[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, vl, st[dt], 0, 0, 0);
       }
@@ -308,17 +334,17 @@ __global__ __launch_bounds__(256) void lightning_chunk_kernel(const char *__rest
     if (i < n) {
       float *dst = a.o + (size_t)(sp.t0 + t0 + i) * a.H * a.vg + (size_t)h * a.vg + c0 + 4 * g;
 #pragma unroll
-      for (int vt = 0; vt < 4; ++vt)
+      for (int vt = 0; vt < VT; ++vt)
         if (vt * 16 < vw) *reinterpret_cast<f4 *>(dst + vt * 16) = o[vt];
     }
     __syncthreads();
     if (t0 + C < sp.n) publish();
   }
 #pragma unroll
-  for (int dt = 0; dt < 2 * KS; ++dt)
-    if (dt * 16 < a.dg && vcol < vw)
+  for (int dt = 0; dt < ND; ++dt)
+    if ((d0 + dt) * 16 < a.dg && vcol < vw)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) S[(size_t)(dt * 16 + 4 * g + e) * a.vg] = st[dt][e];
+      for (int e = 0; e < 4; ++e) S[(size_t)((d0 + dt) * 16 + 4 * g + e) * a.vg] = st[dt][e];
 }
 
 hipError_t launch_lightning_chunks(const char *blob, int off_spans, int num_spans, const Lightning &a,
@@ -328,14 +354,23 @@ hipError_t launch_lightning_chunks(const char *blob, int off_spans, int num_span
   const int cols = a.H * (2 * a.dg + a.vg);
   const long n = (long)a.T * (cols / 8);
   hipLaunchKernelGGL(lightning_qkv_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, a, cols);
-  const dim3 grid((a.vg + 63) / 64, a.H, num_spans);
-#define FFMI_LC(KS)                                                                                   \
-  hipLaunchKernelGGL((lightning_chunk_kernel<KS>), grid, dim3(256), 0, s, blob, off_spans, a, limit)
+  // narrow workgroups where the spans and heads alone do not fill the chip
+  const long wide = (long)a.H * num_spans * ((a.vg + 63) / 64);
+#define FFMI_LC2(KS, VS)                                                                                  \
+  hipLaunchKernelGGL((lightning_chunk_kernel<KS, VS>), dim3((a.vg + VS - 1) / VS, a.H, num_spans), dim3(256), \
+                     0, s, blob, off_spans, a, limit)
+#define FFMI_LC(KS)                        \
+  do {                                     \
+    if (wide <= 128) FFMI_LC2(KS, 16);     \
+    else if (wide <= 256) FFMI_LC2(KS, 32); \
+    else FFMI_LC2(KS, 64);                 \
+  } while (0)
   if (a.dg <= 32) FFMI_LC(1);
   else if (a.dg <= 64) FFMI_LC(2);
   else if (a.dg <= 128) FFMI_LC(4);
   else FFMI_LC(8);
 #undef FFMI_LC
+#undef FFMI_LC2
   return hipGetLastError();
 }
 

@@ -57,7 +57,7 @@ struct AttnArgs {
 // rows a slot, [slot][G][16][vp] and [slot][G][16][2]
 hipError_t launch_paged_attn(const char *blob, const PagedLists &pl, const AttnArgs &a, float *slabs,
                              float *ml, hipStream_t s);
-constexpr int kAttnTiles = 8;  // row tiles of a workgroup in prompts
+constexpr int kAttnTiles = 4;  // row tiles of a workgroup in prompts
 // any width up to kAttnRowsMax, one workgroup per row of every block (fp32, or
 // bf16 with scale and bias for base-2 exponents as above)
 constexpr int kAttnRowsMax = 1024;

@@ -8,11 +8,12 @@
 namespace ffmi {
 
 typedef uint32_t u4 __attribute__((ext_vector_type(4)));
+typedef float f2 __attribute__((ext_vector_type(2)));
 
 int attn_width(int dim) { return dim <= 64 ? 64 : dim <= 128 ? 128 : dim <= 256 ? 256 : 0; }
 
 // ---------------------------------------------------------------------------
-// queries, keys, values: one wave per (token, head)
+// queries, keys, values: one wave per (tokens, head)
 // ---------------------------------------------------------------------------
 // column n of a row of deferred sums; several slabs: their loads together
 __device__ __forceinline__ float slab_sum(const Partials &y, size_t slab, size_t at) {
@@ -28,55 +29,144 @@ __device__ __forceinline__ float slab_sum(const Partials &y, size_t slab, size_t
   return v;
 }
 
-template <class E, int NE>
+__device__ __forceinline__ void store4(uint16_t *p, float a, float b, float c, float d) {
+  *reinterpret_cast<uint2 *>(p) =
+      make_uint2(f2bf(a) | ((uint32_t)f2bf(b) << 16), f2bf(c) | ((uint32_t)f2bf(d) << 16));
+}
+__device__ __forceinline__ void store4(float *p, float a, float b, float c, float d) {
+  *reinterpret_cast<f4 *>(p) = f4{a, b, c, d};
+}
+
+__device__ __forceinline__ f2 slab_sum2(const Partials &y, size_t slab, size_t at) {
+  f2 v = *reinterpret_cast<const f2 *>(y.p + at);
+  if (y.S > 1) {
+    f2 p[7];
+#pragma unroll
+    for (int s = 1; s < 8; ++s)
+      p[s - 1] = *reinterpret_cast<const f2 *>(y.p + at + (size_t)min(s, y.S - 1) * slab);
+#pragma unroll
+    for (int s = 1; s < 8; ++s)
+      if (s < y.S) v[0] += p[s - 1][0], v[1] += p[s - 1][1];
+  }
+  return v;
+}
+__device__ __forceinline__ void store2(uint16_t *p, f2 v) {
+  *reinterpret_cast<uint32_t *>(p) = f2bf(v[0]) | ((uint32_t)f2bf(v[1]) << 16);
+}
+__device__ __forceinline__ void store2(float *p, f2 v) { *reinterpret_cast<f2 *>(p) = v; }
+
+// A wave takes NT consecutive batch tokens of one head, a lane NE columns in
+// neighbouring pairs (NE == 1: one).
+template <class E, int NE, int NT>
 __global__ __launch_bounds__(256) void attn_prep_kernel(const PagedToken *__restrict__ tok, int T,
                                                         AttnPrep a) {
   const int heads = a.H + 2 * a.G, lane = threadIdx.x & 63;
   const long id = blockIdx.x * 4L + (threadIdx.x >> 6);
-  const int hd = (int)(id % heads);
-  const long t = id / heads;
-  if (t >= T) return;
+  const int hd = (int)(id % heads), t0 = (int)(id / heads) * NT;
+  if (t0 >= T) return;
   const bool isv = hd >= a.H + a.G, isq = hd < a.H;
   const int g = isq ? 0 : (hd - a.H) % a.G;
   const int wd = isv ? a.vg : a.dg;  // columns of this head
   const int col = isv ? (a.H + a.G) * a.dg + g * a.vg : hd * a.dg;
-  const PagedToken tk = tok[t];
-  const size_t slab = (size_t)T * a.y.NP, row = (size_t)t * a.y.NP + col;
-  float v[NE], ss = 0.f;
+  const size_t slab = (size_t)T * a.y.NP;
+  const auto column = [&](int i) { return NE == 1 ? lane : (i >> 1) * 128 + lane * 2 + (i & 1); };
+  PagedToken tk[NT];
+  float v[NT][NE], ss[NT];
+#pragma unroll
+  for (int k = 0; k < NT; ++k) tk[k] = tok[min(t0 + k, T - 1)];
+#pragma unroll
+  for (int k = 0; k < NT; ++k) {
+    const size_t row = (size_t)min(t0 + k, T - 1) * a.y.NP + col;
+    if constexpr (NE == 1) {
+      v[k][0] = lane < wd ? slab_sum(a.y, slab, row + lane) : 0.f;
+    } else {
+#pragma unroll
+      for (int i = 0; i < NE; i += 2) {
+        const int c = column(i);  // (the widths are even)
+        f2 p = f2{0.f, 0.f};
+        if (c < wd) p = slab_sum2(a.y, slab, row + c);
+        v[k][i] = p[0], v[k][i + 1] = p[1];
+      }
+    }
+  }
 #pragma unroll
   for (int i = 0; i < NE; ++i) {
-    const int c = lane + i * 64;
-    v[i] = 0.f;
-    if (c < wd) v[i] = slab_sum(a.y, slab, row + c) + a.bias[col + c];
-    ss = fmaf(v[i], v[i], ss);
+    const int c = column(i);
+    const float b = c < wd ? a.bias[col + c] : 0.f;
+#pragma unroll
+    for (int k = 0; k < NT; ++k) v[k][i] += b;
   }
-  const size_t page = (size_t)(tk.row / kPageTokens), key = tk.row % kPageTokens;
   if (isv) {
-    E *dst = (E *)a.vc + (page * a.G + g) * kPageTokens * a.vp;
-    const float lam = a.vmix ? *a.vmix : 0.f;
-    float *first = a.first ? a.first + ((size_t)t * a.G + g) * a.vg : nullptr;
+    if (a.first) {
+      const float lam = a.vmix ? *a.vmix : 0.f;
+#pragma unroll
+      for (int k = 0; k < NT; ++k) {
+        if (t0 + k >= T) break;
+        float *first = a.first + ((size_t)(t0 + k) * a.G + g) * a.vg;
+#pragma unroll
+        for (int i = 0; i < NE; ++i) {
+          const int c = column(i);
+          if (c >= wd) continue;
+          if (a.vmix) v[k][i] = (1.0f - lam) * v[k][i] + lam * first[c];
+          else first[c] = v[k][i];
+        }
+      }
+    }
+    // four tokens in one aligned run of a page: their values lie side by side
+    bool run = NT == 4 && t0 + NT <= T && tk[0].row % 4 == 0;
+#pragma unroll
+    for (int k = 1; k < NT; ++k) run = run && tk[k].row == tk[0].row + k;
 #pragma unroll
     for (int i = 0; i < NE; ++i) {
-      const int c = lane + i * 64;
-      if (c < wd && first) {
-        if (a.vmix) v[i] = (1.0f - lam) * v[i] + lam * first[c];
-        else first[c] = v[i];
+      const int c = column(i);
+      if (c >= a.vp) continue;
+      if (run) {
+        E *dst = (E *)a.vc + ((size_t)(tk[0].row / kPageTokens) * a.G + g) * kPageTokens * a.vp +
+                 val_off(tk[0].row % kPageTokens, c, a.vp);
+        store4(dst, v[0][i], v[NT > 1 ? 1 : 0][i], v[NT > 2 ? 2 : 0][i], v[NT > 3 ? 3 : 0][i]);
+        continue;
       }
-      if (c < a.vp) st_elem(dst + val_off((int)key, c, a.vp), v[i]);
+#pragma unroll
+      for (int k = 0; k < NT; ++k)
+        if (t0 + k < T)
+          st_elem((E *)a.vc + ((size_t)(tk[k].row / kPageTokens) * a.G + g) * kPageTokens * a.vp +
+                      val_off(tk[k].row % kPageTokens, c, a.vp),
+                  v[k][i]);
     }
     return;
   }
 #pragma unroll
-  for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
-  float r = inv_rms(ss, a.dim, a.eps);
-  if (isq && a.coef != 0.f) r *= 1.0f + a.coef * logf((float)((tk.pos + 1) / a.every + 1));
-  const float *w = isq ? a.qnorm : a.knorm;
-  E *dst = isq ? (E *)a.q + ((size_t)t * a.H + hd) * a.dp
-               : (E *)a.kc + (page * a.G + g) * kPageTokens * a.dp;
+  for (int k = 0; k < NT; ++k) {
+    ss[k] = 0.f;
 #pragma unroll
-  for (int i = 0; i < NE; ++i) {
-    const int c = lane + i * 64;
-    if (c < a.dp) st_elem(dst + (isq ? c : key_off((int)key, c, a.dp)), c < wd ? v[i] * r * w[c] : 0.f);
+    for (int i = 0; i < NE; ++i) ss[k] = fmaf(v[k][i], v[k][i], ss[k]);
+  }
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1)
+#pragma unroll
+    for (int k = 0; k < NT; ++k) ss[k] += __shfl_xor(ss[k], o);
+  const float *w = isq ? a.qnorm : a.knorm;
+#pragma unroll
+  for (int k = 0; k < NT; ++k) {
+    if (t0 + k >= T) break;
+    float r = inv_rms(ss[k], a.dim, a.eps);
+    if (isq && a.coef != 0.f) r *= 1.0f + a.coef * logf((float)((tk[k].pos + 1) / a.every + 1));
+    const int key = tk[k].row % kPageTokens;
+    E *dst = isq ? (E *)a.q + ((size_t)(t0 + k) * a.H + hd) * a.dp
+                 : (E *)a.kc + ((size_t)(tk[k].row / kPageTokens) * a.G + g) * kPageTokens * a.dp;
+    if constexpr (NE == 1) {
+      if (lane < a.dp)
+        st_elem(dst + (isq ? lane : key_off(key, lane, a.dp)), lane < wd ? v[k][0] * r * w[lane] : 0.f);
+    } else {
+#pragma unroll
+      for (int i = 0; i < NE; i += 2) {
+        const int c = column(i);
+        if (c >= a.dp) continue;
+        f2 o = f2{0.f, 0.f};
+        if (c < wd) o = f2{v[k][i] * r * w[c], v[k][i + 1] * r * w[c + 1]};
+        store2(dst + (isq ? c : key_off(key, c, a.dp)), o);
+      }
+    }
   }
 }
 
@@ -86,17 +176,25 @@ hipError_t launch_attn_prep(const char *blob, int off_tokens, int T, const AttnP
   const int wide = std::max(std::max(a.dp, a.vp), std::max(a.dg, a.vg));
   if (wide > 1024 || a.y.S < 1 || a.y.S > 8 || a.every < 1) return hipErrorInvalidValue;
   const PagedToken *tok = reinterpret_cast<const PagedToken *>(blob + off_tokens);
-  const dim3 grid((unsigned)(((long)T * (a.H + 2 * a.G) + 3) / 4));
-#define FFMI_AP(E, NE) hipLaunchKernelGGL((attn_prep_kernel<E, NE>), grid, dim3(256), 0, s, tok, T, a)
+#define FFMI_AP(E, NE, NT)                                                                           \
+  hipLaunchKernelGGL((attn_prep_kernel<E, NE, NT>),                                                \
+                     dim3((unsigned)(((long)((T + NT - 1) / NT) * (a.H + 2 * a.G) + 3) / 4)),      \
+                     dim3(256), 0, s, tok, T, a)
+#define FFMI_APN(E, NE)           \
+  do {                            \
+    if (T >= 128) FFMI_AP(E, NE, 4); \
+    else FFMI_AP(E, NE, 1);       \
+  } while (0)
   if (f32) {
-    if (wide <= 256) FFMI_AP(float, 4);
-    else FFMI_AP(float, 16);
+    if (wide <= 256) FFMI_AP(float, 4, 1);
+    else FFMI_AP(float, 16, 1);
   } else {
-    if (wide <= 64) FFMI_AP(uint16_t, 1);
-    else if (wide <= 128) FFMI_AP(uint16_t, 2);
-    else if (wide <= 256) FFMI_AP(uint16_t, 4);
-    else FFMI_AP(uint16_t, 16);
+    if (wide <= 64) FFMI_APN(uint16_t, 1);
+    else if (wide <= 128) FFMI_APN(uint16_t, 2);
+    else if (wide <= 256) FFMI_APN(uint16_t, 4);
+    else FFMI_AP(uint16_t, 16, 1);
   }
+#undef FFMI_APN
 #undef FFMI_AP
   return hipGetLastError();
 }
@@ -112,30 +210,31 @@ hipError_t launch_attn_prep(const char *blob, int off_tokens, int T, const AttnP
 //
 // Up to 16 rows (decoding, short portions): operands straight from memory, the
 // workgroup's four waves over half-pages, their results merged through LDS.
-// More rows (prompts): four waves of two row tiles each over pages staged in
-// LDS, double-buffered, the next page's loads in flight through registers.
-template <int KS, int NK>
-__device__ __forceinline__ void score_bias(const float *bh, int D, bool far, bool whole, int qpos,
-                                           int key0, float scale, f4 (&s)[NK], float &mx) {
+// More rows (prompts): four waves of 16 rows each over pages staged in LDS,
+// double-buffered, the next page's loads in flight through registers.
+//
+// A lane's four keys ask for four consecutive distances: one 16-byte read of the
+// bias table, issued a page ahead like the page itself.
+__device__ __forceinline__ f4 bias4(const float *bh, int D, int qpos, int k0) {
+  const float *p = bh + (D - min(max(qpos - k0 - 3, -4), D));
+  return f4{p[0], p[1], p[2], p[3]};
+}
+// s = s * scale + b, keys after the query out (whole: none of the wave's are);
+// the maximum taken along
+template <int NK>
+__device__ __forceinline__ void bias_and_mask(const f4 (&b)[NK], bool whole, int qpos, int key0,
+                                              float scale, f4 (&s)[NK], float &mx) {
 #pragma unroll
-  for (int i = 0; i < NK; ++i) {
-    const int k0 = key0 + i * 16;
-    f4 b;
-    if (far) {
-      const float f = bh[0];
-      b = f4{f, f, f, f};
-    } else {
-      const float *p = bh + (D - min(max(qpos - k0 - 3, -4), D));
-      b = f4{p[0], p[1], p[2], p[3]};
-    }
+  for (int i = 0; i < NK; ++i)
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      float v = fmaf(s[i][e], scale, b[e]);
-      if (!whole && k0 + e > qpos) v = -INFINITY;
-      s[i][e] = v;
-      mx = fmaxf(mx, v);
-    }
-  }
+    for (int e = 0; e < 4; ++e) s[i][e] = fmaf(s[i][e], scale, b[i][e]);
+  if (!whole)
+#pragma unroll
+    for (int i = 0; i < NK; ++i)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s[i][e] = key0 + i * 16 + e > qpos ? -INFINITY : s[i][e];
+#pragma unroll
+  for (int i = 0; i < NK; ++i) mx = fmaxf(fmaxf(fmaxf(mx, s[i][0]), fmaxf(s[i][1], s[i][2])), s[i][3]);
 }
 __device__ __forceinline__ bf8 pack_weights(const f4 &lo, const f4 &hi) {
   bf8 p;
@@ -167,8 +266,19 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
   const uint16_t *Kc = (const uint16_t *)a.kc, *Vc = (const uint16_t *)a.vc;
   const int units = 2 * bk.ntiles;
 
+  // (the queries first: loads return in order, so the loop never waits for
+  // them behind a prefetch)
+  bf8 q[KS];
+  {
+    const uint16_t *qr = (const uint16_t *)a.q + ((size_t)token * a.H + head) * DP + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) q[ks] = *reinterpret_cast<const bf8 *>(qr + ks * 32);
+  }
   bf8 k[2][KS], v[VT];
+  f4 b[2];
   auto fetch = [&](int u) {
+    const int k0 = bk.tile0 * 64 + u * 32 + 4 * g;
+    b[0] = bias4(bh, a.D, qpos, k0), b[1] = bias4(bh, a.D, qpos, k0 + 16);
     const size_t page = (size_t)(u < 2 ? bk.page0 : table[bk.tile0 + (u >> 1)]) * a.G + grp;
     const uint16_t *kp = Kc + page * (64 * DP) + (size_t)(u & 1) * (2 * KS * 512) + lane * 8;
     const uint16_t *vp = Vc + page * (64 * VP) + (size_t)(u & 1) * (VP * 32) + l15 * 32 + g * 8;
@@ -181,33 +291,26 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
     for (int d = 0; d < VT; ++d) v[d] = *reinterpret_cast<const bf8 *>(vp + d * 512);
   };
   if (wave < units) fetch(wave);
-  bf8 q[KS];
-  {
-    const uint16_t *qr = (const uint16_t *)a.q + ((size_t)token * a.H + head) * DP + 8 * g;
-#pragma unroll
-    for (int ks = 0; ks < KS; ++ks) q[ks] = *reinterpret_cast<const bf8 *>(qr + ks * 32);
-  }
   f4 acc[VT];
 #pragma unroll
   for (int d = 0; d < VT; ++d) acc[d] = f4{0.f, 0.f, 0.f, 0.f};
   float m = -1e30f, l = 0.f;
   for (int u = wave; u < units; u += 4) {
     f4 s[2];
+    s[0] = s[1] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      s[i] = f4{0.f, 0.f, 0.f, 0.f};
+    for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks)
+      for (int i = 0; i < 2; ++i)
         s[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k[i][ks], q[ks], s[i], 0, 0, 0);
-    }
     bf8 vv[VT];
 #pragma unroll
     for (int d = 0; d < VT; ++d) vv[d] = v[d];
+    const f4 bb[2] = {b[0], b[1]};
     if (u + 4 < units) fetch(u + 4);
     const int base = bk.tile0 * 64 + u * 32;
     float mx = -1e30f;
-    score_bias<KS, 2>(bh, a.D, qmin - (base + 31) >= a.D, base + 31 <= qmin, qpos, base + 4 * g,
-                      a.scale, s, mx);
+    bias_and_mask<2>(bb, base + 31 <= qmin, qpos, base + 4 * g, a.scale, s, mx);
     mx = fmaxf(mx, __shfl_xor(mx, 16));
     mx = fmaxf(mx, __shfl_xor(mx, 32));
     const float mn = fmaxf(m, mx), alpha = __builtin_amdgcn_exp2f(m - mn);
@@ -283,21 +386,45 @@ template <int DP, int VP>
 __device__ __forceinline__ void attn_many_rows(const char *__restrict__ blob, const PagedBlock &bk,
                                                const AttnArgs &a, float *__restrict__ slabs,
                                                float *__restrict__ ml, char *lds) {
-  constexpr int KS = DP / 32, VT = VP / 16, MR = 2;
+  constexpr int KS = DP / 32, VT = VP / 16;
   uint16_t *sK = reinterpret_cast<uint16_t *>(lds), *sV = sK + 2 * 64 * DP;
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int grp = blockIdx.y, R = a.H / a.G;
   const int32_t *table = reinterpret_cast<const int32_t *>(blob) + bk.table;
   const uint16_t *Kc = (const uint16_t *)a.kc, *Vc = (const uint16_t *)a.vc;
+  // this wave's rows (past the block: its last row again)
+  const bool idle = wave * 16 >= bk.nrows;
+  const int wrow0 = min(wave * 16, bk.nrows - 1), wrow1 = min(wave * 16 + 16, bk.nrows) - 1;
+  const int qmin = bk.pos0 + (bk.row0 + wrow0 - bk.seg_row) / R;
+  const int qmax = bk.pos0 + (bk.row0 + wrow1 - bk.seg_row) / R;
+  const int row = bk.row0 + min(wave * 16 + l15, bk.nrows - 1);
+  const int token = row / R, head = grp * R + row % R;
+  const int qpos = bk.pos0 + token - bk.seg_row / R;
+  const float *bh = a.bias + (size_t)head * (a.D + 8);
+  const float far_bias = bh[0];
 
+  // (the queries first, as above)
+  bf8 q[KS];
+  {
+    const uint16_t *qr = (const uint16_t *)a.q + ((size_t)token * a.H + head) * DP + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) q[ks] = *reinterpret_cast<const bf8 *>(qr + ks * 32);
+  }
   // pages are stored as their operands: staging is a straight copy
   constexpr int NKC = DP / 32, NVC = VP / 32;  // 16-byte chunks per thread
   u4 pk[NKC], pv[NVC];
+  f4 pb[4];
   auto fetch = [&](int it) {
     const size_t page = (size_t)(it == 0 ? bk.page0 : table[bk.tile0 + it]) * a.G + grp;
     const u4 *kp = reinterpret_cast<const u4 *>(Kc + page * (64 * DP)) + tid;
     const u4 *vp = reinterpret_cast<const u4 *>(Vc + page * (64 * VP)) + tid;
+    const int base = (bk.tile0 + it) * 64;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) pb[j] = f4{far_bias, far_bias, far_bias, far_bias};
+    if (qmin - (base + 63) < a.D)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) pb[j] = bias4(bh, a.D, qpos, base + j * 16 + 4 * g);
 #pragma unroll
     for (int i = 0; i < NKC; ++i) pk[i] = kp[i * 256];
 #pragma unroll
@@ -312,124 +439,102 @@ __device__ __forceinline__ void attn_many_rows(const char *__restrict__ blob, co
     for (int i = 0; i < NVC; ++i) vd[i * 256] = pv[i];
   };
   fetch(0);
-  // this wave's rows (past the block: its last row again)
-  bf8 q[MR][KS];
-  int qpos[MR];
-  const float *bh[MR];
-  const int wrow0 = min(wave * MR * 16, bk.nrows - 1), wrow1 = min(wave * MR * 16 + MR * 16, bk.nrows) - 1;
-  const int qmin = bk.pos0 + (bk.row0 + wrow0 - bk.seg_row) / R;
-  const int qmax = bk.pos0 + (bk.row0 + wrow1 - bk.seg_row) / R;
-  const bool idle = wave * MR * 16 >= bk.nrows;
+  f4 acc[VT];
+  float m = -1e30f, l = 0.f;
 #pragma unroll
-  for (int i = 0; i < MR; ++i) {
-    const int row = bk.row0 + min((wave * MR + i) * 16 + l15, bk.nrows - 1);
-    const int token = row / R, head = grp * R + row % R;
-    qpos[i] = bk.pos0 + token - bk.seg_row / R;
-    bh[i] = a.bias + (size_t)head * (a.D + 8);
-    const uint16_t *qr = (const uint16_t *)a.q + ((size_t)token * a.H + head) * DP + 8 * g;
-#pragma unroll
-    for (int ks = 0; ks < KS; ++ks) q[i][ks] = *reinterpret_cast<const bf8 *>(qr + ks * 32);
-  }
-  f4 acc[MR][VT];
-  float m[MR], l[MR];
-#pragma unroll
-  for (int i = 0; i < MR; ++i) {
-    m[i] = -1e30f, l[i] = 0.f;
-#pragma unroll
-    for (int d = 0; d < VT; ++d) acc[i][d] = f4{0.f, 0.f, 0.f, 0.f};
-  }
+  for (int d = 0; d < VT; ++d) acc[d] = f4{0.f, 0.f, 0.f, 0.f};
   stage(0);
+  f4 b[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) b[j] = pb[j];
   if (bk.ntiles > 1) fetch(1);
   __syncthreads();
   for (int it = 0; it < bk.ntiles; ++it) {
-    if (it + 1 < bk.ntiles) {
-      stage((it + 1) & 1);  // (its buffer was last read before the previous barrier)
-      if (it + 2 < bk.ntiles) fetch(it + 2);
-    }
     const int base = (bk.tile0 + it) * 64;
-    if (!idle && base <= qmax) {
+    const bool work = !idle && base <= qmax;
+    f4 s[4];
+    if (work) {
       const uint16_t *kt = sK + (it & 1) * 64 * DP + lane * 8;
-      const uint16_t *vt = sV + (it & 1) * 64 * VP + l15 * 32 + g * 8;
-      f4 s[MR][4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
+      for (int j = 0; j < 4; ++j) s[j] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int i = 0; i < MR; ++i) s[i][j] = f4{0.f, 0.f, 0.f, 0.f};
+      for (int ks = 0; ks < KS; ++ks) {
+        bf8 kf[4];
 #pragma unroll
-        for (int ks = 0; ks < KS; ++ks) {
-          const bf8 kf = *reinterpret_cast<const bf8 *>(kt + (j * KS + ks) * 512);
-#pragma unroll
-          for (int i = 0; i < MR; ++i)
-            s[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, q[i][ks], s[i][j], 0, 0, 0);
-        }
-      }
-      const bool far = qmin - (base + 63) >= a.D, whole = base + 63 <= qmin;
-      bf8 p[MR][2];
-#pragma unroll
-      for (int i = 0; i < MR; ++i) {
-        float mx = -1e30f;
-        score_bias<KS, 4>(bh[i], a.D, far, whole, qpos[i], base + 4 * g, a.scale, s[i], mx);
-        mx = fmaxf(mx, __shfl_xor(mx, 16));
-        mx = fmaxf(mx, __shfl_xor(mx, 32));
-        const float mn = fmaxf(m[i], mx), alpha = __builtin_amdgcn_exp2f(m[i] - mn);
-        m[i] = mn;
-        float sum = 0.f;
+        for (int j = 0; j < 4; ++j) kf[j] = *reinterpret_cast<const bf8 *>(kt + (j * KS + ks) * 512);
 #pragma unroll
         for (int j = 0; j < 4; ++j)
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            s[i][j][e] = __builtin_amdgcn_exp2f(s[i][j][e] - mn);
-            sum += s[i][j][e];
-          }
-        l[i] = l[i] * alpha + sum;
-        if (!__all(alpha == 1.0f))
-#pragma unroll
-          for (int d = 0; d < VT; ++d) acc[i][d] *= alpha;
-#pragma unroll
-        for (int h = 0; h < 2; ++h) p[i][h] = pack_weights(s[i][2 * h], s[i][2 * h + 1]);
+          s[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j], q[ks], s[j], 0, 0, 0);
       }
+    }
+    f4 bb[4];
 #pragma unroll
-      for (int h = 0; h < 2; ++h)
+    for (int j = 0; j < 4; ++j) bb[j] = b[j];
+    if (it + 1 < bk.ntiles) {
+      stage((it + 1) & 1);  // (its buffer was last read before the previous barrier)
 #pragma unroll
-        for (int d = 0; d < VT; ++d) {
-          const bf8 vf = *reinterpret_cast<const bf8 *>(vt + h * VP * 32 + d * 512);
+      for (int j = 0; j < 4; ++j) b[j] = pb[j];
+      if (it + 2 < bk.ntiles) fetch(it + 2);
+    }
+    if (work) {
+      const uint16_t *vt = sV + (it & 1) * 64 * VP + l15 * 32 + g * 8;
+      float mx = -1e30f;
+      bias_and_mask<4>(bb, base + 63 <= qmin, qpos, base + 4 * g, a.scale, s, mx);
+      mx = fmaxf(mx, __shfl_xor(mx, 16));
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      const float mn = fmaxf(m, mx), alpha = __builtin_amdgcn_exp2f(m - mn);
+      m = mn;
+      float sum = 0.f;
 #pragma unroll
-          for (int i = 0; i < MR; ++i)
-            acc[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, p[i][h], acc[i][d], 0, 0, 0);
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          s[j][e] = __builtin_amdgcn_exp2f(s[j][e] - mn);
+          sum += s[j][e];
         }
+      l = l * alpha + sum;
+      if (!__all(alpha == 1.0f))
+#pragma unroll
+        for (int d = 0; d < VT; ++d) acc[d] *= alpha;
+#pragma unroll
+      for (int h = 0; h < 2; ++h) {
+        const bf8 p = pack_weights(s[2 * h], s[2 * h + 1]);
+#pragma unroll
+        for (int d = 0; d < VT; ++d)
+          acc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              *reinterpret_cast<const bf8 *>(vt + h * VP * 32 + d * 512), p, acc[d], 0, 0, 0);
+      }
     }
     __syncthreads();
   }
+  l += __shfl_xor(l, 16);
+  l += __shfl_xor(l, 32);
+  const int r = wave * 16 + l15;
+  if (r >= bk.nrows) return;
+  if (bk.slot >= 0) {
+    const size_t pr = ((size_t)(bk.slot + wave) * a.G + grp) * 16 + l15;
 #pragma unroll
-  for (int i = 0; i < MR; ++i) {
-    float L = l[i];
-    L += __shfl_xor(L, 16);
-    L += __shfl_xor(L, 32);
-    const int r = (wave * MR + i) * 16 + l15;
-    if (r >= bk.nrows) continue;
-    if (bk.slot >= 0) {
-      const size_t pr = ((size_t)(bk.slot + wave * MR + i) * a.G + grp) * 16 + l15;
+    for (int d = 0; d < VT; ++d) *reinterpret_cast<f4 *>(slabs + pr * VP + d * 16 + 4 * g) = acc[d];
+    if (g == 0) ml[pr * 2] = m, ml[pr * 2 + 1] = l;
+    return;
+  }
+  const float inv = __fdiv_rn(1.0f, l);
+  const int hc = head * a.vg + 4 * g;
 #pragma unroll
-      for (int d = 0; d < VT; ++d) *reinterpret_cast<f4 *>(slabs + pr * VP + d * 16 + 4 * g) = acc[i][d];
-      if (g == 0) ml[pr * 2] = m[i], ml[pr * 2 + 1] = L;
-      continue;
-    }
-    const float inv = __fdiv_rn(1.0f, L);
-    const int gr = bk.row0 + r, tk = gr / R, hc = (grp * R + gr % R) * a.vg + 4 * g;
-#pragma unroll
-    for (int d = 0; d < VT; ++d) {
-      if (d * 16 >= a.vg) continue;
-      const f4 v4 = acc[i][d] * inv;
-      *reinterpret_cast<uint2 *>((uint16_t *)a.o + act_packed_off(tk, hc + d * 16, a.H * a.vg)) =
-          make_uint2(f2bf(v4[0]) | ((uint32_t)f2bf(v4[1]) << 16),
-                     f2bf(v4[2]) | ((uint32_t)f2bf(v4[3]) << 16));
-    }
+  for (int d = 0; d < VT; ++d) {
+    if (d * 16 >= a.vg) continue;
+    const f4 v4 = acc[d] * inv;
+    *reinterpret_cast<uint2 *>((uint16_t *)a.o + act_packed_off(token, hc + d * 16, a.H * a.vg)) =
+        make_uint2(f2bf(v4[0]) | ((uint32_t)f2bf(v4[1]) << 16),
+                   f2bf(v4[2]) | ((uint32_t)f2bf(v4[3]) << 16));
   }
 }
 
 // MANY: the step has blocks of more than 16 rows (and maybe others)
+// (two workgroups per CU = 256 registers a wave where the widths allow it: the
+// accumulators then stay in the registers the softmax works on)
 template <int DP, int VP, bool MANY>
-__global__ __launch_bounds__(256) void paged_attn_kernel(const char *__restrict__ blob, int off_blocks,
+__global__ __launch_bounds__(256, DP + VP <= 256 ? 2 : 1) void paged_attn_kernel(const char *__restrict__ blob, int off_blocks,
                                                          AttnArgs a, float *__restrict__ slabs,
                                                          float *__restrict__ ml) {
   __shared__ __attribute__((aligned(16))) char

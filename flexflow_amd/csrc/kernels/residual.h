@@ -4,12 +4,17 @@
 
 namespace ffmi {
 
-// x = embed[token] * scale + pos[p] in fp32 (pos null: no positions); xb
-// (optional) the bf16 packed tiles.  blob_src: the step's staging in mapped
-// host memory, copied to blob_dst by this first kernel of the step.
+// x = embed[token] + pos[p] in fp32; xb (optional) the bf16 packed tiles.
+// blob_src: the step's staging in mapped host memory, copied to blob_dst by
+// this first kernel of the step.
 hipError_t launch_embed_pos(const char *blob_src, char *blob_dst, size_t blob_bytes,
-                            const uint16_t *embed, float scale, const uint16_t *pos, float *x,
-                            uint16_t *xb, int T, int H, hipStream_t s);
+                            const uint16_t *embed, const uint16_t *pos, float *x, uint16_t *xb,
+                            int T, int H, hipStream_t s);
+// x = embed[token] * scale in fp32, h = x / rms(x) * w as launch_add_norm's; the
+// first kernel of a step, as above
+hipError_t launch_embed_norm(const char *blob_src, char *blob_dst, size_t blob_bytes,
+                             const uint16_t *embed, float scale, const float *w, float *x,
+                             uint16_t *hb, float *hf, int T, int H, int n, float eps, hipStream_t s);
 // x += y / rms(y) * w on n columns (row stride H); y = sum of the fp32 slabs;
 // xb (optional): the new x in bf16 packed tiles
 hipError_t launch_post_norm(Partials y, const float *w, float *x, uint16_t *xb, int T, int H, int n,

@@ -10,21 +10,17 @@ namespace ffmi {
 
 __global__ __launch_bounds__(256) void embed_pos_kernel(
     const char *__restrict__ blob_src, uint4 *__restrict__ blob_dst, int blob_n16,
-    const uint16_t *__restrict__ embed, float scale, const uint16_t *__restrict__ pos,
-    float *__restrict__ x, uint16_t *__restrict__ xb, int H) {
+    const uint16_t *__restrict__ embed, const uint16_t *__restrict__ pos, float *__restrict__ x,
+    uint16_t *__restrict__ xb, int H) {
   const int t = blockIdx.x;
   const PagedToken tk = reinterpret_cast<const PagedToken *>(blob_src)[t];  // tokens come first
   const uint4 *src = reinterpret_cast<const uint4 *>(blob_src);
   for (int i = t * 256 + threadIdx.x; i < blob_n16; i += gridDim.x * 256) blob_dst[i] = src[i];
   for (int c = threadIdx.x; c < H / 8; c += 256) {
-    f4 a, b;
+    f4 a, b, pa, pb;
     unpack8_bf16(*reinterpret_cast<const uint4 *>(embed + (size_t)tk.token * H + c * 8), a, b);
-    a *= scale, b *= scale;
-    if (pos) {
-      f4 pa, pb;
-      unpack8_bf16(*reinterpret_cast<const uint4 *>(pos + (size_t)tk.pos * H + c * 8), pa, pb);
-      a += pa, b += pb;
-    }
+    unpack8_bf16(*reinterpret_cast<const uint4 *>(pos + (size_t)tk.pos * H + c * 8), pa, pb);
+    a += pa, b += pb;
     *reinterpret_cast<f4 *>(x + (size_t)t * H + c * 8) = a;
     *reinterpret_cast<f4 *>(x + (size_t)t * H + c * 8 + 4) = b;
     if (xb) *reinterpret_cast<uint4 *>(xb + act_packed_off(t, c * 8, H)) = pack8_bf16(a, b);
@@ -32,29 +28,43 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(
 }
 
 hipError_t launch_embed_pos(const char *blob_src, char *blob_dst, size_t blob_bytes,
-                            const uint16_t *embed, float scale, const uint16_t *pos, float *x,
-                            uint16_t *xb, int T, int H, hipStream_t s) {
+                            const uint16_t *embed, const uint16_t *pos, float *x, uint16_t *xb,
+                            int T, int H, hipStream_t s) {
   if (T <= 0) return hipSuccess;
   if (H % 32) return hipErrorInvalidValue;
   hipLaunchKernelGGL(embed_pos_kernel, dim3(T), dim3(256), 0, s, blob_src,
-                     reinterpret_cast<uint4 *>(blob_dst), (int)((blob_bytes + 15) / 16), embed, scale,
-                     pos, x, xb, H);
+                     reinterpret_cast<uint4 *>(blob_dst), (int)((blob_bytes + 15) / 16), embed, pos,
+                     x, xb, H);
   return hipGetLastError();
 }
 
 // One workgroup per row; the slab, x and w loads of a chunk are all issued
 // before the reduction.
 //   PRE == false: x += y / rms(y) * w, hb the new x
-//   PRE == true:  x += y, h = x / rms(x) * w to hb or hf (w null: the sum only)
+//   PRE == true:  x += y, h = x / rms(x) * w to hb or hf (w null: the sum only);
+//   without slabs x is, where em.table is given, an embedding row
+struct EmbedRows {
+  const char *blob_src = nullptr;  // staging, tokens first; copied to blob_dst
+  uint4 *blob_dst = nullptr;
+  int blob_n16 = 0;
+  const uint16_t *table = nullptr;
+  float scale = 1.f;
+};
 template <int NT, int MAXC, int MAXS, bool PRE>
 __global__ __launch_bounds__(NT) void stream_norm_kernel(const float *__restrict__ yp, int S, int NP,
                                                          const float *__restrict__ w,
                                                          float *__restrict__ x,
                                                          uint16_t *__restrict__ hb,
                                                          float *__restrict__ hf, int H, int n,
-                                                         float eps) {
+                                                         float eps, EmbedRows em) {
   __shared__ float sh[NT / 64];
   const int row = blockIdx.x, T = gridDim.x, nchunk = H >> 3;
+  const uint16_t *er = nullptr;
+  if (PRE && MAXS == 0 && em.table) {
+    er = em.table + (size_t)reinterpret_cast<const PagedToken *>(em.blob_src)[row].token * H;
+    const uint4 *src = reinterpret_cast<const uint4 *>(em.blob_src);
+    for (int i = row * NT + threadIdx.x; i < em.blob_n16; i += T * NT) em.blob_dst[i] = src[i];
+  }
   f4 y[MAXC][2], xv[MAXC][2], wv[MAXC][2];
   float ss = 0.f;
 #pragma unroll
@@ -70,9 +80,13 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(const float *__restrict
     }
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
-      xv[c][h] = *reinterpret_cast<const f4 *>(x + (size_t)row * H + ch * 8 + 4 * h);
+      if (!er) xv[c][h] = *reinterpret_cast<const f4 *>(x + (size_t)row * H + ch * 8 + 4 * h);
       wv[c][h] = f4{0.f, 0.f, 0.f, 0.f};
       if (!PRE || w) wv[c][h] = *reinterpret_cast<const f4 *>(w + ch * 8 + 4 * h);
+    }
+    if (er) {
+      unpack8_bf16(*reinterpret_cast<const uint4 *>(er + ch * 8), xv[c][0], xv[c][1]);
+      xv[c][0] *= em.scale, xv[c][1] *= em.scale;
     }
     y[c][0] = lo[0], y[c][1] = hi[0];
 #pragma unroll
@@ -101,7 +115,7 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(const float *__restrict
         if constexpr (PRE) y[c][h][e] = v;
         else y[c][h][e] = xv[c][h][e] += v;
       }
-    if (!PRE || MAXS) {
+    if (!PRE || MAXS || er) {
       *reinterpret_cast<f4 *>(x + (size_t)row * H + ch * 8) = xv[c][0];
       *reinterpret_cast<f4 *>(x + (size_t)row * H + ch * 8 + 4) = xv[c][1];
     }
@@ -117,14 +131,15 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(const float *__restrict
 
 template <bool PRE>
 static hipError_t run_stream_norm(Partials y, const float *w, float *x, uint16_t *hb, float *hf,
-                                  int T, int H, int n, float eps, hipStream_t s) {
+                                  int T, int H, int n, float eps, hipStream_t s,
+                                  const EmbedRows &em = EmbedRows()) {
   if (T <= 0) return hipSuccess;
   if (H % 32 || y.S < (PRE ? 0 : 1) || y.S > 8) return hipErrorInvalidValue;
   if (y.S > 0 && (y.NP < H || y.NP % 4 || !y.p)) return hipErrorInvalidValue;
   const int nchunk = H / 8;
 #define FFMI_SN(NT, MC, MS)                                                                       \
   hipLaunchKernelGGL((stream_norm_kernel<NT, MC, MS, PRE>), dim3(T), dim3(NT), 0, s, y.p, y.S, \
-                     y.NP, w, x, hb, hf, H, n, eps)
+                     y.NP, w, x, hb, hf, H, n, eps, em)
 #define FFMI_SNS(NT, MC)                   \
   do {                                     \
     if (PRE && y.S == 0) FFMI_SN(NT, MC, (PRE ? 0 : 1)); \
@@ -146,6 +161,14 @@ static hipError_t run_stream_norm(Partials y, const float *w, float *x, uint16_t
 hipError_t launch_post_norm(Partials y, const float *w, float *x, uint16_t *xb, int T, int H, int n,
                             float eps, hipStream_t s) {
   return run_stream_norm<false>(y, w, x, xb, nullptr, T, H, n, eps, s);
+}
+hipError_t launch_embed_norm(const char *blob_src, char *blob_dst, size_t blob_bytes,
+                             const uint16_t *embed, float scale, const float *w, float *x,
+                             uint16_t *hb, float *hf, int T, int H, int n, float eps, hipStream_t s) {
+  EmbedRows em;
+  em.blob_src = blob_src, em.blob_dst = reinterpret_cast<uint4 *>(blob_dst);
+  em.blob_n16 = (int)((blob_bytes + 15) / 16), em.table = embed, em.scale = scale;
+  return run_stream_norm<true>(Partials(), w, x, hb, hf, T, H, n, eps, s, em);
 }
 hipError_t launch_add_norm(Partials y, const float *w, float *x, uint16_t *hb, float *hf, int T,
                            int H, int n, float eps, hipStream_t s) {

@@ -329,9 +329,9 @@ struct Fesenex : public PagedDecoder {
     return FFMI_OK;
   }
   ffmi_status run_layers() override {
-    FFMI_HIP(launch_embed_pos(step.host, step.dev, step.bytes, embed, embed_scale, nullptr, x, nullptr,
-                              step.T, Wp, stream));
-    FFMI_TRY(add_norm(Partials(), layers[0].norm1));
+    FFMI_HIP(launch_embed_norm(step.host, step.dev, step.bytes, embed, embed_scale, layers[0].norm1, x,
+                               f32 ? nullptr : (uint16_t *)h, f32 ? (float *)h : nullptr, step.T, Wp, W, eps,
+                               stream));
     for (size_t i = 0; i < layers.size(); ++i) {
       const FesenexLayer &L = layers[i];
       const float *next = i + 1 < layers.size() ? layers[i + 1].norm1 : nullptr;

@@ -215,7 +215,7 @@ struct Vapipel : public PagedDecoder {
   }
   ffmi_status run_layers() override {
     const int T = step.T;
-    FFMI_HIP(launch_embed_pos(step.host, step.dev, step.bytes, embed, 1.0f, pos, x, xb, T, Wp, stream));
+    FFMI_HIP(launch_embed_pos(step.host, step.dev, step.bytes, embed, pos, x, xb, T, Wp, stream));
     for (size_t i = 0; i < layers.size(); ++i) {
       const VapipelLayer &L = layers[i];
       Partials y;
