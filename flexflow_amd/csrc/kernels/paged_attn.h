@@ -54,9 +54,11 @@ struct AttnArgs {
   float scale = 0.f;
 };
 // bf16, widths that attn_width gave; slabs / ml: partials of split blocks, 16
-// rows a slot, [slot][G][16][vp] and [slot][G][16][2]
+// rows a slot, [slot][G][16][vp] and [slot][G][16][2].  pr: the launch makes
+// queries, keys and values itself (launch_attn_prep's work; a.q is not read) --
+// steps whose blocks have at most 16 rows only (pl.row_tiles == 1)
 hipError_t launch_paged_attn(const char *blob, const PagedLists &pl, const AttnArgs &a, float *slabs,
-                             float *ml, hipStream_t s);
+                             float *ml, hipStream_t s, const AttnPrep *pr = nullptr, int T = 0);
 constexpr int kAttnTiles = 4;  // row tiles of a workgroup in prompts
 // any width up to kAttnRowsMax, one workgroup per row of every block (fp32, or
 // bf16 with scale and bias for base-2 exponents as above)

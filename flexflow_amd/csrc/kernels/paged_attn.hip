@@ -55,117 +55,171 @@ __device__ __forceinline__ void store2(uint16_t *p, f2 v) {
 }
 __device__ __forceinline__ void store2(float *p, f2 v) { *reinterpret_cast<f2 *>(p) = v; }
 
-// A wave takes NT consecutive batch tokens of one head, a lane NE columns in
-// neighbouring pairs (NE == 1: one).
+// One head of one token across a wave: a lane holds NE columns in neighbouring
+// pairs (NE == 1: one column).  Heads in the order of the columns: q, k, v.
+template <int NE>
+__device__ __forceinline__ int head_column(int i) {
+  const int lane = threadIdx.x & 63;
+  return NE == 1 ? lane : (i >> 1) * 128 + lane * 2 + (i & 1);
+}
+__device__ __forceinline__ int head_width(const AttnPrep &a, int hd) {
+  return hd >= a.H + a.G ? a.vg : a.dg;
+}
+__device__ __forceinline__ int head_start(const AttnPrep &a, int hd) {
+  return hd >= a.H + a.G ? (a.H + a.G) * a.dg + (hd - a.H - a.G) * a.vg : hd * a.dg;
+}
+template <int NE>
+__device__ __forceinline__ void load_bias(const AttnPrep &a, int hd, float (&b)[NE]) {
+  const float *p = a.bias + head_start(a, hd);
+  if constexpr (NE == 1) {
+    const int c = head_column<NE>(0);
+    b[0] = 0.f;
+    if (c < head_width(a, hd)) b[0] = p[c];
+  } else {
+#pragma unroll
+    for (int i = 0; i < NE; i += 2) {
+      const int c = head_column<NE>(i);
+      f2 v = f2{0.f, 0.f};
+      if (c < head_width(a, hd)) v = *reinterpret_cast<const f2 *>(p + c);
+      b[i] = v[0], b[i + 1] = v[1];
+    }
+  }
+}
+// its product, with the bias
+template <int NE>
+__device__ __forceinline__ void load_head(const AttnPrep &a, int T, int t, int hd, const float (&b)[NE],
+                                          float (&v)[NE]) {
+  const int wd = head_width(a, hd);
+  const size_t slab = (size_t)T * a.y.NP, row = (size_t)t * a.y.NP + head_start(a, hd);
+  if constexpr (NE == 1) {
+    const int c = head_column<NE>(0);
+    v[0] = 0.f;
+    if (c < wd) v[0] = slab_sum(a.y, slab, row + c) + b[0];
+  } else {
+#pragma unroll
+    for (int i = 0; i < NE; i += 2) {
+      const int c = head_column<NE>(i);  // (the widths are even)
+      v[i] = v[i + 1] = 0.f;
+      if (c < wd) {
+        const f2 p = slab_sum2(a.y, slab, row + c);
+        v[i] = p[0] + b[i], v[i + 1] = p[1] + b[i + 1];
+      }
+    }
+  }
+}
+// values: mixed with, or kept as, the first mixing layer's (lam: *a.vmix)
+template <int NE>
+__device__ __forceinline__ void mix_head(const AttnPrep &a, int t, int g, float lam, float (&v)[NE]) {
+  if (!a.first) return;
+  float *first = a.first + ((size_t)t * a.G + g) * a.vg;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int c = head_column<NE>(i);
+    if (c >= a.vg) continue;
+    if (a.vmix) v[i] = (1.0f - lam) * v[i] + lam * first[c];
+    else first[c] = v[i];
+  }
+}
+// queries and keys: norm, query temperature
+template <int NE>
+__device__ __forceinline__ void norm_head(const AttnPrep &a, bool isq, int pos, float (&v)[NE]) {
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) ss = fmaf(v[i], v[i], ss);
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
+  float r = inv_rms(ss, a.dim, a.eps);
+  if (isq && a.coef != 0.f) r *= 1.0f + a.coef * logf((float)((pos + 1) / a.every + 1));
+  const float *w = isq ? a.qnorm : a.knorm;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int c = head_column<NE>(i);
+    v[i] = c < a.dg ? v[i] * r * w[c] : 0.f;
+  }
+}
+// columns below `width` to dst(column), pairs lying side by side
+template <class E, int NE, class D>
+__device__ __forceinline__ void store_head(D dst, int width, const float (&v)[NE]) {
+  if constexpr (NE == 1) {
+    const int c = head_column<NE>(0);
+    if (c < width) st_elem((E *)dst(c), v[0]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < NE; i += 2) {
+      const int c = head_column<NE>(i);
+      if (c < width) store2((E *)dst(c), f2{v[i], v[i + 1]});
+    }
+  }
+}
+template <class E, int NE>
+__device__ __forceinline__ void store_value(const AttnPrep &a, int crow, int g, const float (&v)[NE]) {
+  E *dst = (E *)a.vc + ((size_t)(crow / kPageTokens) * a.G + g) * kPageTokens * a.vp;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int c = head_column<NE>(i);
+    if (c < a.vp) st_elem(dst + val_off(crow % kPageTokens, c, a.vp), v[i]);
+  }
+}
+template <class E, int NE>
+__device__ __forceinline__ void store_key(const AttnPrep &a, int crow, int g, const float (&v)[NE]) {
+  E *dst = (E *)a.kc + ((size_t)(crow / kPageTokens) * a.G + g) * kPageTokens * a.dp;
+  const int key = crow % kPageTokens;
+  store_head<E, NE>([&](int c) { return dst + key_off(key, c, a.dp); }, a.dp, v);
+}
+
+// A wave takes NT consecutive batch tokens of one head.
 template <class E, int NE, int NT>
 __global__ __launch_bounds__(256) void attn_prep_kernel(const PagedToken *__restrict__ tok, int T,
                                                         AttnPrep a) {
-  const int heads = a.H + 2 * a.G, lane = threadIdx.x & 63;
+  const int heads = a.H + 2 * a.G;
   const long id = blockIdx.x * 4L + (threadIdx.x >> 6);
-  const int hd = (int)(id % heads), t0 = (int)(id / heads) * NT;
-  if (t0 >= T) return;
+  // (a workgroup's waves side by side in the sequence: the cache lines that
+  // they share are written on one CU)
+  const int nt = (T + NT - 1) / NT, hd = (int)(id / nt), t0 = (int)(id % nt) * NT;
+  if (hd >= heads) return;
   const bool isv = hd >= a.H + a.G, isq = hd < a.H;
   const int g = isq ? 0 : (hd - a.H) % a.G;
-  const int wd = isv ? a.vg : a.dg;  // columns of this head
-  const int col = isv ? (a.H + a.G) * a.dg + g * a.vg : hd * a.dg;
-  const size_t slab = (size_t)T * a.y.NP;
-  const auto column = [&](int i) { return NE == 1 ? lane : (i >> 1) * 128 + lane * 2 + (i & 1); };
   PagedToken tk[NT];
-  float v[NT][NE], ss[NT];
+  float v[NT][NE], bias[NE];
+  const float lam = isv && a.vmix ? *a.vmix : 0.f;
+  load_bias<NE>(a, hd, bias);
 #pragma unroll
   for (int k = 0; k < NT; ++k) tk[k] = tok[min(t0 + k, T - 1)];
 #pragma unroll
-  for (int k = 0; k < NT; ++k) {
-    const size_t row = (size_t)min(t0 + k, T - 1) * a.y.NP + col;
-    if constexpr (NE == 1) {
-      v[k][0] = lane < wd ? slab_sum(a.y, slab, row + lane) : 0.f;
-    } else {
-#pragma unroll
-      for (int i = 0; i < NE; i += 2) {
-        const int c = column(i);  // (the widths are even)
-        f2 p = f2{0.f, 0.f};
-        if (c < wd) p = slab_sum2(a.y, slab, row + c);
-        v[k][i] = p[0], v[k][i + 1] = p[1];
-      }
-    }
-  }
-#pragma unroll
-  for (int i = 0; i < NE; ++i) {
-    const int c = column(i);
-    const float b = c < wd ? a.bias[col + c] : 0.f;
-#pragma unroll
-    for (int k = 0; k < NT; ++k) v[k][i] += b;
-  }
+  for (int k = 0; k < NT; ++k) load_head<NE>(a, T, min(t0 + k, T - 1), hd, bias, v[k]);
   if (isv) {
-    if (a.first) {
-      const float lam = a.vmix ? *a.vmix : 0.f;
 #pragma unroll
-      for (int k = 0; k < NT; ++k) {
-        if (t0 + k >= T) break;
-        float *first = a.first + ((size_t)(t0 + k) * a.G + g) * a.vg;
-#pragma unroll
-        for (int i = 0; i < NE; ++i) {
-          const int c = column(i);
-          if (c >= wd) continue;
-          if (a.vmix) v[k][i] = (1.0f - lam) * v[k][i] + lam * first[c];
-          else first[c] = v[k][i];
-        }
-      }
-    }
+    for (int k = 0; k < NT; ++k)
+      if (t0 + k < T) mix_head<NE>(a, t0 + k, g, lam, v[k]);
     // four tokens in one aligned run of a page: their values lie side by side
     bool run = NT == 4 && t0 + NT <= T && tk[0].row % 4 == 0;
 #pragma unroll
     for (int k = 1; k < NT; ++k) run = run && tk[k].row == tk[0].row + k;
-#pragma unroll
-    for (int i = 0; i < NE; ++i) {
-      const int c = column(i);
-      if (c >= a.vp) continue;
-      if (run) {
-        E *dst = (E *)a.vc + ((size_t)(tk[0].row / kPageTokens) * a.G + g) * kPageTokens * a.vp +
-                 val_off(tk[0].row % kPageTokens, c, a.vp);
-        store4(dst, v[0][i], v[NT > 1 ? 1 : 0][i], v[NT > 2 ? 2 : 0][i], v[NT > 3 ? 3 : 0][i]);
-        continue;
-      }
+    if (!run) {
 #pragma unroll
       for (int k = 0; k < NT; ++k)
-        if (t0 + k < T)
-          st_elem((E *)a.vc + ((size_t)(tk[k].row / kPageTokens) * a.G + g) * kPageTokens * a.vp +
-                      val_off(tk[k].row % kPageTokens, c, a.vp),
-                  v[k][i]);
+        if (t0 + k < T) store_value<E, NE>(a, tk[k].row, g, v[k]);
+      return;
+    }
+    E *dst = (E *)a.vc + ((size_t)(tk[0].row / kPageTokens) * a.G + g) * kPageTokens * a.vp;
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int c = head_column<NE>(i);
+      if (c < a.vp)
+        store4(dst + val_off(tk[0].row % kPageTokens, c, a.vp), v[0][i], v[NT > 1 ? 1 : 0][i],
+               v[NT > 2 ? 2 : 0][i], v[NT > 3 ? 3 : 0][i]);
     }
     return;
   }
 #pragma unroll
   for (int k = 0; k < NT; ++k) {
-    ss[k] = 0.f;
-#pragma unroll
-    for (int i = 0; i < NE; ++i) ss[k] = fmaf(v[k][i], v[k][i], ss[k]);
-  }
-#pragma unroll
-  for (int o = 32; o > 0; o >>= 1)
-#pragma unroll
-    for (int k = 0; k < NT; ++k) ss[k] += __shfl_xor(ss[k], o);
-  const float *w = isq ? a.qnorm : a.knorm;
-#pragma unroll
-  for (int k = 0; k < NT; ++k) {
     if (t0 + k >= T) break;
-    float r = inv_rms(ss[k], a.dim, a.eps);
-    if (isq && a.coef != 0.f) r *= 1.0f + a.coef * logf((float)((tk[k].pos + 1) / a.every + 1));
-    const int key = tk[k].row % kPageTokens;
-    E *dst = isq ? (E *)a.q + ((size_t)(t0 + k) * a.H + hd) * a.dp
-                 : (E *)a.kc + ((size_t)(tk[k].row / kPageTokens) * a.G + g) * kPageTokens * a.dp;
-    if constexpr (NE == 1) {
-      if (lane < a.dp)
-        st_elem(dst + (isq ? lane : key_off(key, lane, a.dp)), lane < wd ? v[k][0] * r * w[lane] : 0.f);
+    norm_head<NE>(a, isq, tk[k].pos, v[k]);
+    if (isq) {
+      E *dst = (E *)a.q + ((size_t)(t0 + k) * a.H + hd) * a.dp;
+      store_head<E, NE>([&](int c) { return dst + c; }, a.dp, v[k]);
     } else {
-#pragma unroll
-      for (int i = 0; i < NE; i += 2) {
-        const int c = column(i);
-        if (c >= a.dp) continue;
-        f2 o = f2{0.f, 0.f};
-        if (c < wd) o = f2{v[k][i] * r * w[c], v[k][i + 1] * r * w[c + 1]};
-        store2(dst + (isq ? c : key_off(key, c, a.dp)), o);
-      }
+      store_key<E, NE>(a, tk[k].row, g, v[k]);
     }
   }
 }
@@ -244,15 +298,24 @@ __device__ __forceinline__ bf8 pack_weights(const f4 &lo, const f4 &hi) {
 }
 
 template <int DP, int VP>
+constexpr int few_rows_lds() {
+  constexpr int q = 16 * (DP + 8) * 2, merge = 4 * 16 * (VP + 4) * 4 + 4 * 16 * 2 * 4;
+  return q > merge ? q : merge;
+}
+template <int DP, int VP>
 constexpr int attn_lds_bytes() {
-  constexpr int prompt = 2 * 64 * (DP + VP) * 2, merge = 4 * 16 * (VP + 4) * 4 + 4 * 16 * 2 * 4;
-  return prompt > merge ? prompt : merge;
+  constexpr int prompt = 2 * 64 * (DP + VP) * 2;
+  return prompt > few_rows_lds<DP, VP>() ? prompt : few_rows_lds<DP, VP>();
 }
 
-template <int DP, int VP>
+// PREP: a step of one block per request (and its splits): the workgroup first
+// makes its own queries (in LDS) and, of the request's new tokens, the keys and
+// values that fall into its pages; no separate launch.
+template <int DP, int VP, bool PREP>
 __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, const PagedBlock &bk,
-                                              const AttnArgs &a, float *__restrict__ slabs,
-                                              float *__restrict__ ml, char *lds) {
+                                              const AttnArgs &a, const AttnPrep &pr, int T,
+                                              float *__restrict__ slabs, float *__restrict__ ml,
+                                              char *lds) {
   constexpr int KS = DP / 32, VT = VP / 16, LDO = VP + 4;
   float *sO = reinterpret_cast<float *>(lds), *sM = sO + 4 * 16 * LDO, *sL = sM + 64;
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
@@ -266,15 +329,7 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
   const uint16_t *Kc = (const uint16_t *)a.kc, *Vc = (const uint16_t *)a.vc;
   const int units = 2 * bk.ntiles;
 
-  // (the queries first: loads return in order, so the loop never waits for
-  // them behind a prefetch)
-  bf8 q[KS];
-  {
-    const uint16_t *qr = (const uint16_t *)a.q + ((size_t)token * a.H + head) * DP + 8 * g;
-#pragma unroll
-    for (int ks = 0; ks < KS; ++ks) q[ks] = *reinterpret_cast<const bf8 *>(qr + ks * 32);
-  }
-  bf8 k[2][KS], v[VT];
+  bf8 q[KS], k[2][KS], v[VT];
   f4 b[2];
   auto fetch = [&](int u) {
     const int k0 = bk.tile0 * 64 + u * 32 + 4 * g;
@@ -290,7 +345,56 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
 #pragma unroll
     for (int d = 0; d < VT; ++d) v[d] = *reinterpret_cast<const bf8 *>(vp + d * 512);
   };
-  if (wave < units) fetch(wave);
+  if constexpr (PREP) {
+    // items: the block's query rows, then a key and a value per new token
+    constexpr int NE = (DP > VP ? DP : VP) / 64, LDQ = DP + 8;
+    uint16_t *sQ = reinterpret_cast<uint16_t *>(lds);
+    const int t0 = bk.seg_row / R, n = bk.nrows / R, nq = bk.nrows, items = nq + 2 * n;
+    auto head_of = [&](int it) {
+      return it < nq ? grp * R + it % R : it < nq + n ? a.H + grp : a.H + a.G + grp;
+    };
+    auto token_of = [&](int it) { return it < nq ? it / R : (it - nq) % n; };
+    auto finish = [&](int it, float (&x)[NE]) {
+      const int tk = token_of(it), pos = bk.pos0 + tk, tile = pos / kPageTokens;
+      if (it < nq) {
+        norm_head<NE>(pr, true, pos, x);
+        store_head<uint16_t, NE>([&](int c) { return sQ + it * LDQ + c; }, DP, x);
+        return;
+      }
+      if (tile < bk.tile0 || tile >= bk.tile0 + bk.ntiles) return;  // another workgroup's page
+      const int crow = table[tile] * kPageTokens + pos % kPageTokens;
+      if (it < nq + n) {
+        norm_head<NE>(pr, false, pos, x);
+        store_key<uint16_t, NE>(pr, crow, grp, x);
+      } else {
+        mix_head<NE>(pr, t0 + tk, grp, pr.vmix ? *pr.vmix : 0.f, x);
+        store_value<uint16_t, NE>(pr, crow, grp, x);
+      }
+    };
+    for (int it = wave; it < items; it += 8) {  // two at a time
+      float x0[NE], x1[NE], b0[NE], b1[NE];
+      const int it1 = min(it + 4, items - 1);
+      load_bias<NE>(pr, head_of(it), b0);
+      load_bias<NE>(pr, head_of(it1), b1);
+      load_head<NE>(pr, T, t0 + token_of(it), head_of(it), b0, x0);
+      load_head<NE>(pr, T, t0 + token_of(it1), head_of(it1), b1, x1);
+      finish(it, x0);
+      if (it + 4 < items) finish(it1, x1);
+    }
+    __syncthreads();  // (the new keys and values are in the cache, for this workgroup)
+    const uint16_t *qr = sQ + min(l15, bk.nrows - 1) * LDQ + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) q[ks] = *reinterpret_cast<const bf8 *>(qr + ks * 32);
+    if (wave < units) fetch(wave);
+    __syncthreads();  // (the merge below reuses the LDS)
+  } else {
+    // (the queries first: loads return in order, so the loop never waits for
+    // them behind a prefetch)
+    const uint16_t *qr = (const uint16_t *)a.q + ((size_t)token * a.H + head) * DP + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) q[ks] = *reinterpret_cast<const bf8 *>(qr + ks * 32);
+    if (wave < units) fetch(wave);
+  }
   f4 acc[VT];
 #pragma unroll
   for (int d = 0; d < VT; ++d) acc[d] = f4{0.f, 0.f, 0.f, 0.f};
@@ -538,7 +642,7 @@ __global__ __launch_bounds__(256, DP + VP <= 256 ? 2 : 1) void paged_attn_kernel
                                                          AttnArgs a, float *__restrict__ slabs,
                                                          float *__restrict__ ml) {
   __shared__ __attribute__((aligned(16))) char
-      lds[MANY ? attn_lds_bytes<DP, VP>() : 4 * 16 * (VP + 4) * 4 + 512];
+      lds[MANY ? attn_lds_bytes<DP, VP>() : few_rows_lds<DP, VP>()];
   const PagedBlock bk = reinterpret_cast<const PagedBlock *>(blob + off_blocks)[blockIdx.x];
   if (bk.nrows <= 0) return;
   if constexpr (MANY) {
@@ -547,7 +651,18 @@ __global__ __launch_bounds__(256, DP + VP <= 256 ? 2 : 1) void paged_attn_kernel
       return;
     }
   }
-  attn_few_rows<DP, VP>(blob, bk, a, slabs, ml, lds);
+  attn_few_rows<DP, VP, false>(blob, bk, a, AttnPrep(), 0, slabs, ml, lds);
+}
+
+// the few-rows form with its queries, keys and values made on the way
+template <int DP, int VP>
+__global__ __launch_bounds__(256, DP + VP <= 256 ? 2 : 1) void paged_attn_prep_kernel(
+    const char *__restrict__ blob, int off_blocks, AttnArgs a, AttnPrep pr, int T,
+    float *__restrict__ slabs, float *__restrict__ ml) {
+  __shared__ __attribute__((aligned(16))) char lds[few_rows_lds<DP, VP>()];
+  const PagedBlock bk = reinterpret_cast<const PagedBlock *>(blob + off_blocks)[blockIdx.x];
+  if (bk.nrows <= 0) return;
+  attn_few_rows<DP, VP, true>(blob, bk, a, pr, T, slabs, ml, lds);
 }
 
 // partials of split blocks, in slot order: a workgroup per 16 rows of a block
@@ -599,9 +714,12 @@ __global__ __launch_bounds__(256) void paged_attn_merge_kernel(const char *__res
 
 template <int DP, int VP>
 static hipError_t run_paged_attn(const char *blob, const PagedLists &pl, const AttnArgs &a,
-                                 float *slabs, float *ml, hipStream_t s) {
+                                 const AttnPrep *pr, int T, float *slabs, float *ml, hipStream_t s) {
   const dim3 grid(pl.num_blocks, a.G);
-  if (pl.row_tiles > 1)
+  if (pr)
+    hipLaunchKernelGGL((paged_attn_prep_kernel<DP, VP>), grid, dim3(256), 0, s, blob, pl.off_blocks, a,
+                       *pr, T, slabs, ml);
+  else if (pl.row_tiles > 1)
     hipLaunchKernelGGL((paged_attn_kernel<DP, VP, true>), grid, dim3(256), 0, s, blob, pl.off_blocks, a,
                        slabs, ml);
   else
@@ -614,13 +732,16 @@ static hipError_t run_paged_attn(const char *blob, const PagedLists &pl, const A
 }
 
 hipError_t launch_paged_attn(const char *blob, const PagedLists &pl, const AttnArgs &a, float *slabs,
-                             float *ml, hipStream_t s) {
+                             float *ml, hipStream_t s, const AttnPrep *pr, int T) {
   if (pl.num_blocks <= 0) return hipSuccess;
+  if (pr && (pl.row_tiles != 1 || pr->H != a.H || pr->G != a.G || pr->dp != a.dp || pr->vp != a.vp ||
+             pr->vg != a.vg || pr->y.S < 1 || pr->y.S > 8 || pr->every < 1))
+    return hipErrorInvalidValue;
   if (a.G < 1 || a.H % a.G || pl.heads != a.H / a.G || pl.groups != a.G || a.vg > a.vp || a.D < 0 ||
       (pl.row_tiles != 1 && pl.row_tiles != kAttnTiles))
     return hipErrorInvalidValue;
 #define FFMI_PA(DP, VP) \
-  if (a.dp == DP && a.vp == VP) return run_paged_attn<DP, VP>(blob, pl, a, slabs, ml, s)
+  if (a.dp == DP && a.vp == VP) return run_paged_attn<DP, VP>(blob, pl, a, pr, T, slabs, ml, s)
   FFMI_PA(64, 64);
   FFMI_PA(64, 128);
   FFMI_PA(64, 256);

@@ -282,16 +282,17 @@ struct Fesenex : public PagedDecoder {
     p.q = q, p.kc = L.kc, p.vc = L.vc;
     p.H = H, p.G = G, p.dim = L.dim, p.dg = L.dg, p.dp = L.dp, p.vg = L.vg, p.vp = L.vp;
     p.eps = eps, p.coef = L.coef, p.every = L.every;
-    FFMI_HIP(launch_attn_prep(step.dev, step.off_tokens, step.T, p, f32, stream));
+    const PagedLists &pl = step.lists(H / G, G);
+    const bool rows = f32 || !attn_width(L.dim) || !attn_width(L.vdim);
+    // decoding and short portions: in the attention's launch
+    const bool fused = !rows && pl.row_tiles == 1;
+    if (!fused) FFMI_HIP(launch_attn_prep(step.dev, step.off_tokens, step.T, p, f32, stream));
     AttnArgs a;
     a.q = q, a.kc = L.kc, a.vc = L.vc, a.bias = L.rel, a.o = att;
     a.H = H, a.G = G, a.dp = L.dp, a.vg = L.vg, a.vp = L.vp, a.D = L.bias_max;
     a.scale = f32 ? L.scale : L.scale * 1.4426950408889634f;
-    const PagedLists &pl = step.lists(H / G, G);
-    if (f32 || !attn_width(L.dim) || !attn_width(L.vdim))
-      FFMI_HIP(launch_paged_attn_rows(step.dev, pl, a, f32, stream));
-    else
-      FFMI_HIP(launch_paged_attn(step.dev, pl, a, slabs, ml, stream));
+    if (rows) FFMI_HIP(launch_paged_attn_rows(step.dev, pl, a, f32, stream));
+    else FFMI_HIP(launch_paged_attn(step.dev, pl, a, slabs, ml, stream, fused ? &p : nullptr, step.T));
     return gemm_sum(att, L.wo, Wp, H * L.vg, y);
   }
   ffmi_status lightning(const FesenexLayer &L, Partials *y) {

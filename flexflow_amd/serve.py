@@ -25,8 +25,8 @@ class Model:
                  weight_init: Union[int, str] = 0, full_precision: bool = False,
                  kv_pool_tokens: int = 0):
         """weights_folder: a checkpoint in the reference's per-tensor format
-        (see checkpoint.convert_hf_model) or the family's own (Vapipel:
-        model.safetensors); None: seeded synthetic weights,
+        (see checkpoint.convert_hf_model) or the family's own (a
+        registry family: model.safetensors); None: seeded synthetic weights,
         `weight_init` "uniform" (0, the bench's), "depth_scaled" (1) or
         "token_chain" (2) -- include/ffmi.h ffmi_model_opts.  full_precision:
         the reference's --use-full-precision (every tensor fp32,
