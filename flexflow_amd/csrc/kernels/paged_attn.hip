@@ -263,7 +263,8 @@ hipError_t launch_attn_prep(const char *blob, int off_tokens, int T, const AttnP
 // sums take them unrounded.
 //
 // Up to 16 rows (decoding, short portions): operands straight from memory, the
-// workgroup's four waves over half-pages, their results merged through LDS.
+// workgroup's waves (eight in a step of such blocks alone, widths allowing) over half-pages, their
+// results merged through LDS.
 // More rows (prompts): four waves of 16 rows each over pages staged in LDS,
 // double-buffered, the next page's loads in flight through registers.
 //
@@ -297,27 +298,27 @@ __device__ __forceinline__ bf8 pack_weights(const f4 &lo, const f4 &hi) {
   return p;
 }
 
-template <int DP, int VP>
+template <int DP, int VP, int NW>
 constexpr int few_rows_lds() {
-  constexpr int q = 16 * (DP + 8) * 2, merge = 4 * 16 * (VP + 4) * 4 + 4 * 16 * 2 * 4;
+  constexpr int q = 16 * (DP + 8) * 2, merge = NW * 16 * (VP + 4) * 4 + NW * 16 * 2 * 4;
   return q > merge ? q : merge;
 }
 template <int DP, int VP>
 constexpr int attn_lds_bytes() {
   constexpr int prompt = 2 * 64 * (DP + VP) * 2;
-  return prompt > few_rows_lds<DP, VP>() ? prompt : few_rows_lds<DP, VP>();
+  return prompt > few_rows_lds<DP, VP, 4>() ? prompt : few_rows_lds<DP, VP, 4>();
 }
 
 // PREP: a step of one block per request (and its splits): the workgroup first
 // makes its own queries (in LDS) and, of the request's new tokens, the keys and
 // values that fall into its pages; no separate launch.
-template <int DP, int VP, bool PREP>
+template <int DP, int VP, int NW, bool PREP>
 __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, const PagedBlock &bk,
                                               const AttnArgs &a, const AttnPrep &pr, int T,
                                               float *__restrict__ slabs, float *__restrict__ ml,
                                               char *lds) {
   constexpr int KS = DP / 32, VT = VP / 16, LDO = VP + 4;
-  float *sO = reinterpret_cast<float *>(lds), *sM = sO + 4 * 16 * LDO, *sL = sM + 64;
+  float *sO = reinterpret_cast<float *>(lds), *sM = sO + NW * 16 * LDO, *sL = sM + NW * 16;
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int grp = blockIdx.y, R = a.H / a.G;
@@ -371,15 +372,15 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
         store_value<uint16_t, NE>(pr, crow, grp, x);
       }
     };
-    for (int it = wave; it < items; it += 8) {  // two at a time
+    for (int it = wave; it < items; it += 2 * NW) {  // two at a time
       float x0[NE], x1[NE], b0[NE], b1[NE];
-      const int it1 = min(it + 4, items - 1);
+      const int it1 = min(it + NW, items - 1);
       load_bias<NE>(pr, head_of(it), b0);
       load_bias<NE>(pr, head_of(it1), b1);
       load_head<NE>(pr, T, t0 + token_of(it), head_of(it), b0, x0);
       load_head<NE>(pr, T, t0 + token_of(it1), head_of(it1), b1, x1);
       finish(it, x0);
-      if (it + 4 < items) finish(it1, x1);
+      if (it + NW < items) finish(it1, x1);
     }
     __syncthreads();  // (the new keys and values are in the cache, for this workgroup)
     const uint16_t *qr = sQ + min(l15, bk.nrows - 1) * LDQ + 8 * g;
@@ -399,7 +400,7 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
 #pragma unroll
   for (int d = 0; d < VT; ++d) acc[d] = f4{0.f, 0.f, 0.f, 0.f};
   float m = -1e30f, l = 0.f;
-  for (int u = wave; u < units; u += 4) {
+  for (int u = wave; u < units; u += NW) {
     f4 s[2];
     s[0] = s[1] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -411,7 +412,7 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
 #pragma unroll
     for (int d = 0; d < VT; ++d) vv[d] = v[d];
     const f4 bb[2] = {b[0], b[1]};
-    if (u + 4 < units) fetch(u + 4);
+    if (u + NW < units) fetch(u + NW);
     const int base = bk.tile0 * 64 + u * 32;
     float mx = -1e30f;
     bias_and_mask<2>(bb, base + 31 <= qmin, qpos, base + 4 * g, a.scale, s, mx);
@@ -443,28 +444,28 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
   {
     float M = sM[l15];
 #pragma unroll
-    for (int w = 1; w < 4; ++w) M = fmaxf(M, sM[w * 16 + l15]);
+    for (int w = 1; w < NW; ++w) M = fmaxf(M, sM[w * 16 + l15]);
     const float f = __builtin_amdgcn_exp2f(m - M);
 #pragma unroll
     for (int d = 0; d < VT; ++d)
       *reinterpret_cast<f4 *>(&sO[(wave * 16 + l15) * LDO + d * 16 + 4 * g]) = acc[d] * f;
   }
   __syncthreads();
-  // the four waves' sums: 16 threads a row, VP / 16 columns each
+  // the waves' sums: 16 threads a row, VP / 16 columns each
   constexpr int NC = VP / 16;
   const int r = tid >> 4, c0 = (tid & 15) * NC;
-  if (r >= bk.nrows) return;
+  if (r >= bk.nrows) return;  // (r: 16 and above in a fifth to eighth wave)
   float M = sM[r], L = 0.f;
 #pragma unroll
-  for (int w = 1; w < 4; ++w) M = fmaxf(M, sM[w * 16 + r]);
+  for (int w = 1; w < NW; ++w) M = fmaxf(M, sM[w * 16 + r]);
 #pragma unroll
-  for (int w = 0; w < 4; ++w) L += sL[w * 16 + r] * __builtin_amdgcn_exp2f(sM[w * 16 + r] - M);
+  for (int w = 0; w < NW; ++w) L += sL[w * 16 + r] * __builtin_amdgcn_exp2f(sM[w * 16 + r] - M);
   f4 o[NC / 4];
 #pragma unroll
   for (int c = 0; c < NC / 4; ++c) {
     o[c] = *reinterpret_cast<const f4 *>(&sO[r * LDO + c0 + c * 4]);
 #pragma unroll
-    for (int w = 1; w < 4; ++w)
+    for (int w = 1; w < NW; ++w)
       o[c] += *reinterpret_cast<const f4 *>(&sO[(w * 16 + r) * LDO + c0 + c * 4]);
   }
   if (bk.slot >= 0) {
@@ -635,34 +636,36 @@ __device__ __forceinline__ void attn_many_rows(const char *__restrict__ blob, co
 }
 
 // MANY: the step has blocks of more than 16 rows (and maybe others)
-// (two workgroups per CU = 256 registers a wave where the widths allow it: the
-// accumulators then stay in the registers the softmax works on)
+// (256 registers a wave where the widths allow it: the accumulators then stay in
+// the registers the softmax works on)
+template <int VP>
+constexpr int kFewWaves = VP <= 128 ? 8 : 4;
 template <int DP, int VP, bool MANY>
-__global__ __launch_bounds__(256, DP + VP <= 256 ? 2 : 1) void paged_attn_kernel(const char *__restrict__ blob, int off_blocks,
-                                                         AttnArgs a, float *__restrict__ slabs,
-                                                         float *__restrict__ ml) {
+__global__ __launch_bounds__(MANY ? 256 : kFewWaves<VP> * 64,
+                             MANY ? (DP + VP <= 256 ? 2 : 1) : kFewWaves<VP> / 4) void
+paged_attn_kernel(const char *__restrict__ blob, int off_blocks, AttnArgs a, float *__restrict__ slabs,
+                  float *__restrict__ ml) {
   __shared__ __attribute__((aligned(16))) char
-      lds[MANY ? attn_lds_bytes<DP, VP>() : few_rows_lds<DP, VP>()];
+      lds[MANY ? attn_lds_bytes<DP, VP>() : few_rows_lds<DP, VP, kFewWaves<VP>>()];
   const PagedBlock bk = reinterpret_cast<const PagedBlock *>(blob + off_blocks)[blockIdx.x];
   if (bk.nrows <= 0) return;
   if constexpr (MANY) {
-    if (bk.nrows > 16) {
-      attn_many_rows<DP, VP>(blob, bk, a, slabs, ml, lds);
-      return;
-    }
+    if (bk.nrows > 16) attn_many_rows<DP, VP>(blob, bk, a, slabs, ml, lds);
+    else attn_few_rows<DP, VP, 4, false>(blob, bk, a, AttnPrep(), 0, slabs, ml, lds);
+  } else {
+    attn_few_rows<DP, VP, kFewWaves<VP>, false>(blob, bk, a, AttnPrep(), 0, slabs, ml, lds);
   }
-  attn_few_rows<DP, VP, false>(blob, bk, a, AttnPrep(), 0, slabs, ml, lds);
 }
 
 // the few-rows form with its queries, keys and values made on the way
 template <int DP, int VP>
-__global__ __launch_bounds__(256, DP + VP <= 256 ? 2 : 1) void paged_attn_prep_kernel(
+__global__ __launch_bounds__(kFewWaves<VP> * 64, kFewWaves<VP> / 4) void paged_attn_prep_kernel(
     const char *__restrict__ blob, int off_blocks, AttnArgs a, AttnPrep pr, int T,
     float *__restrict__ slabs, float *__restrict__ ml) {
-  __shared__ __attribute__((aligned(16))) char lds[few_rows_lds<DP, VP>()];
+  __shared__ __attribute__((aligned(16))) char lds[few_rows_lds<DP, VP, kFewWaves<VP>>()];
   const PagedBlock bk = reinterpret_cast<const PagedBlock *>(blob + off_blocks)[blockIdx.x];
   if (bk.nrows <= 0) return;
-  attn_few_rows<DP, VP, true>(blob, bk, a, pr, T, slabs, ml, lds);
+  attn_few_rows<DP, VP, kFewWaves<VP>, true>(blob, bk, a, pr, T, slabs, ml, lds);
 }
 
 // partials of split blocks, in slot order: a workgroup per 16 rows of a block
@@ -717,14 +720,14 @@ static hipError_t run_paged_attn(const char *blob, const PagedLists &pl, const A
                                  const AttnPrep *pr, int T, float *slabs, float *ml, hipStream_t s) {
   const dim3 grid(pl.num_blocks, a.G);
   if (pr)
-    hipLaunchKernelGGL((paged_attn_prep_kernel<DP, VP>), grid, dim3(256), 0, s, blob, pl.off_blocks, a,
-                       *pr, T, slabs, ml);
+    hipLaunchKernelGGL((paged_attn_prep_kernel<DP, VP>), grid, dim3(kFewWaves<VP> * 64), 0, s, blob,
+                       pl.off_blocks, a, *pr, T, slabs, ml);
   else if (pl.row_tiles > 1)
     hipLaunchKernelGGL((paged_attn_kernel<DP, VP, true>), grid, dim3(256), 0, s, blob, pl.off_blocks, a,
                        slabs, ml);
   else
-    hipLaunchKernelGGL((paged_attn_kernel<DP, VP, false>), grid, dim3(256), 0, s, blob, pl.off_blocks, a,
-                       slabs, ml);
+    hipLaunchKernelGGL((paged_attn_kernel<DP, VP, false>), grid, dim3(kFewWaves<VP> * 64), 0, s, blob,
+                       pl.off_blocks, a, slabs, ml);
   if (pl.num_merges > 0)
     hipLaunchKernelGGL((paged_attn_merge_kernel<VP>), dim3(pl.num_merges, pl.row_tiles, a.G), dim3(256),
                        0, s, blob, pl.off_merges, a, slabs, ml);

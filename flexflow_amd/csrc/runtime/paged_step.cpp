@@ -10,9 +10,10 @@ namespace ffmi {
 static size_t up16(size_t v) { return (v + 15) & ~(size_t)15; }
 // workgroups that fill the chip; fewer blocks than this are split over keys --
 // from kSplitTiles pages on (a page costs a workgroup ~1.6 us, the merge of the
-// partials ~5 us).  The per-block form runs two workgroups per CU, and its waves
-// share out half-pages: pairs of pages keep them even.
+// partials ~5 us).  The per-block form shares half-pages out to a workgroup's
+// waves: it is split later, into whole rounds of them.
 constexpr int kTargetBlocks = 256, kSplitTiles = 5;
+constexpr int kBlockSplitTiles = 32, kBlockRound = 8;
 
 ffmi_status PagedStep::init(int max_tokens, int max_requests, int max_positions,
                             const std::vector<RowShape> &shapes, int max_slots) {
@@ -159,9 +160,9 @@ ffmi_status PagedStep::stage(const int32_t *token_ids, const std::vector<Seg> &i
         const int last = s.pos0 + (r + b.nrows - 1) / l.heads;  // last visible position
         const int tiles = last / kPageTokens + 1;
         const int units = rs.per_block && b.nrows > 16 ? rs.max_tiles : 1;  // slots of a partial
-        int ns = tiles < kSplitTiles ? 1 : std::min(want, tiles);
+        int ns = tiles < (rs.per_block ? kBlockSplitTiles : kSplitTiles) ? 1 : std::min(want, tiles);
         int per = (tiles + ns - 1) / ns;
-        if (rs.per_block && ns > 1) per = (per + 1) & ~1;
+        if (rs.per_block && ns > 1) per = (per + kBlockRound - 1) / kBlockRound * kBlockRound;
         ns = (tiles + per - 1) / per;
         if (slots + ns * units > max_slots_) ns = 1, per = tiles;
         if (ns > 1) merges_.push_back({b.row0, b.nrows, slots, ns});

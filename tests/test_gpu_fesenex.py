@@ -16,15 +16,16 @@ import flexflow_amd as fa
 pytestmark = pytest.mark.gpu
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
-# sizes that are no multiples of the kernels' tiles, layers that all differ
+# sizes that are no multiples of the kernels' tiles, layers that all differ, 1 to
+# 40 query heads to a key/value head
 ODD = FM.model_config(77, 72, [
     FM.lightning(3, 24, 40, [0.5, 0.93, 0.9995]),
-    FM.attention(6, 3, 24, 12, 0.3, bias_max=40, q_temp=(0.4, 5), ff=50, limit=0.7, rel_rows=6),
+    FM.attention(6, 2, 24, 12, 0.3, bias_max=40, q_temp=(0.4, 5), ff=50, limit=0.7, rel_rows=6),
     FM.attention(4, 1, 40, 20, 0.11, bias_max=150, v_mix=True, rel_rows=24),
     FM.lightning(1, 72, 8, [0.98], ff=33, limit=2.5),
     FM.attention(2, 1, 88, 20, 0.2, bias_max=333, q_temp=(-0.2, 64), v_mix=True, ff=130),
-    FM.attention(1, 1, 12, 20, 0.4, bias_max=7, v_mix=True, rel_rows=8)], scale=0.5)
-# full heads of the widths large models have, groups of one and of many rows
+    FM.attention(40, 1, 12, 20, 0.4, bias_max=7, v_mix=True, rel_rows=8)], scale=0.5)
+# full heads of the widths large models have
 WIDE = FM.model_config(300, 256, [
     FM.attention(8, 8, 128, 128, 0.09, bias_max=128, q_temp=(0.1, 32), v_mix=True, ff=320, rel_rows=32),
     FM.lightning(2, 128, 160, [0.9, 0.999], ff=96),
@@ -46,12 +47,12 @@ def tokens(model, n, seed):
     return [int(t) for t in np.random.default_rng(seed).integers(0, model[0]["vocab"], n)]
 
 
-def make_engine(folder, full, pool=12 * 64, batch=256):
+def make_engine(folder, full, pool=12 * 64, batch=256, positions=POSITIONS):
     cfg = fa.load_config(folder)
-    m = fa.Model(cfg, "inc", max_requests=4, max_tokens=batch, max_seq_len=POSITIONS, weights_folder=folder,
+    m = fa.Model(cfg, "inc", max_requests=4, max_tokens=batch, max_seq_len=positions, weights_folder=folder,
                  full_precision=full, kv_pool_tokens=pool)
     return fa.RequestManager(max_requests_per_batch=4, max_tokens_per_batch=batch, max_spec_tree_token_num=0,
-                             max_sequence_length=POSITIONS), m
+                             max_sequence_length=positions), m
 
 
 @pytest.fixture(scope="module")
@@ -226,12 +227,40 @@ def test_portions(engine, name, full):
 @pytest.mark.parametrize("full", [True, False])
 @pytest.mark.parametrize("name", ["odd", "wide"])
 def test_long_contexts(engine, name, full):
-    """Contexts whose blocks are split over their pages: single tokens, short
-    portions and portions of several blocks, far into the sequence."""
+    """Single tokens, short portions and portions of several blocks, far into the
+    sequence."""
     toks = tokens(MODELS[name], 740, 6)
     want, _ = reference(name, toks)
     for cuts in ([740], [640, 40, 2, 18, 1, 1, 1, 37], [319, 1, 1, 130, 3, 65, 200, 21]):
         close(run(engine(name, full), toks, cuts), want, full)
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_split_blocks(tmp_path, full):
+    """Contexts long enough that a block's pages are split over workgroups and
+    merged: single tokens, short portions, portions of several blocks, beside a
+    request that is not split."""
+    model = FM.model_config(90, 64, [FM.attention(8, 2, 24, 20, 0.2, bias_max=300, v_mix=True, q_temp=(0.3, 100)),
+                                     FM.lightning(2, 16, 24, [0.9, 0.999]),
+                                     FM.attention(20, 2, 88, 20, 0.1, bias_max=3000, v_mix=True, ff=64)])
+    w = FM.random_weights(model, 3, sharp=2.0)
+    rm, m = make_engine(FM.write_checkpoint(tmp_path / "m", model[0], w), full, pool=45 * 64, batch=1024,
+                        positions=2600)
+    toks, other = tokens(model, 2420, 1), tokens(model, 90, 2)
+    want, want2 = R.forward(model[0], w, toks), R.forward(model[0], w, other)
+    at, got = 0, []
+    for n in (1000, 1000, 47, 1, 1, 2, 3, 130, 1, 40, 66, 1, 1, 127):
+        entries = [(1, toks[at:at + n], range(n))]
+        if at == 2000:
+            entries.insert(0, (2, other, range(90)))
+        out = rm.replay_step(m, entries)
+        if at == 2000:
+            close(out[:90], want2, full)
+            out = out[90:]
+        got.append(out)
+        at += n
+    assert at == len(toks)
+    close(np.concatenate(got), want, full)
 
 
 @pytest.mark.parametrize("full", [True, False])
