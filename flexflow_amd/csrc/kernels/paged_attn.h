@@ -31,7 +31,7 @@ int attn_width(int dim);
 struct AttnPrep {
   Partials y;
   const float *bias = nullptr;                    // [columns]
-  const float *qnorm = nullptr, *knorm = nullptr;  // [dg]
+  const float *norms = nullptr;                   // [dg] of the queries, [dg] of the keys
   const float *vmix = nullptr;  // null: v as it is
   float *first = nullptr;       // values [T][G][vg]: written (vmix null) or read
   void *q = nullptr, *kc = nullptr, *vc = nullptr;

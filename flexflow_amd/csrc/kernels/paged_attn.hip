@@ -130,7 +130,7 @@ __device__ __forceinline__ void norm_head(const AttnPrep &a, bool isq, int pos, 
   for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
   float r = inv_rms(ss, a.dim, a.eps);
   if (isq && a.coef != 0.f) r *= 1.0f + a.coef * logf((float)((pos + 1) / a.every + 1));
-  const float *w = isq ? a.qnorm : a.knorm;
+  const float *w = a.norms + (isq ? 0 : a.dg);
 #pragma unroll
   for (int i = 0; i < NE; ++i) {
     const int c = head_column<NE>(i);

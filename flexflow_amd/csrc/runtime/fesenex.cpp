@@ -44,7 +44,7 @@ struct FesenexLayer {
   int dg = 0, vg = 0, dp = 0, vp = 0, nq = 0, fp = 0;
   void *win = nullptr, *wo = nullptr, *wgu = nullptr, *wdown = nullptr;
   float *norm1 = nullptr, *norm2 = nullptr;
-  float *bias = nullptr, *qnorm = nullptr, *knorm = nullptr, *vmix = nullptr, *rel = nullptr;
+  float *bias = nullptr, *norms = nullptr, *vmix = nullptr, *rel = nullptr;
   float *powers = nullptr, *onorm = nullptr;
   void *kc = nullptr, *vc = nullptr;  // [pages][groups] blocks (kernels/paged_attn.h)
   float *state = nullptr;             // [slots][heads][dg][vg]
@@ -212,8 +212,9 @@ struct Fesenex : public PagedDecoder {
       FFMI_TRY(vec_to(L.bias, m + "q.b", H, L.dim, L.dg, 0));
       FFMI_TRY(vec_to(L.bias + off_k, m + "k.b", G, L.dim, L.dg, 0));
       FFMI_TRY(vec_to(L.bias + off_v, m + "v.b", G, L.vdim, L.vg, 0));
-      FFMI_TRY(vec(&L.qnorm, m + "q.norm", 1, L.dim, L.dg));
-      FFMI_TRY(vec(&L.knorm, m + "k.norm", 1, L.dim, L.dg));
+      FFMI_TRY(alloc(&L.norms, (size_t)2 * L.dg * 4));
+      FFMI_TRY(vec_to(L.norms, m + "q.norm", 1, L.dim, L.dg));
+      FFMI_TRY(vec_to(L.norms + L.dg, m + "k.norm", 1, L.dim, L.dg));
       if (L.v_mix && !L.v_first) {
         std::vector<long> s;
         FFMI_TRY(shape_of(m + "vmix", {}, &s));
@@ -277,7 +278,7 @@ struct Fesenex : public PagedDecoder {
     const int H = L.heads, G = L.groups;
     FFMI_TRY(gemm_sum(h, L.win, L.nq, Wp, y));
     AttnPrep p;
-    p.y = *y, p.bias = L.bias, p.qnorm = L.qnorm, p.knorm = L.knorm;
+    p.y = *y, p.bias = L.bias, p.norms = L.norms;
     if (L.v_mix) p.first = first_v, p.vmix = L.vmix;
     p.q = q, p.kc = L.kc, p.vc = L.vc;
     p.H = H, p.G = G, p.dim = L.dim, p.dg = L.dg, p.dp = L.dp, p.vg = L.vg, p.vp = L.vp;
