@@ -6,17 +6,8 @@
 #include "../kernels/latent.h"
 #include "../kernels/packing.h"
 #include "../kernels/residual.h"
+#include "device_buf.h"
 #include "paged_step.h"
-
-namespace {
-struct DeviceBuf {
-  void *p = nullptr;
-  ~DeviceBuf() {
-    if (p) (void)hipFree(p);
-  }
-  bool get(size_t bytes) { return hipMalloc(&p, bytes ? bytes : 16) == hipSuccess; }
-};
-}  // namespace
 
 extern "C" ffmi_status ffmi_linear_bf16(const void *X, const void *W, void *Y, int T, int out_dim,
                                         int in_dim, int epilogue, ffmi_stream stream) {

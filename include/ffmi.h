@@ -336,7 +336,7 @@ ffmi_status ffmi_silu_mul_f32(const float *a, const float *b, float *out, size_t
 ffmi_status ffmi_arg_topk_f32(const float *logits, int T, int V, int k, int32_t *ids,
                               float *probs, ffmi_stream stream);
 /* ------------------------------------------------------------------------ */
-/* bf16 products and latent attention (the Vapipel family's operators)       */
+/* bf16 products and latent attention (operators of the registry's families) */
 /* ------------------------------------------------------------------------ */
 typedef enum {
   FFMI_BF16_PLAIN = 0, /* Y bf16 = X W^T                                      */
@@ -348,6 +348,10 @@ typedef enum {
  * packed. */
 ffmi_status ffmi_linear_bf16(const void *X, const void *W, void *Y, int T, int out_dim, int in_dim,
                              int epilogue, ffmi_stream stream);
+/* W [2 out][in]: gate rows, then up rows.  With g = min(gate, limit) and u = up
+ * within +-limit, Y [T][out] bf16 = g sigmoid(1.702 g) (u + 1) */
+ffmi_status ffmi_linear_bf16_glu(const void *X, const void *W, void *Y, int T, int out_dim,
+                                 int in_dim, float limit, ffmi_stream stream);
 /* x[T][H] += y / rms(y) * w in fp32, y the sum of `slabs` [T][H] matrices, the
  * mean over the first n columns (the rest zero); H % 32 == 0, slabs <= 8 */
 ffmi_status ffmi_post_rmsnorm(const float *y, int slabs, const float *w, float *x, int T, int H,

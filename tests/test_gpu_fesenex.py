@@ -365,6 +365,28 @@ def test_each_bucket_of_the_distance_bias_decides(tmp_path, full):
             close(run(eng, toks, cuts), want, full)
 
 
+@pytest.mark.parametrize("dim,vdim", [(24, 72), (56, 24), (120, 40), (200, 64)])
+def test_many_heads_of_linear_attention(tmp_path, dim, vdim):
+    """Heads and requests enough for every width of the chunked form: one, two
+    and four long portions together, states carried on, one of them short."""
+    heads = 100
+    model = FM.model_config(64, 32, [FM.lightning(heads, dim, vdim, [0.7 + 0.003 * h for h in range(heads)])])
+    w = FM.random_weights(model, 4)
+    rm, m = make_engine(FM.write_checkpoint(tmp_path / "m", model[0], w), False, pool=24 * 64, batch=512)
+    reqs = {rid: tokens(model, n, rid) for rid, n in ((1, 290), (2, 250), (3, 210), (4, 150))}
+    at, got = dict.fromkeys(reqs, 0), {rid: [] for rid in reqs}
+    for part in ({1: 100}, {1: 90, 2: 130}, {1: 20, 2: 100, 3: 65, 4: 64}, {1: 80, 2: 20, 3: 145, 4: 2}, {4: 84}):
+        entries = [(rid, reqs[rid][at[rid]:at[rid] + n], range(n)) for rid, n in part.items()]
+        out, r = rm.replay_step(m, entries), 0
+        for rid, toks, _ in entries:
+            got[rid].append(out[r:r + len(toks)])
+            at[rid] += len(toks)
+            r += len(toks)
+    for rid, toks in reqs.items():
+        assert at[rid] == len(toks)
+        close(np.concatenate(got[rid]), R.forward(model[0], w, toks), False)
+
+
 @pytest.mark.parametrize("full", [True, False])
 def test_state_remembers_a_marked_token(tmp_path, full):
     """Without decay a marked token's value stays in the state: it shows at any
