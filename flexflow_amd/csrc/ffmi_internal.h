@@ -197,11 +197,16 @@ struct FuseArgs {
   const uint16_t *wnorm = nullptr;  // consumer: norm weight [K]
   float eps = 0.f;
   float limit = 0.f;                // clamped gated unit (bf16 paired tiles)
+  int y_width = 0;                  // packed output: width of the rows Y is part of (0: N)
 };
 // g = min(gate, limit), u = up within +-limit: g sigmoid(1.702 g) (u + 1)
 __device__ __forceinline__ float clamped_glu(float gate, float up, float limit) {
   const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
   return g * __fdiv_rn(1.0f, 1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
+// g sigmoid(g) u
+__device__ __forceinline__ float silu_glu(float gate, float up) {
+  return gate * __fdiv_rn(1.0f, 1.0f + expf(-gate)) * up;
 }
 hipError_t launch_gemm(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
                        size_t ws_bytes, int T, int N, int K, int epilogue, hipStream_t s,
@@ -226,6 +231,11 @@ size_t gemm_bf16_glu_workspace_bytes(int T, int N, int K);
 hipError_t launch_gemm_bf16_glu(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
                                 size_t ws_bytes, int T, int N, int K, int flags, float limit,
                                 hipStream_t s);
+// The same with a SiLU gate.  y_width: width of the packed rows that Y is the
+// first N columns of (0: N)
+hipError_t launch_gemm_bf16_swiglu(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
+                                   size_t ws_bytes, int T, int N, int K, int flags, int y_width,
+                                   hipStream_t s);
 // fp16 Y[T][N] (row-major) of deferred split-K slabs, summed in slab order and
 // rounded once: the value every consumer of the slabs computes (tensor capture)
 hipError_t launch_partials_reduce(const Partials &p, uint16_t *Y, int T, int N, hipStream_t s);

@@ -1,0 +1,355 @@
+// conv_norm.hip -- sums of parallel sublayers, group norm, causal convolution
+// (conv_norm.h).
+#include "conv_norm.h"
+
+#include <algorithm>
+
+#include "device_util.h"
+
+namespace ffmi {
+
+struct ConvNormStep {
+  const char *blob = nullptr;
+  uint4 *blob_dst = nullptr;  // null: nothing to copy
+  int blob_n16 = 0, off_tokens = 0, T = 0;
+  const int32_t *out_rows = nullptr;  // null: all tokens, C per workgroup
+  int C = 1;
+  int unit = 8, parts = 0;  // columns of a partial sum, partials of a row
+  bool waves = false;       // (unit 512: a partial per wave and chunk)
+};
+
+// A workgroup takes C consecutive tokens, one after the other; a thread has chunks
+// of 8 columns.  The rows h that its first tokens convolve with are made again
+// from x_in (so x and x_in are different buffers) or come from `carry`.
+// MAXS == 0: x is an embedding row.
+// REGS: they are kept in registers (taps <= 4), else in LDS, each thread its own.
+template <int NT, int MAXC, int MAXS, bool REGS>
+__global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm a, EmbedPairs em) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, H = a.H, nchunk = H >> 3, T = st.T;
+  const PagedToken *tok = reinterpret_cast<const PagedToken *>(st.blob + st.off_tokens);
+  if (st.blob_dst) {
+    const uint4 *src = reinterpret_cast<const uint4 *>(st.blob);
+    for (int i = blockIdx.x * NT + tid; i < st.blob_n16; i += gridDim.x * NT) st.blob_dst[i] = src[i];
+  }
+  const int gs = a.n / a.groups, per = st.waves ? (gs + 511) / 512 : gs / st.unit;
+  float *part = lds, *inv = lds + 2 * st.parts;
+  f4 *ring = reinterpret_cast<f4 *>(lds + ((2 * st.parts + a.groups + 3) & ~3));
+  constexpr int KH = REGS ? 3 : 1;
+  f4 hist[KH][MAXC][2];
+  const int past = a.conv ? a.taps - 1 : 0;
+  // the row k + 1 tokens back
+  int head = 0;  // (LDS) slot of the latest row
+  auto old_row = [&](int k, int c, int h) {
+    if constexpr (REGS) return hist[k][c][h];
+    int s = head - k;
+    if (s < 0) s += past;
+    return ring[(s * 2 + h) * nchunk + min(tid + c * NT, nchunk - 1)];
+  };
+  const int first = st.out_rows ? st.out_rows[blockIdx.x] : (int)blockIdx.x * st.C;
+  const int end = st.out_rows ? first + 1 : min(first + st.C, T);
+  for (int t = first - min(tok[first].back, past), odd = 0; t < end; ++t, odd ^= 1) {
+    PagedToken tk = tok[t];  // (one token for the whole workgroup)
+    tk.token = __builtin_amdgcn_readfirstlane(tk.token), tk.prev = __builtin_amdgcn_readfirstlane(tk.prev);
+    tk.pos = __builtin_amdgcn_readfirstlane(tk.pos), tk.back = __builtin_amdgcn_readfirstlane(tk.back);
+    tk.ahead = __builtin_amdgcn_readfirstlane(tk.ahead), tk.slot = __builtin_amdgcn_readfirstlane(tk.slot);
+    tk.bank = __builtin_amdgcn_readfirstlane(tk.bank);
+    const int out = st.out_rows ? (int)blockIdx.x : t;
+    const bool mine = t >= first;
+    f4 x[MAXC][2];
+    float ss[MAXC];
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int ch = min(tid + c * NT, nchunk - 1);
+      if constexpr (MAXS == 0) {
+        unpack8_bf16(*reinterpret_cast<const uint4 *>(em.embed + (size_t)tk.token * H + ch * 8), x[c][0],
+                     x[c][1]);
+        x[c][0] *= em.scale, x[c][1] *= em.scale;
+        if (em.pairs) {
+          const int64_t b = tk.prev < 0 ? em.buckets
+                                        : (tk.prev * em.mul_prev + tk.token * em.mul_cur) % em.buckets;
+          f4 p, q;
+          unpack8_bf16(*reinterpret_cast<const uint4 *>(em.pairs + (size_t)b * H + ch * 8), p, q);
+          x[c][0] += p, x[c][1] += q;
+        }
+      } else {
+        constexpr int SB = MAXC > 1 ? 1 : NT > 512 ? (MAXS < 2 ? 1 : 2) : (MAXS < 1 ? 1 : MAXS);  // slabs in flight
+        f4 y[2], s[SB][2];
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+          x[c][h] = *reinterpret_cast<const f4 *>(a.x_in + (size_t)t * H + ch * 8 + 4 * h);
+          y[h] = f4{0.f, 0.f, 0.f, 0.f};
+        }
+        if (a.y.S > 0) {
+          const float *p = a.y.p + (size_t)t * a.y.NP + ch * 8;
+#pragma unroll
+          for (int s0 = 0; s0 < MAXS; s0 += SB) {
+            if (s0 >= a.y.S) break;
+#pragma unroll
+            for (int sl = 0; sl < SB; ++sl)
+#pragma unroll
+              for (int h = 0; h < 2; ++h)
+                s[sl][h] = *reinterpret_cast<const f4 *>(p + (size_t)min(s0 + sl, a.y.S - 1) * T * a.y.NP + 4 * h);
+#pragma unroll
+            for (int sl = 0; sl < SB; ++sl)
+              if (s0 + sl < a.y.S) y[0] += s[sl][0], y[1] += s[sl][1];
+          }
+        }
+        if (a.rows) {
+          const int32_t *at = a.at + (size_t)t * a.top;
+          const float *wt = a.wt + (size_t)t * a.top;
+          constexpr int U = MAXC > 1 ? 1 : NT > 512 ? 2 : 4;
+          for (int k0 = 0; k0 < a.top; k0 += U) {
+            f4 r[U][2];
+            float w4[U];
+#pragma unroll
+            for (int k = 0; k < U; ++k) {
+              const int kk = min(k0 + k, a.top - 1);
+              const size_t o = (size_t)at[kk] * H + ch * 8;
+              w4[k] = k0 + k < a.top ? wt[kk] : 0.f;
+              if (a.rows_f32) {
+                const float *p = (const float *)a.rows + o;
+                r[k][0] = *reinterpret_cast<const f4 *>(p), r[k][1] = *reinterpret_cast<const f4 *>(p + 4);
+              } else {
+                unpack8_bf16(*reinterpret_cast<const uint4 *>((const uint16_t *)a.rows + o), r[k][0], r[k][1]);
+              }
+            }
+#pragma unroll
+            for (int k = 0; k < U; ++k) y[0] += r[k][0] * w4[k], y[1] += r[k][1] * w4[k];
+          }
+        }
+#pragma unroll
+        for (int h = 0; h < 2; ++h) x[c][h] += y[h] * a.mult;
+      }
+      ss[c] = 0.f;
+      if (tid + c * NT < nchunk) {
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) ss[c] = fmaf(x[c][h][e], x[c][h][e], ss[c]);
+          if (a.x && mine) *reinterpret_cast<f4 *>(a.x + (size_t)t * H + ch * 8 + 4 * h) = x[c][h];
+        }
+      }
+    }
+    if (!a.w) continue;
+    // the groups' norms
+    f4 r[MAXC][2];
+    if (st.waves) {  // a wave's 512 columns lie in one group
+      float *pb = part + odd * st.parts;
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        float v = ss[c];
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
+        const int u = wave + c * (NT / 64);
+        if (lane == 0 && u < st.parts) pb[u] = v;
+      }
+      __syncthreads();
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        const int g = min((wave + c * (NT / 64)) / per, a.groups - 1);
+        float v = 0.f;
+        for (int u = 0; u < per; ++u) v += pb[g * per + u];
+        v = inv_rms(v, gs, a.eps);
+        r[c][0] = r[c][1] = f4{v, v, v, v};
+      }
+    } else {
+      const int us = st.unit, np = 8 / us;
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        const int ch = tid + c * NT;
+        if (ch >= nchunk) continue;
+        if (us == 8) {
+          if (ch < st.parts) part[ch] = ss[c];
+          continue;
+        }
+        int u = ch * np;
+        float v = 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {  // (us divides 8: runs of us columns)
+          v = fmaf(x[c][e >> 2][e & 3], x[c][e >> 2][e & 3], v);
+          if ((e + 1) & (us - 1)) continue;
+          if (u < st.parts) part[u] = v;
+          ++u, v = 0.f;
+        }
+      }
+      __syncthreads();
+      for (int g = wave; g < a.groups; g += NT / 64) {
+        float v = 0.f;
+        for (int u = lane; u < per; u += 64) v += part[g * per + u];
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
+        if (lane == 0) inv[g] = inv_rms(v, gs, a.eps);
+      }
+      __syncthreads();
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        const int ch = min(tid + c * NT, nchunk - 1);
+        int g = ch * 8 / gs, next = (g + 1) * gs;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          if (ch * 8 + e >= next) ++g, next += gs;
+          r[c][e >> 2][e & 3] = inv[min(g, a.groups - 1)];
+        }
+      }
+    }
+    if (past > 0 && tk.back == 0) {  // rows of earlier steps, zeros before the sequence
+#pragma unroll
+      for (int k = 0; k < (REGS ? 3 : 1); ++k)
+        for (int q = k; q < (REGS ? k + 1 : past); ++q) {
+          const float *cr = a.carry + ((size_t)(tk.slot * 2 + tk.bank) * past + min(q, past - 1)) * H;
+#pragma unroll
+          for (int c = 0; c < MAXC; ++c) {
+            const int ch = min(tid + c * NT, nchunk - 1);
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+              f4 v = f4{0.f, 0.f, 0.f, 0.f};
+              if (q < past && tk.pos > q) v = *reinterpret_cast<const f4 *>(cr + ch * 8 + 4 * h);
+              if constexpr (REGS) {
+                hist[k][c][h] = v;
+              } else {  // (chunk by chunk: the threads past the row write what its last owner does not read)
+                head = 0;
+                if (tid + c * NT < nchunk) ring[((q ? past - q : 0) * 2 + h) * nchunk + ch] = v;
+              }
+            }
+          }
+        }
+    }
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int ch = tid + c * NT;
+      if (ch >= nchunk) continue;
+      f4 hv[2], cv[2];
+#pragma unroll
+      for (int h = 0; h < 2; ++h) {
+        hv[h] = x[c][h] * r[c][h] * *reinterpret_cast<const f4 *>(a.w + ch * 8 + 4 * h);
+        x[c][h] = hv[h];
+      }
+      if (!mine) continue;
+      if (a.hb) *reinterpret_cast<uint4 *>(a.hb + act_packed_off(out, ch * 8, H)) = pack8_bf16(hv[0], hv[1]);
+      if (a.hrow) *reinterpret_cast<uint4 *>(a.hrow + (size_t)out * H + ch * 8) = pack8_bf16(hv[0], hv[1]);
+      if (a.hf) {
+        *reinterpret_cast<f4 *>(a.hf + (size_t)out * H + ch * 8) = hv[0];
+        *reinterpret_cast<f4 *>(a.hf + (size_t)out * H + ch * 8 + 4) = hv[1];
+      }
+      if (!a.conv) continue;
+      const bool last = tk.ahead == 0;
+      float *cr = a.carry + ((size_t)(tk.slot * 2 + (tk.bank ^ 1)) * past) * H + ch * 8;
+#pragma unroll
+      for (int h = 0; h < 2; ++h) {
+        // (oldest first, the token's own tap last)
+        f4 v = f4{0.f, 0.f, 0.f, 0.f};
+        if constexpr (REGS) {
+#pragma unroll
+          for (int k = 2; k >= 0; --k)
+            if (k < past) {
+              v += hist[k][c][h] * *reinterpret_cast<const f4 *>(a.conv + (size_t)(past - 1 - k) * H + ch * 8 + 4 * h);
+              if (last && k + 1 < past) *reinterpret_cast<f4 *>(cr + (size_t)(k + 1) * H + 4 * h) = hist[k][c][h];
+            }
+        } else {
+          for (int k = past - 1; k >= 0; --k) {
+            const f4 o = old_row(k, c, h);
+            v += o * *reinterpret_cast<const f4 *>(a.conv + (size_t)(past - 1 - k) * H + ch * 8 + 4 * h);
+            if (last && k + 1 < past) *reinterpret_cast<f4 *>(cr + (size_t)(k + 1) * H + 4 * h) = o;
+          }
+        }
+        v += hv[h] * *reinterpret_cast<const f4 *>(a.conv + (size_t)past * H + ch * 8 + 4 * h);
+        if (last && past > 0) *reinterpret_cast<f4 *>(cr + 4 * h) = hv[h];
+        cv[h] = hv[h] + v;
+      }
+      if (a.cb) *reinterpret_cast<uint4 *>(a.cb + act_packed_off(out, ch * 8, H)) = pack8_bf16(cv[0], cv[1]);
+      if (a.cf) {
+        *reinterpret_cast<f4 *>(a.cf + (size_t)out * H + ch * 8) = cv[0];
+        *reinterpret_cast<f4 *>(a.cf + (size_t)out * H + ch * 8 + 4) = cv[1];
+      }
+    }
+    // h becomes the latest earlier row
+    if (past > 0) {
+      if constexpr (REGS) {
+#pragma unroll
+        for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+          for (int h = 0; h < 2; ++h)
+            hist[2][c][h] = hist[1][c][h], hist[1][c][h] = hist[0][c][h], hist[0][c][h] = x[c][h];
+      } else {
+        head = head + 1 == past ? 0 : head + 1;
+#pragma unroll
+        for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+          for (int h = 0; h < 2; ++h)
+            if (tid + c * NT < nchunk) ring[(head * 2 + h) * nchunk + tid + c * NT] = x[c][h];
+      }
+    }
+  }
+}
+
+static hipError_t run_conv_norm(ConvNormStep st, const ConvNorm &a, const EmbedPairs &em, int blocks,
+                                hipStream_t s) {
+  const int nchunk = a.H / 8;
+  if (a.H % 32 || a.n > a.H || a.groups < 1 || a.n % a.groups || a.y.S < 0 || a.y.S > 8) return hipErrorInvalidValue;
+  if (a.y.S > 0 && (a.y.NP < a.H || a.y.NP % 4 || !a.y.p)) return hipErrorInvalidValue;
+  if (a.rows && (!a.at || !a.wt || a.top < 1)) return hipErrorInvalidValue;
+  if (!em.embed && (!a.x_in || a.x_in == a.x)) return hipErrorInvalidValue;
+  if (a.conv && (a.taps < 1 || (a.taps > 1 && !a.carry))) return hipErrorInvalidValue;
+  const int gs = a.n / a.groups;
+  st.waves = a.groups == 1 || gs % 512 == 0;
+  st.unit = st.waves ? 512 : gs % 8 == 0 ? 8 : gs % 4 == 0 ? 4 : gs % 2 == 0 ? 2 : 1;
+  st.parts = st.waves ? (a.n + 511) / 512 : a.n / st.unit;
+  const bool regs = (!a.conv || a.taps <= 4) && nchunk <= 1024;  // (wider rows: in LDS)
+  size_t lds = (size_t)((2 * st.parts + a.groups + 3) & ~3) * 4;
+  if (!regs && a.conv) lds += (size_t)(a.taps - 1) * a.H * 4;
+  if (lds > 160 * 1024) return hipErrorInvalidValue;
+#define FFMI_CN2(NT, MC, MS, RG)                                                                       \
+  do {                                                                                                 \
+    if (lds > 64 * 1024) {                                                                             \
+      const hipError_t e = hipFuncSetAttribute((const void *)(conv_norm_kernel<NT, MC, MS, RG>),       \
+                                               hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
+      if (e != hipSuccess) return e;                                                                   \
+    }                                                                                                  \
+    hipLaunchKernelGGL((conv_norm_kernel<NT, MC, MS, RG>), dim3(blocks), dim3(NT), lds, s, st, a, em); \
+  } while (0)
+#define FFMI_CN(NT, MC)                                            \
+  do {                                                             \
+    if (em.embed) {                                                \
+      if (MC == 1 && regs) FFMI_CN2(NT, MC, 0, (MC == 1));         \
+      else FFMI_CN2(NT, MC, 0, false);                             \
+    } else if (MC == 1 && regs) {                                  \
+      if (a.y.S <= 1) FFMI_CN2(NT, MC, (MC == 1 ? 1 : 8), (MC == 1)); \
+      else FFMI_CN2(NT, MC, 8, (MC == 1));                         \
+    } else {                                                       \
+      FFMI_CN2(NT, MC, 8, false);                                  \
+    }                                                              \
+  } while (0)
+  if (nchunk <= 128) FFMI_CN(128, 1);
+  else if (nchunk <= 256) FFMI_CN(256, 1);
+  else if (nchunk <= 512) FFMI_CN(512, 1);
+  else if (nchunk <= 1024) FFMI_CN(1024, 1);
+  else if (nchunk <= 2048) FFMI_CN(1024, 2);
+  else return hipErrorInvalidValue;
+#undef FFMI_CN
+#undef FFMI_CN2
+  return hipGetLastError();
+}
+
+hipError_t launch_conv_norm(const char *blob_src, char *blob_dst, size_t blob_bytes, int off_tokens,
+                            const ConvNorm &a, const EmbedPairs *em, int T, hipStream_t s) {
+  if (T <= 0) return hipSuccess;
+  if (em && off_tokens) return hipErrorInvalidValue;
+  ConvNormStep st;
+  st.blob = blob_src, st.off_tokens = off_tokens, st.T = T;
+  if (em) st.blob_dst = reinterpret_cast<uint4 *>(blob_dst), st.blob_n16 = (int)((blob_bytes + 15) / 16);
+  st.C = T <= 256 ? 1 : T <= 1024 ? 4 : 8;
+  return run_conv_norm(st, a, em ? *em : EmbedPairs(), (T + st.C - 1) / st.C, s);
+}
+
+hipError_t launch_conv_norm_rows(const char *blob, int off_tokens, int off_rows, const ConvNorm &a, int T,
+                                 int R, hipStream_t s) {
+  if (R <= 0) return hipSuccess;
+  if (a.conv || a.x) return hipErrorInvalidValue;
+  ConvNormStep st;
+  st.blob = blob, st.off_tokens = off_tokens, st.T = T;
+  st.out_rows = reinterpret_cast<const int32_t *>(blob + off_rows);
+  return run_conv_norm(st, a, EmbedPairs(), R, s);
+}
+
+}  // namespace ffmi

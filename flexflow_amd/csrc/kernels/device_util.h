@@ -44,4 +44,9 @@ __device__ __forceinline__ float inv_rms(float ss, int n, float eps) {
   return __fdiv_rn(1.0f, sqrtf(__fdiv_rn(ss, (float)n) + eps));
 }
 
+// cosine and sine of so many turns
+__device__ __forceinline__ void turn_by(double turns, float &c, float &s) {
+  sincospif(2.0f * (float)(turns - rint(turns)), &s, &c);
+}
+
 }  // namespace ffmi

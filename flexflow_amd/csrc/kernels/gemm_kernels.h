@@ -64,12 +64,13 @@ __device__ __forceinline__ uint16_t silu_mul_h(float gacc, float uacc) {
 //   (4 always writes the split-K slab layout, S = 1 included: its consumer
 //   takes the fp32 sums unrounded)
 //   5 bf16, clamped gated unit of paired [gate|up] tiles (`lim`: its limit)
+//   6 bf16, SiLU gate of paired [gate|up] tiles, fp32 up to the product
 template <int EPI>
 constexpr bool epi_bf16 = EPI >= 2;
 template <int EPI>
 constexpr bool epi_f32 = EPI == 4;
 template <int EPI>
-constexpr bool epi_paired = EPI == 1 || EPI == 5;
+constexpr bool epi_paired = EPI == 1 || EPI == 5 || EPI == 6;
 // (fragments are 16 raw bytes per lane in either format)
 template <int EPI>
 __device__ __forceinline__ f4 mma16(h8 a, h8 b, f4 c) {
@@ -93,6 +94,7 @@ __device__ __forceinline__ uint16_t out16(float v) {
 template <int EPI>
 __device__ __forceinline__ uint16_t pair16(float g, float u, float lim) {
   if constexpr (EPI == 5) return f2bf(clamped_glu(g, u, lim));
+  else if constexpr (EPI == 6) return f2bf(silu_glu(g, u));
   else return silu_mul_h(g, u);
 }
 
@@ -474,7 +476,7 @@ __global__ __launch_bounds__(KW * 64) void gemm_skinny_kernel(
         for (int r = 0; r < 4; ++r) {
           int m = m0 + i * 16 + (lane >> 4) * 4 + r;
           if (m < T)
-            Y[yp ? act_packed_off(m, n, N) : (size_t)m * N + n] = out16<EPI>(acc[i][j][r]);
+            Y[yp ? act_packed_off(m, n, yp) : (size_t)m * N + n] = out16<EPI>(acc[i][j][r]);
         }
     }
   } else {
@@ -487,7 +489,7 @@ __global__ __launch_bounds__(KW * 64) void gemm_skinny_kernel(
         for (int r = 0; r < 4; ++r) {
           int m = m0 + i * 16 + (lane >> 4) * 4 + r;
           if (m >= T) continue;
-          Y[yp ? act_packed_off(m, n, N) : (size_t)m * N + n] =
+          Y[yp ? act_packed_off(m, n, yp) : (size_t)m * N + n] =
               pair16<EPI>(acc[i][0][r], acc[i][1][r], fz.limit);
         }
     }
@@ -608,7 +610,7 @@ __global__ __launch_bounds__(WPG * 64) void gemm_wave_kernel(const uint16_t *__r
         const int m = i * 16 + (lane >> 4) * 4 + r;
         if (m >= T) continue;
         if constexpr (epi_f32<EPI>) Yf[(size_t)m * (NTILES * 16) + n] = acc[i][j][r];
-        else Y[yp ? act_packed_off(m, n, N) : (size_t)m * N + n] = out16<EPI>(acc[i][j][r]);
+        else Y[yp ? act_packed_off(m, n, yp) : (size_t)m * N + n] = out16<EPI>(acc[i][j][r]);
       }
   }
 }
@@ -808,7 +810,7 @@ __device__ __forceinline__ void mid_store(const f4 (&acc)[MTW][NTW], uint16_t *_
       for (int r = 0; r < 4; ++r)
         if constexpr (epi_paired<EPI>) o[r] = pair16<EPI>(acc[i][j][r], acc[i][j + 1][r], lim);
         else o[r] = out16<EPI>(acc[i][j][r]);
-      uint16_t *dst = yp ? Y + act_packed_off(m, n, N) : Y + (size_t)m * N + n;
+      uint16_t *dst = yp ? Y + act_packed_off(m, n, yp) : Y + (size_t)m * N + n;
       if (n + 4 <= N && (((uintptr_t)dst & 7) == 0)) {
         *reinterpret_cast<uint2 *>(dst) =
             make_uint2(o[0] | ((uint32_t)o[1] << 16), o[2] | ((uint32_t)o[3] << 16));
@@ -1101,7 +1103,7 @@ __global__ void gemm_reduce_kernel(const float *__restrict__ Ypart, uint16_t *__
 #pragma unroll
   for (int r = 0; r < 4; ++r)
     o[r] = epi_paired<EPI> ? pair16<EPI>(acc[r], up[r], lim) : out16<EPI>(acc[r]);
-  uint16_t *dst = yp ? Y + act_packed_off(m, n, N) : Y + (size_t)m * N + n;
+  uint16_t *dst = yp ? Y + act_packed_off(m, n, yp) : Y + (size_t)m * N + n;
   if (n + 4 <= N && (((uintptr_t)dst & 7) == 0)) {
     *reinterpret_cast<uint2 *>(dst) =
         make_uint2(o[0] | ((uint32_t)o[1] << 16), o[2] | ((uint32_t)o[3] << 16));
@@ -1311,13 +1313,14 @@ static hipError_t launch_gemm_kind(const uint16_t *X, const uint16_t *Wp, uint16
   const int KT = K / 32;
   const int mtiles = (T + 15) / 16;
   const bool xp = (epilogue & FFMI_X_PACKED) != 0;
-  const int yp = (epilogue & FFMI_Y_PACKED) ? 1 : 0;
+  // packed output: the width of the packed rows (N, or wider: fuse->y_width)
+  const int yp = !(epilogue & FFMI_Y_PACKED) ? 0 : fuse && fuse->y_width ? fuse->y_width : N;
   const bool nt = (epilogue & FFMI_W_STREAM) != 0;
   constexpr int paired = epi_paired<E> ? 1 : 0;
   const float lim = fuse ? fuse->limit : 0.f;
   if (epi_f32<E> && (!ws || ws_bytes < (size_t)T * ((N + 15) / 16) * 16 * sizeof(float)))
     return hipErrorInvalidValue;
-  if ((xp && K % 32) || (yp && N % 32)) return hipErrorInvalidValue;
+  if ((xp && K % 32) || (yp && (N % 32 || yp % 32 || yp < N))) return hipErrorInvalidValue;
   if constexpr (E < 2)
   if (fuse && fuse->kind) {
     // producer: row-major residual out, plain epilogue; consumer: row-major X

@@ -1,0 +1,77 @@
+// moe.h -- mixture of experts: routing, row lists, products by expert: launchers
+// (moe.hip).
+//
+// A token's chosen experts are rows ("slots") of products grouped by expert: every
+// expert's slots lie together, from a multiple of 16 on.  A shared expert that runs
+// for every token is one more group, its slots the tokens in order after all
+// others (from `shared_slot` on in what the second product leaves).
+#pragma once
+#include "../ffmi_internal.h"
+
+namespace ffmi {
+
+struct MoeTile {
+  int32_t expert;  // == number of experts: the shared one
+  int32_t slot0, rows, pad;
+};
+constexpr int kMoeFew = 16, kMoeMany = 128;  // rows of a tile in the two forms
+constexpr int kMoeMaxExperts = 1024, kMoeMaxTop = 64;
+
+// a step's sizes: T tokens of which each takes `top` of `experts`
+struct MoeSizes {
+  int T = 0, experts = 0, top = 0;
+  bool shared = false;
+  int gate_col = 0;  // column of the shared expert's gate in the router's product
+  int tile_rows() const {
+    return (long)T * top >= 32L * experts ? kMoeMany : kMoeFew;
+  }
+  // upper bounds: slots of the experts (whole 16s), tiles
+  __host__ __device__ int expert_slots() const {
+    const int a = T * top, e = a < experts ? a : experts;
+    return (a + 15 * e + 15) / 16 * 16;
+  }
+  __host__ __device__ int shared_slot() const { return expert_slots(); }
+  int slots() const { return expert_slots() + (shared ? (T + 15) / 16 * 16 : 0); }
+  int max_tiles(int rows) const {
+    const int a = T * top, e = a < experts ? a : experts;
+    return (a - e) / rows + e + (shared ? (T + rows - 1) / rows : 0);
+  }
+  __host__ __device__ int picks() const { return top + (shared ? 1 : 0); }
+};
+struct MoeLists {
+  int32_t *picked = nullptr;      // [T][top] experts
+  int32_t *at = nullptr;          // [T][picks] slots, the shared expert's last
+  float *wt = nullptr;            // [T][picks] their weights
+  int32_t *slot_token = nullptr;  // [expert slots]
+  MoeTile *tiles = nullptr;
+  int32_t *num_tiles = nullptr;
+};
+// z: router products, the experts' columns first.  The `top` largest z + bias (the
+// lowest index among equals), softmax over them; the shared expert's weight is the
+// sigmoid of its gate.
+hipError_t launch_moe_route(const Partials &z, const float *bias, const MoeSizes &n, const MoeLists &l,
+                            hipStream_t s);
+
+// One product of every slot with its expert's matrix.
+//   first  (gated): Y[slot] = silu(X W_gate) (X W_up), X the token's row (row-major),
+//          Y bf16 in packed tiles of width N per group (fp32: rows)
+//   second: Y[slot] = X W_down, X the first product's Y; Y rows of N, bf16 (fp32)
+// W: bf16 packed weights, gate / up tiles in turn (fp32: rows, gate then up), expert
+// after expert.
+struct MoeGroup {
+  const void *X = nullptr, *W = nullptr;
+  void *Y = nullptr;
+  int N = 0, K = 0;
+  size_t w_stride = 0;  // elements from expert to expert
+};
+struct MoeGemm {
+  MoeGroup g[2];  // experts, shared
+  int experts = 0;
+  const int32_t *slot_token = nullptr;
+  const MoeTile *tiles = nullptr;
+  const int32_t *num_tiles = nullptr;
+};
+hipError_t launch_moe_gemm(const MoeGemm &a, const MoeSizes &n, bool gated, bool f32, bool stream_weights,
+                           hipStream_t s);
+
+}  // namespace ffmi

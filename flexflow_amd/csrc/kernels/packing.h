@@ -8,10 +8,16 @@ namespace ffmi {
 // head n / np's row n % np (zero from nb on; heads * np rows), column k
 // likewise from (kb, kp).  transpose: src holds [heads][K][N] blocks.
 // perhead: each head its own tile-major packed block (head products).
+// row_pairs / col_pairs: of every head's first so many rows (columns), m and
+// m + half of them come to lie side by side (rotations that pair halves).
+// k0 / kt: the matrix is k-steps k0 .. of a destination of kt k-steps, 32
+// columns each (0: the destination is this matrix alone).
 struct PackSpec {
   int rows = 0, nb = 0, np = 0;  // heads, real rows per head, padded rows per head
   int cols = 0, kb = 0, kp = 0;
   bool transpose = false;
+  int row_pairs = 0, col_pairs = 0;
+  int k0 = 0, kt = 0;
 };
 hipError_t launch_pack_bf16(const uint16_t *src, int ld, const PackSpec &p, uint16_t *dst,
                             int tile_offset, int pitch, bool perhead, hipStream_t s,

@@ -6,7 +6,10 @@ namespace ffmi {
 
 __device__ __forceinline__ uint16_t pack_elem(const uint16_t *src, int ld, const PackSpec &p, int n,
                                               int k) {
-  const int hn = n / p.np, jn = n % p.np, hk = k / p.kp, jk = k % p.kp;
+  const int hn = n / p.np, hk = k / p.kp;
+  int jn = n % p.np, jk = k % p.kp;
+  if (jn < p.row_pairs) jn = (jn >> 1) + (jn & 1) * (p.row_pairs >> 1);
+  if (jk < p.col_pairs) jk = (jk >> 1) + (jk & 1) * (p.col_pairs >> 1);
   if (hn >= p.rows || jn >= p.nb || hk >= p.cols || jk >= p.kb) return 0;
   if (p.transpose) return src[((size_t)hn * p.kb + jk) * ld + jn];
   return src[(size_t)(hn * p.nb + jn) * ld + hk * p.kb + jk];
@@ -30,24 +33,25 @@ hipError_t launch_pack_bf16(const uint16_t *src, int ld, const PackSpec &p, uint
   const int N = p.rows * p.np, K = p.cols * p.kp;
   if (N % 16 || K % 32) return hipErrorInvalidValue;
   const int NT = N / 16, KT = K / 32;
-  const size_t ts = perhead ? (size_t)KT * 512 : w_tile_stride(KT);
+  const size_t ts = perhead ? (size_t)KT * 512 : w_tile_stride(p.kt ? p.kt : KT);
   const size_t ks = perhead ? 512 : w_k_stride(pitch);
+  dst += p.k0 * ks;
   hipLaunchKernelGGL(pack_bf16_kernel, dim3((unsigned)(((long)NT * KT * 64 + 255) / 256)),
                      dim3(256), 0, s, src, ld, p, dst + tile_offset * ts, NT, KT,
                      tile_step * ts, ks);
   return hipGetLastError();
 }
 __global__ void pack_f32_kernel(const uint16_t *__restrict__ src, int ld, PackSpec p,
-                                float *__restrict__ dst, int N, int K) {
+                                float *__restrict__ dst, int N, int K, int ldd) {
   const long i = blockIdx.x * (long)blockDim.x + threadIdx.x;
   if (i >= (long)N * K) return;
-  dst[i] = bf2f(pack_elem(src, ld, p, (int)(i / K), (int)(i % K)));
+  dst[i / K * ldd + i % K] = bf2f(pack_elem(src, ld, p, (int)(i / K), (int)(i % K)));
 }
 hipError_t launch_pack_f32(const uint16_t *src, int ld, const PackSpec &p, float *dst,
                            hipStream_t s) {
   const int N = p.rows * p.np, K = p.cols * p.kp;
   hipLaunchKernelGGL(pack_f32_kernel, dim3((unsigned)(((long)N * K + 255) / 256)), dim3(256), 0, s,
-                     src, ld, p, dst, N, K);
+                     src, ld, p, dst + p.k0 * 32, N, K, p.kt ? p.kt * 32 : K);
   return hipGetLastError();
 }
 

@@ -12,7 +12,12 @@ constexpr int kPageTokens = 64;
 struct PagedToken {
   int32_t token, pos;  // embedding row, position in the sequence
   int32_t row;         // cache row: page * kPageTokens + offset
-  int32_t pad;
+  int32_t prev;        // the token before it in the sequence (-1: none)
+  // its place among its request's tokens in the batch: so many before and after
+  int32_t back, ahead;
+  // rows that a layer carries from step to step lie in two banks per request
+  // slot: this step reads one and writes the other
+  int32_t slot, bank;
 };
 
 // One workgroup of the attention: `nrows` consecutive (token, head) rows of a
@@ -45,6 +50,7 @@ constexpr int kShortSpan = 16;
 struct PagedLists {  // the block lists of the layers with one row shape
   int heads = 0;      // rows per token
   int groups = 1;     // copies of the list a launch runs (key/value heads)
+  int window = 0;     // the last positions that a query sees, itself included (0: all)
   int row_tiles = 0;  // rows of the largest block / 16
   int num_blocks = 0, num_merges = 0, off_blocks = 0, off_merges = 0;
 };

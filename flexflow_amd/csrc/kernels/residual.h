@@ -29,5 +29,9 @@ hipError_t launch_row_norm(const char *blob, int off_rows, const float *x, const
 hipError_t launch_relu2_f32(float *u, size_t n, hipStream_t s);
 // Y[T][F] = clamped_glu of gu [T][gate F | up F]
 hipError_t launch_glu_f32(const float *gu, float *Y, int T, int F, float limit, hipStream_t s);
+// the same with a SiLU gate, Y rows of ldy
+hipError_t launch_swiglu_f32(const float *gu, float *Y, int T, int F, int ldy, hipStream_t s);
+// z = cap tanh(z / cap) on n columns of rows of ld
+hipError_t launch_soft_cap(float *z, int R, int n, int ld, float cap, hipStream_t s);
 
 }  // namespace ffmi

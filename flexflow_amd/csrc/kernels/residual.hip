@@ -244,4 +244,30 @@ hipError_t launch_glu_f32(const float *gu, float *Y, int T, int F, float limit, 
   return hipGetLastError();
 }
 
+__global__ void swiglu_f32_kernel(const float *__restrict__ gu, float *__restrict__ Y, int F, size_t n, int ldy) {
+  for (size_t i = blockIdx.x * (size_t)blockDim.x + threadIdx.x; i < n;
+       i += (size_t)gridDim.x * blockDim.x) {
+    const size_t t = i / F, c = i % F;
+    Y[t * ldy + c] = silu_glu(gu[t * 2 * F + c], gu[t * 2 * F + F + c]);
+  }
+}
+hipError_t launch_swiglu_f32(const float *gu, float *Y, int T, int F, int ldy, hipStream_t s) {
+  const size_t n = (size_t)T * F;
+  if (n == 0) return hipSuccess;
+  hipLaunchKernelGGL(swiglu_f32_kernel, dim3((unsigned)std::min<size_t>((n + 255) / 256, 16384)),
+                     dim3(256), 0, s, gu, Y, F, n, ldy);
+  return hipGetLastError();
+}
+
+__global__ void soft_cap_kernel(float *z, int n, int ld, float cap) {
+  float *row = z + (size_t)blockIdx.y * ld;
+  for (int c = blockIdx.x * 256 + threadIdx.x; c < n; c += gridDim.x * 256) row[c] = cap * tanhf(__fdiv_rn(row[c], cap));
+}
+hipError_t launch_soft_cap(float *z, int R, int n, int ld, float cap, hipStream_t s) {
+  if (R <= 0) return hipSuccess;
+  if (!(cap > 0.f)) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(soft_cap_kernel, dim3(std::min((n + 255) / 256, 64), R), dim3(256), 0, s, z, n, ld, cap);
+  return hipGetLastError();
+}
+
 }  // namespace ffmi

@@ -92,7 +92,7 @@ ffmi_status PagedDecoder::shape_of(const std::string &name, const std::vector<lo
 
 ffmi_status PagedDecoder::pack_rows(const PackSpec &p, int ld, void *dst, int row0, int N) {
   if (f32)
-    FFMI_HIP(launch_pack_f32(tmp, ld, p, (float *)dst + (size_t)row0 * p.cols * p.kp, stream));
+    FFMI_HIP(launch_pack_f32(tmp, ld, p, (float *)dst + (size_t)row0 * (p.kt ? p.kt * 32 : p.cols * p.kp), stream));
   else
     FFMI_HIP(launch_pack_bf16(tmp, ld, p, (uint16_t *)dst, row0 / 16, N / 16, false, stream));
   return FFMI_OK;
@@ -184,10 +184,16 @@ ffmi_status PagedDecoder::gemm_sum(const void *X, const void *Wt, int N, int K, 
   return FFMI_OK;
 }
 
-ffmi_status PagedDecoder::capture_layer(int i) {
+ffmi_status PagedDecoder::capture(int i, const float *rows) {
   if (dbg)
-    FFMI_HIP(hipMemcpyAsync(dbg_x + (size_t)i * Tm * Wp, x, (size_t)step.T * Wp * 4,
+    FFMI_HIP(hipMemcpyAsync(dbg_x + (size_t)i * Tm * Wp, rows, (size_t)step.T * Wp * 4,
                             hipMemcpyDeviceToDevice, stream));
+  return FFMI_OK;
+}
+
+ffmi_status PagedDecoder::output_rows() {
+  FFMI_HIP(launch_row_norm(step.dev, step.off_rows, x, final_norm, f32 ? nullptr : (uint16_t *)h,
+                           f32 ? (float *)h : nullptr, step.R, Wp, W, eps, stream));
   return FFMI_OK;
 }
 
@@ -195,13 +201,13 @@ ffmi_status PagedDecoder::enqueue(bool sample) {
   FFMI_TRY(run_layers());
   const int R = step.R;
   if (R == 0) return FFMI_OK;
-  FFMI_HIP(launch_row_norm(step.dev, step.off_rows, x, final_norm, f32 ? nullptr : (uint16_t *)h,
-                           f32 ? (float *)h : nullptr, R, Wp, W, eps, stream));
+  FFMI_TRY(output_rows());
   if (f32)
     FFMI_HIP(launch_gemm_f32((const float *)h, (const float *)head, logits, R, Vp, Wp, stream));
   else
     FFMI_HIP(launch_gemm_bf16_f32((const uint16_t *)h, (const uint16_t *)head, nullptr, logits,
                                   (size_t)Tm * Vp * 4, R, Vp, Wp, FFMI_X_PACKED | wstream, stream));
+  if (logit_cap > 0.f) FFMI_HIP(launch_soft_cap(logits, R, V, Vp, logit_cap, stream));
   if (sample)  // greedy: argmax of the softmax, straight into pinned memory
     FFMI_HIP(launch_softmax_topk_f32(logits, R, V, 1, res_h, (float *)(res_h + Tm), stream, Vp));
   return FFMI_OK;
@@ -226,7 +232,7 @@ ffmi_status PagedDecoder::forward(const BatchConfig &bc, const int *rows, int n,
                                 tk.abs_depth_in_request),
                  FFMI_ERR_INVALID);
     }
-  FFMI_TRY(step.stage(bc, pool, rows, n));
+  FFMI_TRY(step.stage(bc, pool, recurrent ? &states : nullptr, rows, n));
   if (step.T == 0) return FFMI_OK;
   if (recurrent)
     for (int t = 0; t < bc.num_tokens; ++t) {
@@ -263,8 +269,11 @@ ffmi_status PagedDecoder::forward(const BatchConfig &bc, const int *rows, int n,
   }
   FFMI_HIP(hipStreamSynchronize(stream));
   if (recurrent)
-    for (int t = 0; t < bc.num_tokens; ++t)
-      states.done(bc.tokensInfo[t].request_index, bc.tokensInfo[t].abs_depth_in_request + 1);
+    for (int t = 0; t < bc.num_tokens; ++t) {
+      const auto &tk = bc.tokensInfo[t];
+      if (t + 1 == bc.num_tokens || bc.tokensInfo[t + 1].request_index != tk.request_index)
+        states.done(tk.request_index, tk.abs_depth_in_request + 1, tk.token_id);
+    }
   if (dbg) dbg_T = step.T, dbg_R = step.R;
   return FFMI_OK;
 }

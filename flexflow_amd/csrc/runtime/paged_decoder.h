@@ -35,6 +35,8 @@ struct PagedDecoder : public ffmi_model {
   virtual ffmi_status init_layers() = 0;
   // the layers of a step: token rows to the residual stream x
   virtual ffmi_status run_layers() = 0;
+  // the output product's rows: h = norm(x) of the step's output rows
+  virtual ffmi_status output_rows();
 
   ffmi_model_opts o{};
   std::string folder;
@@ -43,6 +45,7 @@ struct PagedDecoder : public ffmi_model {
   int Vp = 0, Wp = 0, Tm = 0;  // padded; batch capacity
   int num_layers = 0;
   float eps = 0.f;
+  float logit_cap = 0.f;  // soft cap of the logits (0: none)
   bool f32 = false;
   bool recurrent = false;  // some layer keeps a state per request slot
   float *final_norm = nullptr;
@@ -114,7 +117,9 @@ struct PagedDecoder : public ffmi_model {
   // ---- steps ----
   // y (fp32 sums) = X . W^T
   ffmi_status gemm_sum(const void *X, const void *Wt, int N, int K, Partials *y);
-  ffmi_status capture_layer(int i);  // (tensor capture) x after layer i
+  ffmi_status capture_layer(int i) { return capture(i, x); }  // (tensor capture) x after layer i
+  ffmi_status capture(int i, const float *rows);
+  bool capturing() const { return dbg != 0; }
   ffmi_status enqueue(bool sample);
   ffmi_status forward(const BatchConfig &bc, const int *rows, int n, bool sample);
 

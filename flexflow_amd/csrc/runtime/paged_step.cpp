@@ -23,10 +23,10 @@ ffmi_status PagedStep::init(int max_tokens, int max_requests, int max_positions,
          (size_t)max_requests * ((max_pages_ + 16) * 4 + sizeof(PagedSpan)) + 256;
   for (const RowShape &h : shapes) {
     bool known = false;
-    for (const RowShape &k : shapes_) known |= k.heads == h.heads && k.groups == h.groups;
+    for (const RowShape &k : shapes_) known |= k.heads == h.heads && k.groups == h.groups && k.window == h.window;
     if (known) continue;
     PagedLists l;
-    l.heads = h.heads, l.groups = h.groups;
+    l.heads = h.heads, l.groups = h.groups, l.window = h.window;
     lists_.push_back(l);
     shapes_.push_back(h);
     const size_t nb = ((size_t)max_tokens * h.heads + 15) / 16 + max_requests + max_slots + 128;
@@ -48,13 +48,14 @@ PagedStep::~PagedStep() {
   if (dev) (void)hipFree(dev);
 }
 
-const PagedLists &PagedStep::lists(int heads, int groups) const {
+const PagedLists &PagedStep::lists(int heads, int groups, int window) const {
   for (const auto &l : lists_)
-    if (l.heads == heads && l.groups == groups) return l;
+    if (l.heads == heads && l.groups == groups && l.window == window) return l;
   return lists_.front();
 }
 
-ffmi_status PagedStep::stage(const BatchConfig &bc, PagePool &pool, const int *rows, int num_rows) {
+ffmi_status PagedStep::stage(const BatchConfig &bc, PagePool &pool, const StateSlots *states, const int *rows,
+                             int num_rows) {
   const int n = bc.num_tokens;
   FFMI_CHECK(n >= 0 && n <= max_tokens_, FFMI_ERR_INVALID);
   std::vector<Seg> segs;
@@ -70,6 +71,10 @@ ffmi_status PagedStep::stage(const BatchConfig &bc, PagePool &pool, const int *r
       pool.set_owner(slot, guid);
     }
     Seg s{0, bc.tokensInfo[t].abs_depth_in_request, nullptr, slot};
+    if (states) {
+      if (s.pos0 > 0) s.prev = states->last(slot);
+      s.bank = states->bank(slot);
+    }
     for (; t < n && bc.tokensInfo[t].request_index == slot; ++t, ++s.n) {
       FFMI_CHECK(bc.tokensInfo[t].abs_depth_in_request == s.pos0 + s.n, FFMI_ERR_INVALID);
       ids_[t] = bc.tokensInfo[t].token_id;
@@ -106,7 +111,8 @@ ffmi_status PagedStep::stage(const int32_t *token_ids, const std::vector<Seg> &i
   for (size_t i = 0; i < in.size(); ++i)
     for (int j = 0; j < in[i].n; ++j) {
       const int p = in[i].pos0 + j, t = segs[i].t0 + j;
-      tok[t] = {token_ids[t], p, in[i].table[p / kPageTokens] * kPageTokens + p % kPageTokens, 0};
+      tok[t] = {token_ids[t], p, in[i].table[p / kPageTokens] * kPageTokens + p % kPageTokens,
+                j > 0 ? token_ids[t - 1] : in[i].prev, j, in[i].n - 1 - j, in[i].slot, in[i].bank};
     }
   size_t off = up16((size_t)T * sizeof(PagedToken));
   off_rows = (int)off;
@@ -158,7 +164,9 @@ ffmi_status PagedStep::stage(const int32_t *token_ids, const std::vector<Seg> &i
         b.row0 = row0 + r, b.nrows = std::min(br, nrows - r);
         b.seg_row = row0, b.pos0 = s.pos0, b.table = s.table;
         const int last = s.pos0 + (r + b.nrows - 1) / l.heads;  // last visible position
-        const int tiles = last / kPageTokens + 1;
+        // the first page that the block's first row sees
+        const int first = l.window ? std::max(0, s.pos0 + r / l.heads - l.window + 1) / kPageTokens : 0;
+        const int tiles = last / kPageTokens + 1 - first;
         const int units = rs.per_block && b.nrows > 16 ? rs.max_tiles : 1;  // slots of a partial
         int ns = tiles < (rs.per_block ? kBlockSplitTiles : kSplitTiles) ? 1 : std::min(want, tiles);
         int per = (tiles + ns - 1) / ns;
@@ -167,7 +175,7 @@ ffmi_status PagedStep::stage(const int32_t *token_ids, const std::vector<Seg> &i
         if (slots + ns * units > max_slots_) ns = 1, per = tiles;
         if (ns > 1) merges_.push_back({b.row0, b.nrows, slots, ns});
         for (int i = 0; i < ns; ++i) {
-          b.tile0 = i * per, b.ntiles = std::min(per, tiles - i * per);
+          b.tile0 = first + i * per, b.ntiles = std::min(per, tiles - i * per);
           b.slot = ns > 1 ? slots : -1;
           if (ns > 1) slots += units;
           b.page0 = reinterpret_cast<const int32_t *>(host)[s.table + b.tile0];

@@ -7,6 +7,7 @@
 #include "../kernels/paged.h"
 #include "batch_config.h"
 #include "page_pool.h"
+#include "state_slots.h"
 
 namespace ffmi {
 
@@ -19,6 +20,7 @@ namespace ffmi {
 struct RowShape {
   int heads = 1, groups = 1, max_tiles = 4;
   bool per_block = false;
+  int window = 0;  // positions a query sees, itself included: earlier pages are left out (0: all)
 };
 
 struct PagedStep {
@@ -33,6 +35,8 @@ struct PagedStep {
     int n, pos0;
     const int32_t *table;  // pages of positions 0 .. pos0 + n
     int slot = 0;          // request slot
+    int prev = -1;         // the token before the first (-1: none or not wanted)
+    int bank = 0;          // of the slot's carried rows (kernels/paged.h)
   };
   // Fills the pinned staging: the segments' tokens in order (token_ids), the
   // output rows and the attention's lists.
@@ -40,9 +44,11 @@ struct PagedStep {
                     int num_rows);
   // The same from an INC batch: takes the pages its tokens
   // need (a slot whose request changed gives its old pages back first) and
-  // lists rows[0, num_rows) for the output.
-  ffmi_status stage(const BatchConfig &bc, PagePool &pool, const int *rows, int num_rows);
-  const PagedLists &lists(int heads, int groups = 1) const;
+  // lists rows[0, num_rows) for the output.  states: where the requests' last
+  // tokens and banks come from (null: no layer asks for them).
+  ffmi_status stage(const BatchConfig &bc, PagePool &pool, const StateSlots *states, const int *rows,
+                    int num_rows);
+  const PagedLists &lists(int heads, int groups = 1, int window = 0) const;
 
   char *host = nullptr, *dev = nullptr;
   size_t bytes = 0;
