@@ -233,6 +233,7 @@ hipError_t launch_gemm_bf16_glu(const uint16_t *X, const uint16_t *Wp, uint16_t 
                                 hipStream_t s);
 // The same with a SiLU gate.  y_width: width of the packed rows that Y is the
 // first N columns of (0: N)
+size_t gemm_bf16_swiglu_workspace_bytes(int T, int N, int K);
 hipError_t launch_gemm_bf16_swiglu(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
                                    size_t ws_bytes, int T, int N, int K, int flags, int y_width,
                                    hipStream_t s);

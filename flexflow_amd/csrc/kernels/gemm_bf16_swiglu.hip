@@ -4,6 +4,8 @@
 
 namespace ffmi {
 
+size_t gemm_bf16_swiglu_workspace_bytes(int T, int N, int K) { return gemm_slab_bytes(T, N, K, 1); }
+
 hipError_t launch_gemm_bf16_swiglu(const uint16_t *X, const uint16_t *Wp, uint16_t *Y, float *ws,
                                    size_t ws_bytes, int T, int N, int K, int flags, int y_width,
                                    hipStream_t s) {

@@ -228,7 +228,7 @@ struct Nomutar : public PagedDecoder {
       if (L.ff && f32) gemms.push_back({2 * L.fp, Wp});
       if (L.ff && !f32)
         for (int t = 16; t <= Tm; t += 16)
-          ws_bytes = std::max(ws_bytes, gemm_bf16_glu_workspace_bytes(t, L.fp, Wp));
+          ws_bytes = std::max(ws_bytes, gemm_bf16_swiglu_workspace_bytes(t, L.fp, Wp));
       if (!L.experts) continue;
       L.efp = up(L.eff, 32), L.sfp = up(L.sff, 32), L.gate_col = up(L.experts, 16);
       L.nr = up(L.gate_col + 1, 32);

@@ -193,6 +193,7 @@ SIGNATURES = {
     "ffmi_model_destroy": (None, [c_void_p]),
     "ffmi_model_vocab_size": (c_int, [c_void_p]),
     "ffmi_linear_bf16": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p]),
+    "ffmi_linear_bf16_swiglu": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p]),
     "ffmi_linear_bf16_glu": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p]),
     "ffmi_post_rmsnorm": (c_int, [c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_float,
                                   c_void_p]),

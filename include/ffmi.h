@@ -352,6 +352,9 @@ ffmi_status ffmi_linear_bf16(const void *X, const void *W, void *Y, int T, int o
  * within +-limit, Y [T][out] bf16 = g sigmoid(1.702 g) (u + 1) */
 ffmi_status ffmi_linear_bf16_glu(const void *X, const void *W, void *Y, int T, int out_dim,
                                  int in_dim, float limit, ffmi_stream stream);
+/* The same with a SiLU gate: Y = gate sigmoid(gate) up */
+ffmi_status ffmi_linear_bf16_swiglu(const void *X, const void *W, void *Y, int T, int out_dim,
+                                    int in_dim, ffmi_stream stream);
 /* x[T][H] += y / rms(y) * w in fp32, y the sum of `slabs` [T][H] matrices, the
  * mean over the first n columns (the rest zero); H % 32 == 0, slabs <= 8 */
 ffmi_status ffmi_post_rmsnorm(const float *y, int slabs, const float *w, float *x, int T, int H,
