@@ -304,6 +304,34 @@ def fesenex_config(width, heads, kv_heads, dim, ff, layers, vocab=32000):
                              mlp=mlp) for i in range(layers)])
 
 
+# --model nomutar: (name, width, heads, key/value heads, head size, ff, layers)
+NOMUTAR_SIZES = [("width2048", 2048, 16, 4, 128, 5632, 8), ("width4096", 4096, 32, 8, 128, 11008, 8)]
+
+
+def nomutar_config(width, heads, kv_heads, dim, ff, layers, vocab=32000):
+    """The three types of attention in turn, a window of 512 in two of them; every
+    fourth layer's feed-forward dense, the others 32 experts of which a token takes 4,
+    beside a shared one (a token's units together: ff)."""
+    part = (ff // 8 + 31) // 32 * 32
+    scalings = {"attention": dict(factor=8.0, low=1.0, high=4.0, original=8192),
+                "attention_2": dict(factor=4.0, original=4096, fast=32.0, slow=1.0)}
+
+    def one(i):
+        kind = ("attention_2", "attention", "attention_3", "attention")[i % 4]
+        mix = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** -0.5,
+                   rot=dict(base=500000.0, dims=dim))
+        if kind in scalings:
+            mix["rot"]["scaling"] = scalings[kind]
+            mix.update(mask=dict(size=512), softcap=50.0)
+        mlp = dict(kind="dense", ff=ff) if i % 4 == 0 else \
+            dict(kind="moe", expert=dict(ff=part), router=dict(experts=32, top=4), shared=dict(ff=ff - 4 * part))
+        return dict(type=kind, mixer=mix, mlp=mlp)
+    return dict(architecture="Nomutar", vocab=vocab, width=width,
+                embedding=dict(scale=width ** 0.5, bigram=dict(buckets=65521, mul_prev=31, mul_cur=7)),
+                norm=dict(eps=1e-6, groups=4), canon=dict(taps=4), residual_mult=0.5, logit_softcap=30.0,
+                layers=[one(i) for i in range(layers)])
+
+
 def bench_decoder(cfg, B, prompt_len, decode, mtb, repeats):
     """Prefill and decode throughput of incremental decoding: generates of one
     new token (the prompts' steps alone) and of `decode`, best of `repeats`."""
@@ -334,38 +362,43 @@ def bench_decoder(cfg, B, prompt_len, decode, mtb, repeats):
 
 
 def bench_family(args):
-    """--model vapipel | fesenex: the family's decoder (random weights) and LLaMA
-    at equal sizes, incremental decoding, one GPU.  One JSON line."""
+    """--model vapipel | fesenex | nomutar: the family's decoder (random weights) and
+    LLaMA (nomutar: Fesenex too) at equal sizes, incremental decoding, one GPU.  One
+    JSON line."""
     legs = []
-    sizes = VAPIPEL_SIZES if args.model == "vapipel" else FESENEX_SIZES
+    sizes = {"vapipel": VAPIPEL_SIZES, "fesenex": FESENEX_SIZES, "nomutar": NOMUTAR_SIZES}[args.model]
     for name, width, heads, *more, ff, layers in sizes:
         if args.only_size and name != args.only_size:
             continue
         if args.model == "vapipel":
             dim, rank = more
-            leg0, own = {"kv_rank": rank}, vapipel_config(width, heads, dim, rank, ff, layers)
+            leg0, cfgs = {"kv_rank": rank}, {"vapipel": vapipel_config(width, heads, dim, rank, ff, layers)}
         else:
             kv_heads, dim = more
-            leg0, own = {"kv_heads": kv_heads}, fesenex_config(width, heads, kv_heads, dim, ff, layers)
-        cfgs = {args.model: own,
-                "llama": dict(num_layers=layers, vocab_size=32000, num_heads=heads,
-                              num_kv_heads=heads, hidden=width, intermediate=ff, rms_eps=1e-6,
-                              rope_theta=10000.0)}
+            grouped = (width, heads, kv_heads, dim, ff, layers)
+            leg0, cfgs = {"kv_heads": kv_heads}, {"fesenex": fesenex_config(*grouped)}
+            if args.model == "nomutar":
+                cfgs = {"nomutar": nomutar_config(*grouped), **cfgs}
+        cfgs["llama"] = dict(num_layers=layers, vocab_size=32000, num_heads=heads, num_kv_heads=heads,
+                             hidden=width, intermediate=ff, rms_eps=1e-6, rope_theta=10000.0)
         for prompt in (args.prefill, 1024):
             leg = {"size": name, **leg0, "layers": layers, "batch": args.batch,
                    "prompt": prompt, "decode": args.decode}
             for fam, cfg in cfgs.items():
-                if args.only_family and (fam == "llama") != (args.only_family == "llama"):
+                if args.only_family and fam != args.only_family:
                     continue
                 leg[fam] = bench_decoder(cfg, args.batch, prompt, args.decode,
                                          args.max_tokens_per_batch, args.steps)
             legs.append(leg)
             print(f"[bench] {json.dumps(leg)}", file=sys.stderr, flush=True)
-    head = legs[-1].get(args.model) or legs[-1]["llama"]
+    ran = args.only_family if args.only_family in cfgs else args.model
+    head = legs[-1][ran]
     what = {"vapipel": "latent-attention decoder",
-            "fesenex": "softmax- and linear-attention decoder"}[args.model]
+            "fesenex": "softmax- and linear-attention decoder",
+            "nomutar": "decoder of parallel layers with experts"}[args.model]
+    beside = "Fesenex and LLaMA" if args.model == "nomutar" else "LLaMA"
     print(json.dumps({
-        "metric": f"decode tokens/s, {what} beside LLaMA at equal size",
+        "metric": f"decode tokens/s, {what} beside {beside} at equal size",
         "value": head["decode_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
         "warmup": 1, "ms_per_step": round(head["decode_step_us"] / 1e3, 4),
         "higher_is_better": True, "scaling": "strong", "vs_baseline": None, "dtype": "bf16",
@@ -454,12 +487,12 @@ def main():
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
     ap.add_argument("--mode", choices=["spec", "incr"], default="spec")
-    ap.add_argument("--model", choices=["llama", "vapipel", "fesenex"], default="llama",
-                    help="llama: the headline workload; vapipel, fesenex: prefill and decode throughput "
+    ap.add_argument("--model", choices=["llama", "vapipel", "fesenex", "nomutar"], default="llama",
+                    help="llama: the headline workload; vapipel, fesenex, nomutar: prefill and decode throughput "
                          "of that family's decoder beside LLaMA at equal sizes (one GPU)")
-    ap.add_argument("--only-family", choices=["llama", "vapipel", "fesenex"], default=None,
-                    help="--model vapipel | fesenex: run one of the two (profiling)")
-    ap.add_argument("--only-size", default=None, help="--model vapipel | fesenex: run one size (profiling)")
+    ap.add_argument("--only-family", choices=["llama", "vapipel", "fesenex", "nomutar"], default=None,
+                    help="--model vapipel | fesenex | nomutar: run one of the models (profiling)")
+    ap.add_argument("--only-size", default=None, help="--model vapipel | fesenex | nomutar: run one size (profiling)")
     ap.add_argument("--batch", type=int, default=8)
     ap.add_argument("--prefill", type=int, default=128)
     ap.add_argument("--decode", type=int, default=128)
