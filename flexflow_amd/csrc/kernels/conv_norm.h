@@ -27,6 +27,7 @@ struct ConvNorm {
   const float *conv = nullptr;  // [taps][H]; null: no convolution
   int taps = 0;
   float *carry = nullptr;
+  float *inv = nullptr;  // [T][groups] scratch (convolution): 1 / rms of the groups
   // h and c in packed tiles, rows of bf16, or rows of fp32 (null: not wanted)
   uint16_t *hb = nullptr, *hrow = nullptr, *cb = nullptr;
   float *hf = nullptr, *cf = nullptr;

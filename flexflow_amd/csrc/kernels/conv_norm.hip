@@ -12,18 +12,19 @@ struct ConvNormStep {
   const char *blob = nullptr;
   uint4 *blob_dst = nullptr;  // null: nothing to copy
   int blob_n16 = 0, off_tokens = 0, T = 0;
-  const int32_t *out_rows = nullptr;  // null: all tokens, C per workgroup
-  int C = 1;
+  const int32_t *out_rows = nullptr;  // null: all tokens
   int unit = 8, parts = 0;  // columns of a partial sum, partials of a row
   bool waves = false;       // (unit 512: a partial per wave and chunk)
 };
 
-// A workgroup takes C consecutive tokens, one after the other; a thread has chunks
-// of 8 columns.  The rows h that its first tokens convolve with are made again
-// from x_in (so x and x_in are different buffers) or come from `carry`.
+// A workgroup takes a token; a thread has chunks of 8 columns.  Few tokens (CONV):
+// the convolution as well; the rows h that it reads are made again from x_in (so x
+// and x_in are different buffers) or come from `carry`.  Many tokens: conv_kernel
+// follows, on the x and inv of this one.
 // MAXS == 0: x is an embedding row.
-// REGS: they are kept in registers (taps <= 4), else in LDS, each thread its own.
-template <int NT, int MAXC, int MAXS, bool REGS>
+// REGS: the earlier rows are kept in registers (taps <= 4), else in LDS, each thread
+// its own.
+template <int NT, int MAXC, int MAXS, bool CONV, bool REGS>
 __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm a, EmbedPairs em) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, H = a.H, nchunk = H >> 3, T = st.T;
@@ -37,7 +38,7 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
   f4 *ring = reinterpret_cast<f4 *>(lds + ((2 * st.parts + a.groups + 3) & ~3));
   constexpr int KH = REGS ? 3 : 1;
   f4 hist[KH][MAXC][2];
-  const int past = a.conv ? a.taps - 1 : 0;
+  const int past = CONV ? a.taps - 1 : 0;
   // the row k + 1 tokens back
   int head = 0;  // (LDS) slot of the latest row
   auto old_row = [&](int k, int c, int h) {
@@ -46,16 +47,38 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
     if (s < 0) s += past;
     return ring[(s * 2 + h) * nchunk + min(tid + c * NT, nchunk - 1)];
   };
-  const int first = st.out_rows ? st.out_rows[blockIdx.x] : (int)blockIdx.x * st.C;
-  const int end = st.out_rows ? first + 1 : min(first + st.C, T);
-  for (int t = first - min(tok[first].back, past), odd = 0; t < end; ++t, odd ^= 1) {
+  const int first = st.out_rows ? st.out_rows[blockIdx.x] : (int)blockIdx.x;
+  for (int t = CONV ? first - min(tok[first].back, past) : first, odd = 0; t <= first; ++t, odd ^= 1) {
     PagedToken tk = tok[t];  // (one token for the whole workgroup)
     tk.token = __builtin_amdgcn_readfirstlane(tk.token), tk.prev = __builtin_amdgcn_readfirstlane(tk.prev);
     tk.pos = __builtin_amdgcn_readfirstlane(tk.pos), tk.back = __builtin_amdgcn_readfirstlane(tk.back);
     tk.ahead = __builtin_amdgcn_readfirstlane(tk.ahead), tk.slot = __builtin_amdgcn_readfirstlane(tk.slot);
     tk.bank = __builtin_amdgcn_readfirstlane(tk.bank);
     const int out = st.out_rows ? (int)blockIdx.x : t;
-    const bool mine = t >= first;
+    const bool mine = t == first;
+    // (rows of earlier steps, zeros before the sequence; first: nothing waits for them)
+    if (CONV && past > 0 && tk.back == 0) {
+#pragma unroll
+      for (int k = 0; k < (REGS ? 3 : 1); ++k)
+        for (int q = k; q < (REGS ? k + 1 : past); ++q) {
+          const float *cr = a.carry + ((size_t)(tk.slot * 2 + tk.bank) * past + min(q, past - 1)) * H;
+#pragma unroll
+          for (int c = 0; c < MAXC; ++c) {
+            const int ch = min(tid + c * NT, nchunk - 1);
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+              f4 v = f4{0.f, 0.f, 0.f, 0.f};
+              if (q < past && tk.pos > q) v = *reinterpret_cast<const f4 *>(cr + ch * 8 + 4 * h);
+              if constexpr (REGS) {
+                hist[k][c][h] = v;
+              } else {  // (chunk by chunk: the threads past the row write what its last owner does not read)
+                head = 0;
+                if (tid + c * NT < nchunk) ring[((q ? past - q : 0) * 2 + h) * nchunk + ch] = v;
+              }
+            }
+          }
+        }
+    }
     f4 x[MAXC][2];
     float ss[MAXC];
 #pragma unroll
@@ -98,7 +121,7 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
         if (a.rows) {
           const int32_t *at = a.at + (size_t)t * a.top;
           const float *wt = a.wt + (size_t)t * a.top;
-          constexpr int U = MAXC > 1 ? 1 : NT > 512 ? 2 : 4;
+          constexpr int U = MAXC > 1 ? 1 : NT > 512 ? 2 : 8;
           for (int k0 = 0; k0 < a.top; k0 += U) {
             f4 r[U][2];
             float w4[U];
@@ -151,6 +174,8 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
         float v = 0.f;
         for (int u = 0; u < per; ++u) v += pb[g * per + u];
         v = inv_rms(v, gs, a.eps);
+        const int u = wave + c * (NT / 64);
+        if (!CONV && a.inv && lane == 0 && u < st.parts && u % per == 0) a.inv[(size_t)t * a.groups + g] = v;
         r[c][0] = r[c][1] = f4{v, v, v, v};
       }
     } else {
@@ -179,7 +204,10 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
         for (int u = lane; u < per; u += 64) v += part[g * per + u];
 #pragma unroll
         for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
-        if (lane == 0) inv[g] = inv_rms(v, gs, a.eps);
+        if (lane == 0) {
+          inv[g] = inv_rms(v, gs, a.eps);
+          if (!CONV && a.inv) a.inv[(size_t)t * a.groups + g] = inv[g];
+        }
       }
       __syncthreads();
 #pragma unroll
@@ -192,28 +220,6 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
           r[c][e >> 2][e & 3] = inv[min(g, a.groups - 1)];
         }
       }
-    }
-    if (past > 0 && tk.back == 0) {  // rows of earlier steps, zeros before the sequence
-#pragma unroll
-      for (int k = 0; k < (REGS ? 3 : 1); ++k)
-        for (int q = k; q < (REGS ? k + 1 : past); ++q) {
-          const float *cr = a.carry + ((size_t)(tk.slot * 2 + tk.bank) * past + min(q, past - 1)) * H;
-#pragma unroll
-          for (int c = 0; c < MAXC; ++c) {
-            const int ch = min(tid + c * NT, nchunk - 1);
-#pragma unroll
-            for (int h = 0; h < 2; ++h) {
-              f4 v = f4{0.f, 0.f, 0.f, 0.f};
-              if (q < past && tk.pos > q) v = *reinterpret_cast<const f4 *>(cr + ch * 8 + 4 * h);
-              if constexpr (REGS) {
-                hist[k][c][h] = v;
-              } else {  // (chunk by chunk: the threads past the row write what its last owner does not read)
-                head = 0;
-                if (tid + c * NT < nchunk) ring[((q ? past - q : 0) * 2 + h) * nchunk + ch] = v;
-              }
-            }
-          }
-        }
     }
 #pragma unroll
     for (int c = 0; c < MAXC; ++c) {
@@ -232,7 +238,7 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
         *reinterpret_cast<f4 *>(a.hf + (size_t)out * H + ch * 8) = hv[0];
         *reinterpret_cast<f4 *>(a.hf + (size_t)out * H + ch * 8 + 4) = hv[1];
       }
-      if (!a.conv) continue;
+      if constexpr (!CONV) continue;
       const bool last = tk.ahead == 0;
       float *cr = a.carry + ((size_t)(tk.slot * 2 + (tk.bank ^ 1)) * past) * H + ch * 8;
 #pragma unroll
@@ -283,6 +289,104 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
   }
 }
 
+// The convolution of many tokens: a thread has 8 columns of C consecutive tokens.
+// TAPS: at most (0: any; earlier rows are then read for every token again).
+template <int C, int TAPS>
+__global__ __launch_bounds__(256) void conv_kernel(const PagedToken *__restrict__ tok, int T, ConvNorm a) {
+  const int H = a.H, col = (blockIdx.y * 256 + threadIdx.x) * 8, t0 = blockIdx.x * C, past = a.taps - 1;
+  if (col >= H) return;
+  const int gs = a.n / a.groups;
+  auto load8 = [](const float *p, f4 (&v)[2]) {
+    v[0] = *reinterpret_cast<const f4 *>(p), v[1] = *reinterpret_cast<const f4 *>(p + 4);
+  };
+  f4 w[2];
+  load8(a.w + col, w);
+  // row h of token t of this step
+  auto scale_row = [&](int t, f4 (&v)[2]) {
+    const float *iv = a.inv + (size_t)t * a.groups;
+    if (gs % 8 == 0) {
+      const float r = iv[min(col / gs, a.groups - 1)];
+      v[0] = v[0] * f4{r, r, r, r} * w[0], v[1] = v[1] * f4{r, r, r, r} * w[1];
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e >> 2][e & 3] = v[e >> 2][e & 3] * iv[min((col + e) / gs, a.groups - 1)] * w[e >> 2][e & 3];
+    }
+  };
+  // the row of q + 1 tokens before the step's first one of the request
+  auto old_row = [&](const PagedToken &tk, int q, f4 (&v)[2]) {
+    v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
+    if (tk.pos - tk.back > q) load8(a.carry + ((size_t)(tk.slot * 2 + tk.bank) * past + q) * H + col, v);
+  };
+  auto finish = [&](int t, const PagedToken &tk, const f4 (&h)[2], f4 (&v)[2]) {
+    f4 cw[2];
+    load8(a.conv + (size_t)past * H + col, cw);
+#pragma unroll
+    for (int k = 0; k < 2; ++k) v[k] = h[k] + (v[k] + h[k] * cw[k]);
+    if (a.cb) *reinterpret_cast<uint4 *>(a.cb + act_packed_off(t, col, H)) = pack8_bf16(v[0], v[1]);
+    if (a.cf) {
+      *reinterpret_cast<f4 *>(a.cf + (size_t)t * H + col) = v[0];
+      *reinterpret_cast<f4 *>(a.cf + (size_t)t * H + col + 4) = v[1];
+    }
+  };
+  auto keep = [&](const PagedToken &tk, int q, const f4 (&h)[2]) {  // h as the q-th row of the next step's carry
+    float *cr = a.carry + ((size_t)(tk.slot * 2 + (tk.bank ^ 1)) * past + q) * H + col;
+    *reinterpret_cast<f4 *>(cr) = h[0], *reinterpret_cast<f4 *>(cr + 4) = h[1];
+  };
+  if constexpr (TAPS > 0) {
+    constexpr int P = TAPS - 1;
+    f4 h[C + P][2], cw[P][2];  // rows t0 - P .., taps of the rows 1 to P tokens back
+#pragma unroll
+    for (int i = 0; i < C + P; ++i) load8(a.x + (size_t)min(max(t0 - P + i, 0), T - 1) * H + col, h[i]);
+#pragma unroll
+    for (int k = 0; k < P; ++k) load8(a.conv + (size_t)max(past - 1 - k, 0) * H + col, cw[k]);
+#pragma unroll
+    for (int i = 0; i < C + P; ++i) scale_row(min(max(t0 - P + i, 0), T - 1), h[i]);
+#pragma unroll
+    for (int i = 0; i < C; ++i) {
+      const int t = t0 + i;
+      if (t >= T) break;
+      const PagedToken tk = tok[t];
+      f4 v[2];
+      v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int k = P - 1; k >= 0; --k)  // (oldest first, the token's own tap last)
+        if (k < past) {
+          f4 o[2];
+          if (tk.back > k) o[0] = h[i + P - 1 - k][0], o[1] = h[i + P - 1 - k][1];
+          else old_row(tk, k - tk.back, o);
+          v[0] += o[0] * cw[k][0], v[1] += o[1] * cw[k][1];
+          if (tk.ahead == 0 && k + 1 < past) keep(tk, k + 1, o);
+        }
+      if (tk.ahead == 0 && past > 0) keep(tk, 0, h[i + P]);
+      finish(t, tk, h[i + P], v);
+    }
+  } else {
+    for (int t = t0; t < min(t0 + C, T); ++t) {
+      const PagedToken tk = tok[t];
+      f4 h[2], v[2];
+      load8(a.x + (size_t)t * H + col, h);
+      scale_row(t, h);
+      v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
+      for (int k = past - 1; k >= 0; --k) {
+        f4 o[2], cw[2];
+        load8(a.conv + (size_t)(past - 1 - k) * H + col, cw);
+        if (tk.back > k) {
+          load8(a.x + (size_t)(t - 1 - k) * H + col, o);
+          scale_row(t - 1 - k, o);
+        } else {
+          old_row(tk, k - tk.back, o);
+        }
+        v[0] += o[0] * cw[0], v[1] += o[1] * cw[1];
+        if (tk.ahead == 0 && k + 1 < past) keep(tk, k + 1, o);
+      }
+      if (tk.ahead == 0 && past > 0) keep(tk, 0, h);
+      finish(t, tk, h, v);
+    }
+  }
+}
+
+// steps of more tokens take the convolution from a launch of its own
+constexpr int kConvFused = 64;
 static hipError_t run_conv_norm(ConvNormStep st, const ConvNorm &a, const EmbedPairs &em, int blocks,
                                 hipStream_t s) {
   const int nchunk = a.H / 8;
@@ -290,35 +394,37 @@ static hipError_t run_conv_norm(ConvNormStep st, const ConvNorm &a, const EmbedP
   if (a.y.S > 0 && (a.y.NP < a.H || a.y.NP % 4 || !a.y.p)) return hipErrorInvalidValue;
   if (a.rows && (!a.at || !a.wt || a.top < 1)) return hipErrorInvalidValue;
   if (!em.embed && (!a.x_in || a.x_in == a.x)) return hipErrorInvalidValue;
-  if (a.conv && (a.taps < 1 || (a.taps > 1 && !a.carry))) return hipErrorInvalidValue;
+  if (a.conv && (!a.w || a.taps < 1 || (a.taps > 1 && !a.carry))) return hipErrorInvalidValue;
+  // many tokens: the convolution in a launch of its own
+  const bool split = a.conv && st.T > kConvFused && a.x && a.inv, conv = a.conv && !split;
   const int gs = a.n / a.groups;
   st.waves = a.groups == 1 || gs % 512 == 0;
   st.unit = st.waves ? 512 : gs % 8 == 0 ? 8 : gs % 4 == 0 ? 4 : gs % 2 == 0 ? 2 : 1;
   st.parts = st.waves ? (a.n + 511) / 512 : a.n / st.unit;
-  const bool regs = (!a.conv || a.taps <= 4) && nchunk <= 1024;  // (wider rows: in LDS)
+  const bool regs = conv && a.taps <= 4 && nchunk <= 1024;  // (wider rows: in LDS)
   size_t lds = (size_t)((2 * st.parts + a.groups + 3) & ~3) * 4;
-  if (!regs && a.conv) lds += (size_t)(a.taps - 1) * a.H * 4;
+  if (conv && !regs) lds += (size_t)(a.taps - 1) * a.H * 4;
   if (lds > 160 * 1024) return hipErrorInvalidValue;
-#define FFMI_CN2(NT, MC, MS, RG)                                                                       \
+#define FFMI_CN2(NT, MC, MS, CV, RG)                                                                   \
   do {                                                                                                 \
     if (lds > 64 * 1024) {                                                                             \
-      const hipError_t e = hipFuncSetAttribute((const void *)(conv_norm_kernel<NT, MC, MS, RG>),       \
+      const hipError_t e = hipFuncSetAttribute((const void *)(conv_norm_kernel<NT, MC, MS, CV, RG>),   \
                                                hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
       if (e != hipSuccess) return e;                                                                   \
     }                                                                                                  \
-    hipLaunchKernelGGL((conv_norm_kernel<NT, MC, MS, RG>), dim3(blocks), dim3(NT), lds, s, st, a, em); \
+    hipLaunchKernelGGL((conv_norm_kernel<NT, MC, MS, CV, RG>), dim3(blocks), dim3(NT), lds, s, st, a, em); \
   } while (0)
-#define FFMI_CN(NT, MC)                                            \
-  do {                                                             \
-    if (em.embed) {                                                \
-      if (MC == 1 && regs) FFMI_CN2(NT, MC, 0, (MC == 1));         \
-      else FFMI_CN2(NT, MC, 0, false);                             \
-    } else if (MC == 1 && regs) {                                  \
-      if (a.y.S <= 1) FFMI_CN2(NT, MC, (MC == 1 ? 1 : 8), (MC == 1)); \
-      else FFMI_CN2(NT, MC, 8, (MC == 1));                         \
-    } else {                                                       \
-      FFMI_CN2(NT, MC, 8, false);                                  \
-    }                                                              \
+#define FFMI_CN1(NT, MC, MS)                                   \
+  do {                                                         \
+    if (!conv) FFMI_CN2(NT, MC, MS, false, false);             \
+    else if (MC == 1 && regs) FFMI_CN2(NT, MC, MS, true, (MC == 1)); \
+    else FFMI_CN2(NT, MC, MS, true, false);                    \
+  } while (0)
+#define FFMI_CN(NT, MC)                                         \
+  do {                                                          \
+    if (em.embed) FFMI_CN1(NT, MC, 0);                          \
+    else if (MC == 1 && a.y.S <= 2) FFMI_CN1(NT, MC, (MC == 1 ? 2 : 8)); \
+    else FFMI_CN1(NT, MC, 8);                                   \
   } while (0)
   if (nchunk <= 128) FFMI_CN(128, 1);
   else if (nchunk <= 256) FFMI_CN(256, 1);
@@ -327,7 +433,18 @@ static hipError_t run_conv_norm(ConvNormStep st, const ConvNorm &a, const EmbedP
   else if (nchunk <= 2048) FFMI_CN(1024, 2);
   else return hipErrorInvalidValue;
 #undef FFMI_CN
+#undef FFMI_CN1
 #undef FFMI_CN2
+  if (split) {
+    // (the first kernel's staging copy is there by now, in any form)
+    const PagedToken *tok =
+        reinterpret_cast<const PagedToken *>((st.blob_dst ? (const char *)st.blob_dst : st.blob) + st.off_tokens);
+#define FFMI_CV(C, TP) \
+  hipLaunchKernelGGL((conv_kernel<C, TP>), dim3((st.T + C - 1) / C, (nchunk + 255) / 256), dim3(256), 0, s, tok, st.T, a)
+    if (a.taps <= 4) FFMI_CV(8, 4);
+    else FFMI_CV(4, 0);
+#undef FFMI_CV
+  }
   return hipGetLastError();
 }
 
@@ -338,8 +455,7 @@ hipError_t launch_conv_norm(const char *blob_src, char *blob_dst, size_t blob_by
   ConvNormStep st;
   st.blob = blob_src, st.off_tokens = off_tokens, st.T = T;
   if (em) st.blob_dst = reinterpret_cast<uint4 *>(blob_dst), st.blob_n16 = (int)((blob_bytes + 15) / 16);
-  st.C = T <= 256 ? 1 : T <= 1024 ? 4 : 8;
-  return run_conv_norm(st, a, em ? *em : EmbedPairs(), (T + st.C - 1) / st.C, s);
+  return run_conv_norm(st, a, em ? *em : EmbedPairs(), T, s);
 }
 
 hipError_t launch_conv_norm_rows(const char *blob, int off_tokens, int off_rows, const ConvNorm &a, int T,

@@ -1176,7 +1176,8 @@ static MidPlan mid_plan(int T, int N, int K, int epi, bool deferred = false) {
   // K = 11008 down projection (gate/up 337 -> 270 us, qkv 149 -> 139,
   // down 148 -> 135, lm_head 428 -> 409); FFMI_PREFILL_PLAN=0 keeps the model
   static const bool prefill_plan = !getenv("FFMI_PREFILL_PLAN") || atoi(getenv("FFMI_PREFILL_PLAN")) != 0;
-  if (prefill_plan && p.mblocks >= 4) {
+  // (N <= 128, a router's columns: a handful of workgroups; the model splits K)
+  if (prefill_plan && p.mblocks >= 4 && !(deferred && ntiles <= 8)) {
     p.NTW = 8;
     p.S = K >= 8192 && KT >= 2 ? 2 : 1;
     // 4-row-tile waves run one workgroup per CU: only where the grid still

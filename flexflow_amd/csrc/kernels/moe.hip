@@ -10,23 +10,32 @@ namespace ffmi {
 // ---------------------------------------------------------------------------
 // routing
 // ---------------------------------------------------------------------------
+// a column's sum over the slabs, their loads together
+__device__ __forceinline__ float slab_total(const Partials &z, const float *p, size_t slab) {
+  float v[8];
+#pragma unroll
+  for (int s = 0; s < 8; ++s) v[s] = p[min(s, z.S - 1) * slab];
+#pragma unroll
+  for (int s = 1; s < 8; ++s)
+    if (s < z.S) v[0] += v[s];
+  return v[0];
+}
 // A wave picks a token's experts: NV logits a lane, the best of the wave `top`
 // times over.
 template <int NV>
 __device__ __forceinline__ void pick_experts(const Partials &z, const float *__restrict__ bias, const MoeSizes &n,
-                                             int t, int32_t *picked, float *wt) {
+                                             int t, const MoeLists &l) {
   const int lane = threadIdx.x & 63;
   const size_t slab = (size_t)n.T * z.NP;
   const float *row = z.p + (size_t)t * z.NP;
+  const float gate = n.shared ? slab_total(z, row + n.gate_col, slab) : 0.f;
   float v[NV];
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
     const int e = i * 64 + lane;
     v[i] = -INFINITY;
     if (e < n.experts) {
-      float x = row[e];
-      for (int s = 1; s < z.S; ++s) x += row[e + s * slab];
-      v[i] = x + bias[e];
+      v[i] = slab_total(z, row + e, slab) + bias[e];
     }
   }
   float top0 = 0.f, sum = 0.f, mine = 0.f;  // lane k: the k-th pick
@@ -52,19 +61,15 @@ __device__ __forceinline__ void pick_experts(const Partials &z, const float *__r
       if (at == i * 64 + lane) v[i] = -INFINITY;
   }
   if (lane < n.top) {
-    picked[lane] = min(mine_e, n.experts - 1);
-    wt[(size_t)t * n.picks() + lane] = __fdiv_rn(mine, sum);
+    l.picked[(size_t)t * n.top + lane] = min(mine_e, n.experts - 1);
+    l.wt[(size_t)t * n.top + lane] = __fdiv_rn(mine, sum);
   }
-  if (n.shared && lane == 0) {
-    float x = row[n.gate_col];
-    for (int s = 1; s < z.S; ++s) x += row[n.gate_col + s * slab];
-    wt[(size_t)t * n.picks() + n.top] = __fdiv_rn(1.0f, 1.0f + expf(-x));
-  }
+  if (n.shared && lane == 0) l.gate[t] = __fdiv_rn(1.0f, 1.0f + expf(-gate));
 }
 template <int NV>
 __global__ __launch_bounds__(256) void moe_pick_kernel(Partials z, const float *bias, MoeSizes n, MoeLists l) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (t < n.T) pick_experts<NV>(z, bias, n, t, l.picked + (size_t)t * n.top, l.wt);
+  if (t < n.T) pick_experts<NV>(z, bias, n, t, l);
 }
 
 // One workgroup: tokens by expert.  PICK: it picks the experts as well (few tokens).
@@ -72,11 +77,11 @@ template <int NV, bool PICK>
 __global__ __launch_bounds__(1024) void moe_lists_kernel(Partials z, const float *bias, MoeSizes n, MoeLists l,
                                                          int rows) {
   __shared__ int count[kMoeMaxExperts], next[kMoeMaxExperts], total;
-  const int tid = threadIdx.x, A = n.T * n.top, picks = n.picks();
+  const int tid = threadIdx.x, A = n.T * n.top, st = n.shared_tiles(rows);
   for (int e = tid; e < n.experts; e += 1024) count[e] = 0;
   if constexpr (PICK)
     for (int t = tid >> 6; t < n.T; t += 16)
-      pick_experts<NV>(z, bias, n, t, l.picked + (size_t)t * n.top, l.wt);
+      pick_experts<NV>(z, bias, n, t, l);
   __syncthreads();
   for (int a = tid; a < A; a += 1024) atomicAdd(&count[l.picked[a]], 1);
   __syncthreads();
@@ -91,7 +96,7 @@ __global__ __launch_bounds__(1024) void moe_lists_kernel(Partials z, const float
       if (tid >= o) slots += a, tiles += b;
     }
     if (tid == 63) total = tiles;
-    slots -= own_s, tiles -= own_t;
+    slots -= own_s, tiles += st - own_t;
     for (int e = e0; e < e1; ++e) {
       next[e] = slots;
       for (int r = 0; r < count[e]; r += rows)
@@ -100,16 +105,13 @@ __global__ __launch_bounds__(1024) void moe_lists_kernel(Partials z, const float
     }
   }
   __syncthreads();
-  const int st = n.shared ? (n.T + rows - 1) / rows : 0;
   for (int i = tid; i < st; i += 1024)
-    l.tiles[total + i] = MoeTile{n.experts, i * rows, min(rows, n.T - i * rows), 0};
-  if (tid == 0) *l.num_tiles = total + st;
-  if (n.shared)
-    for (int t = tid; t < n.T; t += 1024) l.at[(size_t)t * picks + n.top] = n.shared_slot() + t;
+    l.tiles[i] = MoeTile{n.experts, i * rows, min(rows, n.T - i * rows), 0};
+  if (tid == 0) *l.num_tiles = st + total;
   for (int a = tid; a < A; a += 1024) {
-    const int slot = atomicAdd(&next[l.picked[a]], 1), t = a / n.top;
-    l.slot_token[slot] = t;
-    l.at[(size_t)t * picks + a % n.top] = slot;
+    const int slot = atomicAdd(&next[l.picked[a]], 1);
+    l.slot_token[slot] = a / n.top;
+    l.at[a] = slot;
   }
 }
 
@@ -117,7 +119,7 @@ hipError_t launch_moe_route(const Partials &z, const float *bias, const MoeSizes
                             hipStream_t s) {
   if (n.T <= 0) return hipSuccess;
   if (n.experts < 1 || n.experts > kMoeMaxExperts || n.top < 1 || n.top > std::min(n.experts, kMoeMaxTop) ||
-      z.S < 1 || z.NP < n.experts || (n.shared && n.gate_col >= z.NP))
+      z.S < 1 || z.S > 8 || z.NP < n.experts || (n.shared && n.gate_col >= z.NP))
     return hipErrorInvalidValue;
   const int rows = n.tile_rows();
 #define FFMI_MR(NV)                                                                                        \
@@ -149,12 +151,13 @@ __device__ __forceinline__ void store_bf16x4(uint16_t *p, float a, float b, floa
       make_uint2(f2bf(a) | ((uint32_t)f2bf(b) << 16), f2bf(c) | ((uint32_t)f2bf(d) << 16));
 }
 // four consecutive output columns n.. of slot row m; gated: of the gate and up sums
+// (f: the row's factor)
 template <bool GATED>
-__device__ __forceinline__ void moe_store(const MoeGroup &g, int m, int n, const f4 &a, const f4 &b) {
+__device__ __forceinline__ void moe_store(const MoeGroup &g, int m, int n, float f, const f4 &a, const f4 &b) {
   uint16_t *Y = (uint16_t *)g.Y;
   if constexpr (GATED)
-    store_bf16x4(Y + act_packed_off(m, n, g.N), silu_glu(a[0], b[0]), silu_glu(a[1], b[1]),
-                 silu_glu(a[2], b[2]), silu_glu(a[3], b[3]));
+    store_bf16x4(Y + act_packed_off(m, n, g.ldy), f * silu_glu(a[0], b[0]), f * silu_glu(a[1], b[1]),
+                 f * silu_glu(a[2], b[2]), f * silu_glu(a[3], b[3]));
   else
     store_bf16x4(Y + (size_t)m * g.N + n, a[0], a[1], a[2], a[3]);
 }
@@ -162,11 +165,11 @@ __device__ __forceinline__ void moe_store(const MoeGroup &g, int m, int n, const
 // Up to 16 rows: a workgroup has two 16-column tiles (a gate / up pair) and splits
 // K over its four waves; weights straight to registers, U k-steps in flight.
 template <bool GATED, bool NTL>
-__global__ __launch_bounds__(256) void moe_few_kernel(MoeGemm a, size_t wts) {
+__global__ __launch_bounds__(256) void moe_few_kernel(MoeGemm a, int first, size_t wts) {
   constexpr int U = 8;
   __shared__ f4 red[3][2][64];
-  if ((int)blockIdx.y >= *a.num_tiles) return;
-  const MoeTile tl = a.tiles[blockIdx.y];
+  if (first + (int)blockIdx.y >= *a.num_tiles) return;
+  const MoeTile tl = a.tiles[first + blockIdx.y];
   const bool shared = tl.expert >= a.experts;
   const MoeGroup &g = a.g[shared];
   const int KT = g.K >> 5, ntiles = (GATED ? 2 : 1) * (g.N >> 4), tile0 = blockIdx.x * 2;
@@ -211,110 +214,138 @@ __global__ __launch_bounds__(256) void moe_few_kernel(MoeGemm a, size_t wts) {
   if (m >= tl.rows) return;
   const int row = tl.slot0 + m, n = (lane >> 4) * 4;
   if constexpr (GATED) {
-    moe_store<true>(g, row, blockIdx.x * 16 + n, acc[0], acc[1]);
+    moe_store<true>(g, row, blockIdx.x * 16 + n, shared ? a.gate[row] : 1.0f, acc[0], acc[1]);
   } else {
-    moe_store<false>(g, row, tile0 * 16 + n, acc[0], acc[0]);
-    if (tile0 + 1 < ntiles) moe_store<false>(g, row, tile0 * 16 + 16 + n, acc[1], acc[1]);
+    moe_store<false>(g, row, tile0 * 16 + n, 1.0f, acc[0], acc[0]);
+    if (tile0 + 1 < ntiles) moe_store<false>(g, row, tile0 * 16 + 16 + n, 1.0f, acc[1], acc[1]);
   }
 }
 
-// Up to 128 rows x 8 tiles a workgroup: four waves of 4 x 4 accumulators; both
-// operands' fragments go to LDS as they are stored (row-major rows: a lane fetches
-// its own row's 16 bytes), NB - 1 k-steps in flight across raw barriers with
-// counted waits, as the dense tile product does.  The column tiles of a row tile
-// share an XCD.
-template <bool GATED, int NB>
-__global__ __launch_bounds__(256, 2) void moe_tile_kernel(MoeGemm a, int ncol, size_t wts) {
-  __shared__ __attribute__((aligned(1024))) h8 lds[NB][16][64];
-  const int nwg = *a.num_tiles * ncol, b = blockIdx.x;
-  if (b >= nwg) return;
+// Up to 256 rows x 16 tiles a workgroup: eight waves as 2 (every other 16 rows) x 4
+// (weight tiles); both operands' fragments go to LDS as they are stored (row-major
+// rows: a lane fetches its own row's 16 bytes), NB - 1 k-steps in flight across raw
+// barriers with counted waits, as the dense tile product does.  NF: 16-row fragments
+// of a wave that hold rows; with up to 128 rows the other half is not fetched either.
+template <bool GATED, int NF, int NB>
+__device__ __forceinline__ void moe_tile(const MoeGemm &a, const MoeTile &tl, int tile0, size_t wts,
+                                         h8 (*lds)[32][64]) {
+  constexpr int OPS = NF > 4 ? 4 : 3;  // fragments that a wave fetches for a k-step
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int xcd = b & 7, q = nwg >> 3, r = nwg & 7;
-  const int L = (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + (b >> 3);
-  const MoeTile tl = a.tiles[L / ncol];
   const bool shared = tl.expert >= a.experts;
   const MoeGroup &g = a.g[shared];
-  const int KT = g.K >> 5, ntiles = (GATED ? 2 : 1) * (g.N >> 4), tile0 = L % ncol * 8;
-  if (tile0 >= ntiles) return;
+  const int KT = g.K >> 5, ntiles = (GATED ? 2 : 1) * (g.N >> 4);
   const size_t wks = wts == 512 ? (size_t)ntiles * 512 : 512, ts = wts == 512 ? 512 : (size_t)KT * 512;
   const uint16_t *W = (const uint16_t *)g.W + (shared ? 0 : tl.expert * g.w_stride) + lane * 8;
-  const uint16_t *src[4];
-  size_t step[4];
+  const uint16_t *src[OPS];
 #pragma unroll
-  for (int p = 0; p < 4; ++p) {
-    const int f = wave + 4 * p;  // fragments 0-7: rows, 8-15: weight tiles
-    if (f >= 8) {
-      src[p] = W + min(tile0 + f - 8, ntiles - 1) * ts, step[p] = wks;
+  for (int p = 0; p < OPS; ++p) {
+    const int f = wave + 8 * p;
+    if (p >= OPS - 2) {  // weight tiles
+      src[p] = W + min(tile0 + f - 8 * (OPS - 2), ntiles - 1) * ts;
     } else if (GATED) {
       const int slot = tl.slot0 + min(f * 16 + (lane & 15), tl.rows - 1);
       src[p] = (const uint16_t *)g.X + (size_t)(shared ? slot : a.slot_token[slot]) * g.K + 8 * (lane >> 4);
-      step[p] = 32;
     } else {
       const int mt = (tl.slot0 >> 4) + min(f, (tl.rows - 1) >> 4);
-      src[p] = (const uint16_t *)g.X + ((size_t)mt * KT * 64 + lane) * 8, step[p] = 512;
+      src[p] = (const uint16_t *)g.X + ((size_t)mt * KT * 64 + lane) * 8;
     }
   }
   auto issue_one = [&](int kt, int p) {
+    const bool w = p >= OPS - 2;
     __builtin_amdgcn_global_load_lds(
-        (const __attribute__((address_space(1))) void *)(src[p] + (size_t)kt * step[p]),
-        (__attribute__((address_space(3))) void *)(&lds[kt % NB][wave + 4 * p][0]), 16, 0, 0);
+        (const __attribute__((address_space(1))) void *)(src[p] + (size_t)kt * (w ? wks : GATED ? 32 : 512)),
+        (__attribute__((address_space(3))) void *)(&lds[kt % NB][wave + 8 * (w ? p - (OPS - 2) + 2 : p)][0]), 16,
+        0, 0);
   };
-  const int wm = wave >> 1, wn = wave & 1;
-  f4 acc[4][4];
+  const int wm = wave >> 2, wn = wave & 3;
+  f4 acc[NF][4];
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+  for (int i = 0; i < NF; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int kt = 0; kt < NB - 1; ++kt)
     if (kt < KT)
 #pragma unroll
-      for (int p = 0; p < 4; ++p) issue_one(kt, p);
-  static_assert(NB == 4, "the waits below count NB - 2 younger stages of 4 loads");
+      for (int p = 0; p < OPS; ++p) issue_one(kt, p);
+  static_assert(NB == 4, "the waits below count NB - 2 younger stages");
   for (int kt = 0; kt < KT; ++kt) {
     // step kt has arrived once at most the younger steps' loads remain; the barrier
     // makes every wave's visible and retires the reads of the buffer filled next
     const int ahead = min(KT - 1 - kt, NB - 2);
-    if (ahead >= 2) asm volatile("s_waitcnt vmcnt(8)" ::: "memory");
-    else if (ahead == 1) asm volatile("s_waitcnt vmcnt(4)" ::: "memory");
-    else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    if (ahead >= 2) {
+      if constexpr (OPS == 4) asm volatile("s_waitcnt vmcnt(8)" ::: "memory");
+      else asm volatile("s_waitcnt vmcnt(6)" ::: "memory");
+    } else if (ahead == 1) {
+      if constexpr (OPS == 4) asm volatile("s_waitcnt vmcnt(4)" ::: "memory");
+      else asm volatile("s_waitcnt vmcnt(3)" ::: "memory");
+    } else {
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();
     asm volatile("" ::: "memory");
     const bool more = kt + NB - 1 < KT;
     const int buf = kt % NB;
-    h8 xf[4], wf[4];
+    h8 xf[NF], wf[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) wf[j] = lds[buf][8 + wn * 4 + j][lane];
+    for (int j = 0; j < 4; ++j) wf[j] = lds[buf][16 + wn * 4 + j][lane];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) xf[i] = lds[buf][wm * 4 + i][lane];
+    for (int i = 0; i < NF; ++i) xf[i] = lds[buf][2 * i + wm][lane];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
+    for (int i = 0; i < NF; ++i) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) acc[i][j] = moe_mma(wf[j], xf[i], acc[i][j]);
-      if (more) issue_one(kt + NB - 1, i);
+      if (more)
+#pragma unroll
+        for (int p = 0; p < OPS; ++p)  // (spread: a fetch's issue hides under the products)
+          if (p * NF / OPS == i) issue_one(kt + NB - 1, p);
     }
   }
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int m = (wm * 4 + i) * 16 + (lane & 15);
+  for (int i = 0; i < NF; ++i) {
+    const int m = (2 * i + wm) * 16 + (lane & 15);
     if (m >= tl.rows) continue;
+    const float f = GATED && shared ? a.gate[tl.slot0 + m] : 1.0f;
 #pragma unroll
     for (int j = 0; j < 4; j += GATED ? 2 : 1) {
       const int tile = tile0 + wn * 4 + j;
       if (tile >= ntiles) continue;
-      moe_store<GATED>(g, tl.slot0 + m, (GATED ? tile >> 1 : tile) * 16 + (lane >> 4) * 4, acc[i][j],
+      moe_store<GATED>(g, tl.slot0 + m, (GATED ? tile >> 1 : tile) * 16 + (lane >> 4) * 4, f, acc[i][j],
                        acc[i][GATED ? j + 1 : j]);
     }
   }
 }
+// The shared expert's workgroups first (the longest), their row tiles of a column
+// tile on one XCD; then the experts', a row tile's columns in turn.
+template <bool GATED>
+__global__ __launch_bounds__(512, 1) void moe_tile_kernel(MoeGemm a, int first, int st, int cols_shared,
+                                                          int cols, size_t wts) {
+  __shared__ __attribute__((aligned(1024))) h8 lds[4][32][64];
+  const int nsh = st * cols_shared, b = blockIdx.x;
+  int tile, col;
+  if (b < nsh) {
+    const int xcd = b & 7, q = nsh >> 3, r = nsh & 7;
+    const int L = (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + (b >> 3);
+    tile = L % st, col = L / st;
+  } else {
+    tile = first + st + (b - nsh) / cols, col = (b - nsh) % cols;
+    if (tile >= *a.num_tiles) return;
+  }
+  const MoeTile tl = a.tiles[tile];
+  const int frags = (tl.rows + 15) >> 4;
+  if (frags <= 4) moe_tile<GATED, 2, 4>(a, tl, col * 16, wts, lds);
+  else if (frags <= 8) moe_tile<GATED, 4, 4>(a, tl, col * 16, wts, lds);
+  else if (frags <= 12) moe_tile<GATED, 6, 4>(a, tl, col * 16, wts, lds);
+  else moe_tile<GATED, 8, 4>(a, tl, col * 16, wts, lds);
+}
 
 // fp32: 16 rows x 64 columns a workgroup
 template <bool GATED>
-__global__ __launch_bounds__(256) void moe_f32_kernel(MoeGemm a) {
+__global__ __launch_bounds__(256) void moe_f32_kernel(MoeGemm a, int first) {
   __shared__ float sx[16][33], sw[GATED ? 2 : 1][64][33];
-  if ((int)blockIdx.y >= *a.num_tiles) return;
-  const MoeTile tl = a.tiles[blockIdx.y];
+  if (first + (int)blockIdx.y >= *a.num_tiles) return;
+  const MoeTile tl = a.tiles[first + blockIdx.y];
   const bool shared = tl.expert >= a.experts;
   const MoeGroup &g = a.g[shared];
   const int n0 = blockIdx.x * 64, tid = threadIdx.x, r = tid & 15, c = tid >> 4;
@@ -349,9 +380,13 @@ __global__ __launch_bounds__(256) void moe_f32_kernel(MoeGemm a) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int n = n0 + c + 16 * j;
-        if (n < g.N)
-          ((float *)g.Y)[(size_t)(tl.slot0 + m0 + r) * g.N + n] =
-              GATED ? silu_glu(acc[0][j], acc[GATED ? 1 : 0][j]) : acc[0][j];
+        const int row = tl.slot0 + m0 + r;
+        if (n >= g.N) continue;
+        if constexpr (GATED)
+          ((float *)g.Y)[(size_t)row * g.ldy + n] =
+              (shared ? a.gate[row] : 1.0f) * silu_glu(acc[0][j], acc[GATED ? 1 : 0][j]);
+        else
+          ((float *)g.Y)[(size_t)row * g.N + n] = acc[0][j];
       }
   }
 }
@@ -359,29 +394,37 @@ __global__ __launch_bounds__(256) void moe_f32_kernel(MoeGemm a) {
 hipError_t launch_moe_gemm(const MoeGemm &a, const MoeSizes &n, bool gated, bool f32, bool stream_weights,
                            hipStream_t s) {
   if (n.T <= 0) return hipSuccess;
+  const bool shared = gated && n.shared;
   int N = 0;
-  for (int i = 0; i < (n.shared ? 2 : 1); ++i) {
-    if (a.g[i].N % 32 || a.g[i].K % 32 || a.g[i].N <= 0 || a.g[i].K <= 0) return hipErrorInvalidValue;
-    N = std::max(N, a.g[i].N);
+  for (int i = 0; i < (shared ? 2 : 1); ++i) {
+    const MoeGroup &g = a.g[i];
+    if (g.N % 32 || g.K % 32 || g.N <= 0 || g.K <= 0 || (gated && (g.ldy < g.N || g.ldy % 32)))
+      return hipErrorInvalidValue;
+    N = std::max(N, g.N);
   }
-  const int rows = n.tile_rows(), tiles = n.max_tiles(rows);
-  if (tiles > 65535) return hipErrorInvalidValue;
+  // (the second product leaves the shared expert's tiles out)
+  const int rows = n.tile_rows(), st = shared ? n.shared_tiles(rows) : 0, first = n.shared_tiles(rows) - st;
+  const int tiles = n.expert_tiles(rows);
+  if (st + tiles > 65535 || (shared && !a.gate)) return hipErrorInvalidValue;
   if (f32) {
-    const dim3 grid((N + 63) / 64, tiles);
-    if (gated) hipLaunchKernelGGL(moe_f32_kernel<true>, grid, dim3(256), 0, s, a);
-    else hipLaunchKernelGGL(moe_f32_kernel<false>, grid, dim3(256), 0, s, a);
+    const dim3 grid((N + 63) / 64, st + tiles);
+    if (gated) hipLaunchKernelGGL(moe_f32_kernel<true>, grid, dim3(256), 0, s, a, first);
+    else hipLaunchKernelGGL(moe_f32_kernel<false>, grid, dim3(256), 0, s, a, first);
     return hipGetLastError();
   }
-  const int ntiles = (gated ? 2 : 1) * N / 16;
+  const int per = gated ? 2 : 1;
   const size_t wts = weights_kmajor() ? 512 : 0;
   if (rows == kMoeMany) {
-    const int ncol = (ntiles + 7) / 8;
-    if (gated) hipLaunchKernelGGL((moe_tile_kernel<true, 4>), dim3(tiles * ncol), dim3(256), 0, s, a, ncol, wts);
-    else hipLaunchKernelGGL((moe_tile_kernel<false, 4>), dim3(tiles * ncol), dim3(256), 0, s, a, ncol, wts);
+    const int cols = (per * a.g[0].N / 16 + 15) / 16, cols_shared = st ? (per * a.g[1].N / 16 + 15) / 16 : 0;
+    const dim3 grid(st * cols_shared + tiles * cols);
+    if (gated)
+      hipLaunchKernelGGL(moe_tile_kernel<true>, grid, dim3(512), 0, s, a, first, st, cols_shared, cols, wts);
+    else
+      hipLaunchKernelGGL(moe_tile_kernel<false>, grid, dim3(512), 0, s, a, first, st, cols_shared, cols, wts);
     return hipGetLastError();
   }
-  const dim3 grid((ntiles + 1) / 2, tiles);
-#define FFMI_MF(G, NL) hipLaunchKernelGGL((moe_few_kernel<G, NL>), grid, dim3(256), 0, s, a, wts)
+  const dim3 grid((per * N / 16 + 1) / 2, st + tiles);
+#define FFMI_MF(G, NL) hipLaunchKernelGGL((moe_few_kernel<G, NL>), grid, dim3(256), 0, s, a, first, wts)
   if (gated && stream_weights) FFMI_MF(true, true);
   else if (gated) FFMI_MF(true, false);
   else if (stream_weights) FFMI_MF(false, true);

@@ -10,7 +10,8 @@
 //           scores cap tanh(q . k * scale / cap) over a window; softmax, optionally
 //           with a sink; optionally values that turn with their positions; W_o
 //   ff:     W_down (silu(W_gate h) * (W_up h)); or the `top` of many such, weighted,
-//           beside a shared one with a sigmoid gate
+//           beside a shared one with a sigmoid gate (on its units, so that its W_down
+//           joins W_o)
 //   logits = cap tanh(head group norm(x) / cap)
 //
 // 32-bit in either precision: residual stream, norms, convolution and its carried
@@ -58,10 +59,11 @@ struct NomutarLayer {
   // feed-forward: dense (ff) or experts
   int ff = 0, experts = 0, top = 0, eff = 0, sff = 0;
   // padded sizes: per-head columns of the products (dg, vg) and of the caches (dp,
-  // vp), first product, attention output, feed-forwards, router
-  int dg = 0, vg = 0, dp = 0, vp = 0, nq = 0, na = 0, fp = 0, efp = 0, sfp = 0, gate_col = 0, nr = 0;
+  // vp), first product, attention output, feed-forwards, router; units (dense or the
+  // shared expert's) beside the attention output in the layer's last product
+  int dg = 0, vg = 0, dp = 0, vp = 0, nq = 0, na = 0, fp = 0, efp = 0, gate_col = 0, nr = 0;
   void *win = nullptr, *wout = nullptr, *wgu = nullptr, *wrouter = nullptr;
-  void *egu = nullptr, *edown = nullptr, *sgu = nullptr, *sdown = nullptr;
+  void *egu = nullptr, *edown = nullptr;
   float *norm = nullptr, *bias = nullptr, *norms = nullptr, *sink = nullptr, *conv = nullptr, *rbias = nullptr;
   double *dfreq = nullptr, *dvfreq = nullptr;
 };
@@ -84,10 +86,10 @@ struct Nomutar : public PagedDecoder {
   bool rows_form = false;  // some layer's attention has no MFMA form
   int max_slots = 0;
   // activations: second residual buffer, mixer input, rows for the experts
-  float *x2 = nullptr, *xs[2] = {};
+  float *x2 = nullptr, *xs[2] = {}, *rms = nullptr;
   void *c = nullptr, *q = nullptr, *cat = nullptr;
   uint16_t *hrow = nullptr;
-  void *eu = nullptr, *su = nullptr, *ey = nullptr;
+  void *eu = nullptr, *ey = nullptr;
   float *slabs = nullptr, *ml = nullptr;
   MoeLists moe;
 
@@ -206,7 +208,7 @@ struct Nomutar : public PagedDecoder {
 
   // ---- buffers and weights ----
   ffmi_status init_layers() override {
-    size_t qw = 32, cw = 32, eu_rows = 0, su_rows = 0, slots = 0, picks = 0, picked = 0, tiles = 0, eslots = 0;
+    size_t qw = 32, cw = 32, units = 0, slots = 0, picks = 0, tiles = 0;
     double wbytes = 0;
     int min_groups = 1 << 30;
     std::vector<RowShape> shapes;
@@ -214,7 +216,7 @@ struct Nomutar : public PagedDecoder {
     FFMI_CHECK((taps <= 4 && Wp <= 8192) || (size_t)taps * Wp * 4 <= 150 * 1024, FFMI_ERR_UNSUPPORTED);
     for (NomutarLayer &L : layers) {
       const int H = L.heads, G = L.groups;
-      L.dg = up(L.dim, 32), L.vg = up(L.vdim, 32), L.fp = up(L.ff, 32);
+      L.dg = up(L.dim, 32), L.vg = up(L.vdim, 32), L.fp = up(L.ff + L.sff, 32);
       FFMI_CHECK(L.dg <= kAttnRowsMax && L.vg <= kAttnRowsMax, FFMI_ERR_UNSUPPORTED);
       L.dp = L.dg, L.vp = L.vg;
       if (!f32 && attn_width(L.dim) && attn_width(L.vdim)) L.dp = attn_width(L.dim), L.vp = attn_width(L.vdim);
@@ -230,38 +232,35 @@ struct Nomutar : public PagedDecoder {
         for (int t = 16; t <= Tm; t += 16)
           ws_bytes = std::max(ws_bytes, gemm_bf16_swiglu_workspace_bytes(t, L.fp, Wp));
       if (!L.experts) continue;
-      L.efp = up(L.eff, 32), L.sfp = up(L.sff, 32), L.gate_col = up(L.experts, 16);
+      L.efp = up(L.eff, 32), L.gate_col = up(L.experts, 16);
       L.nr = up(L.gate_col + 1, 32);
       gemms.push_back({L.nr, Wp});
-      wbytes += 6.0 * Wp * ((double)L.experts * L.efp + L.sfp);
+      wbytes += 6.0 * Wp * L.experts * L.efp;
       for (int t = 1; t <= Tm; ++t) {
         const MoeSizes n = sizes(L, t);
-        // (a tile of the first product may be read past its last slot)
-        eu_rows = std::max(eu_rows, (size_t)(n.expert_slots() + kMoeMany) * L.efp);
-        eslots = std::max(eslots, (size_t)n.expert_slots());
-        slots = std::max(slots, (size_t)n.slots());
-        picks = std::max(picks, (size_t)t * n.picks()), picked = std::max(picked, (size_t)t * L.top);
-        tiles = std::max(tiles, (size_t)n.max_tiles(n.tile_rows()));
+        units = std::max(units, (size_t)n.slots() * L.efp);
+        slots = std::max(slots, (size_t)n.slots()), picks = std::max(picks, (size_t)t * L.top);
+        tiles = std::max(tiles, (size_t)(n.expert_tiles(n.tile_rows()) + n.shared_tiles(n.tile_rows())));
       }
-      su_rows = std::max(su_rows, (size_t)(Tm + kMoeMany) * L.sfp);
     }
     // 16-row slots for the splits of a step whose blocks do not fill the chip
     max_slots = rows_form ? 0 : 512 * kAttnTiles / min_groups;
     FFMI_TRY(init_step(shapes, max_slots, gemms, wbytes));
     FFMI_TRY(alloc_zero(&x2, (size_t)Tm * Wp * 4));
     xs[0] = x, xs[1] = x2;
+    FFMI_TRY(alloc_zero(&rms, (size_t)Tm * groups * 4));
     FFMI_TRY(alloc_zero(&c, (size_t)Tm * Wp * es()));
     FFMI_TRY(alloc_zero(&q, (size_t)Tm * qw * es()));
     FFMI_TRY(alloc_zero(&cat, (size_t)Tm * cw * es()));
     if (slots) {
       if (!f32) FFMI_TRY(alloc_zero(&hrow, (size_t)Tm * Wp * 2));
-      FFMI_TRY(alloc_zero(&eu, eu_rows * es()));
-      FFMI_TRY(alloc_zero(&su, su_rows * es()));
+      FFMI_TRY(alloc_zero(&eu, units * es()));
       FFMI_TRY(alloc_zero(&ey, slots * Wp * es()));
-      FFMI_TRY(alloc_zero(&moe.picked, picked * 4));
+      FFMI_TRY(alloc_zero(&moe.picked, picks * 4));
       FFMI_TRY(alloc_zero(&moe.at, picks * 4));
       FFMI_TRY(alloc_zero(&moe.wt, picks * 4));
-      FFMI_TRY(alloc_zero(&moe.slot_token, eslots * 4));
+      FFMI_TRY(alloc_zero(&moe.gate, (size_t)Tm * 4));
+      FFMI_TRY(alloc_zero(&moe.slot_token, slots * 4));
       FFMI_TRY(alloc_zero(&moe.tiles, tiles * sizeof(MoeTile)));
       FFMI_TRY(alloc_zero(&moe.num_tiles, 16));
     }
@@ -366,19 +365,22 @@ struct Nomutar : public PagedDecoder {
       }
       FFMI_TRY(upload(&L.sink, s));
     }
-    // one product for the sublayers' outputs: W_o and a dense W_down side by side
+    // one product for the sublayers' outputs: W_o and a W_down that every token takes
+    // (dense or the shared expert's) side by side
     FFMI_TRY(alloc(&L.wout, (size_t)Wp * (L.na + L.fp) * es()));
     PackSpec so = spec(1, W, Wp, H, L.vdim, L.vg);
     so.col_pairs = vpairs, so.kt = (L.na + L.fp) / 32;
     FFMI_TRY(raw(m + "o", {W, (long)H * L.vdim}));
     FFMI_TRY(pack_rows(so, H * L.vdim, L.wout, 0, Wp));
-    if (L.ff) {
-      PackSpec sd = spec(1, W, Wp, 1, L.ff, L.fp);
+    if (L.fp) {
+      const std::string d = L.ff ? f : f + "shared.";
+      const int ff = L.ff + L.sff;  // (one of the two)
+      PackSpec sd = spec(1, W, Wp, 1, ff, L.fp);
       sd.k0 = L.na / 32, sd.kt = so.kt;
-      FFMI_TRY(raw(f + "down", {W, L.ff}));
-      FFMI_TRY(pack_rows(sd, L.ff, L.wout, 0, Wp));
+      FFMI_TRY(raw(d + "down", {W, ff}));
+      FFMI_TRY(pack_rows(sd, ff, L.wout, 0, Wp));
       FFMI_TRY(alloc(&L.wgu, (size_t)2 * L.fp * Wp * es()));
-      FFMI_TRY(gate_up(L.wgu, f, L.ff, L.fp));
+      FFMI_TRY(gate_up(L.wgu, d, ff, L.fp));
     }
     return L.experts ? load_experts(f, L) : FFMI_OK;
   }
@@ -398,10 +400,7 @@ struct Nomutar : public PagedDecoder {
     }
     if (!L.sff) return FFMI_OK;
     FFMI_TRY(raw(f + "shared.sg", {1, W}));
-    FFMI_TRY(pack_rows(spec(1, 1, 16, 1, W, Wp), W, L.wrouter, L.gate_col, L.nr));
-    FFMI_TRY(alloc(&L.sgu, (size_t)2 * L.sfp * Wp * es()));
-    FFMI_TRY(gate_up(L.sgu, f + "shared.", L.sff, L.sfp));
-    return linear(&L.sdown, f + "shared.down", W, Wp, 1, L.sff, L.sfp);
+    return pack_rows(spec(1, 1, 16, 1, W, Wp), W, L.wrouter, L.gate_col, L.nr);
   }
 
   // ---- one step ----
@@ -432,14 +431,18 @@ struct Nomutar : public PagedDecoder {
     else FFMI_HIP(launch_rotary_attn(step.dev, pl, a, slabs, ml, stream, fused ? &p : nullptr, step.T));
     return FFMI_OK;
   }
+  // the columns after the attention output
+  void *units_of(const NomutarLayer &L) {
+    return (char *)cat + (f32 ? (size_t)L.na * 4 : (size_t)L.na / 32 * 512 * 2);
+  }
   ffmi_status dense(const NomutarLayer &L) {
     const int T = step.T, ld = L.na + L.fp;
     if (f32) {
       FFMI_HIP(launch_gemm_f32((const float *)h, (const float *)L.wgu, ws, T, 2 * L.fp, Wp, stream));
-      FFMI_HIP(launch_swiglu_f32(ws, (float *)cat + L.na, T, L.fp, ld, stream));
+      FFMI_HIP(launch_swiglu_f32(ws, (float *)units_of(L), T, L.fp, ld, stream));
     } else {
       FFMI_HIP(launch_gemm_bf16_swiglu((const uint16_t *)h, (const uint16_t *)L.wgu,
-                                       (uint16_t *)cat + (size_t)L.na / 32 * 512, ws, ws_bytes, T, L.fp, Wp,
+                                       (uint16_t *)units_of(L), ws, ws_bytes, T, L.fp, Wp,
                                        FFMI_X_PACKED | FFMI_Y_PACKED | wstream, ld, stream));
     }
     return FFMI_OK;
@@ -451,22 +454,22 @@ struct Nomutar : public PagedDecoder {
     FFMI_HIP(launch_moe_route(z, L.rbias, n, moe, stream));
     MoeGemm a;
     a.experts = L.experts, a.slot_token = moe.slot_token, a.tiles = moe.tiles, a.num_tiles = moe.num_tiles;
+    a.gate = moe.gate;
     const void *rows = f32 ? h : hrow;
-    a.g[0] = {rows, L.egu, eu, L.efp, Wp, (size_t)2 * L.efp * Wp};
-    a.g[1] = {rows, L.sgu, su, L.sfp, Wp, 0};
+    a.g[0] = {rows, L.egu, eu, L.efp, Wp, L.efp, (size_t)2 * L.efp * Wp};
+    a.g[1] = {rows, L.wgu, units_of(L), L.fp, Wp, L.na + L.fp, 0};
     FFMI_HIP(launch_moe_gemm(a, n, true, f32, wstream != 0, stream));
-    a.g[0] = {eu, L.edown, ey, Wp, L.efp, (size_t)L.efp * Wp};
-    a.g[1] = {su, L.sdown, (char *)ey + (size_t)n.shared_slot() * Wp * es(), Wp, L.sfp, 0};
+    a.g[0] = {eu, L.edown, ey, Wp, L.efp, 0, (size_t)L.efp * Wp};
     FFMI_HIP(launch_moe_gemm(a, n, false, f32, wstream != 0, stream));
     return FFMI_OK;
   }
   // x of the sums that layer `prev` (null: none) left, for the norm `w`
   ConvNorm sum_norm(const NomutarLayer *prev, const Partials &y, const float *w) {
     ConvNorm n;
-    n.H = Wp, n.n = W, n.groups = groups, n.eps = eps, n.mult = mult, n.w = w, n.x_in = xs[0];
+    n.H = Wp, n.n = W, n.groups = groups, n.eps = eps, n.mult = mult, n.w = w, n.x_in = xs[0], n.inv = rms;
     if (prev) n.y = y;
     if (prev && prev->experts) {
-      n.rows = ey, n.rows_f32 = f32, n.at = moe.at, n.wt = moe.wt, n.top = sizes(*prev, step.T).picks();
+      n.rows = ey, n.rows_f32 = f32, n.at = moe.at, n.wt = moe.wt, n.top = prev->top;
     }
     return n;
   }

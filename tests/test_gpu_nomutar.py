@@ -403,10 +403,11 @@ def test_wide_rows(tmp_path, width, groups, taps, full):
     close(out, np.concatenate([want2, want[:250]]), full)
 
 
-@pytest.mark.parametrize("n,top,T", [(64, 64, 3), (65, 2, 200), (130, 8, 64), (300, 3, 40), (4, 1, 1000), (24, 6, 129)])
+@pytest.mark.parametrize("n,top,T", [(64, 64, 3), (65, 2, 200), (130, 8, 64), (300, 3, 40), (4, 1, 1000), (24, 6, 129),
+                                     (6, 2, 300), (4, 1, 700), (3, 2, 1010)])
 def test_many_experts(tmp_path, n, top, T):
     """Routers of one to sixteen logits a lane, steps of few and of many rows an
-    expert, experts that no token takes."""
+    expert (up to 64, 128, 192, 256 and more), experts that no token takes."""
     cfg = NM.model_config(90, 320, [NM.experts(NM.plain(2, 1, 16, 16, 0.2), n, top, 40, shared=70)], bigram=None)
     w = NM.random_weights(cfg, 7)
     toks = tokens(cfg, T, 5)
