@@ -19,8 +19,8 @@ struct ConvNormStep {
 
 // A workgroup takes a token; a thread has chunks of 8 columns.  Few tokens (CONV):
 // the convolution as well; the rows h that it reads are made again from x_in (so x
-// and x_in are different buffers) or come from `carry`.  Many tokens: conv_kernel
-// follows, on the x and inv of this one.
+// and x_in are different buffers), after the token's own, or come from `carry`.  Many
+// tokens: conv_kernel follows, on the x and inv of this one.
 // MAXS == 0: x is an embedding row.
 // REGS: the earlier rows are kept in registers (taps <= 4), else in LDS, each thread
 // its own.
@@ -29,6 +29,9 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, H = a.H, nchunk = H >> 3, T = st.T;
   const PagedToken *tok = reinterpret_cast<const PagedToken *>(st.blob + st.off_tokens);
+  const int first = st.out_rows ? st.out_rows[blockIdx.x] : (int)blockIdx.x;
+  const int out = blockIdx.x;
+  const PagedToken raw = tok[first];  // (one token for the whole workgroup)
   if (st.blob_dst) {
     const uint4 *src = reinterpret_cast<const uint4 *>(st.blob);
     for (int i = blockIdx.x * NT + tid; i < st.blob_n16; i += gridDim.x * NT) st.blob_dst[i] = src[i];
@@ -36,106 +39,79 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
   const int gs = a.n / a.groups, per = st.waves ? (gs + 511) / 512 : gs / st.unit;
   float *part = lds, *inv = lds + 2 * st.parts;
   f4 *ring = reinterpret_cast<f4 *>(lds + ((2 * st.parts + a.groups + 3) & ~3));
+  const int past = CONV ? a.taps - 1 : 0;
+  auto chunk = [&](int c) { return min(tid + c * NT, nchunk - 1); };
+  auto load8 = [](const float *p, f4 (&v)[2]) {
+    v[0] = *reinterpret_cast<const f4 *>(p), v[1] = *reinterpret_cast<const f4 *>(p + 4);
+  };
+  // the row k + 1 tokens back
   constexpr int KH = REGS ? 3 : 1;
   f4 hist[KH][MAXC][2];
-  const int past = CONV ? a.taps - 1 : 0;
-  // the row k + 1 tokens back
   int head = 0;  // (LDS) slot of the latest row
+  auto ring_at = [&](int slot, int c, int h) -> f4 & { return ring[(slot * 2 + h) * nchunk + chunk(c)]; };
   auto old_row = [&](int k, int c, int h) {
     if constexpr (REGS) return hist[k][c][h];
-    int s = head - k;
-    if (s < 0) s += past;
-    return ring[(s * 2 + h) * nchunk + min(tid + c * NT, nchunk - 1)];
+    return ring_at(head - k < 0 ? head - k + past : head - k, c, h);
   };
-  const int first = st.out_rows ? st.out_rows[blockIdx.x] : (int)blockIdx.x;
-  for (int t = CONV ? first - min(tok[first].back, past) : first, odd = 0; t <= first; ++t, odd ^= 1) {
-    PagedToken tk = tok[t];  // (one token for the whole workgroup)
-    tk.token = __builtin_amdgcn_readfirstlane(tk.token), tk.prev = __builtin_amdgcn_readfirstlane(tk.prev);
-    tk.pos = __builtin_amdgcn_readfirstlane(tk.pos), tk.back = __builtin_amdgcn_readfirstlane(tk.back);
-    tk.ahead = __builtin_amdgcn_readfirstlane(tk.ahead), tk.slot = __builtin_amdgcn_readfirstlane(tk.slot);
-    tk.bank = __builtin_amdgcn_readfirstlane(tk.bank);
-    const int out = st.out_rows ? (int)blockIdx.x : t;
-    const bool mine = t == first;
-    // (rows of earlier steps, zeros before the sequence; first: nothing waits for them)
-    if (CONV && past > 0 && tk.back == 0) {
-#pragma unroll
-      for (int k = 0; k < (REGS ? 3 : 1); ++k)
-        for (int q = k; q < (REGS ? k + 1 : past); ++q) {
-          const float *cr = a.carry + ((size_t)(tk.slot * 2 + tk.bank) * past + min(q, past - 1)) * H;
-#pragma unroll
-          for (int c = 0; c < MAXC; ++c) {
-            const int ch = min(tid + c * NT, nchunk - 1);
-#pragma unroll
-            for (int h = 0; h < 2; ++h) {
-              f4 v = f4{0.f, 0.f, 0.f, 0.f};
-              if (q < past && tk.pos > q) v = *reinterpret_cast<const f4 *>(cr + ch * 8 + 4 * h);
-              if constexpr (REGS) {
-                hist[k][c][h] = v;
-              } else {  // (chunk by chunk: the threads past the row write what its last owner does not read)
-                head = 0;
-                if (tid + c * NT < nchunk) ring[((q ? past - q : 0) * 2 + h) * nchunk + ch] = v;
-              }
-            }
-          }
-        }
-    }
-    f4 x[MAXC][2];
-    float ss[MAXC];
+  // x of row t; meanwhile() runs while its first loads are under way
+  auto sum_row = [&](int t, auto meanwhile, f4 (&x)[MAXC][2]) {
 #pragma unroll
     for (int c = 0; c < MAXC; ++c) {
-      const int ch = min(tid + c * NT, nchunk - 1);
+      const int ch = chunk(c);
       if constexpr (MAXS == 0) {
-        unpack8_bf16(*reinterpret_cast<const uint4 *>(em.embed + (size_t)tk.token * H + ch * 8), x[c][0],
-                     x[c][1]);
-        x[c][0] *= em.scale, x[c][1] *= em.scale;
+        PagedToken tk = t == first ? raw : tok[t];
+        const int token = __builtin_amdgcn_readfirstlane(tk.token), prev = __builtin_amdgcn_readfirstlane(tk.prev);
+        unpack8_bf16(*reinterpret_cast<const uint4 *>(em.embed + (size_t)token * H + ch * 8), x[c][0], x[c][1]);
+        f4 p[2];
+        p[0] = p[1] = f4{0.f, 0.f, 0.f, 0.f};
         if (em.pairs) {
-          const int64_t b = tk.prev < 0 ? em.buckets
-                                        : (tk.prev * em.mul_prev + tk.token * em.mul_cur) % em.buckets;
-          f4 p, q;
-          unpack8_bf16(*reinterpret_cast<const uint4 *>(em.pairs + (size_t)b * H + ch * 8), p, q);
-          x[c][0] += p, x[c][1] += q;
+          const int64_t b = prev < 0 ? em.buckets : (prev * em.mul_prev + token * em.mul_cur) % em.buckets;
+          unpack8_bf16(*reinterpret_cast<const uint4 *>(em.pairs + (size_t)b * H + ch * 8), p[0], p[1]);
         }
+        if (c == 0) meanwhile();
+#pragma unroll
+        for (int h = 0; h < 2; ++h) x[c][h] = x[c][h] * em.scale + p[h];
       } else {
         constexpr int SB = MAXC > 1 ? 1 : NT > 512 ? (MAXS < 2 ? 1 : 2) : (MAXS < 1 ? 1 : MAXS);  // slabs in flight
+        constexpr int U = MAXC > 1 ? 1 : NT > 512 ? 2 : 4;                                      // expert rows
         f4 y[2], s[SB][2];
+        const int32_t *at = a.at + (size_t)t * a.top;
+        const float *wt = a.wt + (size_t)t * a.top;
+        int at0[U];
+        float wt0[U];
+        if (a.rows)
 #pragma unroll
-        for (int h = 0; h < 2; ++h) {
-          x[c][h] = *reinterpret_cast<const f4 *>(a.x_in + (size_t)t * H + ch * 8 + 4 * h);
-          y[h] = f4{0.f, 0.f, 0.f, 0.f};
-        }
+          for (int k = 0; k < U; ++k) at0[k] = at[min(k, a.top - 1)], wt0[k] = wt[min(k, a.top - 1)];
+        load8(a.x_in + (size_t)t * H + ch * 8, x[c]);
+        y[0] = y[1] = f4{0.f, 0.f, 0.f, 0.f};
+        const float *p = a.y.p + (size_t)t * a.y.NP + ch * 8;
+        if (a.y.S > 0)
+#pragma unroll
+          for (int sl = 0; sl < SB; ++sl) load8(p + (size_t)min(sl, a.y.S - 1) * T * a.y.NP, s[sl]);
+        if (c == 0) meanwhile();
         if (a.y.S > 0) {
-          const float *p = a.y.p + (size_t)t * a.y.NP + ch * 8;
 #pragma unroll
           for (int s0 = 0; s0 < MAXS; s0 += SB) {
             if (s0 >= a.y.S) break;
+            if (s0 > 0)
 #pragma unroll
-            for (int sl = 0; sl < SB; ++sl)
-#pragma unroll
-              for (int h = 0; h < 2; ++h)
-                s[sl][h] = *reinterpret_cast<const f4 *>(p + (size_t)min(s0 + sl, a.y.S - 1) * T * a.y.NP + 4 * h);
+              for (int sl = 0; sl < SB; ++sl) load8(p + (size_t)min(s0 + sl, a.y.S - 1) * T * a.y.NP, s[sl]);
 #pragma unroll
             for (int sl = 0; sl < SB; ++sl)
               if (s0 + sl < a.y.S) y[0] += s[sl][0], y[1] += s[sl][1];
           }
         }
         if (a.rows) {
-          const int32_t *at = a.at + (size_t)t * a.top;
-          const float *wt = a.wt + (size_t)t * a.top;
-          constexpr int U = MAXC > 1 ? 1 : NT > 512 ? 2 : 8;
           for (int k0 = 0; k0 < a.top; k0 += U) {
             f4 r[U][2];
             float w4[U];
 #pragma unroll
             for (int k = 0; k < U; ++k) {
               const int kk = min(k0 + k, a.top - 1);
-              const size_t o = (size_t)at[kk] * H + ch * 8;
-              w4[k] = k0 + k < a.top ? wt[kk] : 0.f;
-              if (a.rows_f32) {
-                const float *p = (const float *)a.rows + o;
-                r[k][0] = *reinterpret_cast<const f4 *>(p), r[k][1] = *reinterpret_cast<const f4 *>(p + 4);
-              } else {
-                unpack8_bf16(*reinterpret_cast<const uint4 *>((const uint16_t *)a.rows + o), r[k][0], r[k][1]);
-              }
+              const size_t o = (size_t)(k0 ? at[kk] : at0[k]) * H + ch * 8;
+              w4[k] = k0 + k >= a.top ? 0.f : k0 ? wt[kk] : wt0[k];
+              if (a.rows_f32) load8((const float *)a.rows + o, r[k]);
+              else unpack8_bf16(*reinterpret_cast<const uint4 *>((const uint16_t *)a.rows + o), r[k][0], r[k][1]);
             }
 #pragma unroll
             for (int k = 0; k < U; ++k) y[0] += r[k][0] * w4[k], y[1] += r[k][1] * w4[k];
@@ -144,19 +120,18 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
 #pragma unroll
         for (int h = 0; h < 2; ++h) x[c][h] += y[h] * a.mult;
       }
-      ss[c] = 0.f;
-      if (tid + c * NT < nchunk) {
-#pragma unroll
-        for (int h = 0; h < 2; ++h) {
-#pragma unroll
-          for (int e = 0; e < 4; ++e) ss[c] = fmaf(x[c][h][e], x[c][h][e], ss[c]);
-          if (a.x && mine) *reinterpret_cast<f4 *>(a.x + (size_t)t * H + ch * 8 + 4 * h) = x[c][h];
-        }
-      }
     }
-    if (!a.w) continue;
-    // the groups' norms
-    f4 r[MAXC][2];
+  };
+  // 1 / rms of every column's group, of row t
+  auto group_rms = [&](int t, int odd, const f4 (&x)[MAXC][2], f4 (&r)[MAXC][2]) {
+    float ss[MAXC];
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      ss[c] = 0.f;
+      if (tid + c * NT < nchunk)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss[c] = fmaf(x[c][e >> 2][e & 3], x[c][e >> 2][e & 3], ss[c]);
+    }
     if (st.waves) {  // a wave's 512 columns lie in one group
       float *pb = part + odd * st.parts;
 #pragma unroll
@@ -170,77 +145,141 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
       __syncthreads();
 #pragma unroll
       for (int c = 0; c < MAXC; ++c) {
-        const int g = min((wave + c * (NT / 64)) / per, a.groups - 1);
+        const int u0 = wave + c * (NT / 64), g = min(u0 / per, a.groups - 1);
         float v = 0.f;
         for (int u = 0; u < per; ++u) v += pb[g * per + u];
         v = inv_rms(v, gs, a.eps);
-        const int u = wave + c * (NT / 64);
-        if (!CONV && a.inv && lane == 0 && u < st.parts && u % per == 0) a.inv[(size_t)t * a.groups + g] = v;
+        if (!CONV && a.inv && lane == 0 && u0 < st.parts && u0 % per == 0) a.inv[(size_t)t * a.groups + g] = v;
         r[c][0] = r[c][1] = f4{v, v, v, v};
       }
-    } else {
-      const int us = st.unit, np = 8 / us;
-#pragma unroll
-      for (int c = 0; c < MAXC; ++c) {
-        const int ch = tid + c * NT;
-        if (ch >= nchunk) continue;
-        if (us == 8) {
-          if (ch < st.parts) part[ch] = ss[c];
-          continue;
-        }
-        int u = ch * np;
-        float v = 0.f;
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {  // (us divides 8: runs of us columns)
-          v = fmaf(x[c][e >> 2][e & 3], x[c][e >> 2][e & 3], v);
-          if ((e + 1) & (us - 1)) continue;
-          if (u < st.parts) part[u] = v;
-          ++u, v = 0.f;
-        }
-      }
-      __syncthreads();
-      for (int g = wave; g < a.groups; g += NT / 64) {
-        float v = 0.f;
-        for (int u = lane; u < per; u += 64) v += part[g * per + u];
-#pragma unroll
-        for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
-        if (lane == 0) {
-          inv[g] = inv_rms(v, gs, a.eps);
-          if (!CONV && a.inv) a.inv[(size_t)t * a.groups + g] = inv[g];
-        }
-      }
-      __syncthreads();
-#pragma unroll
-      for (int c = 0; c < MAXC; ++c) {
-        const int ch = min(tid + c * NT, nchunk - 1);
-        int g = ch * 8 / gs, next = (g + 1) * gs;
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          if (ch * 8 + e >= next) ++g, next += gs;
-          r[c][e >> 2][e & 3] = inv[min(g, a.groups - 1)];
-        }
-      }
+      return;
     }
+    const int us = st.unit, np = 8 / us;
 #pragma unroll
     for (int c = 0; c < MAXC; ++c) {
       const int ch = tid + c * NT;
       if (ch >= nchunk) continue;
-      f4 hv[2], cv[2];
+      if (us == 8) {
+        if (ch < st.parts) part[ch] = ss[c];
+        continue;
+      }
+      int u = ch * np;
+      float v = 0.f;
 #pragma unroll
-      for (int h = 0; h < 2; ++h) {
-        hv[h] = x[c][h] * r[c][h] * *reinterpret_cast<const f4 *>(a.w + ch * 8 + 4 * h);
-        x[c][h] = hv[h];
+      for (int e = 0; e < 8; ++e) {  // (us divides 8: runs of us columns)
+        v = fmaf(x[c][e >> 2][e & 3], x[c][e >> 2][e & 3], v);
+        if ((e + 1) & (us - 1)) continue;
+        if (u < st.parts) part[u] = v;
+        ++u, v = 0.f;
       }
-      if (!mine) continue;
-      if (a.hb) *reinterpret_cast<uint4 *>(a.hb + act_packed_off(out, ch * 8, H)) = pack8_bf16(hv[0], hv[1]);
-      if (a.hrow) *reinterpret_cast<uint4 *>(a.hrow + (size_t)out * H + ch * 8) = pack8_bf16(hv[0], hv[1]);
+    }
+    __syncthreads();
+    for (int g = wave; g < a.groups; g += NT / 64) {
+      float v = 0.f;
+      for (int u = lane; u < per; u += 64) v += part[g * per + u];
+#pragma unroll
+      for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
+      if (lane == 0) {
+        inv[g] = inv_rms(v, gs, a.eps);
+        if (!CONV && a.inv) a.inv[(size_t)t * a.groups + g] = inv[g];
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int ch = chunk(c);
+      int g = ch * 8 / gs, next = (g + 1) * gs;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        if (ch * 8 + e >= next) ++g, next += gs;
+        r[c][e >> 2][e & 3] = inv[min(g, a.groups - 1)];
+      }
+    }
+  };
+
+  int pos = 0, back = 0, ahead = 0, bank = 0;
+  size_t slot = 0;
+  // rows of earlier steps, zeros before the sequence (read while the token's own
+  // row is summed)
+  auto carried = [&]() {
+    if constexpr (!CONV) return;
+    pos = __builtin_amdgcn_readfirstlane(raw.pos), back = __builtin_amdgcn_readfirstlane(raw.back);
+    ahead = __builtin_amdgcn_readfirstlane(raw.ahead), bank = __builtin_amdgcn_readfirstlane(raw.bank);
+    slot = __builtin_amdgcn_readfirstlane(raw.slot);
+    if (past == 0 || back > past) return;
+    const float *cr = a.carry + (slot * 2 + bank) * past * H;
+    for (int k = 0; k < (REGS ? 1 : past); ++k)
+#pragma unroll
+      for (int kr = 0; kr < KH; ++kr)
+#pragma unroll
+        for (int c = 0; c < MAXC; ++c) {
+          const int q = REGS ? kr : k;
+          f4 v[2];
+          v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
+          if (q < past && pos - back > q) load8(cr + (size_t)q * H + chunk(c) * 8, v);
+#pragma unroll
+          for (int h = 0; h < 2; ++h) {
+            if constexpr (REGS) hist[kr][c][h] = v[h];
+            else if (tid + c * NT < nchunk) ring_at(q ? past - q : 0, c, h) = v[h];
+          }
+        }
+  };
+  f4 hown[MAXC][2], w[MAXC][2];
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    w[c][0] = w[c][1] = f4{0.f, 0.f, 0.f, 0.f};
+    if (a.w) load8(a.w + chunk(c) * 8, w[c]);
+  }
+  {
+    f4 r[MAXC][2];
+    sum_row(first, carried, hown);
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+      for (int h = 0; h < 2; ++h)
+        if (a.x && tid + c * NT < nchunk)
+          *reinterpret_cast<f4 *>(a.x + (size_t)first * H + (tid + c * NT) * 8 + 4 * h) = hown[c][h];
+    if (!a.w) return;
+    group_rms(first, 0, hown, r);
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+#pragma unroll
+      for (int h = 0; h < 2; ++h) hown[c][h] = hown[c][h] * r[c][h] * w[c][h];
+      const int ch = tid + c * NT;
+      if (ch >= nchunk) continue;
+      const uint4 hp = pack8_bf16(hown[c][0], hown[c][1]);
+      if (a.hb) *reinterpret_cast<uint4 *>(a.hb + act_packed_off(out, ch * 8, H)) = hp;
+      if (a.hrow) *reinterpret_cast<uint4 *>(a.hrow + (size_t)out * H + ch * 8) = hp;
       if (a.hf) {
-        *reinterpret_cast<f4 *>(a.hf + (size_t)out * H + ch * 8) = hv[0];
-        *reinterpret_cast<f4 *>(a.hf + (size_t)out * H + ch * 8 + 4) = hv[1];
+        *reinterpret_cast<f4 *>(a.hf + (size_t)out * H + ch * 8) = hown[c][0];
+        *reinterpret_cast<f4 *>(a.hf + (size_t)out * H + ch * 8 + 4) = hown[c][1];
       }
-      if constexpr (!CONV) continue;
-      const bool last = tk.ahead == 0;
-      float *cr = a.carry + ((size_t)(tk.slot * 2 + (tk.bank ^ 1)) * past) * H + ch * 8;
+    }
+  }
+  if constexpr (CONV) {
+    // the rows before it that this step brought, oldest first
+    for (int t = first - min(back, past), odd = 1; t < first; ++t, odd ^= 1) {
+      f4 x[MAXC][2], r[MAXC][2];
+      sum_row(t, []() {}, x);
+      group_rms(t, odd, x, r);
+      if constexpr (!REGS) head = head + 1 == past ? 0 : head + 1;
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+          const f4 v = x[c][h] * r[c][h] * w[c][h];
+          if constexpr (REGS) hist[2][c][h] = hist[1][c][h], hist[1][c][h] = hist[0][c][h], hist[0][c][h] = v;
+          else if (tid + c * NT < nchunk) ring_at(head, c, h) = v;
+        }
+    }
+    const bool last = ahead == 0;
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int ch = tid + c * NT;
+      if (ch >= nchunk) continue;
+      f4 cv[2];
+      float *cr = a.carry + ((slot * 2 + (bank ^ 1)) * past) * H + ch * 8;
+      const float *cw = a.conv + ch * 8;
 #pragma unroll
       for (int h = 0; h < 2; ++h) {
         // (oldest first, the token's own tap last)
@@ -249,41 +288,24 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
 #pragma unroll
           for (int k = 2; k >= 0; --k)
             if (k < past) {
-              v += hist[k][c][h] * *reinterpret_cast<const f4 *>(a.conv + (size_t)(past - 1 - k) * H + ch * 8 + 4 * h);
+              v += hist[k][c][h] * *reinterpret_cast<const f4 *>(cw + (size_t)(past - 1 - k) * H + 4 * h);
               if (last && k + 1 < past) *reinterpret_cast<f4 *>(cr + (size_t)(k + 1) * H + 4 * h) = hist[k][c][h];
             }
         } else {
           for (int k = past - 1; k >= 0; --k) {
             const f4 o = old_row(k, c, h);
-            v += o * *reinterpret_cast<const f4 *>(a.conv + (size_t)(past - 1 - k) * H + ch * 8 + 4 * h);
+            v += o * *reinterpret_cast<const f4 *>(cw + (size_t)(past - 1 - k) * H + 4 * h);
             if (last && k + 1 < past) *reinterpret_cast<f4 *>(cr + (size_t)(k + 1) * H + 4 * h) = o;
           }
         }
-        v += hv[h] * *reinterpret_cast<const f4 *>(a.conv + (size_t)past * H + ch * 8 + 4 * h);
-        if (last && past > 0) *reinterpret_cast<f4 *>(cr + 4 * h) = hv[h];
-        cv[h] = hv[h] + v;
+        v += hown[c][h] * *reinterpret_cast<const f4 *>(cw + (size_t)past * H + 4 * h);
+        if (last && past > 0) *reinterpret_cast<f4 *>(cr + 4 * h) = hown[c][h];
+        cv[h] = hown[c][h] + v;
       }
       if (a.cb) *reinterpret_cast<uint4 *>(a.cb + act_packed_off(out, ch * 8, H)) = pack8_bf16(cv[0], cv[1]);
       if (a.cf) {
         *reinterpret_cast<f4 *>(a.cf + (size_t)out * H + ch * 8) = cv[0];
         *reinterpret_cast<f4 *>(a.cf + (size_t)out * H + ch * 8 + 4) = cv[1];
-      }
-    }
-    // h becomes the latest earlier row
-    if (past > 0) {
-      if constexpr (REGS) {
-#pragma unroll
-        for (int c = 0; c < MAXC; ++c)
-#pragma unroll
-          for (int h = 0; h < 2; ++h)
-            hist[2][c][h] = hist[1][c][h], hist[1][c][h] = hist[0][c][h], hist[0][c][h] = x[c][h];
-      } else {
-        head = head + 1 == past ? 0 : head + 1;
-#pragma unroll
-        for (int c = 0; c < MAXC; ++c)
-#pragma unroll
-          for (int h = 0; h < 2; ++h)
-            if (tid + c * NT < nchunk) ring[(head * 2 + h) * nchunk + tid + c * NT] = x[c][h];
       }
     }
   }
@@ -441,7 +463,7 @@ static hipError_t run_conv_norm(ConvNormStep st, const ConvNorm &a, const EmbedP
         reinterpret_cast<const PagedToken *>((st.blob_dst ? (const char *)st.blob_dst : st.blob) + st.off_tokens);
 #define FFMI_CV(C, TP) \
   hipLaunchKernelGGL((conv_kernel<C, TP>), dim3((st.T + C - 1) / C, (nchunk + 255) / 256), dim3(256), 0, s, tok, st.T, a)
-    if (a.taps <= 4) FFMI_CV(8, 4);
+    if (a.taps <= 4) FFMI_CV(4, 4);
     else FFMI_CV(4, 0);
 #undef FFMI_CV
   }
