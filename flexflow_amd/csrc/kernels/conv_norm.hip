@@ -311,98 +311,84 @@ __global__ __launch_bounds__(NT) void conv_norm_kernel(ConvNormStep st, ConvNorm
   }
 }
 
-// The convolution of many tokens: a thread has 8 columns of C consecutive tokens.
+// The convolution of many tokens: a thread has 4 columns of C consecutive tokens,
+// a workgroup 4 C tokens side by side (16: whole lines of the packed tiles).
 // TAPS: at most (0: any; earlier rows are then read for every token again).
 template <int C, int TAPS>
 __global__ __launch_bounds__(256) void conv_kernel(const PagedToken *__restrict__ tok, int T, ConvNorm a) {
-  const int H = a.H, col = (blockIdx.y * 256 + threadIdx.x) * 8, t0 = blockIdx.x * C, past = a.taps - 1;
-  if (col >= H) return;
-  const int gs = a.n / a.groups;
-  auto load8 = [](const float *p, f4 (&v)[2]) {
-    v[0] = *reinterpret_cast<const f4 *>(p), v[1] = *reinterpret_cast<const f4 *>(p + 4);
-  };
-  f4 w[2];
-  load8(a.w + col, w);
-  // row h of token t of this step
-  auto scale_row = [&](int t, f4 (&v)[2]) {
+  const int H = a.H, past = a.taps - 1, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int col = (blockIdx.y * 64 + lane) * 4, t0 = (blockIdx.x * 4 + wave) * C;
+  if (col >= H || t0 >= T) return;
+  const int gs = a.n / a.groups, g0 = min(col / gs, a.groups - 1);
+  const bool one = min((col + 3) / gs, a.groups - 1) == g0;  // (else the columns lie in several groups)
+  auto load4 = [](const float *p) { return *reinterpret_cast<const f4 *>(p); };
+  const f4 w = load4(a.w + col), own = load4(a.conv + (size_t)past * H + col);
+  auto inv_of = [&](int t) {
     const float *iv = a.inv + (size_t)t * a.groups;
-    if (gs % 8 == 0) {
-      const float r = iv[min(col / gs, a.groups - 1)];
-      v[0] = v[0] * f4{r, r, r, r} * w[0], v[1] = v[1] * f4{r, r, r, r} * w[1];
-    } else {
+    const float r = iv[g0];
+    f4 v = {r, r, r, r};
+    if (!one)
 #pragma unroll
-      for (int e = 0; e < 8; ++e) v[e >> 2][e & 3] = v[e >> 2][e & 3] * iv[min((col + e) / gs, a.groups - 1)] * w[e >> 2][e & 3];
-    }
+      for (int e = 1; e < 4; ++e) v[e] = iv[min((col + e) / gs, a.groups - 1)];
+    return v;
+  };
+  auto carry_at = [&](const PagedToken &tk, int bank, int q) {
+    return a.carry + ((size_t)(tk.slot * 2 + bank) * past + q) * H + col;
   };
   // the row of q + 1 tokens before the step's first one of the request
-  auto old_row = [&](const PagedToken &tk, int q, f4 (&v)[2]) {
-    v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
-    if (tk.pos - tk.back > q) load8(a.carry + ((size_t)(tk.slot * 2 + tk.bank) * past + q) * H + col, v);
+  auto old_row = [&](const PagedToken &tk, int q) {
+    return tk.pos - tk.back > q ? load4(carry_at(tk, tk.bank, q)) : f4{0.f, 0.f, 0.f, 0.f};
   };
-  auto finish = [&](int t, const PagedToken &tk, const f4 (&h)[2], f4 (&v)[2]) {
-    f4 cw[2];
-    load8(a.conv + (size_t)past * H + col, cw);
-#pragma unroll
-    for (int k = 0; k < 2; ++k) v[k] = h[k] + (v[k] + h[k] * cw[k]);
-    if (a.cb) *reinterpret_cast<uint4 *>(a.cb + act_packed_off(t, col, H)) = pack8_bf16(v[0], v[1]);
-    if (a.cf) {
-      *reinterpret_cast<f4 *>(a.cf + (size_t)t * H + col) = v[0];
-      *reinterpret_cast<f4 *>(a.cf + (size_t)t * H + col + 4) = v[1];
-    }
+  auto keep = [&](const PagedToken &tk, int q, const f4 &h) {
+    if (tk.ahead == 0 && q < past) *reinterpret_cast<f4 *>(carry_at(tk, tk.bank ^ 1, q)) = h;
   };
-  auto keep = [&](const PagedToken &tk, int q, const f4 (&h)[2]) {  // h as the q-th row of the next step's carry
-    float *cr = a.carry + ((size_t)(tk.slot * 2 + (tk.bank ^ 1)) * past + q) * H + col;
-    *reinterpret_cast<f4 *>(cr) = h[0], *reinterpret_cast<f4 *>(cr + 4) = h[1];
+  auto finish = [&](int t, const PagedToken &tk, const f4 &h, f4 v) {
+    keep(tk, 0, h);
+    v = h + (v + h * own);
+    if (a.cb)
+      *reinterpret_cast<uint2 *>(a.cb + act_packed_off(t, col, H)) =
+          make_uint2(f2bf(v[0]) | ((uint32_t)f2bf(v[1]) << 16), f2bf(v[2]) | ((uint32_t)f2bf(v[3]) << 16));
+    if (a.cf) *reinterpret_cast<f4 *>(a.cf + (size_t)t * H + col) = v;
   };
   if constexpr (TAPS > 0) {
     constexpr int P = TAPS - 1;
-    f4 h[C + P][2], cw[P][2];  // rows t0 - P .., taps of the rows 1 to P tokens back
+    f4 h[C + P], r[C + P], cw[P];  // rows t0 - P .., taps of the rows 1 to P tokens back
+    PagedToken tk[C];
 #pragma unroll
-    for (int i = 0; i < C + P; ++i) load8(a.x + (size_t)min(max(t0 - P + i, 0), T - 1) * H + col, h[i]);
+    for (int i = 0; i < C + P; ++i) {
+      const int t = min(max(t0 - P + i, 0), T - 1);
+      h[i] = load4(a.x + (size_t)t * H + col), r[i] = inv_of(t);
+    }
 #pragma unroll
-    for (int k = 0; k < P; ++k) load8(a.conv + (size_t)max(past - 1 - k, 0) * H + col, cw[k]);
+    for (int k = 0; k < P; ++k) cw[k] = load4(a.conv + (size_t)max(past - 1 - k, 0) * H + col);
 #pragma unroll
-    for (int i = 0; i < C + P; ++i) scale_row(min(max(t0 - P + i, 0), T - 1), h[i]);
+    for (int i = 0; i < C; ++i) tk[i] = tok[min(t0 + i, T - 1)];
+#pragma unroll
+    for (int i = 0; i < C + P; ++i) h[i] = h[i] * r[i] * w;
 #pragma unroll
     for (int i = 0; i < C; ++i) {
-      const int t = t0 + i;
-      if (t >= T) break;
-      const PagedToken tk = tok[t];
-      f4 v[2];
-      v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
+      if (t0 + i >= T) break;
+      f4 v = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int k = P - 1; k >= 0; --k)  // (oldest first, the token's own tap last)
         if (k < past) {
-          f4 o[2];
-          if (tk.back > k) o[0] = h[i + P - 1 - k][0], o[1] = h[i + P - 1 - k][1];
-          else old_row(tk, k - tk.back, o);
-          v[0] += o[0] * cw[k][0], v[1] += o[1] * cw[k][1];
-          if (tk.ahead == 0 && k + 1 < past) keep(tk, k + 1, o);
+          const f4 o = tk[i].back > k ? h[i + P - 1 - k] : old_row(tk[i], k - tk[i].back);
+          v += o * cw[k];
+          keep(tk[i], k + 1, o);
         }
-      if (tk.ahead == 0 && past > 0) keep(tk, 0, h[i + P]);
-      finish(t, tk, h[i + P], v);
+      finish(t0 + i, tk[i], h[i + P], v);
     }
   } else {
     for (int t = t0; t < min(t0 + C, T); ++t) {
       const PagedToken tk = tok[t];
-      f4 h[2], v[2];
-      load8(a.x + (size_t)t * H + col, h);
-      scale_row(t, h);
-      v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
+      f4 v = {0.f, 0.f, 0.f, 0.f};
       for (int k = past - 1; k >= 0; --k) {
-        f4 o[2], cw[2];
-        load8(a.conv + (size_t)(past - 1 - k) * H + col, cw);
-        if (tk.back > k) {
-          load8(a.x + (size_t)(t - 1 - k) * H + col, o);
-          scale_row(t - 1 - k, o);
-        } else {
-          old_row(tk, k - tk.back, o);
-        }
-        v[0] += o[0] * cw[0], v[1] += o[1] * cw[1];
-        if (tk.ahead == 0 && k + 1 < past) keep(tk, k + 1, o);
+        const int s = t - 1 - k;
+        const f4 o = tk.back > k ? load4(a.x + (size_t)s * H + col) * inv_of(s) * w : old_row(tk, k - tk.back);
+        v += o * load4(a.conv + (size_t)(past - 1 - k) * H + col);
+        keep(tk, k + 1, o);
       }
-      if (tk.ahead == 0 && past > 0) keep(tk, 0, h);
-      finish(t, tk, h, v);
+      finish(t, tk, load4(a.x + (size_t)t * H + col) * inv_of(t) * w, v);
     }
   }
 }
@@ -462,7 +448,7 @@ static hipError_t run_conv_norm(ConvNormStep st, const ConvNorm &a, const EmbedP
     const PagedToken *tok =
         reinterpret_cast<const PagedToken *>((st.blob_dst ? (const char *)st.blob_dst : st.blob) + st.off_tokens);
 #define FFMI_CV(C, TP) \
-  hipLaunchKernelGGL((conv_kernel<C, TP>), dim3((st.T + C - 1) / C, (nchunk + 255) / 256), dim3(256), 0, s, tok, st.T, a)
+  hipLaunchKernelGGL((conv_kernel<C, TP>), dim3((st.T + 4 * C - 1) / (4 * C), (a.H / 4 + 63) / 64), dim3(256), 0, s, tok, st.T, a)
     if (a.taps <= 4) FFMI_CV(4, 4);
     else FFMI_CV(4, 0);
 #undef FFMI_CV
