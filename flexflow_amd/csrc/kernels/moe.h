@@ -24,7 +24,7 @@ struct MoeSizes {
   bool shared = false;
   int gate_col = 0;  // column of the shared expert's gate in the router's product
   int tile_rows() const {
-    return (long)T * top >= 12L * experts && T >= 64 ? kMoeMany : kMoeFew;
+    return T > 32 && (long)T * top >= 4L * experts ? kMoeMany : kMoeFew;
   }
   // upper bounds: slots of the experts (whole 16s), tiles
   __host__ __device__ int slots() const {
