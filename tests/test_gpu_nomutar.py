@@ -408,7 +408,7 @@ def test_wide_rows(tmp_path, width, groups, taps, full):
 def test_many_experts(tmp_path, n, top, T):
     """Routers of one to sixteen logits a lane, steps of few and of many rows an
     expert (up to 64, 128, 192, 256 and more), experts that no token takes."""
-    cfg = NM.model_config(90, 320, [NM.experts(NM.plain(2, 1, 16, 16, 0.2), n, top, 40, shared=70)], bigram=None)
+    cfg = NM.model_config(90, 352, [NM.experts(NM.plain(2, 1, 16, 16, 0.2), n, top, 40, shared=70)], bigram=None)
     w = NM.random_weights(cfg, 7)
     toks = tokens(cfg, T, 5)
     want = R.forward(cfg, w, toks)
