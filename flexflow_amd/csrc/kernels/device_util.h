@@ -29,6 +29,20 @@ __device__ __forceinline__ float ld_elem(const float *p) { return *p; }
 __device__ __forceinline__ void st_elem(uint16_t *p, float v) { *p = f2bf(v); }
 __device__ __forceinline__ void st_elem(float *p, float v) { *p = v; }
 
+__device__ __forceinline__ float sigmoid_f(float v) { return __fdiv_rn(1.0f, 1.0f + expf(-v)); }
+__device__ __forceinline__ float silu_f(float v) { return v * sigmoid_f(v); }
+// value and remainder in bf16
+__device__ __forceinline__ void split2(float v, __bf16 &hi, __bf16 &lo) {
+  hi = (__bf16)v;
+  lo = (__bf16)(v - (float)hi);
+}
+// element `at` of deferred sums
+__device__ __forceinline__ float sum_at(const Partials &y, size_t slab, size_t at) {
+  float v = y.p[at];
+  for (int s = 1; s < y.S; ++s) v += y.p[at + s * slab];
+  return v;
+}
+
 template <int NT>
 __device__ __forceinline__ float row_sum(float v, float *sh) {
 #pragma unroll

@@ -10,14 +10,6 @@ namespace ffmi {
 typedef short s4 __attribute__((ext_vector_type(4)));
 typedef uint32_t u4 __attribute__((ext_vector_type(4)));
 
-__device__ __forceinline__ float sigmoid_f(float v) { return __fdiv_rn(1.0f, 1.0f + expf(-v)); }
-__device__ __forceinline__ float silu_f(float v) { return v * sigmoid_f(v); }
-__device__ __forceinline__ float sum_at(const Partials &y, size_t slab, size_t at) {
-  float v = y.p[at];
-  for (int s = 1; s < y.S; ++s) v += y.p[at + s * slab];
-  return v;
-}
-
 // ---------------------------------------------------------------------------
 // token by token: a workgroup per (32 value columns, head, span), the state in
 // registers: thread = (row ri of every 32 rows, 4 columns)
@@ -128,11 +120,6 @@ __global__ __launch_bounds__(256) void lightning_qkv_kernel(Lightning a, int col
   *reinterpret_cast<uint4 *>(a.qkv + (size_t)t * cols + c) = pack8_bf16(lo, hi);
 }
 
-// value and remainder in bf16
-__device__ __forceinline__ void split2(float v, __bf16 &hi, __bf16 &lo) {
-  hi = (__bf16)v;
-  lo = (__bf16)(v - (float)hi);
-}
 // operand of 8 k-values from row-major LDS rows: column c0 + (lane & 15), rows
 // kb * 32 + {4g .. 4g + 3, 16 + 4g ..}
 template <int LD>

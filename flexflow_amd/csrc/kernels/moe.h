@@ -21,6 +21,7 @@ constexpr int kMoeMaxExperts = 1024, kMoeMaxTop = 64;
 // a step's sizes: T tokens of which each takes `top` of `experts`
 struct MoeSizes {
   int T = 0, experts = 0, top = 0;
+  int identity = 0;  // further outputs of the router, after the experts': the row itself
   bool shared = false;
   int gate_col = 0;  // column of the shared expert's gate in the router's product
   int tile_rows() const {
@@ -39,9 +40,10 @@ struct MoeSizes {
 };
 struct MoeLists {
   int32_t *picked = nullptr;      // [T][top] experts
-  int32_t *at = nullptr;          // [T][top] slots
+  int32_t *at = nullptr;          // [T][top] slots (-1: none, an identity expert)
   float *wt = nullptr;            // [T][top] their weights
   float *gate = nullptr;          // [T] the shared expert's
+  float *own = nullptr;           // [T] the identity experts' weights together
   int32_t *slot_token = nullptr;  // [slots]
   MoeTile *tiles = nullptr;       // the shared expert's first
   int32_t *num_tiles = nullptr;
@@ -50,11 +52,22 @@ struct MoeLists {
 // lowest index among equals), softmax over them; gate: the sigmoid of its column.
 hipError_t launch_moe_route(const Partials &z, const float *bias, const MoeSizes &n, const MoeLists &l,
                             hipStream_t s);
+// Another choice: scores s = softmax of all columns (identity experts' included); the
+// `top` largest s + correction among the columns of the best `keep` of `groups` equal
+// groups of neighbours (a group counts as its best column); weights scale s / (sum of
+// the chosen s + 1e-20).
+struct MoeScores {
+  const float *correction = nullptr;  // [experts + identity]
+  int groups = 1, keep = 1;
+  float scale = 1.f;
+};
+hipError_t launch_moe_route_scores(const Partials &z, const MoeScores &sc, const MoeSizes &n, const MoeLists &l,
+                                   hipStream_t s);
 
 // One product of every slot with its expert's matrix.
 //   first  (gated): Y[slot] = silu(X W_gate) (X W_up), X the token's row (row-major),
 //          Y bf16 in packed tiles of width ldy (fp32: rows); the shared expert's
-//          times gate[token]
+//          times gate[token].  limit > 0: the clamped gated unit instead
 //   second: Y[slot] = X W_down, X the first product's Y; Y rows of N, bf16 (fp32)
 // W: bf16 packed weights, gate / up tiles in turn (fp32: rows, gate then up), expert
 // after expert.
@@ -71,6 +84,7 @@ struct MoeGemm {
   const MoeTile *tiles = nullptr;
   const int32_t *num_tiles = nullptr;
   const float *gate = nullptr;
+  float limit = 0.f;
 };
 hipError_t launch_moe_gemm(const MoeGemm &a, const MoeSizes &n, bool gated, bool f32, bool stream_weights,
                            hipStream_t s);

@@ -20,6 +20,23 @@ __device__ __forceinline__ float slab_total(const Partials &z, const float *p, s
     if (s < z.S) v[0] += v[s];
   return v[0];
 }
+// the wave's largest value, NV a lane (column i * 64 + lane; the lowest among equals)
+template <int NV>
+__device__ __forceinline__ int best_column(const float (&v)[NV], float &best) {
+  const int lane = threadIdx.x & 63;
+  int at = lane;
+  best = v[0];
+#pragma unroll
+  for (int i = 1; i < NV; ++i)
+    if (v[i] > best) best = v[i], at = i * 64 + lane;
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) {
+    const float b = __shfl_xor(best, o);
+    const int w = __shfl_xor(at, o);
+    if (b > best || (b == best && w < at)) best = b, at = w;
+  }
+  return at;
+}
 // A wave picks a token's experts: NV logits a lane, the best of the wave `top`
 // times over.
 template <int NV>
@@ -41,17 +58,8 @@ __device__ __forceinline__ void pick_experts(const Partials &z, const float *__r
   float top0 = 0.f, sum = 0.f, mine = 0.f;  // lane k: the k-th pick
   int mine_e = 0;
   for (int k = 0; k < n.top; ++k) {
-    float best = v[0];
-    int at = lane;
-#pragma unroll
-    for (int i = 1; i < NV; ++i)
-      if (v[i] > best) best = v[i], at = i * 64 + lane;
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float b = __shfl_xor(best, o);
-      const int w = __shfl_xor(at, o);
-      if (b > best || (b == best && w < at)) best = b, at = w;
-    }
+    float best;
+    const int at = best_column<NV>(v, best);
     if (k == 0) top0 = best;
     const float p = expf(best - top0);
     sum += p;
@@ -66,24 +74,90 @@ __device__ __forceinline__ void pick_experts(const Partials &z, const float *__r
   }
   if (n.shared && lane == 0) l.gate[t] = __fdiv_rn(1.0f, 1.0f + expf(-gate));
 }
+// the same by scores
 template <int NV>
-__global__ __launch_bounds__(256) void moe_pick_kernel(Partials z, const float *bias, MoeSizes n, MoeLists l) {
+__device__ __forceinline__ void pick_experts(const Partials &z, const MoeScores &sc, const MoeSizes &n, int t,
+                                             const MoeLists &l) {
+  const int lane = threadIdx.x & 63, cols = n.experts + n.identity, size = cols / sc.groups;
+  const size_t slab = (size_t)n.T * z.NP;
+  const float *row = z.p + (size_t)t * z.NP;
+  float s[NV], v[NV];
+  float mx = -INFINITY, sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int e = i * 64 + lane;
+    s[i] = e < cols ? slab_total(z, row + e, slab) : -INFINITY;
+    mx = fmaxf(mx, s[i]);
+  }
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
+#pragma unroll
+  for (int i = 0; i < NV; ++i) s[i] = expf(s[i] - mx), sum += s[i];
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) sum += __shfl_xor(sum, o);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int e = i * 64 + lane;
+    s[i] = __fdiv_rn(s[i], sum);
+    v[i] = e < cols ? s[i] + sc.correction[e] : -INFINITY;
+  }
+  if (sc.keep < sc.groups) {  // the group of the best column left, `keep` times over
+    float left[NV];
+    bool in[NV];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) left[i] = v[i], in[i] = false;
+    for (int k = 0; k < sc.keep; ++k) {
+      float best;
+      const int g = best_column<NV>(left, best) / size;
+#pragma unroll
+      for (int i = 0; i < NV; ++i)
+        if ((i * 64 + lane) / size == g) in[i] = true, left[i] = -INFINITY;
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+      if (!in[i]) v[i] = -INFINITY;
+  }
+  float mine = 0.f, total = 0.f, own = 0.f;
+  int mine_e = 0;
+  for (int k = 0; k < n.top; ++k) {
+    float best, w = 0.f;
+    const int at = best_column<NV>(v, best);
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+      if (at == i * 64 + lane) v[i] = -INFINITY, w = s[i];
+    w = __shfl(w, at & 63);
+    total += w;
+    if (at >= n.experts) own += w;
+    if (lane == k) mine = w, mine_e = at;
+  }
+  const float f = __fdiv_rn(sc.scale, total + 1e-20f);
+  if (lane < n.top) {
+    const bool real = mine_e < n.experts;
+    l.picked[(size_t)t * n.top + lane] = real ? mine_e : -1;
+    l.wt[(size_t)t * n.top + lane] = real ? mine * f : 0.f;
+  }
+  if (n.identity && lane == 0) l.own[t] = own * f;
+}
+// How: `const float *` (bias) or MoeScores
+template <int NV, class How>
+__global__ __launch_bounds__(256) void moe_pick_kernel(Partials z, How how, MoeSizes n, MoeLists l) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (t < n.T) pick_experts<NV>(z, bias, n, t, l);
+  if (t < n.T) pick_experts<NV>(z, how, n, t, l);
 }
 
 // One workgroup: tokens by expert.  PICK: it picks the experts as well (few tokens).
-template <int NV, bool PICK>
-__global__ __launch_bounds__(1024) void moe_lists_kernel(Partials z, const float *bias, MoeSizes n, MoeLists l,
+template <int NV, bool PICK, class How>
+__global__ __launch_bounds__(1024) void moe_lists_kernel(Partials z, How how, MoeSizes n, MoeLists l,
                                                          int rows) {
   __shared__ int count[kMoeMaxExperts], next[kMoeMaxExperts], total;
   const int tid = threadIdx.x, A = n.T * n.top, st = n.shared_tiles(rows);
   for (int e = tid; e < n.experts; e += 1024) count[e] = 0;
   if constexpr (PICK)
     for (int t = tid >> 6; t < n.T; t += 16)
-      pick_experts<NV>(z, bias, n, t, l);
+      pick_experts<NV>(z, how, n, t, l);
   __syncthreads();
-  for (int a = tid; a < A; a += 1024) atomicAdd(&count[l.picked[a]], 1);
+  for (int a = tid; a < A; a += 1024)
+    if (l.picked[a] >= 0) atomicAdd(&count[l.picked[a]], 1);
   __syncthreads();
   if (tid < 64) {  // first slot and first tile of every expert: a scan over the wave
     const int per = (n.experts + 63) / 64, e0 = tid * per, e1 = min(e0 + per, n.experts);
@@ -109,34 +183,53 @@ __global__ __launch_bounds__(1024) void moe_lists_kernel(Partials z, const float
     l.tiles[i] = MoeTile{n.experts, i * rows, min(rows, n.T - i * rows), 0};
   if (tid == 0) *l.num_tiles = st + total;
   for (int a = tid; a < A; a += 1024) {
+    if (l.picked[a] < 0) {
+      l.at[a] = -1;
+      continue;
+    }
     const int slot = atomicAdd(&next[l.picked[a]], 1);
     l.slot_token[slot] = a / n.top;
     l.at[a] = slot;
   }
 }
 
-hipError_t launch_moe_route(const Partials &z, const float *bias, const MoeSizes &n, const MoeLists &l,
-                            hipStream_t s) {
+template <class How>
+static hipError_t route(const Partials &z, How how, const MoeSizes &n, const MoeLists &l, hipStream_t s) {
   if (n.T <= 0) return hipSuccess;
-  if (n.experts < 1 || n.experts > kMoeMaxExperts || n.top < 1 || n.top > std::min(n.experts, kMoeMaxTop) ||
-      z.S < 1 || z.S > 8 || z.NP < n.experts || (n.shared && n.gate_col >= z.NP))
+  const int cols = n.experts + n.identity;
+  if (n.experts < 1 || n.identity < 0 || cols > kMoeMaxExperts || n.top < 1 ||
+      n.top > std::min(cols, kMoeMaxTop) || z.S < 1 || z.S > 8 || z.NP < cols ||
+      (n.shared && n.gate_col >= z.NP) || (n.identity && !l.own))
     return hipErrorInvalidValue;
   const int rows = n.tile_rows();
-#define FFMI_MR(NV)                                                                                        \
-  do {                                                                                                     \
-    if (n.T <= 64) {                                                                                       \
-      hipLaunchKernelGGL((moe_lists_kernel<NV, true>), dim3(1), dim3(1024), 0, s, z, bias, n, l, rows);    \
-    } else {                                                                                               \
-      hipLaunchKernelGGL(moe_pick_kernel<NV>, dim3((n.T + 3) / 4), dim3(256), 0, s, z, bias, n, l);        \
-      hipLaunchKernelGGL((moe_lists_kernel<1, false>), dim3(1), dim3(1024), 0, s, z, bias, n, l, rows);    \
-    }                                                                                                      \
+#define FFMI_MR(NV)                                                                                          \
+  do {                                                                                                       \
+    if (n.T <= 64) {                                                                                         \
+      hipLaunchKernelGGL((moe_lists_kernel<NV, true, How>), dim3(1), dim3(1024), 0, s, z, how, n, l, rows);  \
+    } else {                                                                                                 \
+      hipLaunchKernelGGL((moe_pick_kernel<NV, How>), dim3((n.T + 3) / 4), dim3(256), 0, s, z, how, n, l);    \
+      hipLaunchKernelGGL((moe_lists_kernel<1, false, How>), dim3(1), dim3(1024), 0, s, z, how, n, l, rows);  \
+    }                                                                                                        \
   } while (0)
-  if (n.experts <= 64) FFMI_MR(1);
-  else if (n.experts <= 128) FFMI_MR(2);
-  else if (n.experts <= 256) FFMI_MR(4);
+  if (cols <= 64) FFMI_MR(1);
+  else if (cols <= 128) FFMI_MR(2);
+  else if (cols <= 256) FFMI_MR(4);
   else FFMI_MR(16);
 #undef FFMI_MR
   return hipGetLastError();
+}
+hipError_t launch_moe_route(const Partials &z, const float *bias, const MoeSizes &n, const MoeLists &l,
+                            hipStream_t s) {
+  if (n.identity) return hipErrorInvalidValue;
+  return route(z, bias, n, l, s);
+}
+hipError_t launch_moe_route_scores(const Partials &z, const MoeScores &sc, const MoeSizes &n, const MoeLists &l,
+                                   hipStream_t s) {
+  const int cols = n.experts + n.identity;
+  if (sc.groups < 1 || cols % sc.groups || sc.keep < 1 || sc.keep > sc.groups ||
+      n.top > cols / sc.groups * sc.keep || n.shared || !sc.correction)
+    return hipErrorInvalidValue;
+  return route(z, sc, n, l, s);
 }
 
 // ---------------------------------------------------------------------------
@@ -152,12 +245,16 @@ __device__ __forceinline__ void store_bf16x4(uint16_t *p, float a, float b, floa
 }
 // four consecutive output columns n.. of slot row m; gated: of the gate and up sums
 // (f: the row's factor)
+__device__ __forceinline__ float moe_unit(float gate, float up, float limit) {
+  return limit > 0.f ? clamped_glu(gate, up, limit) : silu_glu(gate, up);
+}
 template <bool GATED>
-__device__ __forceinline__ void moe_store(const MoeGroup &g, int m, int n, float f, const f4 &a, const f4 &b) {
+__device__ __forceinline__ void moe_store(const MoeGroup &g, int m, int n, float f, float limit, const f4 &a,
+                                          const f4 &b) {
   uint16_t *Y = (uint16_t *)g.Y;
   if constexpr (GATED)
-    store_bf16x4(Y + act_packed_off(m, n, g.ldy), f * silu_glu(a[0], b[0]), f * silu_glu(a[1], b[1]),
-                 f * silu_glu(a[2], b[2]), f * silu_glu(a[3], b[3]));
+    store_bf16x4(Y + act_packed_off(m, n, g.ldy), f * moe_unit(a[0], b[0], limit), f * moe_unit(a[1], b[1], limit),
+                 f * moe_unit(a[2], b[2], limit), f * moe_unit(a[3], b[3], limit));
   else
     store_bf16x4(Y + (size_t)m * g.N + n, a[0], a[1], a[2], a[3]);
 }
@@ -214,10 +311,10 @@ __global__ __launch_bounds__(256) void moe_few_kernel(MoeGemm a, int first, size
   if (m >= tl.rows) return;
   const int row = tl.slot0 + m, n = (lane >> 4) * 4;
   if constexpr (GATED) {
-    moe_store<true>(g, row, blockIdx.x * 16 + n, shared ? a.gate[row] : 1.0f, acc[0], acc[1]);
+    moe_store<true>(g, row, blockIdx.x * 16 + n, shared ? a.gate[row] : 1.0f, a.limit, acc[0], acc[1]);
   } else {
-    moe_store<false>(g, row, tile0 * 16 + n, 1.0f, acc[0], acc[0]);
-    if (tile0 + 1 < ntiles) moe_store<false>(g, row, tile0 * 16 + 16 + n, 1.0f, acc[1], acc[1]);
+    moe_store<false>(g, row, tile0 * 16 + n, 1.0f, 0.f, acc[0], acc[0]);
+    if (tile0 + 1 < ntiles) moe_store<false>(g, row, tile0 * 16 + 16 + n, 1.0f, 0.f, acc[1], acc[1]);
   }
 }
 
@@ -311,8 +408,8 @@ __device__ __forceinline__ void moe_tile(const MoeGemm &a, const MoeTile &tl, in
     for (int j = 0; j < 4; j += GATED ? 2 : 1) {
       const int tile = tile0 + wn * 4 + j;
       if (tile >= ntiles) continue;
-      moe_store<GATED>(g, tl.slot0 + m, (GATED ? tile >> 1 : tile) * 16 + (lane >> 4) * 4, f, acc[i][j],
-                       acc[i][GATED ? j + 1 : j]);
+      moe_store<GATED>(g, tl.slot0 + m, (GATED ? tile >> 1 : tile) * 16 + (lane >> 4) * 4, f, a.limit,
+                       acc[i][j], acc[i][GATED ? j + 1 : j]);
     }
   }
 }
@@ -384,7 +481,7 @@ __global__ __launch_bounds__(256) void moe_f32_kernel(MoeGemm a, int first) {
         if (n >= g.N) continue;
         if constexpr (GATED)
           ((float *)g.Y)[(size_t)row * g.ldy + n] =
-              (shared ? a.gate[row] : 1.0f) * silu_glu(acc[0][j], acc[GATED ? 1 : 0][j]);
+              (shared ? a.gate[row] : 1.0f) * moe_unit(acc[0][j], acc[GATED ? 1 : 0][j], a.limit);
         else
           ((float *)g.Y)[(size_t)row * g.N + n] = acc[0][j];
       }

@@ -6,7 +6,8 @@ namespace ffmi {
 
 // dst = the [N][K] matrix a kernel wants, from the checkpoint's src: row n =
 // head n / np's row n % np (zero from nb on; heads * np rows), column k
-// likewise from (kb, kp).  transpose: src holds [heads][K][N] blocks.
+// likewise from (kb, kp).  transpose: src holds [heads][cols][kb][N] blocks.
+// plus: added to every element that is not padding (pack_f32).
 // perhead: each head its own tile-major packed block (head products).
 // row_pairs / col_pairs: of every head's first so many rows (columns), m and
 // m + half of them come to lie side by side (rotations that pair halves).
@@ -18,6 +19,7 @@ struct PackSpec {
   bool transpose = false;
   int row_pairs = 0, col_pairs = 0;
   int k0 = 0, kt = 0;
+  float plus = 0.f;
 };
 hipError_t launch_pack_bf16(const uint16_t *src, int ld, const PackSpec &p, uint16_t *dst,
                             int tile_offset, int pitch, bool perhead, hipStream_t s,

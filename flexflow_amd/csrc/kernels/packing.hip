@@ -4,15 +4,20 @@
 
 namespace ffmi {
 
-__device__ __forceinline__ uint16_t pack_elem(const uint16_t *src, int ld, const PackSpec &p, int n,
-                                              int k) {
+// the index of destination element (n, k) in src; -1: padding
+__device__ __forceinline__ long pack_index(int ld, const PackSpec &p, int n, int k) {
   const int hn = n / p.np, hk = k / p.kp;
   int jn = n % p.np, jk = k % p.kp;
   if (jn < p.row_pairs) jn = (jn >> 1) + (jn & 1) * (p.row_pairs >> 1);
   if (jk < p.col_pairs) jk = (jk >> 1) + (jk & 1) * (p.col_pairs >> 1);
-  if (hn >= p.rows || jn >= p.nb || hk >= p.cols || jk >= p.kb) return 0;
-  if (p.transpose) return src[((size_t)hn * p.kb + jk) * ld + jn];
-  return src[(size_t)(hn * p.nb + jn) * ld + hk * p.kb + jk];
+  if (hn >= p.rows || jn >= p.nb || hk >= p.cols || jk >= p.kb) return -1;
+  if (p.transpose) return ((long)(hn * p.cols + hk) * p.kb + jk) * ld + jn;
+  return (long)(hn * p.nb + jn) * ld + hk * p.kb + jk;
+}
+__device__ __forceinline__ uint16_t pack_elem(const uint16_t *src, int ld, const PackSpec &p, int n,
+                                              int k) {
+  const long at = pack_index(ld, p, n, k);
+  return at < 0 ? 0 : src[at];
 }
 __global__ void pack_bf16_kernel(const uint16_t *__restrict__ src, int ld, PackSpec p,
                                  uint16_t *__restrict__ dst, int NT, int KT, size_t ts, size_t ks) {
@@ -45,7 +50,8 @@ __global__ void pack_f32_kernel(const uint16_t *__restrict__ src, int ld, PackSp
                                 float *__restrict__ dst, int N, int K, int ldd) {
   const long i = blockIdx.x * (long)blockDim.x + threadIdx.x;
   if (i >= (long)N * K) return;
-  dst[i / K * ldd + i % K] = bf2f(pack_elem(src, ld, p, (int)(i / K), (int)(i % K)));
+  const long at = pack_index(ld, p, (int)(i / K), (int)(i % K));
+  dst[i / K * ldd + i % K] = at < 0 ? 0.f : bf2f(src[at]) + p.plus;
 }
 hipError_t launch_pack_f32(const uint16_t *src, int ld, const PackSpec &p, float *dst,
                            hipStream_t s) {

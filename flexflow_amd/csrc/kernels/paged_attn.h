@@ -49,6 +49,16 @@ struct AttnPrep {
   const double *freq = nullptr, *vfreq = nullptr;
   int rot = 0;
   float rot_mult = 1.f;
+  // rotary kind: taps > 0: a causal convolution of every product column over time,
+  // before norm and rotation; conv [taps][columns] (columns (H + G) dg + G vg), the
+  // last row the current token's.  The last taps - 1 product rows of a request are
+  // carried: carry [slots][2 banks][taps - 1][columns], the latest first.  off_tokens:
+  // the step's tokens in its metadata
+  const float *conv = nullptr;
+  int taps = 0;
+  float *carry = nullptr;
+  int off_tokens = 0;
+  bool unit = false;  // rotated queries and keys over their rms, per head
 };
 hipError_t launch_attn_prep(const char *blob, int off_tokens, int T, const AttnPrep &a, bool f32,
                             hipStream_t s);
@@ -77,6 +87,7 @@ struct AttnArgs {
   const float *sink = nullptr;
   const double *vfreq = nullptr;
   int off_tokens = 0;
+  float mult = 1.f;  // of the outputs
 };
 // bf16, widths that attn_width gave; slabs / ml: partials of split blocks, 16
 // rows a slot, [slot][G][16][vp] and [slot][G][16][2].  pr: the launch makes

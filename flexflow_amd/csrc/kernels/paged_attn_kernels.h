@@ -115,6 +115,34 @@ __device__ __forceinline__ void load_head(const AttnPrep &a, int T, int t, int h
     }
   }
 }
+// (rotary kind) the convolution over time: v, token t's product, becomes the sum over
+// its taps; the rows that later steps need go to the other bank
+template <int NE>
+__device__ __forceinline__ void conv_head(const AttnPrep &a, int T, int t, const PagedToken &tk, int hd,
+                                          float (&v)[NE]) {
+  const int wd = head_width(a, hd), c0 = head_start(a, hd), past = a.taps - 1;
+  const size_t C = (size_t)(a.H + a.G) * a.dg + (size_t)a.G * a.vg;
+  const float *old = a.carry + ((size_t)tk.slot * 2 + tk.bank) * past * C;
+  float *now = a.carry + ((size_t)tk.slot * 2 + (tk.bank ^ 1)) * past * C;
+  const size_t slab = (size_t)T * a.y.NP;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int c = head_column<NE>(i);
+    if (c >= wd) continue;
+    const size_t col = c0 + c;
+    if (tk.ahead < past) now[tk.ahead * C + col] = v[i];
+    if (tk.back == 0)  // (a short portion: earlier rows move on)
+      for (int p = tk.ahead + 1; p < past; ++p)
+        now[p * C + col] = p - tk.ahead <= tk.pos ? old[(p - tk.ahead - 1) * C + col] : 0.f;
+    float sum = v[i] * a.conv[past * C + col];
+    for (int d = 1; d <= past && d <= tk.pos; ++d) {
+      const float u = tk.back >= d ? slab_sum(a.y, slab, (size_t)(t - d) * a.y.NP + col)
+                                   : old[(d - tk.back - 1) * C + col];
+      sum = fmaf(u, a.conv[(past - d) * C + col], sum);
+    }
+    v[i] = sum;
+  }
+}
 // values: mixed with, or kept as, the first mixing layer's (lam: *a.vmix)
 template <int NE>
 __device__ __forceinline__ void mix_head(const AttnPrep &a, int t, int g, float lam, float (&v)[NE]) {
@@ -180,6 +208,16 @@ __device__ __forceinline__ void rotary_head(const AttnPrep &a, int hd, int pos, 
     }
   }
   if (a.rot > 0) rotate_head<NE>(a.freq, a.rot, a.rot_mult, pos, v);
+  if (a.unit) {  // (columns past the head are zero)
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NE; ++i) ss = fmaf(v[i], v[i], ss);
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
+    const float f = inv_rms(ss, a.dim, a.eps);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) v[i] *= f;
+  }
 }
 // sums of squares of a token's whole query and key rows: this thread's columns
 template <int NTH>
@@ -322,6 +360,10 @@ __global__ __launch_bounds__(512) void rotary_prep_kernel(const PagedToken *__re
     load_bias<NE>(a, hd, bias);
 #pragma unroll
     for (int k = 0; k < NT; ++k) load_head<NE>(a, T, min(t0 + k, T - 1), hd, bias, v[k]);
+    if (a.taps > 0)
+#pragma unroll
+      for (int k = 0; k < NT; ++k)
+        if (t0 + k < T) conv_head<NE>(a, T, t0 + k, tk[k], hd, v[k]);
     if (isv) {
       if (a.vfreq)
 #pragma unroll
@@ -429,8 +471,9 @@ __device__ __forceinline__ float row_factor(const AttnArgs &a, int head, float M
   if constexpr (KIND == kRotary) {
     if (a.sink) {
       const float sk = a.sink[head], top = fmaxf(M, sk), f = __builtin_amdgcn_exp2f(M - top);
-      return __fdiv_rn(f, fmaf(L, f, __builtin_amdgcn_exp2f(sk - top)));
+      return __fdiv_rn(a.mult * f, fmaf(L, f, __builtin_amdgcn_exp2f(sk - top)));
     }
+    return __fdiv_rn(a.mult, L);
   }
   return __fdiv_rn(1.0f, L);
 }
@@ -538,6 +581,10 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
     };
     auto finish = [&](int it, float (&x)[NE]) {
       const int tk = token_of(it), pos = bk.pos0 + tk, tile = pos / kPageTokens;
+      if constexpr (KIND == kRotary)  // (split blocks carry the same rows)
+        if (pr.taps > 0)
+          conv_head<NE>(pr, T, t0 + tk, reinterpret_cast<const PagedToken *>(blob + pr.off_tokens)[t0 + tk],
+                        head_of(it), x);
       if (it < nq) {
         make(it, pos, x);
         store_head<uint16_t, NE>([&](int c) { return sQ + it * LDQ + c; }, DP, x);
@@ -1025,12 +1072,12 @@ __global__ __launch_bounds__(256) void paged_attn_rows_kernel(const char *__rest
       acc[i] = s;
     }
   }
-  float inv = __fdiv_rn(1.0f, l);
+  float inv = __fdiv_rn(KIND == kRotary ? a.mult : 1.0f, l);
   if constexpr (KIND == kRotary)
     if (a.sink) {
       const float sk = a.sink[head], top = fmaxf(m, sk);
       const float f = base2 ? exp2f(m - top) : expf(m - top);
-      inv = __fdiv_rn(f, l * f + (base2 ? exp2f(sk - top) : expf(sk - top)));
+      inv = __fdiv_rn(a.mult * f, l * f + (base2 ? exp2f(sk - top) : expf(sk - top)));
     }
 #pragma unroll
   for (int i = 0; i < kAttnRowsMax / 256; ++i) {

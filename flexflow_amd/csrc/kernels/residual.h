@@ -4,7 +4,8 @@
 
 namespace ffmi {
 
-// x = embed[token] + pos[p] in fp32; xb (optional) the bf16 packed tiles.
+// x = embed[token] + pos[p] (pos null: the embedding alone) in fp32; xb (optional) the
+// bf16 packed tiles.
 // blob_src: the step's staging in mapped host memory, copied to blob_dst by
 // this first kernel of the step.
 hipError_t launch_embed_pos(const char *blob_src, char *blob_dst, size_t blob_bytes,
@@ -26,6 +27,27 @@ hipError_t launch_add_norm(Partials y, const float *w, float *x, uint16_t *hb, f
 // h[i] = x[rows[i]] / rms * w: bf16 packed tiles (hb) or fp32 rows (hf)
 hipError_t launch_row_norm(const char *blob, int off_rows, const float *x, const float *w,
                            uint16_t *hb, float *hf, int R, int H, int n, float eps, hipStream_t s);
+// The stream normed after every sum:
+//   x = norm(alpha x + sum of y's slabs + sum over k of wt[t][k] rows[at[t][k]]
+//            + own[t] x) w
+// rows (of experts; at < 0: none): bf16 or (rows_f32) fp32, [.][H].  Besides x: bf16
+// packed tiles (hb) and bf16 rows (hrow) of it.
+struct SumNorm {
+  Partials y;  // S == 0: none
+  const void *rows = nullptr;
+  bool rows_f32 = false;
+  const int32_t *at = nullptr;
+  const float *wt = nullptr, *own = nullptr;
+  int top = 0;
+  float alpha = 1.f, eps = 0.f;
+  const float *w = nullptr;
+  float *x = nullptr;
+  uint16_t *hb = nullptr, *hrow = nullptr;
+  int T = 0, H = 0, n = 0;  // columns, the first n of them real
+};
+hipError_t launch_sum_norm(const SumNorm &a, hipStream_t s);
+// packed bf16 rows of the columns [col, col + n) of deferred sums, n a multiple of 32
+hipError_t launch_pack_sums(const Partials &y, int col, uint16_t *out, int T, int n, hipStream_t s);
 hipError_t launch_relu2_f32(float *u, size_t n, hipStream_t s);
 // Y[T][F] = clamped_glu of gu [T][gate F | up F]
 hipError_t launch_glu_f32(const float *gu, float *Y, int T, int F, float limit, hipStream_t s);

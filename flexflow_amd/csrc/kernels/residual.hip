@@ -19,8 +19,10 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(
   for (int c = threadIdx.x; c < H / 8; c += 256) {
     f4 a, b, pa, pb;
     unpack8_bf16(*reinterpret_cast<const uint4 *>(embed + (size_t)tk.token * H + c * 8), a, b);
-    unpack8_bf16(*reinterpret_cast<const uint4 *>(pos + (size_t)tk.pos * H + c * 8), pa, pb);
-    a += pa, b += pb;
+    if (pos) {
+      unpack8_bf16(*reinterpret_cast<const uint4 *>(pos + (size_t)tk.pos * H + c * 8), pa, pb);
+      a += pa, b += pb;
+    }
     *reinterpret_cast<f4 *>(x + (size_t)t * H + c * 8) = a;
     *reinterpret_cast<f4 *>(x + (size_t)t * H + c * 8 + 4) = b;
     if (xb) *reinterpret_cast<uint4 *>(xb + act_packed_off(t, c * 8, H)) = pack8_bf16(a, b);
@@ -211,6 +213,127 @@ hipError_t launch_row_norm(const char *blob, int off_rows, const float *x, const
   if (H % 32) return hipErrorInvalidValue;
   hipLaunchKernelGGL(row_norm_kernel, dim3(R), dim3(256), 0, s,
                      reinterpret_cast<const int32_t *>(blob + off_rows), x, w, hb, hf, H, n, eps);
+  return hipGetLastError();
+}
+
+// One workgroup per row, a thread's chunks of 8 columns; all loads before the
+// reduction.
+template <int NT, int MAXC, int MAXS>
+__global__ __launch_bounds__(NT) void sum_norm_kernel(SumNorm a) {
+  constexpr int U = 4;  // expert rows in flight
+  __shared__ float sh[NT / 64];
+  const int row = blockIdx.x, H = a.H, nchunk = H >> 3;
+  f4 x[MAXC][2], wv[MAXC][2];
+  float ss = 0.f;
+  const float alpha = a.own ? a.alpha + a.own[row] : a.alpha;
+  const int32_t *at = a.rows ? a.at + (size_t)row * a.top : nullptr;
+  const float *wt = a.rows ? a.wt + (size_t)row * a.top : nullptr;
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = min((int)threadIdx.x + c * NT, nchunk - 1);
+    f4 p[MAXS ? MAXS : 1][2];
+#pragma unroll
+    for (int sl = 0; sl < MAXS; ++sl) {
+      const float *q = a.y.p + (size_t)row * a.y.NP + ch * 8 + (size_t)min(sl, a.y.S - 1) * a.T * a.y.NP;
+      p[sl][0] = *reinterpret_cast<const f4 *>(q), p[sl][1] = *reinterpret_cast<const f4 *>(q + 4);
+    }
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      x[c][h] = *reinterpret_cast<const f4 *>(a.x + (size_t)row * H + ch * 8 + 4 * h) * alpha;
+      wv[c][h] = *reinterpret_cast<const f4 *>(a.w + ch * 8 + 4 * h);
+    }
+    f4 y[2];
+    y[0] = y[1] = f4{0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; at && k0 < a.top; k0 += U) {
+      f4 r[U][2];
+      float w[U];
+#pragma unroll
+      for (int k = 0; k < U; ++k) {
+        const int kk = min(k0 + k, a.top - 1), slot = at[kk];
+        w[k] = k0 + k < a.top && slot >= 0 ? wt[kk] : 0.f;
+        const size_t o = (size_t)max(slot, 0) * H + ch * 8;
+        if (a.rows_f32) {
+          const float *q = (const float *)a.rows + o;
+          r[k][0] = *reinterpret_cast<const f4 *>(q), r[k][1] = *reinterpret_cast<const f4 *>(q + 4);
+        } else {
+          unpack8_bf16(*reinterpret_cast<const uint4 *>((const uint16_t *)a.rows + o), r[k][0], r[k][1]);
+        }
+      }
+#pragma unroll
+      for (int k = 0; k < U; ++k)
+        if (w[k] != 0.f) y[0] += r[k][0] * w[k], y[1] += r[k][1] * w[k];
+    }
+#pragma unroll
+    for (int sl = 0; sl < MAXS; ++sl)
+      if (sl < a.y.S) y[0] += p[sl][0], y[1] += p[sl][1];
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      x[c][h] += y[h];
+      if ((int)threadIdx.x + c * NT < nchunk)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss = fmaf(x[c][h][e], x[c][h][e], ss);
+    }
+  }
+  const float r = inv_rms(row_sum<NT>(ss, sh), a.n, a.eps);
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = threadIdx.x + c * NT;
+    if (ch >= nchunk) continue;
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) x[c][h][e] = x[c][h][e] * r * wv[c][h][e];
+      *reinterpret_cast<f4 *>(a.x + (size_t)row * H + ch * 8 + 4 * h) = x[c][h];
+    }
+    const uint4 b = pack8_bf16(x[c][0], x[c][1]);
+    if (a.hb) *reinterpret_cast<uint4 *>(a.hb + act_packed_off(row, ch * 8, H)) = b;
+    if (a.hrow) *reinterpret_cast<uint4 *>(a.hrow + (size_t)row * H + ch * 8) = b;
+  }
+}
+hipError_t launch_sum_norm(const SumNorm &a, hipStream_t s) {
+  if (a.T <= 0) return hipSuccess;
+  if (a.H % 32 || !a.x || !a.w || a.y.S < 0 || a.y.S > 8 || (a.y.S > 0 && (a.y.NP < a.H || a.y.NP % 4)) ||
+      (a.rows && (a.top < 1 || !a.at || !a.wt)))
+    return hipErrorInvalidValue;
+  const int nchunk = a.H / 8;
+#define FFMI_SM(NT, MC, MS) hipLaunchKernelGGL((sum_norm_kernel<NT, MC, MS>), dim3(a.T), dim3(NT), 0, s, a)
+#define FFMI_SMS(NT, MC)                 \
+  do {                                   \
+    if (a.y.S == 0) FFMI_SM(NT, MC, 0);  \
+    else if (a.y.S == 1) FFMI_SM(NT, MC, 1); \
+    else if (a.y.S <= 4) FFMI_SM(NT, MC, 4); \
+    else FFMI_SM(NT, MC, 8);             \
+  } while (0)
+  if (nchunk <= 128) FFMI_SMS(128, 1);
+  else if (nchunk <= 256) FFMI_SMS(256, 1);
+  else if (nchunk <= 512) FFMI_SMS(512, 1);
+  else if (nchunk <= 1024) FFMI_SMS(1024, 1);
+  else if (nchunk <= 2048) FFMI_SMS(1024, 2);
+  else return hipErrorInvalidValue;
+#undef FFMI_SMS
+#undef FFMI_SM
+  return hipGetLastError();
+}
+
+__global__ __launch_bounds__(256) void pack_sums_kernel(Partials y, int col, uint16_t *__restrict__ out, int T,
+                                                        int n) {
+  const int n8 = n >> 3;
+  const long id = blockIdx.x * 256L + threadIdx.x;
+  if (id >= (long)T * n8) return;
+  const int t = (int)(id / n8), c = (int)(id % n8) * 8;
+  const float *p = y.p + (size_t)t * y.NP + col + c;
+  f4 lo = *reinterpret_cast<const f4 *>(p), hi = *reinterpret_cast<const f4 *>(p + 4);
+  for (int s = 1; s < y.S; ++s) {
+    const float *ps = p + (size_t)s * T * y.NP;
+    lo += *reinterpret_cast<const f4 *>(ps), hi += *reinterpret_cast<const f4 *>(ps + 4);
+  }
+  *reinterpret_cast<uint4 *>(out + act_packed_off(t, c, n)) = pack8_bf16(lo, hi);
+}
+hipError_t launch_pack_sums(const Partials &y, int col, uint16_t *out, int T, int n, hipStream_t s) {
+  if (T <= 0) return hipSuccess;
+  if (n <= 0 || n % 32 || col % 4 || y.NP % 4 || y.S < 1 || col + n > y.NP) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(pack_sums_kernel, dim3((unsigned)(((long)T * (n / 8) + 255) / 256)), dim3(256), 0, s, y, col,
+                     out, T, n);
   return hipGetLastError();
 }
 

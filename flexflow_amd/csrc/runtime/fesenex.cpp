@@ -239,13 +239,7 @@ struct Fesenex : public PagedDecoder {
     if (!L.ff) return FFMI_OK;
     FFMI_TRY(vec(&L.norm2, p + "norm2", 1, W, Wp));
     FFMI_TRY(alloc(&L.wgu, (size_t)2 * L.fp * Wp * es()));
-    const PackSpec gu = spec(1, L.ff, L.fp, 1, W, Wp);
-    for (int k = 0; k < 2; ++k) {  // bf16: gate and up tiles in turn
-      FFMI_TRY(raw(p + (k ? "mlp.up" : "mlp.gate"), {L.ff, W}));
-      if (f32) FFMI_TRY(pack_rows(gu, W, L.wgu, k * L.fp, 2 * L.fp));
-      else
-        FFMI_HIP(launch_pack_bf16(raw_tensor(), W, gu, (uint16_t *)L.wgu, k, 2 * L.fp / 16, false, stream, 2));
-    }
+    FFMI_TRY(gate_up(L.wgu, p + "mlp.", L.ff, L.fp));
     return linear(&L.wdown, p + "mlp.down", W, Wp, 1, L.ff, L.fp);
   }
   // the bias of every distance, per head, in the attention's order (AttnArgs)

@@ -89,9 +89,7 @@ struct Nomutar : public PagedDecoder {
   float *x2 = nullptr, *xs[2] = {}, *rms = nullptr;
   void *c = nullptr, *q = nullptr, *cat = nullptr;
   uint16_t *hrow = nullptr;
-  void *eu = nullptr, *ey = nullptr;
   float *slabs = nullptr, *ml = nullptr;
-  MoeLists moe;
 
   // ---- configuration ----
   ffmi_status configure_rotation(const Json &r, const std::string &at, NomutarLayer *L) {
@@ -208,7 +206,7 @@ struct Nomutar : public PagedDecoder {
 
   // ---- buffers and weights ----
   ffmi_status init_layers() override {
-    size_t qw = 32, cw = 32, units = 0, slots = 0, picks = 0, tiles = 0;
+    size_t qw = 32, cw = 32;
     double wbytes = 0;
     int min_groups = 1 << 30;
     std::vector<RowShape> shapes;
@@ -236,12 +234,7 @@ struct Nomutar : public PagedDecoder {
       L.nr = up(L.gate_col + 1, 32);
       gemms.push_back({L.nr, Wp});
       wbytes += 6.0 * Wp * L.experts * L.efp;
-      for (int t = 1; t <= Tm; ++t) {
-        const MoeSizes n = sizes(L, t);
-        units = std::max(units, (size_t)n.slots() * L.efp);
-        slots = std::max(slots, (size_t)n.slots()), picks = std::max(picks, (size_t)t * L.top);
-        tiles = std::max(tiles, (size_t)(n.expert_tiles(n.tile_rows()) + n.shared_tiles(n.tile_rows())));
-      }
+      need_experts(sizes(L, 0), L.efp);
     }
     // 16-row slots for the splits of a step whose blocks do not fill the chip
     max_slots = rows_form ? 0 : 512 * kAttnTiles / min_groups;
@@ -252,18 +245,8 @@ struct Nomutar : public PagedDecoder {
     FFMI_TRY(alloc_zero(&c, (size_t)Tm * Wp * es()));
     FFMI_TRY(alloc_zero(&q, (size_t)Tm * qw * es()));
     FFMI_TRY(alloc_zero(&cat, (size_t)Tm * cw * es()));
-    if (slots) {
-      if (!f32) FFMI_TRY(alloc_zero(&hrow, (size_t)Tm * Wp * 2));
-      FFMI_TRY(alloc_zero(&eu, units * es()));
-      FFMI_TRY(alloc_zero(&ey, slots * Wp * es()));
-      FFMI_TRY(alloc_zero(&moe.picked, picks * 4));
-      FFMI_TRY(alloc_zero(&moe.at, picks * 4));
-      FFMI_TRY(alloc_zero(&moe.wt, picks * 4));
-      FFMI_TRY(alloc_zero(&moe.gate, (size_t)Tm * 4));
-      FFMI_TRY(alloc_zero(&moe.slot_token, slots * 4));
-      FFMI_TRY(alloc_zero(&moe.tiles, tiles * sizeof(MoeTile)));
-      FFMI_TRY(alloc_zero(&moe.num_tiles, 16));
-    }
+    if (moe.num_slots && !f32) FFMI_TRY(alloc_zero(&hrow, (size_t)Tm * Wp * 2));
+    FFMI_TRY(alloc_experts());
     size_t part = 0, rows = 0;
     for (NomutarRun &r : runs) {
       const NomutarLayer &L = layers[r.layer];
@@ -291,12 +274,6 @@ struct Nomutar : public PagedDecoder {
     n.T = T, n.experts = L.experts, n.top = L.top, n.shared = L.sff > 0, n.gate_col = L.gate_col;
     return n;
   }
-  template <class T>
-  ffmi_status upload(T **dst, const std::vector<T> &v) {
-    FFMI_TRY(alloc(dst, v.size() * sizeof(T)));
-    if (!v.empty()) FFMI_HIP(hipMemcpy(*dst, v.data(), v.size() * sizeof(T), hipMemcpyHostToDevice));
-    return FFMI_OK;
-  }
   // rows of the first product's weight: `heads` of n rows, padded to np
   ffmi_status in_rows(NomutarLayer &L, const std::string &name, int heads, int n, int np, int pairs, int row0) {
     FFMI_TRY(raw(name, {(long)heads * n, W}));
@@ -310,15 +287,6 @@ struct Nomutar : public PagedDecoder {
     PackSpec p = spec(heads, 1, 1, 1, n, np);
     p.col_pairs = pairs;
     FFMI_HIP(launch_pack_f32(raw_tensor(), n, p, dst, stream));
-    return FFMI_OK;
-  }
-  ffmi_status gate_up(void *dst, const std::string &p, int ff, int fp) {
-    const PackSpec gu = spec(1, ff, fp, 1, W, Wp);
-    for (int k = 0; k < 2; ++k) {  // bf16: gate and up tiles in turn
-      FFMI_TRY(raw(p + (k ? "up" : "gate"), {ff, W}));
-      if (f32) FFMI_TRY(pack_rows(gu, W, dst, k * fp, 2 * fp));
-      else FFMI_HIP(launch_pack_bf16(raw_tensor(), W, gu, (uint16_t *)dst, k, 2 * fp / 16, false, stream, 2));
-    }
     return FFMI_OK;
   }
   ffmi_status load_layer(const std::string &p, NomutarLayer &L) {
@@ -353,15 +321,9 @@ struct Nomutar : public PagedDecoder {
     if (L.type->sink) {
       std::vector<float> s(H, 0.f);
       if (L.type->learned_sink) {
-        FFMI_TRY(raw(m + "sink", {H}));
-        FFMI_HIP(hipStreamSynchronize(stream));
-        std::vector<uint16_t> t(H);
-        FFMI_HIP(hipMemcpy(t.data(), raw_tensor(), t.size() * 2, hipMemcpyDeviceToHost));
-        for (int i = 0; i < H; ++i) {
-          const uint32_t bits = (uint32_t)t[i] << 16;
-          memcpy(&s[i], &bits, 4);
-          if (!f32) s[i] *= kLog2e;
-        }
+        FFMI_TRY(host_vec(&s, m + "sink", H));
+        if (!f32)
+          for (float &v : s) v *= kLog2e;
       }
       FFMI_TRY(upload(&L.sink, s));
     }
@@ -389,15 +351,7 @@ struct Nomutar : public PagedDecoder {
     FFMI_TRY(raw(f + "router", {L.experts, W}));
     FFMI_TRY(pack_rows(spec(1, L.experts, L.gate_col, 1, W, Wp), W, L.wrouter, 0, L.nr));
     FFMI_TRY(vec(&L.rbias, f + "router.b", 1, L.experts, L.gate_col));
-    const size_t gu = (size_t)2 * L.efp * Wp * es(), dn = (size_t)Wp * L.efp * es();
-    FFMI_TRY(alloc(&L.egu, gu * L.experts));
-    FFMI_TRY(alloc(&L.edown, dn * L.experts));
-    for (int e = 0; e < L.experts; ++e) {
-      const std::string p = f + "e" + std::to_string(e) + ".";
-      FFMI_TRY(gate_up((char *)L.egu + gu * e, p, L.eff, L.efp));
-      FFMI_TRY(raw(p + "down", {W, L.eff}));
-      FFMI_TRY(pack_rows(spec(1, W, Wp, 1, L.eff, L.efp), L.eff, (char *)L.edown + dn * e, 0, Wp));
-    }
+    FFMI_TRY(expert_matrices(f, L.experts, L.eff, L.efp, &L.egu, &L.edown));
     if (!L.sff) return FFMI_OK;
     FFMI_TRY(raw(f + "shared.sg", {1, W}));
     return pack_rows(spec(1, 1, 16, 1, W, Wp), W, L.wrouter, L.gate_col, L.nr);
@@ -451,15 +405,16 @@ struct Nomutar : public PagedDecoder {
     const MoeSizes n = sizes(L, step.T);
     Partials z;
     FFMI_TRY(gemm_sum(h, L.wrouter, L.nr, Wp, &z));
-    FFMI_HIP(launch_moe_route(z, L.rbias, n, moe, stream));
+    FFMI_HIP(launch_moe_route(z, L.rbias, n, moe.lists, stream));
     MoeGemm a;
-    a.experts = L.experts, a.slot_token = moe.slot_token, a.tiles = moe.tiles, a.num_tiles = moe.num_tiles;
-    a.gate = moe.gate;
+    const MoeLists &l = moe.lists;
+    a.experts = L.experts, a.slot_token = l.slot_token, a.tiles = l.tiles, a.num_tiles = l.num_tiles;
+    a.gate = l.gate;
     const void *rows = f32 ? h : hrow;
-    a.g[0] = {rows, L.egu, eu, L.efp, Wp, L.efp, (size_t)2 * L.efp * Wp};
+    a.g[0] = {rows, L.egu, moe.units, L.efp, Wp, L.efp, (size_t)2 * L.efp * Wp};
     a.g[1] = {rows, L.wgu, units_of(L), L.fp, Wp, L.na + L.fp, 0};
     FFMI_HIP(launch_moe_gemm(a, n, true, f32, wstream != 0, stream));
-    a.g[0] = {eu, L.edown, ey, Wp, L.efp, 0, (size_t)L.efp * Wp};
+    a.g[0] = {moe.units, L.edown, moe.rows, Wp, L.efp, 0, (size_t)L.efp * Wp};
     FFMI_HIP(launch_moe_gemm(a, n, false, f32, wstream != 0, stream));
     return FFMI_OK;
   }
@@ -469,7 +424,7 @@ struct Nomutar : public PagedDecoder {
     n.H = Wp, n.n = W, n.groups = groups, n.eps = eps, n.mult = mult, n.w = w, n.x_in = xs[0], n.inv = rms;
     if (prev) n.y = y;
     if (prev && prev->experts) {
-      n.rows = ey, n.rows_f32 = f32, n.at = moe.at, n.wt = moe.wt, n.top = prev->top;
+      n.rows = moe.rows, n.rows_f32 = f32, n.at = moe.lists.at, n.wt = moe.lists.wt, n.top = prev->top;
     }
     return n;
   }

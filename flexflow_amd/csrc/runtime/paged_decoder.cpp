@@ -105,6 +105,66 @@ ffmi_status PagedDecoder::linear(void **dst, const std::string &name, int nb, in
   return pack_rows(spec(1, nb, np, cols, kb, kp), cols * kb, *dst, 0, np);
 }
 
+ffmi_status PagedDecoder::host_vec(std::vector<float> *v, const std::string &name, int n, int kind) {
+  FFMI_TRY(raw(name, {n}, kind));
+  FFMI_HIP(hipStreamSynchronize(stream));
+  std::vector<uint16_t> t(n);
+  FFMI_HIP(hipMemcpy(t.data(), tmp, t.size() * 2, hipMemcpyDeviceToHost));
+  v->resize(n);
+  for (int i = 0; i < n; ++i) {
+    const uint32_t bits = (uint32_t)t[i] << 16;
+    memcpy(&(*v)[i], &bits, 4);
+  }
+  return FFMI_OK;
+}
+
+ffmi_status PagedDecoder::gate_up(void *dst, const std::string &p, int ff, int fp) {
+  const PackSpec gu = spec(1, ff, fp, 1, W, Wp);
+  for (int k = 0; k < 2; ++k) {  // bf16: gate and up tiles in turn
+    FFMI_TRY(raw(p + (k ? "up" : "gate"), {ff, W}));
+    if (f32) FFMI_TRY(pack_rows(gu, W, dst, k * fp, 2 * fp));
+    else FFMI_HIP(launch_pack_bf16(tmp, W, gu, (uint16_t *)dst, k, 2 * fp / 16, false, stream, 2));
+  }
+  return FFMI_OK;
+}
+
+ffmi_status PagedDecoder::expert_matrices(const std::string &p, int experts, int ff, int fp, void **gated,
+                                          void **down) {
+  const size_t gu = (size_t)2 * fp * Wp * es(), dn = (size_t)Wp * fp * es();
+  FFMI_TRY(alloc(gated, gu * experts));
+  FFMI_TRY(alloc(down, dn * experts));
+  for (int e = 0; e < experts; ++e) {
+    const std::string pe = p + "e" + std::to_string(e) + ".";
+    FFMI_TRY(gate_up((char *)*gated + gu * e, pe, ff, fp));
+    FFMI_TRY(raw(pe + "down", {W, ff}));
+    FFMI_TRY(pack_rows(spec(1, W, Wp, 1, ff, fp), ff, (char *)*down + dn * e, 0, Wp));
+  }
+  return FFMI_OK;
+}
+
+void PagedDecoder::need_experts(MoeSizes n, int fp) {
+  for (n.T = 1; n.T <= Tm; ++n.T) {
+    moe.num_units = std::max(moe.num_units, (size_t)n.slots() * fp);
+    moe.num_slots = std::max(moe.num_slots, (size_t)n.slots());
+    moe.num_picks = std::max(moe.num_picks, (size_t)n.T * n.top);
+    moe.num_tiles = std::max(moe.num_tiles, (size_t)(n.expert_tiles(n.tile_rows()) + n.shared_tiles(n.tile_rows())));
+  }
+}
+ffmi_status PagedDecoder::alloc_experts() {
+  if (!moe.num_slots) return FFMI_OK;
+  MoeLists &l = moe.lists;
+  FFMI_TRY(alloc_zero(&moe.units, moe.num_units * es()));
+  FFMI_TRY(alloc_zero(&moe.rows, moe.num_slots * Wp * es()));
+  FFMI_TRY(alloc_zero(&l.picked, moe.num_picks * 4));
+  FFMI_TRY(alloc_zero(&l.at, moe.num_picks * 4));
+  FFMI_TRY(alloc_zero(&l.wt, moe.num_picks * 4));
+  FFMI_TRY(alloc_zero(&l.gate, (size_t)Tm * 4));
+  FFMI_TRY(alloc_zero(&l.own, (size_t)Tm * 4));
+  FFMI_TRY(alloc_zero(&l.slot_token, moe.num_slots * 4));
+  FFMI_TRY(alloc_zero(&l.tiles, moe.num_tiles * sizeof(MoeTile)));
+  return alloc_zero(&l.num_tiles, 16);
+}
+
 ffmi_status PagedDecoder::vec(float **dst, const std::string &name, int rows, int n, int np, int kind) {
   FFMI_TRY(alloc(dst, (size_t)rows * np * 4));
   return vec_to(*dst, name, rows, n, np, kind);
@@ -137,7 +197,7 @@ ffmi_status PagedDecoder::init() {
   Wp = up(W, 32), Vp = up(V, 32);
   FFMI_TRY(init_layers());
   FFMI_TRY(table(&embed, "embed", V));
-  FFMI_TRY(vec(&final_norm, "final.norm", 1, W, Wp));
+  FFMI_TRY(load_final());
   FFMI_TRY(linear(&head, "head", V, Vp, 1, W, Wp));
   FFMI_HIP(hipStreamSynchronize(stream));
   if (tmp) (void)hipFree(tmp);
@@ -160,12 +220,7 @@ ffmi_status PagedDecoder::init_step(const std::vector<RowShape> &shapes, int max
   FFMI_TRY(alloc_zero(&h, (size_t)Tm * Wp * es()));
   FFMI_TRY(alloc(&logits, (size_t)Tm * Vp * 4));
   ws_bytes = std::max(ws_bytes, (size_t)Tm * Wp * 4);
-  for (const auto &g : gemms) {
-    ws_bytes = std::max(ws_bytes, (size_t)Tm * g.first * 4);
-    if (!f32)
-      for (int t = 16; t <= Tm; t += 16)
-        ws_bytes = std::max(ws_bytes, gemm_bf16_workspace_bytes(t, g.first, g.second));
-  }
+  for (const auto &g : gemms) ws_bytes = std::max(ws_bytes, sum_bytes(g.first, g.second));
   FFMI_TRY(alloc(&ws, ws_bytes));
   FFMI_HIP(hipHostMalloc((void **)&res_h, (size_t)Tm * 8,
                          hipHostMallocCoherent | hipHostMallocMapped));
@@ -173,13 +228,21 @@ ffmi_status PagedDecoder::init_step(const std::vector<RowShape> &shapes, int max
 }
 
 // ---- one step ----
-ffmi_status PagedDecoder::gemm_sum(const void *X, const void *Wt, int N, int K, Partials *y) {
+size_t PagedDecoder::sum_bytes(int N, int K) const {
+  size_t n = (size_t)Tm * N * 4;
+  if (!f32)
+    for (int t = 16; t <= Tm; t += 16) n = std::max(n, gemm_bf16_workspace_bytes(t, N, K));
+  return n;
+}
+
+ffmi_status PagedDecoder::gemm_sum_to(const void *X, const void *Wt, int N, int K, Partials *y, float *to,
+                                      size_t to_bytes) {
   if (f32) {
-    FFMI_HIP(launch_gemm_f32((const float *)X, (const float *)Wt, ws, step.T, N, K, stream));
-    y->p = ws, y->S = 1, y->NP = N;
+    FFMI_HIP(launch_gemm_f32((const float *)X, (const float *)Wt, to, step.T, N, K, stream));
+    y->p = to, y->S = 1, y->NP = N;
     return FFMI_OK;
   }
-  FFMI_HIP(launch_gemm_bf16_f32((const uint16_t *)X, (const uint16_t *)Wt, nullptr, ws, ws_bytes,
+  FFMI_HIP(launch_gemm_bf16_f32((const uint16_t *)X, (const uint16_t *)Wt, nullptr, to, to_bytes,
                                 step.T, N, K, FFMI_X_PACKED | wstream, stream, y));
   return FFMI_OK;
 }

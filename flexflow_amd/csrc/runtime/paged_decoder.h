@@ -10,6 +10,7 @@
 #include <string>
 #include <vector>
 
+#include "../kernels/moe.h"
 #include "../kernels/packing.h"
 #include "../kernels/residual.h"
 #include "json.h"
@@ -37,6 +38,8 @@ struct PagedDecoder : public ffmi_model {
   virtual ffmi_status run_layers() = 0;
   // the output product's rows: h = norm(x) of the step's output rows
   virtual ffmi_status output_rows();
+  // "final.norm"
+  virtual ffmi_status load_final() { return vec(&final_norm, "final.norm", 1, W, Wp); }
 
   ffmi_model_opts o{};
   std::string folder;
@@ -113,10 +116,37 @@ struct PagedDecoder : public ffmi_model {
   // [rows][W] table, bf16 rows of Wp
   ffmi_status table(uint16_t **dst, const std::string &name, int rows);
   const uint16_t *raw_tensor() const { return tmp; }
+  // a vector's n values on the host
+  ffmi_status host_vec(std::vector<float> *v, const std::string &name, int n, int kind = 0);
+  template <class T>
+  ffmi_status upload(T **dst, const std::vector<T> &v) {
+    FFMI_TRY(alloc(dst, v.size() * sizeof(T)));
+    if (!v.empty()) FFMI_HIP(hipMemcpy(*dst, v.data(), v.size() * sizeof(T), hipMemcpyHostToDevice));
+    return FFMI_OK;
+  }
+  // "<p>gate" and "<p>up" [ff][W] as one gated product's weight
+  ffmi_status gate_up(void *dst, const std::string &p, int ff, int fp);
+  // "<p>e0.", "<p>e1.", ...: the experts' gated and down matrices, expert after expert
+  ffmi_status expert_matrices(const std::string &p, int experts, int ff, int fp, void **gated, void **down);
+
+  // ---- mixture of experts: a step's buffers, sized for every layer (kernels/moe.h) ----
+  struct ExpertBuffers {
+    void *units = nullptr, *rows = nullptr;  // the first product's, the second's
+    MoeLists lists;
+    size_t num_units = 0, num_slots = 0, num_picks = 0, num_tiles = 0;
+  } moe;
+  // room for a layer's steps of 1 .. Tm tokens (n: its sizes, T aside; fp: padded units)
+  void need_experts(MoeSizes n, int fp);
+  ffmi_status alloc_experts();
 
   // ---- steps ----
   // y (fp32 sums) = X . W^T
-  ffmi_status gemm_sum(const void *X, const void *Wt, int N, int K, Partials *y);
+  ffmi_status gemm_sum(const void *X, const void *Wt, int N, int K, Partials *y) {
+    return gemm_sum_to(X, Wt, N, K, y, ws, ws_bytes);
+  }
+  ffmi_status gemm_sum_to(const void *X, const void *Wt, int N, int K, Partials *y, float *to, size_t to_bytes);
+  // least bytes of the sums of a product with N columns
+  size_t sum_bytes(int N, int K) const;
   ffmi_status capture_layer(int i) { return capture(i, x); }  // (tensor capture) x after layer i
   ffmi_status capture(int i, const float *rows);
   bool capturing() const { return dbg != 0; }
