@@ -190,3 +190,13 @@ def forward(cfg, w, tokens, layers=None):
         if layers is not None:
             layers.append(x)
     return zero_centred_norm(x, w["final.norm"], eps) @ w["head"].T
+
+
+def greedy(cfg, w, prompt, length):
+    """(tokens up to `length`, the smallest lead of a pick over the runner-up)"""
+    toks, lead = list(prompt), np.inf
+    while len(toks) < length:
+        z = np.sort(forward(cfg, w, toks)[-1])
+        lead = min(lead, z[-1] - z[-2])
+        toks.append(int(forward(cfg, w, toks)[-1].argmax()))
+    return toks, lead
