@@ -332,6 +332,28 @@ def nomutar_config(width, heads, kv_heads, dim, ff, layers, vocab=32000):
                 layers=[one(i) for i in range(layers)])
 
 
+# --model pekarax: (name, width, heads, key/value heads, head size, ff, layers)
+PEKARAX_SIZES = NOMUTAR_SIZES
+
+
+def pekarax_config(width, heads, kv_heads, dim, ff, layers, vocab=32000):
+    """Two delta-rule layers, one of attention beside a normalised memory, one gated
+    memory with few wide heads, and so on; Nomutar's experts, without a shared one and with
+    identity experts, in every layer."""
+    wide = max(1, heads // 4)
+    mixers = {"channel_delta": dict(heads=heads, kv_heads=heads, dim=dim, vdim=dim, conv=4),
+              "parallel": dict(left_scale=0.8, right_scale=0.5,
+                               left=dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=1.0, conv=4,
+                                         rot=dict(base=500000.0, dims=dim)),
+                               right=dict(heads=wide, dim=dim, vdim=2 * dim, gate_cap=15.0)),
+              "gla": dict(heads=wide, dim=2 * dim, vdim=4 * dim, tau=16.0)}
+    mlp = dict(kind="moe", expert=dict(ff=(ff // 8 + 31) // 32 * 32, limit=7.0),
+               router=dict(experts=32, identity=4, top=4, groups=dict(count=4, keep=2), scale=2.5))
+    kinds = ("channel_delta", "channel_delta", "parallel", "gla")
+    return dict(architecture="Pekarax", vocab=vocab, width=width, norm=dict(eps=1e-6), postln_alpha=3.0,
+                layers=[dict(type=kinds[i % 4], mixer=mixers[kinds[i % 4]], mlp=mlp) for i in range(layers)])
+
+
 def bench_decoder(cfg, B, prompt_len, decode, mtb, repeats):
     """Prefill and decode throughput of incremental decoding: generates of one
     new token (the prompts' steps alone) and of `decode`, best of `repeats`."""
@@ -362,11 +384,12 @@ def bench_decoder(cfg, B, prompt_len, decode, mtb, repeats):
 
 
 def bench_family(args):
-    """--model vapipel | fesenex | nomutar: the family's decoder (random weights) and
-    LLaMA (nomutar: Fesenex too) at equal sizes, incremental decoding, one GPU.  One
-    JSON line."""
+    """--model vapipel | fesenex | nomutar | pekarax: the family's decoder (random weights)
+    and LLaMA (nomutar: Fesenex too; pekarax: Nomutar and Fesenex) at equal sizes,
+    incremental decoding, one GPU.  One JSON line."""
     legs = []
-    sizes = {"vapipel": VAPIPEL_SIZES, "fesenex": FESENEX_SIZES, "nomutar": NOMUTAR_SIZES}[args.model]
+    sizes = {"vapipel": VAPIPEL_SIZES, "fesenex": FESENEX_SIZES, "nomutar": NOMUTAR_SIZES,
+             "pekarax": PEKARAX_SIZES}[args.model]
     for name, width, heads, *more, ff, layers in sizes:
         if args.only_size and name != args.only_size:
             continue
@@ -377,8 +400,10 @@ def bench_family(args):
             kv_heads, dim = more
             grouped = (width, heads, kv_heads, dim, ff, layers)
             leg0, cfgs = {"kv_heads": kv_heads}, {"fesenex": fesenex_config(*grouped)}
-            if args.model == "nomutar":
+            if args.model in ("nomutar", "pekarax"):
                 cfgs = {"nomutar": nomutar_config(*grouped), **cfgs}
+            if args.model == "pekarax":
+                cfgs = {"pekarax": pekarax_config(*grouped), **cfgs}
         cfgs["llama"] = dict(num_layers=layers, vocab_size=32000, num_heads=heads, num_kv_heads=heads,
                              hidden=width, intermediate=ff, rms_eps=1e-6, rope_theta=10000.0)
         for prompt in (args.prefill, 1024):
@@ -395,8 +420,9 @@ def bench_family(args):
     head = legs[-1][ran]
     what = {"vapipel": "latent-attention decoder",
             "fesenex": "softmax- and linear-attention decoder",
-            "nomutar": "decoder of parallel layers with experts"}[args.model]
-    beside = "Fesenex and LLaMA" if args.model == "nomutar" else "LLaMA"
+            "nomutar": "decoder of parallel layers with experts",
+            "pekarax": "decoder of matrix memories with experts"}[args.model]
+    beside = {"nomutar": "Fesenex and LLaMA", "pekarax": "Nomutar, Fesenex and LLaMA"}.get(args.model, "LLaMA")
     print(json.dumps({
         "metric": f"decode tokens/s, {what} beside {beside} at equal size",
         "value": head["decode_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
@@ -487,12 +513,12 @@ def main():
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
     ap.add_argument("--mode", choices=["spec", "incr"], default="spec")
-    ap.add_argument("--model", choices=["llama", "vapipel", "fesenex", "nomutar"], default="llama",
-                    help="llama: the headline workload; vapipel, fesenex, nomutar: prefill and decode throughput "
-                         "of that family's decoder beside LLaMA at equal sizes (one GPU)")
-    ap.add_argument("--only-family", choices=["llama", "vapipel", "fesenex", "nomutar"], default=None,
-                    help="--model vapipel | fesenex | nomutar: run one of the models (profiling)")
-    ap.add_argument("--only-size", default=None, help="--model vapipel | fesenex | nomutar: run one size (profiling)")
+    ap.add_argument("--model", choices=["llama", "vapipel", "fesenex", "nomutar", "pekarax"], default="llama",
+                    help="llama: the headline workload; vapipel, fesenex, nomutar, pekarax: prefill and decode "
+                         "throughput of that family's decoder beside LLaMA at equal sizes (one GPU)")
+    ap.add_argument("--only-family", choices=["llama", "vapipel", "fesenex", "nomutar", "pekarax"], default=None,
+                    help="any other than --model llama: run one of the models (profiling)")
+    ap.add_argument("--only-size", default=None, help="any other than --model llama: run one size (profiling)")
     ap.add_argument("--batch", type=int, default=8)
     ap.add_argument("--prefill", type=int, default=128)
     ap.add_argument("--decode", type=int, default=128)

@@ -68,30 +68,38 @@ struct Memory {
   int ldo = 0, out_col = 0;
   int off_tokens = 0;  // the step's tokens in its metadata
 };
-constexpr int kMemoryChunk = 64;
+constexpr int kMemoryChunk = kSpanChunk;
 constexpr int kMemoryMaxDim = 512, kMemoryMaxVdim = 2048;  // token by token
 constexpr int kMemoryMaxChunkDim = 256;                    // chunks
 inline int memory_state_columns(MemoryRule r, int vdim) {
   return (vdim + (r == kMemoryNormed) + 31) / 32 * 32;
 }
 
-// token by token: spans of at most `limit` tokens, everything in one launch
-hipError_t launch_memory_steps(const char *blob, int off_spans, int num_spans, const Memory &a, bool f32,
-                               int limit, hipStream_t s);
-
-// Chunks: spans of more than `limit` tokens (bf16 model).  Scratch, from the step's
-// bounds: per (chunk, head) the operands of the pass over the chunks.
+// Scratch, from the step's bounds: per (chunk, head) the operands of the pass over the
+// chunks, per token what the launches after it take.
 struct MemoryScratch {
-  uint16_t *qg = nullptr, *kd = nullptr, *w = nullptr;  // [64][DK], [DK][64], [64][DK]
+  uint16_t *rows = nullptr;                             // delta: [T][columns of q | k | v]
+  uint16_t *qg = nullptr, *kd = nullptr, *w = nullptr;  // [64][DK], [DK][64], [64][DK] (delta)
   uint16_t *p = nullptr;                                // [64][64]
-  void *u = nullptr;                                    // [64][vs] fp32 (delta) or bf16
+  float *u = nullptr;                                   // delta: [64][vs]
   float *last = nullptr;                                // [DK]
   float *gates = nullptr;                               // normed: [T][H][3]
   float *o = nullptr;                                   // [T][H][vs]
 };
 inline int memory_chunk_width(int dg) { return dg <= 32 ? 32 : dg <= 64 ? 64 : dg <= 128 ? 128 : 256; }
+// most chunks that a step of T tokens in so many spans has
 inline size_t memory_chunks_max(int T, int spans) { return (size_t)T / kMemoryChunk + spans; }
-hipError_t launch_memory_chunks(const char *blob, int off_spans, int num_spans, const Memory &a,
+
+// Token by token: spans of at most `limit` tokens, everything in one launch, unless the
+// heads are few and wide: with scratch (w) their columns are then split, the outputs are
+// left in w.o (*left) and launch_memory_out has to follow.
+hipError_t launch_memory_steps(const char *blob, int off_spans, int num_spans, const Memory &a,
+                               const MemoryScratch *w, bool f32, int limit, bool *left, hipStream_t s);
+// Chunks (bf16 model): spans of more than `limit` >= kShortSpan tokens; num_chunks: the
+// step's (PagedSpan::chunk0 counts them).  The outputs are left in w.o.
+hipError_t launch_memory_chunks(const char *blob, int off_spans, int num_spans, int num_chunks, const Memory &a,
                                 const MemoryScratch &w, int limit, hipStream_t s);
+// norm and gate of w.o, for the tokens of spans of more than `above` tokens
+hipError_t launch_memory_out(const char *blob, const Memory &a, const MemoryScratch &w, int above, hipStream_t s);
 
 }  // namespace ffmi

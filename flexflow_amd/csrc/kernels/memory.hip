@@ -2,6 +2,7 @@
 #include "memory_util.h"
 
 #include <algorithm>
+#include <type_traits>
 
 namespace ffmi {
 
@@ -9,156 +10,236 @@ namespace {
 
 constexpr int NT = 512, NW = NT / 64;
 
-__device__ __forceinline__ float dot_part(const uint16_t *w, const float *x) {
-  const uint2 v = *reinterpret_cast<const uint2 *>(w);
-  const f4 u = *reinterpret_cast<const f4 *>(x);
-  return fmaf(__builtin_bit_cast(float, v.x << 16), u[0],
-              fmaf(__builtin_bit_cast(float, v.x & 0xffff0000u), u[1],
-                   fmaf(__builtin_bit_cast(float, v.y << 16), u[2],
-                        __builtin_bit_cast(float, v.y & 0xffff0000u) * u[3])));
-}
-__device__ __forceinline__ float dot_part(const float *w, const float *x) {
-  const f4 v = *reinterpret_cast<const f4 *>(w), u = *reinterpret_cast<const f4 *>(x);
-  return fmaf(v[0], u[0], fmaf(v[1], u[1], fmaf(v[2], u[2], v[3] * u[3])));
-}
-// rows [row0, row0 + n) of a second product, for np tokens whose inputs are in LDS
-// (x [np][r]): done(token, row, value); eight lanes a row
-template <class E, class D>
-__device__ __forceinline__ void low_rank(const LowRank &l, int row0, int n, int np, const float *x, D done) {
-  const int j = threadIdx.x & 7;
-  for (int id = threadIdx.x >> 3; id < np * n; id += NT / 8) {
-    const int t = id / n, c = id - t * n;
-    const E *w = (const E *)l.w + (size_t)(row0 + c) * l.r + j * 4;
-    float v = 0.f;
-    for (int k = 0; k < l.r; k += 32) v += dot_part(w + k, x + t * l.r + j * 4 + k);
-#pragma unroll
-    for (int o = 1; o < 8; o <<= 1) v += __shfl_xor(v, o);
-    if (j == 0) done(t, c, v);
+// 8 elements of a row in registers, and their product with 8 fp32 values
+struct Row8 {
+  uint4 v;
+  __device__ __forceinline__ void load(const uint16_t *p) { v = *reinterpret_cast<const uint4 *>(p); }
+  __device__ __forceinline__ float dot(const float *x) const {
+    f4 a, b;
+    unpack8_bf16(v, a, b);
+    const f4 u = *reinterpret_cast<const f4 *>(x), w = *reinterpret_cast<const f4 *>(x + 4);
+    return fmaf(a[0], u[0], fmaf(a[1], u[1], fmaf(a[2], u[2], a[3] * u[3]))) +
+           fmaf(b[0], w[0], fmaf(b[1], w[1], fmaf(b[2], w[2], b[3] * w[3])));
   }
-}
+};
+struct Row8F {
+  f4 a, b;
+  __device__ __forceinline__ void load(const float *p) {
+    a = *reinterpret_cast<const f4 *>(p), b = *reinterpret_cast<const f4 *>(p + 4);
+  }
+  __device__ __forceinline__ float dot(const float *x) const {
+    const f4 u = *reinterpret_cast<const f4 *>(x), w = *reinterpret_cast<const f4 *>(x + 4);
+    return fmaf(a[0], u[0], fmaf(a[1], u[1], fmaf(a[2], u[2], a[3] * u[3]))) +
+           fmaf(b[0], w[0], fmaf(b[1], w[1], fmaf(b[2], w[2], b[3] * w[3])));
+  }
+};
+// A narrow second product: four lanes a row, 32 columns at a time.  The first rows' first
+// 128 columns are fetched ahead (head), before the product's input is there.
+template <class E>
+struct LowRankRows {
+  typedef typename std::conditional<sizeof(E) == 2, Row8, Row8F>::type Row;
+  static constexpr int kAhead = 4, kRows = NT / 4;
+  Row head[kAhead];
+  static __device__ __forceinline__ const E *row(const LowRank &l, int r) {
+    return (const E *)l.w + (size_t)r * l.r + (threadIdx.x & 3) * 8;
+  }
+  __device__ __forceinline__ void fetch(const LowRank &l, int row0, int n) {
+    const int c = min((int)threadIdx.x >> 2, n - 1);
+#pragma unroll
+    for (int i = 0; i < kAhead; ++i)
+      if (i * 32 < l.r) head[i].load(row(l, row0 + c) + i * 32);
+  }
+  // rows [row0, row0 + n) for np tokens whose inputs are in LDS (x [np][r])
+  template <class D>
+  __device__ __forceinline__ void run(const LowRank &l, int row0, int n, int np, const float *x, D done) {
+    const int j = threadIdx.x & 3;
+    for (int c0 = 0; c0 < n; c0 += kRows) {
+      const int c = c0 + ((int)threadIdx.x >> 2), cc = min(c, n - 1);
+      const E *w = row(l, row0 + cc);
+      Row cur[kAhead];
+#pragma unroll
+      for (int i = 0; i < kAhead; ++i) {
+        cur[i] = head[i];
+        if (c0 > 0 && i * 32 < l.r) cur[i].load(w + i * 32);
+      }
+      for (int t = 0; t < np; ++t) {
+        const float *xt = x + t * l.r + j * 8;
+        float v = 0.f;
+#pragma unroll
+        for (int i = 0; i < kAhead; ++i)
+          if (i * 32 < l.r) v += cur[i].dot(xt + i * 32);
+        for (int k = kAhead * 32; k < l.r; k += 32) {
+          Row more;
+          more.load(w + k);
+          v += more.dot(xt + k);
+        }
+        v += __shfl_xor(v, 1);
+        v += __shfl_xor(v, 2);
+        if (j == 0 && c < n) done(t, c, v);
+      }
+    }
+  }
+};
 
 // LDS of a piece of tokens, in floats
 __host__ __device__ inline int piece_floats(const Memory &a) {
   return 3 * a.dg + 2 * a.vs + a.vg + a.decay.r + a.gate.r + 8;
 }
 
-// A workgroup per (head, span).  The state's columns in slices of 4 << cw, a slice in
-// registers: thread = (4 columns, every (NT >> cw)-th row), P rows a thread; tokens in
-// pieces that fit the LDS.  Per piece: projections, convolution, gates and norms of all
-// its tokens; then slice by slice the tokens in turn, one barrier each (two sets of
-// partial sums alternate); then the outputs' norm and gate.
-template <MemoryRule RULE, class E, int P>
+// A workgroup per (head, span, part of the state's columns: `cols` of them).  The columns
+// in slices of 4 << cw, a slice in registers: thread = (4 columns, every (NT >> cw)-th
+// row), P rows a thread; tokens in pieces that fit the LDS.  Per piece: projections,
+// convolution, gates and norms of all its tokens; then slice by slice the tokens in turn,
+// one barrier each (two sets of partial sums alternate); then the outputs' norm and gate.
+// SPLIT: more than one part; outputs (and m) are left in scratch instead.
+// What memory has to give comes in the order it is waited for: narrow matrices, the
+// products' columns, the state.
+template <MemoryRule RULE, class E, int P, bool SPLIT>
 __global__ __launch_bounds__(NT) void memory_steps_kernel(const char *__restrict__ blob, int off_spans, Memory a,
-                                                          int limit, int piece, int cw) {
+                                                          MemoryScratch w, int limit, int piece, int cw, int cols) {
+  constexpr int TAPS = 4;  // up to here without a loop
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const PagedSpan sp = reinterpret_cast<const PagedSpan *>(blob + off_spans)[blockIdx.y];
   if (sp.n > limit) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x;
-  const int dg = a.dg, vs = a.vs, vg = a.vg, hq = h / (a.H / a.G);
+  const int dg = a.dg, vs = a.vs, vg = a.vg, hq = h / (a.H / a.G), bank = sp.bank;
+  const int cb = SPLIT ? blockIdx.z * cols : 0, ce = SPLIT ? min(cb + cols, vs) : vs;
   const int CW = 1 << cw, SW = CW * 4, NG = NT >> cw;
+  const int r1 = a.decay.r, r2 = SPLIT ? 0 : a.gate.r;
   float *sq = lds, *sk = sq + piece * dg, *sg = sk + piece * dg, *sv = sg + piece * dg, *so = sv + piece * vs;
-  float *sgate = so + piece * vs, *sx = sgate + piece * vg, *sx2 = sx + piece * a.decay.r;
-  float *scal = sx2 + piece * a.gate.r;  // [token][8]: beta or i, f, k . q, m, key factor, decay
+  float *sgate = so + piece * vs, *sx = sgate + piece * vg, *sx2 = sx + piece * r1;
+  float *scal = sx2 + piece * a.gate.r;  // [token][8]: beta or i, f, k . q, m
   float *red = scal + piece * 8;         // [2][2][NW][SW]
   const int cl = (tid & (CW - 1)) * 4, rg = tid >> cw;
-  const bool one = vs <= SW;  // the whole state stays in registers
+  const bool one = ce - cb <= SW;  // all the columns stay in registers
+  const bool first = h % (a.H / a.G) == 0 && cb == 0;  // (query and key heads are shared)
   float *S = a.state + ((size_t)sp.slot * a.H + h) * dg * vs;
-  const int bank = reinterpret_cast<const PagedToken *>(blob + a.off_tokens)[sp.t0].bank;
+
+  LowRankRows<E> decay, gate;
+  if constexpr (RULE != kMemoryNormed) decay.fetch(a.decay, h * a.dim, a.dim);
+  if (r2 > 0) gate.fetch(a.gate, h * a.vdim, a.vdim);
+  float nw[4];  // the norm's weights of this lane's columns
+  if constexpr (!SPLIT)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) nw[i] = a.norm[(a.norm_heads ? h * vg : 0) + min(lane + 64 * i, vg - 1)];
+  float m = 0.f;
+  if constexpr (RULE == kMemoryNormed)
+    if (sp.pos0 > 0) m = a.peak[((size_t)sp.slot * 2 + bank) * a.H + h];
+
   f4 st[P];
   auto load = [&](int c0, bool fresh) {
 #pragma unroll
     for (int p = 0; p < P; ++p) {
       const int row = p * NG + rg;
       st[p] = f4{0.f, 0.f, 0.f, 0.f};
-      if (!fresh && row < dg && c0 + cl < vs) st[p] = *reinterpret_cast<const f4 *>(S + (size_t)row * vs + c0 + cl);
+      if (!fresh && row < dg && c0 + cl < ce) st[p] = *reinterpret_cast<const f4 *>(S + (size_t)row * vs + c0 + cl);
     }
   };
   auto store = [&](int c0) {
 #pragma unroll
     for (int p = 0; p < P; ++p) {
       const int row = p * NG + rg;
-      if (row < dg && c0 + cl < vs) *reinterpret_cast<f4 *>(S + (size_t)row * vs + c0 + cl) = st[p];
+      if (row < dg && c0 + cl < ce) *reinterpret_cast<f4 *>(S + (size_t)row * vs + c0 + cl) = st[p];
     }
   };
-  if (one) load(0, sp.pos0 == 0);
-  float m = 0.f;
-  if constexpr (RULE == kMemoryNormed)
-    if (sp.pos0 > 0) m = a.peak[((size_t)sp.slot * 2 + bank) * a.H + h];
 
   const size_t slab = (size_t)a.T * a.y.NP, C = memory_columns(a);
   const int past = max(a.taps - 1, 0);
   const float *old = a.carry + ((size_t)sp.slot * 2 + bank) * past * C;
   float *now = a.carry + ((size_t)sp.slot * 2 + (bank ^ 1)) * past * C;
-  // column c of q | k | v for token t of the span; keep: this workgroup carries it on
-  auto project = [&](int t, int c, bool keep) {
-    const size_t at = (size_t)(sp.t0 + t) * a.y.NP + a.col + c;
-    const float u = sum_at(a.y, slab, at);
+  // column c of q | k | v for token t of the span, u its product; keep: it is carried on
+  auto project = [&](int t, int c, float u, bool keep) {
     float v = u;
     if (a.taps > 0) {
-      if (keep) {
-        const int ahead = sp.n - 1 - t;
-        if (ahead < past) now[ahead * C + c] = u;
-        if (t == 0)  // (a short span: earlier rows move on)
+      const size_t at = (size_t)(sp.t0 + t) * a.y.NP + a.col + c;
+      const auto before = [&](int d) {  // d tokens back
+        if (t < d) return old[(d - t - 1) * C + c];
+        return sum_at(a.y, slab, at - (size_t)d * a.y.NP);
+      };
+      const int n = min(past, sp.pos0 + t);
+      v = u * a.conv[past * C + c];
+      if (past < TAPS) {
+        float x[TAPS - 1], cv[TAPS - 1];
+#pragma unroll
+        for (int d = 1; d < TAPS; ++d) {
+          x[d - 1] = cv[d - 1] = 0.f;
+          if (d <= n) x[d - 1] = before(d), cv[d - 1] = a.conv[(past - d) * C + c];
+        }
+        if (keep && t == 0)  // (a short span: earlier rows move on)
+#pragma unroll
+          for (int d = 1; d < TAPS; ++d)
+            if (sp.n + d - 1 < past) now[(sp.n + d - 1) * C + c] = x[d - 1];
+#pragma unroll
+        for (int d = 1; d < TAPS; ++d) v = fmaf(x[d - 1], cv[d - 1], v);
+      } else {
+        for (int d = 1; d <= n; ++d) v = fmaf(before(d), a.conv[(past - d) * C + c], v);
+        if (keep && t == 0)
           for (int p = sp.n; p < past; ++p) now[p * C + c] = p - sp.n < sp.pos0 ? old[(p - sp.n) * C + c] : 0.f;
       }
-      v = u * a.conv[past * C + c];
-      for (int d = 1; d <= past && d <= sp.pos0 + t; ++d)
-        v = fmaf(t >= d ? sum_at(a.y, slab, at - (size_t)d * a.y.NP) : old[(d - t - 1) * C + c],
-                 a.conv[(past - d) * C + c], v);
+      if (keep && sp.n - 1 - t < past) now[(sp.n - 1 - t) * C + c] = u;
     }
     return a.silu ? silu_f(v) : v;
+  };
+  // what a token needs of the first product, item by item: its column, and where it goes
+  const int nv = ce - cb, e1 = 2 * dg, e2 = e1 + nv, e3 = e2 + r1 + r2, e4 = e3 + (SPLIT || r2 > 0 ? 0 : vg);
+  const int items = e4 + (RULE == kMemoryDelta ? 1 : RULE == kMemoryNormed ? 2 : 0);
+  auto column = [&](int c) {
+    if (c < e1) return a.col + (c < dg ? hq * dg + c : (a.G + hq) * dg + c - dg);
+    if (c < e2) return cb + c - e1 < vg ? a.col + 2 * a.G * dg + h * vg + cb + c - e1 : -1;
+    if (c < e3) return c - e2 < r1 ? a.decay.col + c - e2 : a.gate.col + c - e2 - r1;
+    if (c < e4) return a.col_gate + h * vg + c - e3;
+    return RULE == kMemoryDelta ? a.col_beta + h : (c == e4 ? a.col_i : a.col_f) + h;
+  };
+  auto place = [&](int p0, int t, int c, float u) {
+    if (c < e1) {
+      const float v = project(p0 + t, c < dg ? hq * dg + c : (a.G + hq) * dg + c - dg, u, first);
+      (c < dg ? sq : sk)[t * dg + (c < dg ? c : c - dg)] = v;
+    } else if (c < e2) {
+      const int vc = cb + c - e1;
+      float v = 0.f;
+      if (vc < vg) v = project(p0 + t, 2 * a.G * dg + h * vg + vc, u, true);
+      if (RULE == kMemoryNormed && vc == a.vdim) v = 1.f;
+      sv[t * vs + vc] = v;
+    } else if (c < e3) {
+      if (c - e2 < r1) sx[t * r1 + c - e2] = u;
+      else sx2[t * r2 + c - e2 - r1] = u;
+    } else if (c < e4) {
+      sgate[t * vg + c - e3] = u;
+    } else if constexpr (RULE == kMemoryDelta) {
+      scal[t * 8] = sigmoid_f(u);
+    } else if constexpr (RULE == kMemoryNormed) {
+      const float z = a.cap * tanhf(__fdiv_rn(u + (c == e4 ? a.bi : a.bf)[h], a.cap));
+      scal[t * 8 + c - e4] = c == e4 ? z : -softplus_f(-z);
+    }
   };
   int turn = 0;
   for (int p0 = 0; p0 < sp.n; p0 += piece) {
     const int np = min(piece, sp.n - p0);
-    // the first product's columns
-    {
-      const int w = 2 * dg + vs;
-      const bool first = h % (a.H / a.G) == 0;  // (query and key heads are shared)
-      for (int id = tid; id < np * w; id += NT) {
-        const int t = id / w, c = id - t * w;
-        if (c < dg) sq[t * dg + c] = project(p0 + t, hq * dg + c, first);
-        else if (c < 2 * dg) sk[t * dg + c - dg] = project(p0 + t, (a.G + hq) * dg + c - dg, first);
-        else {
-          const int vc = c - 2 * dg;
-          float v = 0.f;
-          if (vc < vg) v = project(p0 + t, 2 * a.G * dg + h * vg + vc, true);
-          if (RULE == kMemoryNormed && vc == a.vdim) v = 1.f;
-          sv[t * vs + vc] = v;
-        }
-      }
-      const int r1 = a.decay.r, r2 = a.gate.r, rr = r1 + r2;
-      for (int id = tid; id < np * rr; id += NT) {
-        const int t = id / rr, c = id - t * rr;
-        const float v = sum_at(a.y, slab, (size_t)(sp.t0 + p0 + t) * a.y.NP + (c < r1 ? a.decay.col + c : a.gate.col + c - r1));
-        if (c < r1) sx[t * r1 + c] = v;
-        else sx2[t * r2 + c - r1] = v;
-      }
-      if (tid < np) {
-        const int t = sp.t0 + p0 + tid;
-        if constexpr (RULE == kMemoryDelta)
-          scal[tid * 8] = sigmoid_f(sum_at(a.y, slab, (size_t)t * a.y.NP + a.col_beta + h));
-        if constexpr (RULE == kMemoryNormed) {
-          float i, f;
-          memory_gates(a, t, h, i, f);
-          scal[tid * 8] = i, scal[tid * 8 + 1] = f;
-        }
-      }
+    for (int id0 = tid; id0 < np * items; id0 += 2 * NT) {  // two at a time
+      const int id1 = id0 + NT;
+      const int ta = id0 / items, ca = id0 - ta * items, tb = id1 / items, cc = id1 - tb * items;
+      const bool both = id1 < np * items;
+      const int ya = column(ca), yb = both ? column(cc) : -1;
+      float ua = 0.f, ub = 0.f;
+      if (ya >= 0) ua = sum_at(a.y, slab, (size_t)(sp.t0 + p0 + ta) * a.y.NP + ya);
+      if (yb >= 0) ub = sum_at(a.y, slab, (size_t)(sp.t0 + p0 + tb) * a.y.NP + yb);
+      place(p0, ta, ca, ua);
+      if (both) place(p0, tb, cc, ub);
     }
+    if (p0 == 0) load(cb, sp.pos0 == 0);
     __syncthreads();
     // gates, norms
     if constexpr (RULE == kMemoryNormed) {
-      float mm = m, mine = 0.f;  // (every wave follows m for its own tokens)
+      float mm = m;  // (every wave follows m for its own tokens)
       for (int t = 0; t < np; ++t) {
         const float i = scal[t * 8], f = scal[t * 8 + 1], mn = fmaxf(f + mm, i);
         if (t % NW == wave) {
           const float d = expf(f + mm - mn), kf = expf(i - mn);
-          for (int c = lane; c < dg; c += 64) sg[t * dg + c] = d;
-          if (lane == 0) scal[t * 8 + 3] = mn, scal[t * 8 + 4] = kf;
-          mine = kf;
+          if (lane == 0) scal[t * 8 + 3] = mn;
           for (int c = lane; c < dg; c += 64) {
+            sg[t * dg + c] = d;
             sq[t * dg + c] *= a.q_scale;
-            sk[t * dg + c] *= mine;
+            sk[t * dg + c] *= kf;
           }
         }
         mm = mn;
@@ -166,43 +247,36 @@ __global__ __launch_bounds__(NT) void memory_steps_kernel(const char *__restrict
       m = mm;
     } else {
       for (int t = wave; t < np; t += NW) {
-        float qq = 0.f, kk = 0.f, kq = 0.f;
-        for (int c = lane; c < dg; c += 64) {
-          const float x = sq[t * dg + c], y = sk[t * dg + c];
-          qq = fmaf(x, x, qq), kk = fmaf(y, y, kk), kq = fmaf(x, y, kq);
-        }
         float fq = a.q_scale, fk = 1.f;
         if (a.unit || RULE == kMemoryDelta) {
+          float qq = 0.f, kk = 0.f, kq = 0.f;
+          for (int c = lane; c < dg; c += 64) {
+            const float x = sq[t * dg + c], y = sk[t * dg + c];
+            qq = fmaf(x, x, qq), kk = fmaf(y, y, kk), kq = fmaf(x, y, kq);
+          }
 #pragma unroll
           for (int o = 32; o > 0; o >>= 1)
             qq += __shfl_xor(qq, o), kk += __shfl_xor(kk, o), kq += __shfl_xor(kq, o);
+          if (a.unit)
+            fq *= __fdiv_rn(1.0f, sqrtf(qq + 1e-6f)), fk = __fdiv_rn(1.0f, sqrtf(kk + 1e-6f));
+          if (lane == 0) scal[t * 8 + 2] = kq * fq * fk;
         }
-        if (a.unit)
-          fq *= __fdiv_rn(1.0f, sqrtf(qq + 1e-6f)), fk = __fdiv_rn(1.0f, sqrtf(kk + 1e-6f));
         for (int c = lane; c < dg; c += 64) {
           sq[t * dg + c] *= fq;
           sk[t * dg + c] *= fk;
         }
-        if (lane == 0) scal[t * 8 + 2] = kq * fq * fk;
       }
-      low_rank<E>(a.decay, h * a.dim, a.dim, np, sx,
-                  [&](int t, int c, float z) { sg[t * dg + c] = expf(log_decay<RULE>(a, h, c, z)); });
+      decay.run(a.decay, h * a.dim, a.dim, np, sx,
+                [&](int t, int c, float z) { sg[t * dg + c] = expf(log_decay<RULE>(a, h, c, z)); });
       for (int id = tid; id < np * (dg - a.dim); id += NT)
         sg[id / (dg - a.dim) * dg + a.dim + id % (dg - a.dim)] = 1.f;
     }
-    if (a.gate.r > 0) {
-      low_rank<E>(a.gate, h * a.vdim, a.vdim, np, sx2, [&](int t, int c, float z) { sgate[t * vg + c] = z; });
-      for (int id = tid; id < np * (vg - a.vdim); id += NT)
-        sgate[id / (vg - a.vdim) * vg + a.vdim + id % (vg - a.vdim)] = 0.f;
-    } else {
-      for (int id = tid; id < np * vg; id += NT)
-        sgate[id] = sum_at(a.y, slab, (size_t)(sp.t0 + p0 + id / vg) * a.y.NP + a.col_gate + h * vg + id % vg);
-    }
+    if (r2 > 0) gate.run(a.gate, h * a.vdim, a.vdim, np, sx2, [&](int t, int c, float z) { sgate[t * vg + c] = z; });
     __syncthreads();
     // the tokens in turn
-    for (int c0 = 0; c0 < vs; c0 += SW) {
-      if (!one) load(c0, sp.pos0 + p0 == 0);
-      const bool col = c0 + cl < vs;
+    for (int c0 = cb; c0 < ce; c0 += SW) {
+      if (!one && (p0 > 0 || c0 > cb)) load(c0, sp.pos0 + p0 == 0);
+      const bool col = c0 + cl < ce;
       for (int t = 0; t < np; ++t, turn ^= 1) {
         float *part = red + turn * 2 * NW * SW;
         f4 v = f4{0.f, 0.f, 0.f, 0.f}, pk = v, pq = v;
@@ -254,36 +328,47 @@ __global__ __launch_bounds__(NT) void memory_steps_kernel(const char *__restrict
 #pragma unroll
           for (int w = 1; w < NW; ++w) o += *reinterpret_cast<const f4 *>(part + w * SW + cl);
           if constexpr (RULE == kMemoryDelta) o += u * scal[t * 8 + 2];
-          *reinterpret_cast<f4 *>(so + t * vs + c0 + cl) = o;
+          if constexpr (SPLIT)
+            *reinterpret_cast<f4 *>(w.o + ((size_t)(sp.t0 + p0 + t) * a.H + h) * vs + c0 + cl) = o;
+          else *reinterpret_cast<f4 *>(so + t * vs + c0 + cl) = o;
         }
       }
       if (!one || p0 + np >= sp.n) store(c0);
     }
-    __syncthreads();
-    // a wave per token: norm and gate
-    for (int t = wave; t < np; t += NW) {
-      float f = 1.f, ss = 0.f;
-      if constexpr (RULE == kMemoryNormed)
-        f = __fdiv_rn(1.0f, fmaxf(fabsf(so[t * vs + a.vdim]), expf(-scal[t * 8 + 3])) + 1e-6f);
-      for (int c = lane; c < a.vdim; c += 64) {
-        const float v = so[t * vs + c] * f;
-        ss = fmaf(v, v, ss);
-      }
+    if constexpr (SPLIT) {
+      if (RULE == kMemoryNormed && cb == 0 && tid < np)
+        w.gates[((size_t)(sp.t0 + p0 + tid) * a.H + h) * 3 + 2] = scal[tid * 8 + 3];
+    } else {
+      __syncthreads();
+      // a wave per token: norm and gate
+      for (int t = wave; t < np; t += NW) {
+        float f = 1.f, ss = 0.f;
+        if constexpr (RULE == kMemoryNormed)
+          f = __fdiv_rn(1.0f, fmaxf(fabsf(so[t * vs + a.vdim]), expf(-scal[t * 8 + 3])) + 1e-6f);
+        for (int c = lane; c < a.vdim; c += 64) {
+          const float v = so[t * vs + c] * f;
+          ss = fmaf(v, v, ss);
+        }
 #pragma unroll
-      for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
-      const float r = f * inv_rms(ss, a.vdim, a.eps);
-      const int row = sp.t0 + p0 + t;
-      for (int c = lane; c < vg; c += 64) {
-        const float gt = sgate[t * vg + c], w = a.norm[(a.norm_heads ? h * vg : 0) + c];
-        const float v = c < a.vdim ? so[t * vs + c] * r * w * (a.gate_silu ? silu_f(gt) : sigmoid_f(gt)) : 0.f;
-        const int oc = a.out_col + h * vg + c;
-        st_elem((E *)a.out + (sizeof(E) == 2 ? act_packed_off(row, oc, a.ldo) : (size_t)row * a.ldo + oc), v);
+        for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
+        const float r = f * inv_rms(ss, a.vdim, a.eps);
+        const int row = sp.t0 + p0 + t;
+        auto put = [&](int c, float wv) {
+          const float gt = sgate[t * vg + c];
+          const float v = c < a.vdim ? so[t * vs + c] * r * wv * (a.gate_silu ? silu_f(gt) : sigmoid_f(gt)) : 0.f;
+          const int oc = a.out_col + h * vg + c;
+          st_elem((E *)a.out + (sizeof(E) == 2 ? act_packed_off(row, oc, a.ldo) : (size_t)row * a.ldo + oc), v);
+        };
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (lane + 64 * i < vg) put(lane + 64 * i, nw[i]);
+        for (int c = lane + 256; c < vg; c += 64) put(c, a.norm[(a.norm_heads ? h * vg : 0) + c]);
       }
     }
     __syncthreads();
   }
   if constexpr (RULE == kMemoryNormed)
-    if (tid == 0) a.peak[((size_t)sp.slot * 2 + (bank ^ 1)) * a.H + h] = m;
+    if (tid == 0 && cb == 0) a.peak[((size_t)sp.slot * 2 + (bank ^ 1)) * a.H + h] = m;
 }
 
 bool bad_shape(const Memory &a) {
@@ -297,7 +382,8 @@ bool bad_shape(const Memory &a) {
 }
 
 template <MemoryRule RULE, class E>
-hipError_t run_steps(const char *blob, int off_spans, int num_spans, const Memory &a, int limit, hipStream_t s) {
+hipError_t run_steps(const char *blob, int off_spans, int num_spans, const Memory &a, const MemoryScratch *w,
+                     int limit, bool *left, hipStream_t s) {
   // the widest power of two of columns that leaves at most 8 rows a thread
   int cw = 3;
   while (cw < 6 && (4 << cw) < a.vs && ((a.dg << (cw + 1)) + NT - 1) / NT <= 8) ++cw;
@@ -306,10 +392,24 @@ hipError_t run_steps(const char *blob, int off_spans, int num_spans, const Memor
   const int piece = std::min({kShortSpan, limit, std::max(1, (budget - red) / each)});
   const size_t bytes = (size_t)(red + piece * each) * 4;
   if (bytes > 64 * 1024) return hipErrorInvalidValue;
-  const dim3 grid(a.H, num_spans);
-#define FFMI_MS(P)                                                                                           \
-  hipLaunchKernelGGL((memory_steps_kernel<RULE, E, P>), grid, dim3(NT), bytes, s, blob, off_spans, a, limit, \
-                     piece, cw)
+  // few wide heads: their slices side by side
+  const int slices = (a.vs + (4 << cw) - 1) / (4 << cw), wgs = a.H * num_spans;
+  const int want = w && a.gate.r == 0 && sizeof(E) == 2 ? std::min(slices, (512 + wgs - 1) / wgs) : 1;
+  const int cols = (slices + want - 1) / want * (4 << cw), parts = (a.vs + cols - 1) / cols;
+  const MemoryScratch none;
+  *left = parts > 1;
+  const dim3 grid(a.H, num_spans, parts);
+#define FFMI_MS(P)                                                                                                    \
+  do {                                                                                                                \
+    if constexpr (sizeof(E) == 2 && RULE != kMemoryDelta)                                                             \
+      if (parts > 1) {                                                                                                \
+        hipLaunchKernelGGL((memory_steps_kernel<RULE, E, P, true>), grid, dim3(NT), bytes, s, blob, off_spans, a, *w,  \
+                           limit, piece, cw, cols);                                                                   \
+        break;                                                                                                        \
+      }                                                                                                               \
+    hipLaunchKernelGGL((memory_steps_kernel<RULE, E, P, false>), grid, dim3(NT), bytes, s, blob, off_spans, a,        \
+                       w ? *w : none, limit, piece, cw, cols);                                                        \
+  } while (0)
   if (rows <= 1) FFMI_MS(1);
   else if (rows <= 2) FFMI_MS(2);
   else if (rows <= 4) FFMI_MS(4);
@@ -321,13 +421,14 @@ hipError_t run_steps(const char *blob, int off_spans, int num_spans, const Memor
 
 }  // namespace
 
-hipError_t launch_memory_steps(const char *blob, int off_spans, int num_spans, const Memory &a, bool f32,
-                               int limit, hipStream_t s) {
+hipError_t launch_memory_steps(const char *blob, int off_spans, int num_spans, const Memory &a,
+                               const MemoryScratch *w, bool f32, int limit, bool *left, hipStream_t s) {
+  *left = false;
   if (num_spans <= 0) return hipSuccess;
-  if (bad_shape(a) || limit < 1) return hipErrorInvalidValue;
-#define FFMI_MR(RULE)                                                                          \
-  return f32 ? run_steps<RULE, float>(blob, off_spans, num_spans, a, limit, s)                 \
-             : run_steps<RULE, uint16_t>(blob, off_spans, num_spans, a, limit, s)
+  if (bad_shape(a) || limit < 1 || (w && (!w->o || (a.rule == kMemoryNormed && !w->gates)))) return hipErrorInvalidValue;
+#define FFMI_MR(RULE)                                                                              \
+  return f32 ? run_steps<RULE, float>(blob, off_spans, num_spans, a, w, limit, left, s)            \
+             : run_steps<RULE, uint16_t>(blob, off_spans, num_spans, a, w, limit, left, s)
   if (a.rule == kMemoryGated) FFMI_MR(kMemoryGated);
   if (a.rule == kMemoryDelta) FFMI_MR(kMemoryDelta);
   FFMI_MR(kMemoryNormed);

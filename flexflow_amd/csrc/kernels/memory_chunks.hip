@@ -8,8 +8,8 @@
 //          T = (1 + beta a)^-1, unit lower triangular
 //   o_i  = (q_i exp(G_i))^T S + sum over j <= i of p_ij u_j
 //   S'   = exp(G_last) S + sum over j of (k_j exp(G_last - G_j)) u_j^T
-// The first launch makes what does not need S, all chunks side by side; the second passes
-// over a span's chunks with the state in registers; the third has the outputs' norm and gate.
+// Launches: delta: convolved rows; normed: gates; then what does not need S, all chunks
+// side by side; then the pass over a span's chunks with the state in registers.
 //
 // No exponent is ever positive beyond kSpread: a chunk's four blocks of 16 tokens take their
 // decays from the blocks' borders, and a block's own 16 x 16 products from its start while
@@ -52,36 +52,102 @@ __device__ __forceinline__ uint2 pack4(const f4 &v) {
   return make_uint2(f2bf(v[0]) | ((uint32_t)f2bf(v[1]) << 16), f2bf(v[2]) | ((uint32_t)f2bf(v[3]) << 16));
 }
 
-// columns c .. c + 7 of q | k | v for token t of the span, convolved
-__device__ __forceinline__ void project8(const Memory &a, const PagedSpan &sp, int bank, int t, int c, bool keep,
-                                         f4 (&v)[2]) {
-  const size_t slab = (size_t)a.T * a.y.NP, at = (size_t)(sp.t0 + t) * a.y.NP + a.col + c;
-  sum8(a.y, slab, at, v);
-  if (a.taps > 0) {
-    const size_t cols = memory_columns(a);
-    const int past = a.taps - 1;
-    const float *old = a.carry + ((size_t)sp.slot * 2 + bank) * past * cols + c;
-    if (keep && sp.n - 1 - t < past) {  // (spans of this form are longer than that)
-      float *now = a.carry + ((size_t)sp.slot * 2 + (bank ^ 1)) * past * cols + (sp.n - 1 - t) * cols + c;
-      *reinterpret_cast<f4 *>(now) = v[0], *reinterpret_cast<f4 *>(now + 4) = v[1];
+__device__ __forceinline__ void load8(const float *p, f4 (&v)[2]) {
+  v[0] = *reinterpret_cast<const f4 *>(p), v[1] = *reinterpret_cast<const f4 *>(p + 4);
+}
+// softplus in base-2 units: log2(1 + 2^(z log2 e))
+__device__ __forceinline__ float softplus2(float z) {
+  z *= kLog2e;
+  return fmaxf(z, 0.f) + __builtin_amdgcn_logf(1.f + ex2(-fabsf(z)));
+}
+template <MemoryRule RULE>
+__device__ __forceinline__ float log2_decay(const Memory &a, float rate, float z) {
+  if constexpr (RULE == kMemoryDelta) return -rate * softplus2(z);
+  else return -a.inv_tau * softplus2(-z);
+}
+
+// the span whose chunk `c` is (counted over the step's long spans); a wave looks for it
+__device__ __forceinline__ int span_of_chunk(const PagedSpan *spans, int num, int c) {
+  for (int b = 0; b < num; b += 64) {
+    const int i = b + (threadIdx.x & 63);
+    bool hit = false;
+    if (i < num) {
+      const PagedSpan sp = spans[i];
+      hit = sp.n > kShortSpan && c >= sp.chunk0 && c < sp.chunk0 + (sp.n + C - 1) / C;
     }
-    const float *w = a.conv + c;
-    v[0] *= *reinterpret_cast<const f4 *>(w + past * cols), v[1] *= *reinterpret_cast<const f4 *>(w + past * cols + 4);
-    for (int d = 1; d <= past && d <= sp.pos0 + t; ++d) {
-      f4 u[2];
-      if (t >= d) {
-        sum8(a.y, slab, at - (size_t)d * a.y.NP, u);
-      } else {
-        const float *o = old + (d - t - 1) * cols;
-        u[0] = *reinterpret_cast<const f4 *>(o), u[1] = *reinterpret_cast<const f4 *>(o + 4);
+    const uint64_t m = __ballot(hit);
+    if (m) return __builtin_amdgcn_readfirstlane(b + __ffsll((unsigned long long)m) - 1);
+  }
+  return -1;
+}
+
+// delta: rows of q | k | v, convolved and through their activation, for the chunks; the
+// rows that are carried on.  A thread has 8 columns of TB tokens; PAST: taps - 1 (earlier
+// rows in registers), or -1: read again.
+template <int PAST>
+__global__ __launch_bounds__(256) void memory_rows_kernel(const char *__restrict__ blob, Memory a, MemoryScratch w,
+                                                          int limit) {
+  constexpr int TB = 8, H = PAST > 0 ? PAST : 1;
+  const int cols = memory_columns(a), c = (blockIdx.x * 256 + threadIdx.x) * 8, t0 = blockIdx.y * TB;
+  if (c >= cols) return;
+  const PagedToken *tok = reinterpret_cast<const PagedToken *>(blob + a.off_tokens);
+  const size_t slab = (size_t)a.T * a.y.NP;
+  const int past = a.taps - 1;
+  const float *cw = a.conv + c;
+  f4 u[TB][2], x[H][2], wt[H + 1][2];
+#pragma unroll
+  for (int k = 0; k < TB; ++k) sum8(a.y, slab, (size_t)min(t0 + k, a.T - 1) * a.y.NP + a.col + c, u[k]);
+  // the row d tokens before token t
+  auto before = [&](const PagedToken &tk, int t, int d, f4 (&v)[2]) {
+    v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
+    if (tk.back >= d) sum8(a.y, slab, (size_t)(t - d) * a.y.NP + a.col + c, v);
+    else if (tk.pos >= d) load8(a.carry + (((size_t)tk.slot * 2 + tk.bank) * past + d - tk.back - 1) * cols + c, v);
+  };
+  if constexpr (PAST >= 0)
+#pragma unroll
+    for (int d = 0; d <= PAST; ++d) load8(cw + (size_t)(PAST - d) * cols, wt[d]);
+#pragma unroll
+  for (int k = 0; k < TB; ++k) {
+    const int t = t0 + k;
+    if (t >= a.T) break;
+    const PagedToken tk = tok[t];
+    if (PAST > 0 && (k == 0 || tk.back == 0))
+#pragma unroll
+      for (int d = 1; d <= PAST; ++d) before(tk, t, d, x[d - 1]);
+    if (tk.back + tk.ahead + 1 > limit) {
+      f4 v[2];
+      if (tk.ahead < past) {
+        float *now = a.carry + (((size_t)tk.slot * 2 + (tk.bank ^ 1)) * past + tk.ahead) * cols + c;
+        *reinterpret_cast<f4 *>(now) = u[k][0], *reinterpret_cast<f4 *>(now + 4) = u[k][1];
       }
-      const float *wd = w + (past - d) * cols;
-      v[0] += u[0] * *reinterpret_cast<const f4 *>(wd), v[1] += u[1] * *reinterpret_cast<const f4 *>(wd + 4);
+      if constexpr (PAST >= 0) {
+        v[0] = u[k][0] * wt[0][0], v[1] = u[k][1] * wt[0][1];
+#pragma unroll
+        for (int d = 1; d <= PAST; ++d) v[0] += x[d - 1][0] * wt[d][0], v[1] += x[d - 1][1] * wt[d][1];
+      } else {
+        f4 f[2], e[2];
+        load8(cw + (size_t)past * cols, f);
+        v[0] = u[k][0] * f[0], v[1] = u[k][1] * f[1];
+        for (int d = 1; d <= past; ++d) {
+          before(tk, t, d, e);
+          load8(cw + (size_t)(past - d) * cols, f);
+          v[0] += e[0] * f[0], v[1] += e[1] * f[1];
+        }
+      }
+      if (a.silu)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const float y = v[e >> 2][e & 3];
+          v[e >> 2][e & 3] = y * __builtin_amdgcn_rcpf(1.f + ex2(-kLog2e * y));
+        }
+      *reinterpret_cast<uint4 *>(w.rows + (size_t)t * cols + c) = pack8_bf16(v[0], v[1]);
+    }
+    if constexpr (PAST > 0) {
+#pragma unroll
+      for (int d = PAST; d > 1; --d) x[d - 1][0] = x[d - 2][0], x[d - 1][1] = x[d - 2][1];
+      x[0][0] = u[k][0], x[0][1] = u[k][1];
     }
   }
-  if (a.silu)
-#pragma unroll
-    for (int e = 0; e < 8; ++e) v[e >> 2][e & 3] = silu_f(v[e >> 2][e & 3]);
 }
 
 // normed: decay, key factor (logs, base 2) and m of every token of a long span; a workgroup
@@ -92,8 +158,7 @@ __global__ __launch_bounds__(256) void memory_gates_kernel(const char *__restric
   const PagedSpan sp = reinterpret_cast<const PagedSpan *>(blob + off_spans)[blockIdx.y];
   if (sp.n <= limit) return;
   const int tid = threadIdx.x, h = blockIdx.x, per = (sp.n + 255) / 256;
-  const int b = min(tid * per, sp.n), e = min(b + per, sp.n);
-  const int bank = reinterpret_cast<const PagedToken *>(blob + a.off_tokens)[sp.t0].bank;
+  const int b = min(tid * per, sp.n), e = min(b + per, sp.n), bank = sp.bank;
   float add = 0.f, top = -INFINITY;
   for (int t = b; t < e; ++t) {
     float i, f;
@@ -124,10 +189,11 @@ __global__ __launch_bounds__(256) void memory_gates_kernel(const char *__restric
   }
 }
 
-// A workgroup per (chunk, head, span); wave b has the chunk's block of 16 tokens b.
+// A workgroup per (chunk, head); wave b has the chunk's block of 16 tokens b.
 template <MemoryRule RULE, int KS>
-__global__ __launch_bounds__(256) void memory_chunk_kernel(const char *__restrict__ blob, int off_spans, Memory a,
-                                                           MemoryScratch w, int limit) {
+__global__ __launch_bounds__(256, KS <= 4 ? 2 : 1) void memory_chunk_kernel(const char *__restrict__ blob, int off_spans,
+                                                                            int num_spans, Memory a, MemoryScratch w,
+                                                                            int limit) {
   constexpr bool DELTA = RULE == kMemoryDelta;
   constexpr int DK = KS * 32, LDK = DK + 8, LDG = DK + 4, LDA = C + 4, VW = 64, LDV = VW + 8;
   constexpr int GB = C * LDG * 4, AB = C * LDA * 4 + C * LDV * 2;
@@ -137,49 +203,128 @@ __global__ __launch_bounds__(256) void memory_chunk_kernel(const char *__restric
   __shared__ float sbeta[C];
   float *sG = reinterpret_cast<float *>(sX), *sA = sG;                       // (one after the other)
   uint16_t *sV = reinterpret_cast<uint16_t *>(sX + C * LDA * 4);
-  const PagedSpan sp = reinterpret_cast<const PagedSpan *>(blob + off_spans)[blockIdx.z];
-  const int t0 = blockIdx.x * C, h = blockIdx.y, n = min(C, sp.n - t0);
-  if (sp.n <= limit || n <= 0) return;
+  const PagedSpan *spans = reinterpret_cast<const PagedSpan *>(blob + off_spans);
+  const int si = span_of_chunk(spans, num_spans, blockIdx.x);
+  if (si < 0) return;
+  const PagedSpan sp = spans[si];
+  const int t0 = (blockIdx.x - sp.chunk0) * C, h = blockIdx.y, n = min(C, sp.n - t0);
+  if (sp.n <= limit) return;
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int bank = reinterpret_cast<const PagedToken *>(blob + a.off_tokens)[sp.t0].bank;
-  const int hq = h / (a.H / a.G);
-  const bool first = h % (a.H / a.G) == 0;  // (query and key heads are shared)
-  const size_t id = ((size_t)(sp.t0 / C) + blockIdx.z + blockIdx.x) * a.H + h;
+  const int hq = h / (a.H / a.G), cols = memory_columns(a);
+  const size_t id = (size_t)blockIdx.x * a.H + h, row0 = sp.t0 + t0;
+  const size_t slab = (size_t)a.T * a.y.NP, zslab = (size_t)a.T * a.z.NP;
 
-  // queries, keys, log decays: sixteen lanes a row
+  // queries, keys, log decays: sixteen lanes a row, a wave's sixteen rows; everything is
+  // asked for before anything is used
   constexpr int NI = (DK + 127) / 128;
-  for (int r4 = 0; r4 < 16; r4 += 4) {
-    const int r = wave * 16 + r4 + g, t = t0 + r;
+  const f4 nil = {0.f, 0.f, 0.f, 0.f};
+  f4 lq[4][NI][2], lk[4][NI][2], lg[4][NI][2];
+  uint4 bq[4][NI], bk[4][NI];
+  f4 gn[4];  // normed: gates of a row
+  float beta = 0.f;
+  constexpr int NV = C * VW / 8 / 256;  // 16-byte pieces of a slice of values per thread
+  uint4 lv[NV];
+  auto fetch_values = [&](int c0) {
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int e = tid + i * 256, r = e / (VW / 8), c = c0 + e % (VW / 8) * 8;
+      lv[i] = make_uint4(0, 0, 0, 0);
+      if (r < n && c < a.vg)
+        lv[i] = *reinterpret_cast<const uint4 *>(w.rows + (row0 + r) * cols + 2 * a.G * a.dg + h * a.vg + c);
+    }
+  };
+#pragma unroll
+  for (int i4 = 0; i4 < 4; ++i4) {
+    const int r = wave * 16 + i4 * 4 + g;
+    const size_t t = row0 + min(r, n - 1);
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const int c = min((l15 + 16 * i) * 8, a.dg - 8);
+      if constexpr (DELTA) {
+        bq[i4][i] = *reinterpret_cast<const uint4 *>(w.rows + t * cols + hq * a.dg + c);
+        bk[i4][i] = *reinterpret_cast<const uint4 *>(w.rows + t * cols + (a.G + hq) * a.dg + c);
+      } else {
+        load8(a.y.p + t * a.y.NP + a.col + hq * a.dg + c, lq[i4][i]);
+        load8(a.y.p + t * a.y.NP + a.col + (a.G + hq) * a.dg + c, lk[i4][i]);
+      }
+      if constexpr (RULE != kMemoryNormed) load8(a.z.p + t * a.z.NP + a.decay.zcol + h * a.dg + c, lg[i4][i]);
+    }
+    if constexpr (RULE == kMemoryNormed) {
+      const float *gt = w.gates + (t * a.H + h) * 3;
+      gn[i4] = f4{gt[0], gt[1], 0.f, 0.f};
+    }
+  }
+  if constexpr (DELTA) {
+    if (tid < n) beta = a.y.p[(row0 + tid) * a.y.NP + a.col_beta + h];
+    fetch_values(0);
+  }
+  f4 lb[NI][2];
+  if constexpr (RULE != kMemoryNormed)
+#pragma unroll
+    for (int i = 0; i < NI; ++i) load8(a.dbias + (size_t)h * a.dg + min((l15 + 16 * i) * 8, a.dg - 8), lb[i]);
+  const float rate = DELTA ? a.rate[h] : 0.f;
+  // (products split over K: the other slabs)
+  for (int s = 1; s < a.y.S; ++s) {
+    if constexpr (DELTA) {
+      if (tid < n) beta += a.y.p[s * slab + (row0 + tid) * a.y.NP + a.col_beta + h];
+    } else {
+#pragma unroll
+      for (int i4 = 0; i4 < 4; ++i4)
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+          const size_t t = row0 + min(wave * 16 + i4 * 4 + g, n - 1);
+          const int c = min((l15 + 16 * i) * 8, a.dg - 8);
+          f4 v[2];
+          load8(a.y.p + s * slab + t * a.y.NP + a.col + hq * a.dg + c, v);
+          lq[i4][i][0] += v[0], lq[i4][i][1] += v[1];
+          load8(a.y.p + s * slab + t * a.y.NP + a.col + (a.G + hq) * a.dg + c, v);
+          lk[i4][i][0] += v[0], lk[i4][i][1] += v[1];
+        }
+    }
+  }
+  if constexpr (RULE != kMemoryNormed)
+    for (int s = 1; s < a.z.S; ++s)
+#pragma unroll
+      for (int i4 = 0; i4 < 4; ++i4)
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+          f4 v[2];
+          load8(a.z.p + s * zslab + (row0 + min(wave * 16 + i4 * 4 + g, n - 1)) * a.z.NP + a.decay.zcol + h * a.dg +
+                    min((l15 + 16 * i) * 8, a.dg - 8), v);
+          lg[i4][i][0] += v[0], lg[i4][i][1] += v[1];
+        }
+  if constexpr (DELTA)
+    if (tid < C) sbeta[tid] = tid < n ? sigmoid_f(beta) : 0.f;
+#pragma unroll
+  for (int i4 = 0; i4 < 4; ++i4) {
+    const int r = wave * 16 + i4 * 4 + g;
     const bool real = r < n;
     f4 q[NI][2], k[NI][2];
     float qq = 0.f, kk = 0.f;
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
-      const int c = (l15 + 16 * i) * 8;
+      if constexpr (DELTA) {
+        unpack8_bf16(bq[i4][i], q[i][0], q[i][1]);
+        unpack8_bf16(bk[i4][i], k[i][0], k[i][1]);
+      } else {
 #pragma unroll
-      for (int j = 0; j < 2; ++j) q[i][j] = k[i][j] = f4{0.f, 0.f, 0.f, 0.f};
-      if (real && c < a.dg) {
-        project8(a, sp, bank, t, hq * a.dg + c, first, q[i]);
-        project8(a, sp, bank, t, (a.G + hq) * a.dg + c, first, k[i]);
+        for (int j = 0; j < 2; ++j) q[i][j] = lq[i4][i][j], k[i][j] = lk[i4][i][j];
       }
+      if (!real || (l15 + 16 * i) * 8 >= a.dg) q[i][0] = q[i][1] = k[i][0] = k[i][1] = nil;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         qq = fmaf(q[i][e >> 2][e & 3], q[i][e >> 2][e & 3], qq);
         kk = fmaf(k[i][e >> 2][e & 3], k[i][e >> 2][e & 3], kk);
       }
     }
-    float fq = a.q_scale, fk = 1.f, gs = 0.f;
+    float fq = a.q_scale, fk = 1.f;
     if (a.unit) {
 #pragma unroll
       for (int o = 1; o < 16; o <<= 1) qq += __shfl_xor(qq, o), kk += __shfl_xor(kk, o);
       fq *= __fdiv_rn(1.0f, sqrtf(qq + 1e-6f)), fk = __fdiv_rn(1.0f, sqrtf(kk + 1e-6f));
     }
-    if constexpr (RULE == kMemoryNormed)
-      if (real) {
-        const float *gt = w.gates + ((size_t)(sp.t0 + t) * a.H + h) * 3;
-        gs = gt[0], fk = ex2(gt[1]);
-      }
+    if constexpr (RULE == kMemoryNormed) fk = ex2(gn[i4][1]);
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
       const int c = (l15 + 16 * i) * 8;
@@ -187,22 +332,15 @@ __global__ __launch_bounds__(256) void memory_chunk_kernel(const char *__restric
       *reinterpret_cast<uint4 *>(&sQ[r * LDK + c]) = pack8_bf16(q[i][0] * fq, q[i][1] * fq);
       *reinterpret_cast<uint4 *>(&sK[r * LDK + c]) = pack8_bf16(k[i][0] * fk, k[i][1] * fk);
       f4 d[2];
-      d[0] = d[1] = f4{gs, gs, gs, gs};
-      if constexpr (RULE != kMemoryNormed)
-        if (real && c < a.dg) {
-          sum8(a.z, (size_t)a.T * a.z.NP, (size_t)(sp.t0 + t) * a.z.NP + a.decay.zcol + h * a.dg + c, d);
 #pragma unroll
-          for (int e = 0; e < 8; ++e) d[e >> 2][e & 3] = log_decay<RULE>(a, h, c + e, d[e >> 2][e & 3]) * kLog2e;
-        }
+      for (int e = 0; e < 8; ++e) {
+        float v = 0.f;
+        if constexpr (RULE == kMemoryNormed) v = gn[i4][0];
+        else v = c + e < a.dim ? log2_decay<RULE>(a, rate, lg[i4][i][e >> 2][e & 3] + lb[i][e >> 2][e & 3]) : 0.f;
+        d[e >> 2][e & 3] = real ? v : 0.f;
+      }
       *reinterpret_cast<f4 *>(&sG[r * LDG + c]) = d[0], *reinterpret_cast<f4 *>(&sG[r * LDG + c + 4]) = d[1];
     }
-  }
-  if (tid < C) {
-    float b = 0.f;
-    if constexpr (DELTA)
-      if (tid < n)
-        b = sigmoid_f(sum_at(a.y, (size_t)a.T * a.y.NP, (size_t)(sp.t0 + t0 + tid) * a.y.NP + a.col_beta + h));
-    sbeta[tid] = b;
   }
   __syncthreads();
   // sums of the log decays within the wave's block
@@ -338,21 +476,7 @@ __global__ __launch_bounds__(256) void memory_chunk_kernel(const char *__restric
     for (int kb = 0; kb < 2; ++kb)
       *reinterpret_cast<bf8 *>(w.kd + (id * DK + ct * 16 + l15) * C + kb * 32 + 8 * g) = read_columns<LDK>(sK, kb, ct * 16);
 
-  if constexpr (!DELTA) {  // the values as they are
-    for (int c = tid; c < C * (a.vs / 8); c += 256) {
-      const int r = c / (a.vs / 8), col = c % (a.vs / 8) * 8;
-      f4 v[2];
-      v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
-      if (r < n) {
-        if (col < a.vg) project8(a, sp, bank, t0 + r, 2 * a.G * a.dg + h * a.vg + col, true, v);
-        if constexpr (RULE == kMemoryNormed)
-#pragma unroll
-          for (int e = 0; e < 8; ++e)
-            if (col + e == a.vdim) v[e >> 2][e & 3] = 1.f;
-      }
-      *reinterpret_cast<uint4 *>((uint16_t *)w.u + (id * C + r) * a.vs + col) = pack8_bf16(v[0], v[1]);
-    }
-  } else {
+  if constexpr (DELTA) {
     // T in A's place.  Its blocks on the diagonal: a lane has a column, rows in turn
     {
       float x[16];
@@ -416,13 +540,12 @@ __global__ __launch_bounds__(256) void memory_chunk_kernel(const char *__restric
     }
     for (int c0 = 0; c0 < a.vs; c0 += VW) {
       __syncthreads();
-      for (int i = tid; i < C * VW / 8; i += 256) {
-        const int r = i / (VW / 8), c = i % (VW / 8) * 8;
-        f4 v[2];
-        v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
-        if (r < n && c0 + c < a.vg) project8(a, sp, bank, t0 + r, 2 * a.G * a.dg + h * a.vg + c0 + c, true, v);
-        *reinterpret_cast<uint4 *>(&sV[r * LDV + c]) = pack8_bf16(v[0], v[1]);
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int e = tid + i * 256;
+        *reinterpret_cast<uint4 *>(&sV[e / (VW / 8) * LDV + e % (VW / 8) * 8]) = lv[i];
       }
+      if (c0 + VW < a.vs) fetch_values(c0 + VW);
       __syncthreads();
 #pragma unroll
       for (int ct = 0; ct < VW / 16; ++ct) {
@@ -435,7 +558,7 @@ __global__ __launch_bounds__(256) void memory_chunk_kernel(const char *__restric
           x = mma(v, th[kb], x);
           x = mma(v, tl[kb], x);
         }
-        *reinterpret_cast<f4 *>((float *)w.u + (id * C + ri) * a.vs + c0 + ct * 16 + 4 * g) = x;
+        *reinterpret_cast<f4 *>(w.u + (id * C + ri) * a.vs + c0 + ct * 16 + 4 * g) = x;
       }
     }
   }
@@ -445,9 +568,10 @@ __global__ __launch_bounds__(256) void memory_chunk_kernel(const char *__restric
 // 16 w .. of u and o, and of the state 16 columns and an even share of the rows, in
 // registers (lane: 4 rows of one column); the state goes to LDS once a chunk as the
 // operand [column][row], u as rows.  What the next chunk needs is fetched a chunk ahead.
-template <bool DELTA, int KS, int VS>
-__global__ __launch_bounds__(256, KS * VS <= (DELTA ? 64 : 128) ? 2 : 1) void memory_scan_kernel(const char *__restrict__ blob, int off_spans,
+template <MemoryRule RULE, int KS, int VS>
+__global__ __launch_bounds__(256, KS * VS <= (RULE == kMemoryDelta ? 64 : 128) ? 2 : 1) void memory_scan_kernel(const char *__restrict__ blob, int off_spans,
                                                                            Memory a, MemoryScratch w, int limit) {
+  constexpr bool DELTA = RULE == kMemoryDelta;
   constexpr int DK = KS * 32, LDK = DK + 8, LDU = VS + 8;
   constexpr int VT = VS / 16, WD = 4 / VT, ND = (2 * KS + WD - 1) / WD;
   __shared__ __attribute__((aligned(16))) uint16_t sHi[VS * LDK], sLo[VS * LDK], sU[C * LDU], sUl[DELTA ? C * LDU : 8];
@@ -457,11 +581,10 @@ __global__ __launch_bounds__(256, KS * VS <= (DELTA ? 64 : 128) ? 2 : 1) void me
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int h = blockIdx.y, c0 = blockIdx.x * VS, vw = min(VS, a.vs - c0);
   const int ri = wave * 16 + l15, vcol = wave % VT * 16 + l15, d0 = wave / VT * ND;
-  const size_t id0 = ((size_t)(sp.t0 / C) + blockIdx.z) * a.H + h;
+  const size_t id0 = (size_t)sp.chunk0 * a.H + h;
 
   bf8 fq[KS], fw[DELTA ? KS : 1], fp[2], fk[ND][2];
   f4 fu[VT], fl[ND];
-  uint2 fv[VT];
   auto fetch = [&](int chunk) {
     const size_t id = id0 + (size_t)chunk * a.H;
 #pragma unroll
@@ -472,9 +595,22 @@ __global__ __launch_bounds__(256, KS * VS <= (DELTA ? 64 : 128) ? 2 : 1) void me
     }
 #pragma unroll
     for (int vt = 0; vt < VT; ++vt) {
-      const size_t at = (id * C + ri) * a.vs + c0 + min(vt * 16, vw - 16) + 4 * g;
-      if constexpr (DELTA) fu[vt] = *reinterpret_cast<const f4 *>((const float *)w.u + at);
-      else fv[vt] = *reinterpret_cast<const uint2 *>((const uint16_t *)w.u + at);
+      const int c = c0 + min(vt * 16, vw - 16) + 4 * g;
+      if constexpr (DELTA) {
+        fu[vt] = *reinterpret_cast<const f4 *>(w.u + (id * C + ri) * a.vs + c);
+      } else {  // the values as the product left them
+        fu[vt] = f4{0.f, 0.f, 0.f, 0.f};
+        const int t = chunk * C + ri;
+        if (t < sp.n && c < a.vg) {
+          const float *p = a.y.p + (size_t)(sp.t0 + t) * a.y.NP + a.col + 2 * a.G * a.dg + h * a.vg + c;
+          fu[vt] = *reinterpret_cast<const f4 *>(p);
+          for (int s = 1; s < a.y.S; ++s) fu[vt] += *reinterpret_cast<const f4 *>(p + (size_t)s * a.T * a.y.NP);
+        }
+        if constexpr (RULE == kMemoryNormed)
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            if (c + e == a.vdim && t < sp.n) fu[vt][e] = 1.f;
+      }
     }
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb) fp[kb] = *reinterpret_cast<const bf8 *>(w.p + (id * C + ri) * C + kb * 32 + 8 * g);
@@ -539,7 +675,7 @@ __global__ __launch_bounds__(256, KS * VS <= (DELTA ? 64 : 128) ? 2 : 1) void me
         *reinterpret_cast<uint2 *>(&sU[at]) = pack4(u[vt]);
         *reinterpret_cast<uint2 *>(&sUl[at]) = pack4(lo);
       } else {
-        *reinterpret_cast<uint2 *>(&sU[at]) = fv[vt];
+        *reinterpret_cast<uint2 *>(&sU[at]) = pack4(fu[vt]);
       }
       o[vt] += olo[vt];
     }
@@ -584,67 +720,98 @@ __global__ __launch_bounds__(256, KS * VS <= (DELTA ? 64 : 128) ? 2 : 1) void me
       for (int e = 0; e < 4; ++e) S[(size_t)((d0 + dt) * 16 + 4 * g + e) * a.vs] = st[dt][e];
 }
 
-// norm and gate of a long span's outputs: sixteen lanes a (token, head)
+// norm and gate: sixteen lanes a (token, head), their columns 64 apart
 template <MemoryRule RULE>
 __global__ __launch_bounds__(256) void memory_out_kernel(const char *__restrict__ blob, Memory a, MemoryScratch w,
-                                                         int limit) {
+                                                         int above) {
   const int l15 = threadIdx.x & 15;
   const long id = blockIdx.x * 16L + (threadIdx.x >> 4);
   const int t = (int)min(id / a.H, (long)a.T - 1), h = (int)(id % a.H);
   const PagedToken tk = reinterpret_cast<const PagedToken *>(blob + a.off_tokens)[t];
-  const bool mine = id < (long)a.T * a.H && tk.back + tk.ahead + 1 > limit;
+  const bool mine = id < (long)a.T * a.H && tk.back + tk.ahead + 1 > above;
   const float *o = w.o + ((size_t)t * a.H + h) * a.vs;
+  const bool second = a.gate.r > 0;
+  const Partials &gp = second ? a.z : a.y;
+  const size_t gat = (size_t)t * gp.NP + (second ? a.gate.zcol : a.col_gate) + h * a.vg;
+  constexpr int NK = 2;  // pieces of 8 columns kept in registers
+  f4 v[NK][2], gt[NK][2];
   float f = 1.f, ss = 0.f;
   if (mine) {
+#pragma unroll
+    for (int k = 0; k < NK; ++k) {
+      const int c = min(l15 * 8 + k * 128, a.vg - 8);
+      load8(o + c, v[k]);
+      sum8(gp, (size_t)a.T * gp.NP, gat + c, gt[k]);
+    }
     if constexpr (RULE == kMemoryNormed)
       f = __fdiv_rn(1.0f, fmaxf(fabsf(o[a.vdim]), expf(-w.gates[((size_t)t * a.H + h) * 3 + 2])) + 1e-6f);
-    for (int c = l15 * 4; c < a.vdim; c += 64) {
-      const f4 v = *reinterpret_cast<const f4 *>(o + c) * f;
+    auto add = [&](const f4 (&x)[2], int c) {
 #pragma unroll
-      for (int e = 0; e < 4; ++e)
-        if (c + e < a.vdim) ss = fmaf(v[e], v[e], ss);
+      for (int e = 0; e < 8; ++e) {
+        const float y = x[e >> 2][e & 3] * f;
+        if (c + e < a.vdim) ss = fmaf(y, y, ss);
+      }
+    };
+#pragma unroll
+    for (int k = 0; k < NK; ++k) add(v[k], l15 * 8 + k * 128);
+    for (int c = l15 * 8 + NK * 128; c < a.vg; c += 128) {
+      f4 x[2];
+      load8(o + c, x);
+      add(x, c);
     }
   }
 #pragma unroll
   for (int k = 1; k < 16; k <<= 1) ss += __shfl_xor(ss, k);
   if (!mine) return;
   const float r = f * inv_rms(ss, a.vdim, a.eps);
-  const bool second = a.gate.r > 0;
-  const Partials &gp = second ? a.z : a.y;
-  const size_t gat = (size_t)t * gp.NP + (second ? a.gate.zcol : a.col_gate) + h * a.vg;
-  for (int c = l15 * 8; c < a.vg; c += 128) {
-    f4 v[2], gt[2];
-    sum8(gp, (size_t)a.T * gp.NP, gat + c, gt);
+  auto put = [&](f4 (&x)[2], const f4 (&y)[2], int c) {
+    f4 wv[2];
+    load8(a.norm + (a.norm_heads ? h * a.vg : 0) + c, wv);
 #pragma unroll
-    for (int j = 0; j < 2; ++j) {
-      v[j] = *reinterpret_cast<const f4 *>(o + c + 4 * j);
-      const f4 wv = *reinterpret_cast<const f4 *>(a.norm + (a.norm_heads ? h * a.vg : 0) + c + 4 * j);
-#pragma unroll
-      for (int e = 0; e < 4; ++e)
-        v[j][e] = c + 4 * j + e < a.vdim ? v[j][e] * r * wv[e] * (a.gate_silu ? silu_f(gt[j][e]) : sigmoid_f(gt[j][e])) : 0.f;
+    for (int e = 0; e < 8; ++e) {
+      const float gv = y[e >> 2][e & 3], sg = __builtin_amdgcn_rcpf(1.f + ex2(-kLog2e * gv));
+      const float z = x[e >> 2][e & 3] * r * wv[e >> 2][e & 3] * (a.gate_silu ? gv * sg : sg);
+      x[e >> 2][e & 3] = c + e < a.vdim ? z : 0.f;
     }
-    *reinterpret_cast<uint4 *>((uint16_t *)a.out + act_packed_off(t, a.out_col + h * a.vg + c, a.ldo)) = pack8_bf16(v[0], v[1]);
+    *reinterpret_cast<uint4 *>((uint16_t *)a.out + act_packed_off(t, a.out_col + h * a.vg + c, a.ldo)) = pack8_bf16(x[0], x[1]);
+  };
+#pragma unroll
+  for (int k = 0; k < NK; ++k)
+    if (l15 * 8 + k * 128 < a.vg) put(v[k], gt[k], l15 * 8 + k * 128);
+  for (int c = l15 * 8 + NK * 128; c < a.vg; c += 128) {
+    f4 x[2], y[2];
+    load8(o + c, x);
+    sum8(gp, (size_t)a.T * gp.NP, gat + c, y);
+    put(x, y, c);
   }
 }
 
 template <MemoryRule RULE>
-hipError_t run_chunks(const char *blob, int off_spans, int num_spans, const Memory &a, const MemoryScratch &w,
-                      int limit, hipStream_t s) {
-  constexpr bool DELTA = RULE == kMemoryDelta;
-  const int chunks = (a.T + C - 1) / C;  // (of the longest span there can be)
+hipError_t run_chunks(const char *blob, int off_spans, int num_spans, int num_chunks, const Memory &a,
+                      const MemoryScratch &w, int limit, hipStream_t s) {
   if (RULE == kMemoryNormed)
     hipLaunchKernelGGL(memory_gates_kernel, dim3(a.H, num_spans), dim3(256), 0, s, blob, off_spans, a, w, limit);
+  if (RULE == kMemoryDelta) {
+    const dim3 grid((2 * a.G * a.dg + a.H * a.vg + 2047) / 2048, (a.T + 7) / 8);
+#define FFMI_MW(PAST) hipLaunchKernelGGL(memory_rows_kernel<PAST>, grid, dim3(256), 0, s, blob, a, w, limit)
+    if (a.taps == 1) FFMI_MW(0);
+    else if (a.taps == 2) FFMI_MW(1);
+    else if (a.taps == 3) FFMI_MW(2);
+    else if (a.taps == 4) FFMI_MW(3);
+    else FFMI_MW(-1);
+#undef FFMI_MW
+  }
   // narrow workgroups where the spans and heads alone do not fill the chip
   const bool wide = (long)a.H * num_spans * (a.vs / 32) >= 256;
-#define FFMI_MS(KS, VS)                                                                                              \
-  hipLaunchKernelGGL((memory_scan_kernel<DELTA, KS, VS>), dim3((a.vs + VS - 1) / VS, a.H, num_spans), dim3(256), 0, s, \
+#define FFMI_MS(KS, VS)                                                                                             \
+  hipLaunchKernelGGL((memory_scan_kernel<RULE, KS, VS>), dim3((a.vs + VS - 1) / VS, a.H, num_spans), dim3(256), 0, s, \
                      blob, off_spans, a, w, limit)
-#define FFMI_MC(KS)                                                                                               \
-  do {                                                                                                            \
-    hipLaunchKernelGGL((memory_chunk_kernel<RULE, KS>), dim3(chunks, a.H, num_spans), dim3(256), 0, s, blob,       \
-                       off_spans, a, w, limit);                                                                   \
-    if (wide) FFMI_MS(KS, 32);                                                                                    \
-    else FFMI_MS(KS, 16);                                                                                         \
+#define FFMI_MC(KS)                                                                                              \
+  do {                                                                                                           \
+    hipLaunchKernelGGL((memory_chunk_kernel<RULE, KS>), dim3(num_chunks, a.H), dim3(256), 0, s, blob, off_spans, \
+                       num_spans, a, w, limit);                                                                  \
+    if (wide) FFMI_MS(KS, 32);                                                                                   \
+    else FFMI_MS(KS, 16);                                                                                        \
   } while (0)
   switch (memory_chunk_width(a.dg)) {
     case 32: FFMI_MC(1); break;
@@ -654,26 +821,39 @@ hipError_t run_chunks(const char *blob, int off_spans, int num_spans, const Memo
   }
 #undef FFMI_MC
 #undef FFMI_MS
-  hipLaunchKernelGGL(memory_out_kernel<RULE>, dim3((unsigned)(((long)a.T * a.H + 15) / 16)), dim3(256), 0, s, blob, a,
-                     w, limit);
   return hipGetLastError();
 }
 
 }  // namespace
 
-hipError_t launch_memory_chunks(const char *blob, int off_spans, int num_spans, const Memory &a,
+hipError_t launch_memory_chunks(const char *blob, int off_spans, int num_spans, int num_chunks, const Memory &a,
                                 const MemoryScratch &w, int limit, hipStream_t s) {
-  if (num_spans <= 0) return hipSuccess;
+  if (num_spans <= 0 || num_chunks <= 0) return hipSuccess;
   if (a.H < 1 || a.G < 1 || a.H % a.G || a.dg % 32 || a.vg % 32 || a.dg > kMemoryMaxChunkDim || a.dim > a.dg ||
       a.vdim > a.vg || a.vs != memory_state_columns(a.rule, a.vdim) || a.y.S < 1 || a.y.NP % 4 || a.col % 4 ||
-      a.col_gate % 4 || a.decay.zcol % 4 || a.gate.zcol % 4 || limit < a.taps || a.ldo % 32 || a.out_col % 32 ||
-      (a.taps > 0 && !a.conv) || (a.taps > 1 && !a.carry) || (a.rule != kMemoryNormed && (a.z.S < 1 || a.z.NP % 4)) ||
-      !w.qg || !w.kd || !w.p || !w.u || !w.last || !w.o || (a.rule == kMemoryDelta && !w.w) ||
-      (a.rule == kMemoryNormed && !w.gates))
+      a.decay.zcol % 4 || limit < a.taps || limit < kShortSpan || (a.rule == kMemoryDelta) != (a.taps > 0) ||
+      (a.taps > 0 && !a.conv) || (a.taps > 1 && !a.carry) ||
+      (a.rule != kMemoryNormed && (a.z.S < 1 || a.z.NP % 4 || !a.dbias)) || !w.qg || !w.kd || !w.p || !w.last ||
+      !w.o || (a.rule == kMemoryDelta && (!w.w || !w.u || !w.rows || !a.rate)) ||
+      (a.rule == kMemoryNormed && !w.gates) || num_chunks > 65535)
     return hipErrorInvalidValue;
-  if (a.rule == kMemoryGated) return run_chunks<kMemoryGated>(blob, off_spans, num_spans, a, w, limit, s);
-  if (a.rule == kMemoryDelta) return run_chunks<kMemoryDelta>(blob, off_spans, num_spans, a, w, limit, s);
-  return run_chunks<kMemoryNormed>(blob, off_spans, num_spans, a, w, limit, s);
+  if (a.rule == kMemoryGated) return run_chunks<kMemoryGated>(blob, off_spans, num_spans, num_chunks, a, w, limit, s);
+  if (a.rule == kMemoryDelta) return run_chunks<kMemoryDelta>(blob, off_spans, num_spans, num_chunks, a, w, limit, s);
+  return run_chunks<kMemoryNormed>(blob, off_spans, num_spans, num_chunks, a, w, limit, s);
+}
+
+hipError_t launch_memory_out(const char *blob, const Memory &a, const MemoryScratch &w, int above, hipStream_t s) {
+  if (a.T <= 0) return hipSuccess;
+  if (!w.o || (a.rule == kMemoryNormed && !w.gates) || a.vg % 32 || a.ldo % 32 || a.out_col % 32 || a.col_gate % 4 ||
+      a.gate.zcol % 4 || (a.gate.r > 0 && a.z.S < 1) || a.out_col + a.H * a.vg > a.ldo)
+    return hipErrorInvalidValue;
+  const dim3 grid((unsigned)(((long)a.T * a.H + 15) / 16));
+#define FFMI_MO(RULE) hipLaunchKernelGGL(memory_out_kernel<RULE>, grid, dim3(256), 0, s, blob, a, w, above)
+  if (a.rule == kMemoryGated) FFMI_MO(kMemoryGated);
+  else if (a.rule == kMemoryDelta) FFMI_MO(kMemoryDelta);
+  else FFMI_MO(kMemoryNormed);
+#undef FFMI_MO
+  return hipGetLastError();
 }
 
 }  // namespace ffmi

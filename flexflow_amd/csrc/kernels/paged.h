@@ -41,9 +41,13 @@ struct PagedMerge {
 // positions pos0 ...
 struct PagedSpan {
   int32_t t0, n, pos0, slot;
+  int32_t bank;    // of the slot's carried rows, as a token's
+  int32_t chunk0;  // its first chunk among those of all spans beyond kShortSpan
+  int32_t pad[2];
 };
 // spans up to this length take the token-by-token form of a recurrence
 constexpr int kShortSpan = 16;
+constexpr int kSpanChunk = 64;  // tokens of a chunk of the others
 
 // Layout of a step's metadata, packed by runtime/paged_step.cpp.  Offsets in
 // bytes from the start of the blob.

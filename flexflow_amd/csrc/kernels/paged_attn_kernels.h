@@ -115,34 +115,79 @@ __device__ __forceinline__ void load_head(const AttnPrep &a, int T, int t, int h
     }
   }
 }
-// (rotary kind) the convolution over time: v, token t's product, becomes the sum over
-// its taps; the rows that later steps need go to the other bank
+// (rotary kind) The convolution over time of one head's columns: v, a token's product,
+// becomes the sum over its taps, and the rows that later steps need go to the other bank.
+// Up to TAPS taps (none in wide heads) their weights and the earlier rows are kept in
+// registers: load(), then the tokens of a run in turn.
 template <int NE>
-__device__ __forceinline__ void conv_head(const AttnPrep &a, int T, int t, const PagedToken &tk, int hd,
-                                          float (&v)[NE]) {
-  const int wd = head_width(a, hd), c0 = head_start(a, hd), past = a.taps - 1;
-  const size_t C = (size_t)(a.H + a.G) * a.dg + (size_t)a.G * a.vg;
-  const float *old = a.carry + ((size_t)tk.slot * 2 + tk.bank) * past * C;
-  float *now = a.carry + ((size_t)tk.slot * 2 + (tk.bank ^ 1)) * past * C;
-  const size_t slab = (size_t)T * a.y.NP;
-#pragma unroll
-  for (int i = 0; i < NE; ++i) {
-    const int c = head_column<NE>(i);
-    if (c >= wd) continue;
-    const size_t col = c0 + c;
-    if (tk.ahead < past) now[tk.ahead * C + col] = v[i];
-    if (tk.back == 0)  // (a short portion: earlier rows move on)
-      for (int p = tk.ahead + 1; p < past; ++p)
-        now[p * C + col] = p - tk.ahead <= tk.pos ? old[(p - tk.ahead - 1) * C + col] : 0.f;
-    float sum = v[i] * a.conv[past * C + col];
-    for (int d = 1; d <= past && d <= tk.pos; ++d) {
-      const float u = tk.back >= d ? slab_sum(a.y, slab, (size_t)(t - d) * a.y.NP + col)
-                                   : old[(d - tk.back - 1) * C + col];
-      sum = fmaf(u, a.conv[(past - d) * C + col], sum);
-    }
-    v[i] = sum;
+struct HeadConv {
+  static constexpr int TAPS = NE <= 4 ? 4 : 1, PAST = TAPS - 1;
+  float w[TAPS][NE], x[PAST > 0 ? PAST : 1][NE];  // of the token d back, and its row
+  static __device__ __forceinline__ size_t columns(const AttnPrep &a) {
+    return (size_t)(a.H + a.G) * a.dg + (size_t)a.G * a.vg;
   }
-}
+  static __device__ __forceinline__ const float *bank(const AttnPrep &a, const PagedToken &tk, int other) {
+    return a.carry + ((size_t)tk.slot * 2 + (tk.bank ^ other)) * (a.taps - 1) * columns(a);
+  }
+  // column col d tokens before token t (0: before the sequence)
+  static __device__ __forceinline__ float before(const AttnPrep &a, int T, int t, const PagedToken &tk, int d,
+                                                 size_t col) {
+    if (d > tk.pos) return 0.f;
+    if (tk.back >= d) return slab_sum(a.y, (size_t)T * a.y.NP, (size_t)(t - d) * a.y.NP + col);
+    return bank(a, tk, 0)[(d - tk.back - 1) * columns(a) + col];
+  }
+  __device__ __forceinline__ void load(const AttnPrep &a, int T, int t, const PagedToken &tk, int hd) {
+    const int wd = head_width(a, hd), c0 = head_start(a, hd), past = a.taps - 1;
+    if (past > PAST) return;
+    const size_t C = columns(a);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int c = head_column<NE>(i);
+#pragma unroll
+      for (int d = 0; d <= PAST; ++d) {
+        w[d][i] = c < wd && d <= past ? a.conv[(past - d) * C + c0 + c] : 0.f;
+        if (d > 0) x[d - 1][i] = c < wd && d <= past ? before(a, T, t, tk, d, c0 + c) : 0.f;
+      }
+    }
+  }
+  // NT > 1: the next token of the run follows
+  template <int NT>
+  __device__ __forceinline__ void apply(const AttnPrep &a, int T, int t, const PagedToken &tk, int hd,
+                                        float (&v)[NE]) {
+    const int wd = head_width(a, hd), c0 = head_start(a, hd), past = a.taps - 1;
+    const size_t C = columns(a);
+    float *now = const_cast<float *>(bank(a, tk, 1));
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int c = head_column<NE>(i);
+      if (c >= wd) continue;
+      const size_t col = c0 + c;
+      const float u = v[i];
+      if (tk.ahead < past) now[tk.ahead * C + col] = u;
+      if (past <= PAST) {
+        if (tk.back == 0)  // (a short portion: earlier rows move on)
+#pragma unroll
+          for (int d = 1; d <= PAST; ++d)
+            if (tk.ahead + d < past) now[(tk.ahead + d) * C + col] = x[d - 1][i];
+        float sum = u * w[0][i];
+#pragma unroll
+        for (int d = 1; d <= PAST; ++d) sum = fmaf(x[d - 1][i], w[d][i], sum);
+        v[i] = sum;
+        if constexpr (NT > 1 && PAST > 0) {
+#pragma unroll
+          for (int d = PAST; d > 1; --d) x[d - 1][i] = x[d - 2][i];
+          x[0][i] = u;
+        }
+      } else {
+        if (tk.back == 0)
+          for (int d = 1; tk.ahead + d < past; ++d) now[(tk.ahead + d) * C + col] = before(a, T, t, tk, d, col);
+        float sum = u * a.conv[past * C + col];
+        for (int d = 1; d <= past; ++d) sum = fmaf(before(a, T, t, tk, d, col), a.conv[(past - d) * C + col], sum);
+        v[i] = sum;
+      }
+    }
+  }
+};
 // values: mixed with, or kept as, the first mixing layer's (lam: *a.vmix)
 template <int NE>
 __device__ __forceinline__ void mix_head(const AttnPrep &a, int t, int g, float lam, float (&v)[NE]) {
@@ -360,10 +405,15 @@ __global__ __launch_bounds__(512) void rotary_prep_kernel(const PagedToken *__re
     load_bias<NE>(a, hd, bias);
 #pragma unroll
     for (int k = 0; k < NT; ++k) load_head<NE>(a, T, min(t0 + k, T - 1), hd, bias, v[k]);
-    if (a.taps > 0)
+    if (a.taps > 0) {
+      HeadConv<NE> cv;
 #pragma unroll
       for (int k = 0; k < NT; ++k)
-        if (t0 + k < T) conv_head<NE>(a, T, t0 + k, tk[k], hd, v[k]);
+        if (t0 + k < T) {
+          if (k == 0 || tk[k].back == 0) cv.load(a, T, t0 + k, tk[k], hd);
+          cv.template apply<NT>(a, T, t0 + k, tk[k], hd, v[k]);
+        }
+    }
     if (isv) {
       if (a.vfreq)
 #pragma unroll
@@ -579,12 +629,17 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
       if constexpr (KIND == kBias) norm_head<NE>(pr, it < nq, pos, x);
       else rotary_head<NE>(pr, head_of(it), pos, pr.norms ? rms[token_of(it)][it < nq ? 0 : 1] : 1.0f, x);
     };
-    auto finish = [&](int it, float (&x)[NE]) {
+    const PagedToken *ptok =
+        KIND == kRotary ? reinterpret_cast<const PagedToken *>(blob + pr.off_tokens) + t0 : nullptr;
+    auto conv = [&](int it, HeadConv<NE> &cv) {
+      if constexpr (KIND == kRotary)
+        if (pr.taps > 0) cv.load(pr, T, t0 + token_of(it), ptok[token_of(it)], head_of(it));
+    };
+    auto finish = [&](int it, HeadConv<NE> &cv, float (&x)[NE]) {
       const int tk = token_of(it), pos = bk.pos0 + tk, tile = pos / kPageTokens;
       if constexpr (KIND == kRotary)  // (split blocks carry the same rows)
         if (pr.taps > 0)
-          conv_head<NE>(pr, T, t0 + tk, reinterpret_cast<const PagedToken *>(blob + pr.off_tokens)[t0 + tk],
-                        head_of(it), x);
+          cv.template apply<1>(pr, T, t0 + tk, ptok[tk], head_of(it), x);
       if (it < nq) {
         make(it, pos, x);
         store_head<uint16_t, NE>([&](int c) { return sQ + it * LDQ + c; }, DP, x);
@@ -608,8 +663,11 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
       load_bias<NE>(pr, head_of(it1), b1);
       load_head<NE>(pr, T, t0 + token_of(it), head_of(it), b0, x0);
       load_head<NE>(pr, T, t0 + token_of(it1), head_of(it1), b1, x1);
-      finish(it, x0);
-      if (it + NW < items) finish(it1, x1);
+      HeadConv<NE> c0, c1;
+      conv(it, c0);
+      conv(it1, c1);
+      finish(it, c0, x0);
+      if (it + NW < items) finish(it1, c1, x1);
     }
     __syncthreads();  // (the new keys and values are in the cache, for this workgroup)
     const uint16_t *qr = sQ + min(l15, bk.nrows - 1) * LDQ + 8 * g;

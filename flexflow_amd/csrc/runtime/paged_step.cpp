@@ -130,13 +130,15 @@ ffmi_status PagedStep::stage(const int32_t *token_ids, const std::vector<Seg> &i
   off_spans = (int)(off = up16(off));
   num_spans = (int)segs.size();
   short_spans = long_spans = false;
+  num_chunks = 0;
   for (size_t i = 0; i < segs.size(); ++i, off += sizeof(PagedSpan)) {
-    const PagedSpan sp{segs[i].t0, segs[i].n, segs[i].pos0, in[i].slot};
+    const PagedSpan sp{segs[i].t0, segs[i].n, segs[i].pos0, in[i].slot, in[i].bank, num_chunks, {0, 0}};
     memcpy(host + off, &sp, sizeof(sp));
     (sp.n <= kShortSpan ? short_spans : long_spans) = true;
+    if (sp.n > kShortSpan) num_chunks += (sp.n + kSpanChunk - 1) / kSpanChunk;
   }
   off = up16(off);
-  shape.assign({T, R, num_spans, stride, short_spans, long_spans});
+  shape.assign({T, R, num_spans, stride, short_spans, long_spans, num_chunks});
   for (size_t li = 0; li < lists_.size(); ++li) {
     PagedLists &l = lists_[li];
     const RowShape &rs = shapes_[li];

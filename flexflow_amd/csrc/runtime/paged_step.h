@@ -54,6 +54,7 @@ struct PagedStep {
   size_t bytes = 0;
   int T = 0, R = 0, off_tokens = 0, off_rows = 0, off_spans = 0, num_spans = 0;
   bool short_spans = false, long_spans = false;  // spans of either kind in the step
+  int num_chunks = 0;                            // of the long ones
   std::vector<int> shape;  // everything a captured graph of this step depends on
 
  private:

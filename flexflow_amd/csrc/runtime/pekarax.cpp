@@ -248,7 +248,7 @@ struct Pekarax : public PagedDecoder {
   }
   ffmi_status alloc_states() {
     const size_t n = o.max_requests, chunks = memory_chunks_max(Tm, o.max_requests);
-    size_t part = 0, rows = 0, keys = 0, solved = 0, pairs = 0, values = 0, last = 0, gates = 0, outs = 0;
+    size_t part = 0, rows = 0, keys = 0, solved = 0, pairs = 0, values = 0, last = 0, gates = 0, outs = 0, cols = 0;
     for (PekaraxLayer &L : layers) {
       PekaraxAttention &A = L.att;
       Memory &M = L.mem;
@@ -267,9 +267,12 @@ struct Pekarax : public PagedDecoder {
       const size_t c = chunks * M.H, wide = memory_chunk_width(M.dg);
       const bool delta = M.rule == kMemoryDelta;
       keys = std::max(keys, c * kMemoryChunk * wide * 2);
-      if (delta) solved = std::max(solved, c * kMemoryChunk * wide * 2);
+      if (delta) {
+        cols = std::max(cols, (size_t)Tm * (2 * M.G * M.dg + M.H * M.vg) * 2);
+        solved = std::max(solved, c * kMemoryChunk * wide * 2);
+        values = std::max(values, c * kMemoryChunk * M.vs * 4);
+      }
       pairs = std::max(pairs, c * kMemoryChunk * kMemoryChunk * 2);
-      values = std::max(values, c * kMemoryChunk * M.vs * (delta ? 4 : 2));
       last = std::max(last, c * wide * 4);
       if (M.rule == kMemoryNormed) gates = std::max(gates, (size_t)Tm * M.H * 12);
       outs = std::max(outs, (size_t)Tm * M.H * M.vs * 4);
@@ -281,9 +284,12 @@ struct Pekarax : public PagedDecoder {
     if (!keys) return FFMI_OK;
     FFMI_TRY(alloc(&scratch.qg, keys));
     FFMI_TRY(alloc(&scratch.kd, keys));
-    if (solved) FFMI_TRY(alloc(&scratch.w, solved));
+    if (solved) {
+      FFMI_TRY(alloc(&scratch.rows, cols));
+      FFMI_TRY(alloc(&scratch.w, solved));
+      FFMI_TRY(alloc(&scratch.u, values));
+    }
     FFMI_TRY(alloc(&scratch.p, pairs));
-    FFMI_TRY(alloc(&scratch.u, values));
     FFMI_TRY(alloc(&scratch.last, last));
     if (gates) FFMI_TRY(alloc(&scratch.gates, gates));
     return alloc(&scratch.o, outs);
@@ -462,8 +468,14 @@ struct Pekarax : public PagedDecoder {
       FFMI_HIP(launch_pack_sums(y, a.decay.col, low, step.T, L.low, stream));
       FFMI_TRY(gemm_sum_to(low, L.wlow, L.nz, L.low, &a.z, zs, zs_bytes));
     }
-    if (shorts) FFMI_HIP(launch_memory_steps(step.dev, step.off_spans, step.num_spans, a, f32, limit, stream));
-    if (longs) FFMI_HIP(launch_memory_chunks(step.dev, step.off_spans, step.num_spans, a, scratch, limit, stream));
+    bool left = false;
+    if (shorts)
+      FFMI_HIP(launch_memory_steps(step.dev, step.off_spans, step.num_spans, a, chunks ? &scratch : nullptr, f32,
+                                   limit, &left, stream));
+    if (longs)
+      FFMI_HIP(launch_memory_chunks(step.dev, step.off_spans, step.num_spans, step.num_chunks, a, scratch, limit,
+                                    stream));
+    if (left || longs) FFMI_HIP(launch_memory_out(step.dev, a, scratch, left ? 0 : limit, stream));
     return FFMI_OK;
   }
   ffmi_status experts(const PekaraxLayer &L) {
