@@ -34,12 +34,12 @@ struct Row8F {
   }
 };
 // A narrow second product: four lanes a row, 32 columns at a time.  The first rows' first
-// 128 columns are fetched ahead (head), before the product's input is there.
-template <class E>
+// 32 kAhead columns are fetched ahead (head), before the product's input is there.
+template <class E, int kAhead>
 struct LowRankRows {
   typedef typename std::conditional<sizeof(E) == 2, Row8, Row8F>::type Row;
-  static constexpr int kAhead = 4, kRows = NT / 4;
-  Row head[kAhead];
+  static constexpr int kRows = NT / 4;
+  Row head[kAhead ? kAhead : 1];
   static __device__ __forceinline__ const E *row(const LowRank &l, int r) {
     return (const E *)l.w + (size_t)r * l.r + (threadIdx.x & 3) * 8;
   }
@@ -56,18 +56,20 @@ struct LowRankRows {
     for (int c0 = 0; c0 < n; c0 += kRows) {
       const int c = c0 + ((int)threadIdx.x >> 2), cc = min(c, n - 1);
       const E *w = row(l, row0 + cc);
-      Row cur[kAhead];
+      Row cur[kAhead ? kAhead : 1];
 #pragma unroll
       for (int i = 0; i < kAhead; ++i) {
         cur[i] = head[i];
         if (c0 > 0 && i * 32 < l.r) cur[i].load(w + i * 32);
       }
+#pragma unroll 1
       for (int t = 0; t < np; ++t) {
         const float *xt = x + t * l.r + j * 8;
         float v = 0.f;
 #pragma unroll
         for (int i = 0; i < kAhead; ++i)
           if (i * 32 < l.r) v += cur[i].dot(xt + i * 32);
+#pragma unroll 1
         for (int k = kAhead * 32; k < l.r; k += 32) {
           Row more;
           more.load(w + k);
@@ -95,9 +97,10 @@ __host__ __device__ inline int piece_floats(const Memory &a) {
 // What memory has to give comes in the order it is waited for: narrow matrices, the
 // products' columns, the state.
 template <MemoryRule RULE, class E, int P, bool SPLIT>
-__global__ __launch_bounds__(NT) void memory_steps_kernel(const char *__restrict__ blob, int off_spans, Memory a,
+__global__ __launch_bounds__(NT, SPLIT ? 4 : 2) void memory_steps_kernel(const char *__restrict__ blob, int off_spans, Memory a,
                                                           MemoryScratch w, int limit, int piece, int cw, int cols) {
-  constexpr int TAPS = 4;  // up to here without a loop
+  constexpr bool CONV = RULE == kMemoryDelta;
+  constexpr int TAPS = CONV ? 4 : 1;  // up to here without a loop
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const PagedSpan sp = reinterpret_cast<const PagedSpan *>(blob + off_spans)[blockIdx.y];
   if (sp.n > limit) return;
@@ -115,9 +118,12 @@ __global__ __launch_bounds__(NT) void memory_steps_kernel(const char *__restrict
   const bool first = h % (a.H / a.G) == 0 && cb == 0;  // (query and key heads are shared)
   float *S = a.state + ((size_t)sp.slot * a.H + h) * dg * vs;
 
-  LowRankRows<E> decay, gate;
+  LowRankRows<E, SPLIT ? 0 : 4> decay, gate;
   if constexpr (RULE != kMemoryNormed) decay.fetch(a.decay, h * a.dim, a.dim);
   if (r2 > 0) gate.fetch(a.gate, h * a.vdim, a.vdim);
+  const float rate = RULE == kMemoryDelta ? a.rate[h] : 0.f;
+  float dbias = 0.f;  // of the first row that this thread finishes
+  if constexpr (RULE != kMemoryNormed) dbias = a.dbias[(size_t)h * dg + min(tid >> 2, a.dim - 1)];
   float nw[4];  // the norm's weights of this lane's columns
   if constexpr (!SPLIT)
 #pragma unroll
@@ -132,14 +138,14 @@ __global__ __launch_bounds__(NT) void memory_steps_kernel(const char *__restrict
     for (int p = 0; p < P; ++p) {
       const int row = p * NG + rg;
       st[p] = f4{0.f, 0.f, 0.f, 0.f};
-      if (!fresh && row < dg && c0 + cl < ce) st[p] = *reinterpret_cast<const f4 *>(S + (size_t)row * vs + c0 + cl);
+      if (!fresh && row < dg && c0 + cl < ce) st[p] = *reinterpret_cast<const f4 *>(S + (uint32_t)(row * vs + c0 + cl));
     }
   };
   auto store = [&](int c0) {
 #pragma unroll
     for (int p = 0; p < P; ++p) {
       const int row = p * NG + rg;
-      if (row < dg && c0 + cl < ce) *reinterpret_cast<f4 *>(S + (size_t)row * vs + c0 + cl) = st[p];
+      if (row < dg && c0 + cl < ce) *reinterpret_cast<f4 *>(S + (uint32_t)(row * vs + c0 + cl)) = st[p];
     }
   };
 
@@ -147,38 +153,16 @@ __global__ __launch_bounds__(NT) void memory_steps_kernel(const char *__restrict
   const int past = max(a.taps - 1, 0);
   const float *old = a.carry + ((size_t)sp.slot * 2 + bank) * past * C;
   float *now = a.carry + ((size_t)sp.slot * 2 + (bank ^ 1)) * past * C;
-  // column c of q | k | v for token t of the span, u its product; keep: it is carried on
-  auto project = [&](int t, int c, float u, bool keep) {
-    float v = u;
-    if (a.taps > 0) {
-      const size_t at = (size_t)(sp.t0 + t) * a.y.NP + a.col + c;
-      const auto before = [&](int d) {  // d tokens back
-        if (t < d) return old[(d - t - 1) * C + c];
-        return sum_at(a.y, slab, at - (size_t)d * a.y.NP);
-      };
-      const int n = min(past, sp.pos0 + t);
-      v = u * a.conv[past * C + c];
-      if (past < TAPS) {
-        float x[TAPS - 1], cv[TAPS - 1];
-#pragma unroll
-        for (int d = 1; d < TAPS; ++d) {
-          x[d - 1] = cv[d - 1] = 0.f;
-          if (d <= n) x[d - 1] = before(d), cv[d - 1] = a.conv[(past - d) * C + c];
-        }
-        if (keep && t == 0)  // (a short span: earlier rows move on)
-#pragma unroll
-          for (int d = 1; d < TAPS; ++d)
-            if (sp.n + d - 1 < past) now[(sp.n + d - 1) * C + c] = x[d - 1];
-#pragma unroll
-        for (int d = 1; d < TAPS; ++d) v = fmaf(x[d - 1], cv[d - 1], v);
-      } else {
-        for (int d = 1; d <= n; ++d) v = fmaf(before(d), a.conv[(past - d) * C + c], v);
-        if (keep && t == 0)
-          for (int p = sp.n; p < past; ++p) now[p * C + c] = p - sp.n < sp.pos0 ? old[(p - sp.n) * C + c] : 0.f;
-      }
-      if (keep && sp.n - 1 - t < past) now[(sp.n - 1 - t) * C + c] = u;
-    }
-    return a.silu ? silu_f(v) : v;
+  // A column of the first product for one token, with what its convolution reads: asked for
+  // (fetch), then finished.
+  struct Item {
+    int t, c, y;  // token of the piece, item, column (-1: none)
+    float u, x[CONV ? TAPS - 1 : 1], w[TAPS];
+  };
+  // the row d tokens before token t, column c of q | k | v
+  auto before = [&](int t, int d, int c) {
+    if (t < d) return old[(d - t - 1) * C + c];
+    return sum_at(a.y, slab, (size_t)(sp.t0 + t - d) * a.y.NP + a.col + c);
   };
   // what a token needs of the first product, item by item: its column, and where it goes
   const int nv = ce - cb, e1 = 2 * dg, e2 = e1 + nv, e3 = e2 + r1 + r2, e4 = e3 + (SPLIT || r2 > 0 ? 0 : vg);
@@ -190,16 +174,54 @@ __global__ __launch_bounds__(NT) void memory_steps_kernel(const char *__restrict
     if (c < e4) return a.col_gate + h * vg + c - e3;
     return RULE == kMemoryDelta ? a.col_beta + h : (c == e4 ? a.col_i : a.col_f) + h;
   };
-  auto place = [&](int p0, int t, int c, float u) {
+  auto fetch = [&](int p0, int np, int id) {
+    Item it;
+    it.t = id / items, it.c = id - it.t * items, it.y = id < np * items ? column(it.c) : -1, it.u = 0.f;
+    const int t = p0 + it.t, n = min(past, sp.pos0 + t), c = it.y - a.col;
+    if (it.y >= 0) it.u = sum_at(a.y, slab, (size_t)(sp.t0 + t) * a.y.NP + it.y);
+    const bool conv = past < TAPS && it.c < e2 && it.y >= 0;
+    if constexpr (CONV)
+#pragma unroll
+      for (int d = 0; d < TAPS; ++d) {
+        it.w[d] = 0.f;
+        if (d > 0) it.x[d - 1] = 0.f;
+        if (conv && d < a.taps) it.w[d] = a.conv[(past - d) * C + c];
+        if (d > 0 && conv && d <= n) it.x[d - 1] = before(t, d, c);
+      }
+    return it;
+  };
+  // through the convolution and the activation; keep: this workgroup carries the row on
+  auto project = [&](const Item &it, int t, bool keep) {
+    if (it.y < 0) return 0.f;
+    float v = it.u;
+    if (CONV && a.taps > 0) {
+      const int c = it.y - a.col;
+      if (past < TAPS) {
+        v *= it.w[0];
+#pragma unroll
+        for (int d = 1; d < TAPS; ++d) v = fmaf(it.x[d - 1], it.w[d], v);
+        if (keep && t == 0)  // (a short span: earlier rows move on)
+#pragma unroll
+          for (int d = 1; d < TAPS; ++d)
+            if (sp.n + d - 1 < past) now[(sp.n + d - 1) * C + c] = it.x[d - 1];
+      } else {
+        v *= a.conv[past * C + c];
+        for (int d = 1; d <= min(past, sp.pos0 + t); ++d) v = fmaf(before(t, d, c), a.conv[(past - d) * C + c], v);
+        if (keep && t == 0)
+          for (int p = sp.n; p < past; ++p) now[p * C + c] = p - sp.n < sp.pos0 ? old[(p - sp.n) * C + c] : 0.f;
+      }
+      if (keep && sp.n - 1 - t < past) now[(sp.n - 1 - t) * C + c] = it.u;
+    }
+    return a.silu ? silu_f(v) : v;
+  };
+  auto finish = [&](int p0, const Item &it) {
+    const int t = it.t, c = it.c;
+    const float u = it.u;
     if (c < e1) {
-      const float v = project(p0 + t, c < dg ? hq * dg + c : (a.G + hq) * dg + c - dg, u, first);
-      (c < dg ? sq : sk)[t * dg + (c < dg ? c : c - dg)] = v;
+      (c < dg ? sq : sk)[t * dg + (c < dg ? c : c - dg)] = project(it, p0 + t, first);
     } else if (c < e2) {
       const int vc = cb + c - e1;
-      float v = 0.f;
-      if (vc < vg) v = project(p0 + t, 2 * a.G * dg + h * vg + vc, u, true);
-      if (RULE == kMemoryNormed && vc == a.vdim) v = 1.f;
-      sv[t * vs + vc] = v;
+      sv[t * vs + vc] = RULE == kMemoryNormed && vc == a.vdim ? 1.f : project(it, p0 + t, true);
     } else if (c < e3) {
       if (c - e2 < r1) sx[t * r1 + c - e2] = u;
       else sx2[t * r2 + c - e2 - r1] = u;
@@ -215,18 +237,21 @@ __global__ __launch_bounds__(NT) void memory_steps_kernel(const char *__restrict
   int turn = 0;
   for (int p0 = 0; p0 < sp.n; p0 += piece) {
     const int np = min(piece, sp.n - p0);
-    for (int id0 = tid; id0 < np * items; id0 += 2 * NT) {  // two at a time
-      const int id1 = id0 + NT;
-      const int ta = id0 / items, ca = id0 - ta * items, tb = id1 / items, cc = id1 - tb * items;
-      const bool both = id1 < np * items;
-      const int ya = column(ca), yb = both ? column(cc) : -1;
-      float ua = 0.f, ub = 0.f;
-      if (ya >= 0) ua = sum_at(a.y, slab, (size_t)(sp.t0 + p0 + ta) * a.y.NP + ya);
-      if (yb >= 0) ub = sum_at(a.y, slab, (size_t)(sp.t0 + p0 + tb) * a.y.NP + yb);
-      place(p0, ta, ca, ua);
-      if (both) place(p0, tb, cc, ub);
+    if constexpr (SPLIT) {
+      for (int id = tid; id < np * items; id += NT) {
+        const Item it = fetch(p0, np, id);
+        if (p0 == 0 && id == tid) load(cb, sp.pos0 == 0);
+        finish(p0, it);
+      }
+    } else {
+      for (int id = tid; id < np * items; id += 2 * NT) {  // two at a time
+        const Item i0 = fetch(p0, np, id), i1 = fetch(p0, np, id + NT);
+        if (p0 == 0 && id == tid) load(cb, sp.pos0 == 0);
+        finish(p0, i0);
+        if (id + NT < np * items) finish(p0, i1);
+      }
     }
-    if (p0 == 0) load(cb, sp.pos0 == 0);
+    if (p0 == 0 && tid >= np * items) load(cb, sp.pos0 == 0);
     __syncthreads();
     // gates, norms
     if constexpr (RULE == kMemoryNormed) {
@@ -267,7 +292,10 @@ __global__ __launch_bounds__(NT) void memory_steps_kernel(const char *__restrict
         }
       }
       decay.run(a.decay, h * a.dim, a.dim, np, sx,
-                [&](int t, int c, float z) { sg[t * dg + c] = expf(log_decay<RULE>(a, h, c, z)); });
+                [&](int t, int c, float z) {
+                  z += c == tid >> 2 ? dbias : a.dbias[(size_t)h * dg + c];
+                  sg[t * dg + c] = sizeof(E) == 2 ? ex2(log2_decay<RULE>(a, rate, z)) : decay_of<RULE>(a, rate, z);
+                });
       for (int id = tid; id < np * (dg - a.dim); id += NT)
         sg[id / (dg - a.dim) * dg + a.dim + id % (dg - a.dim)] = 1.f;
     }
@@ -375,7 +403,7 @@ bool bad_shape(const Memory &a) {
   return a.H < 1 || a.G < 1 || a.H % a.G || a.dg % 32 || a.vg % 32 || a.dg < a.dim || a.vg < a.vdim ||
          a.dim < 1 || a.vdim < 1 || a.vs != memory_state_columns(a.rule, a.vdim) || a.vs < a.vg ||
          a.dg > kMemoryMaxDim || a.vs > kMemoryMaxVdim + 32 || a.y.S < 1 || a.y.S > 8 || a.y.NP % 4 || a.col % 4 ||
-         a.taps < 0 || (a.taps > 0 && !a.conv) || (a.taps > 1 && !a.carry) || a.decay.r % 32 || a.gate.r % 32 ||
+         (a.rule == kMemoryDelta) != (a.taps > 0) || (a.taps > 0 && !a.conv) || (a.taps > 1 && !a.carry) || a.decay.r % 32 || a.gate.r % 32 ||
          (a.rule == kMemoryNormed ? !a.peak || !a.bi || !a.bf || a.decay.r : !a.decay.w || !a.dbias || !a.decay.r) ||
          (a.rule == kMemoryDelta && !a.rate) || !a.norm || !a.state || a.ldo % 32 || a.out_col % 32 ||
          a.out_col + a.H * a.vg > a.ldo;

@@ -17,6 +17,7 @@
 // Logs of decays have base 2.
 #include <algorithm>
 
+#include "conv_rows.h"
 #include "memory_util.h"
 
 namespace ffmi {
@@ -25,10 +26,8 @@ namespace {
 
 typedef short s4 __attribute__((ext_vector_type(4)));
 constexpr int C = kMemoryChunk;
-constexpr float kLog2e = 1.4426950408889634f;
 constexpr float kSpread = 80.f;  // base 2: far from fp32's and bf16's range on either side
 
-__device__ __forceinline__ float ex2(float v) { return __builtin_amdgcn_exp2f(v); }
 __device__ __forceinline__ f4 mma(bf8 a, bf8 b, f4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
 
 // operand of 8 k-values from row-major LDS rows of LD: column c0 + (lane & 15), rows
@@ -55,17 +54,6 @@ __device__ __forceinline__ uint2 pack4(const f4 &v) {
 __device__ __forceinline__ void load8(const float *p, f4 (&v)[2]) {
   v[0] = *reinterpret_cast<const f4 *>(p), v[1] = *reinterpret_cast<const f4 *>(p + 4);
 }
-// softplus in base-2 units: log2(1 + 2^(z log2 e))
-__device__ __forceinline__ float softplus2(float z) {
-  z *= kLog2e;
-  return fmaxf(z, 0.f) + __builtin_amdgcn_logf(1.f + ex2(-fabsf(z)));
-}
-template <MemoryRule RULE>
-__device__ __forceinline__ float log2_decay(const Memory &a, float rate, float z) {
-  if constexpr (RULE == kMemoryDelta) return -rate * softplus2(z);
-  else return -a.inv_tau * softplus2(-z);
-}
-
 // the span whose chunk `c` is (counted over the step's long spans); a wave looks for it
 __device__ __forceinline__ int span_of_chunk(const PagedSpan *spans, int num, int c) {
   for (int b = 0; b < num; b += 64) {
@@ -79,75 +67,6 @@ __device__ __forceinline__ int span_of_chunk(const PagedSpan *spans, int num, in
     if (m) return __builtin_amdgcn_readfirstlane(b + __ffsll((unsigned long long)m) - 1);
   }
   return -1;
-}
-
-// delta: rows of q | k | v, convolved and through their activation, for the chunks; the
-// rows that are carried on.  A thread has 8 columns of TB tokens; PAST: taps - 1 (earlier
-// rows in registers), or -1: read again.
-template <int PAST>
-__global__ __launch_bounds__(256) void memory_rows_kernel(const char *__restrict__ blob, Memory a, MemoryScratch w,
-                                                          int limit) {
-  constexpr int TB = 8, H = PAST > 0 ? PAST : 1;
-  const int cols = memory_columns(a), c = (blockIdx.x * 256 + threadIdx.x) * 8, t0 = blockIdx.y * TB;
-  if (c >= cols) return;
-  const PagedToken *tok = reinterpret_cast<const PagedToken *>(blob + a.off_tokens);
-  const size_t slab = (size_t)a.T * a.y.NP;
-  const int past = a.taps - 1;
-  const float *cw = a.conv + c;
-  f4 u[TB][2], x[H][2], wt[H + 1][2];
-#pragma unroll
-  for (int k = 0; k < TB; ++k) sum8(a.y, slab, (size_t)min(t0 + k, a.T - 1) * a.y.NP + a.col + c, u[k]);
-  // the row d tokens before token t
-  auto before = [&](const PagedToken &tk, int t, int d, f4 (&v)[2]) {
-    v[0] = v[1] = f4{0.f, 0.f, 0.f, 0.f};
-    if (tk.back >= d) sum8(a.y, slab, (size_t)(t - d) * a.y.NP + a.col + c, v);
-    else if (tk.pos >= d) load8(a.carry + (((size_t)tk.slot * 2 + tk.bank) * past + d - tk.back - 1) * cols + c, v);
-  };
-  if constexpr (PAST >= 0)
-#pragma unroll
-    for (int d = 0; d <= PAST; ++d) load8(cw + (size_t)(PAST - d) * cols, wt[d]);
-#pragma unroll
-  for (int k = 0; k < TB; ++k) {
-    const int t = t0 + k;
-    if (t >= a.T) break;
-    const PagedToken tk = tok[t];
-    if (PAST > 0 && (k == 0 || tk.back == 0))
-#pragma unroll
-      for (int d = 1; d <= PAST; ++d) before(tk, t, d, x[d - 1]);
-    if (tk.back + tk.ahead + 1 > limit) {
-      f4 v[2];
-      if (tk.ahead < past) {
-        float *now = a.carry + (((size_t)tk.slot * 2 + (tk.bank ^ 1)) * past + tk.ahead) * cols + c;
-        *reinterpret_cast<f4 *>(now) = u[k][0], *reinterpret_cast<f4 *>(now + 4) = u[k][1];
-      }
-      if constexpr (PAST >= 0) {
-        v[0] = u[k][0] * wt[0][0], v[1] = u[k][1] * wt[0][1];
-#pragma unroll
-        for (int d = 1; d <= PAST; ++d) v[0] += x[d - 1][0] * wt[d][0], v[1] += x[d - 1][1] * wt[d][1];
-      } else {
-        f4 f[2], e[2];
-        load8(cw + (size_t)past * cols, f);
-        v[0] = u[k][0] * f[0], v[1] = u[k][1] * f[1];
-        for (int d = 1; d <= past; ++d) {
-          before(tk, t, d, e);
-          load8(cw + (size_t)(past - d) * cols, f);
-          v[0] += e[0] * f[0], v[1] += e[1] * f[1];
-        }
-      }
-      if (a.silu)
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          const float y = v[e >> 2][e & 3];
-          v[e >> 2][e & 3] = y * __builtin_amdgcn_rcpf(1.f + ex2(-kLog2e * y));
-        }
-      *reinterpret_cast<uint4 *>(w.rows + (size_t)t * cols + c) = pack8_bf16(v[0], v[1]);
-    }
-    if constexpr (PAST > 0) {
-#pragma unroll
-      for (int d = PAST; d > 1; --d) x[d - 1][0] = x[d - 2][0], x[d - 1][1] = x[d - 2][1];
-      x[0][0] = u[k][0], x[0][1] = u[k][1];
-    }
-  }
 }
 
 // normed: decay, key factor (logs, base 2) and m of every token of a long span; a workgroup
@@ -792,17 +711,13 @@ hipError_t run_chunks(const char *blob, int off_spans, int num_spans, int num_ch
   if (RULE == kMemoryNormed)
     hipLaunchKernelGGL(memory_gates_kernel, dim3(a.H, num_spans), dim3(256), 0, s, blob, off_spans, a, w, limit);
   if (RULE == kMemoryDelta) {
-    const dim3 grid((2 * a.G * a.dg + a.H * a.vg + 2047) / 2048, (a.T + 7) / 8);
-#define FFMI_MW(PAST) hipLaunchKernelGGL(memory_rows_kernel<PAST>, grid, dim3(256), 0, s, blob, a, w, limit)
-    if (a.taps == 1) FFMI_MW(0);
-    else if (a.taps == 2) FFMI_MW(1);
-    else if (a.taps == 3) FFMI_MW(2);
-    else if (a.taps == 4) FFMI_MW(3);
-    else FFMI_MW(-1);
-#undef FFMI_MW
+    ConvRows c;
+    c.u = a.y, c.T = a.T, c.col = a.col, c.cols = 2 * a.G * a.dg + a.H * a.vg, c.taps = a.taps, c.conv = a.conv;
+    c.carry = a.carry, c.silu = a.silu, c.hb = w.rows, c.off_tokens = a.off_tokens, c.above = limit;
+    if (const hipError_t e = launch_conv_rows(blob, c, s)) return e;
   }
   // narrow workgroups where the spans and heads alone do not fill the chip
-  const bool wide = (long)a.H * num_spans * (a.vs / 32) >= 256;
+  const bool wide = (long)a.H * num_spans * (a.vs / 16) > 512;
 #define FFMI_MS(KS, VS)                                                                                             \
   hipLaunchKernelGGL((memory_scan_kernel<RULE, KS, VS>), dim3((a.vs + VS - 1) / VS, a.H, num_spans), dim3(256), 0, s, \
                      blob, off_spans, a, w, limit)

@@ -8,13 +8,24 @@ namespace ffmi {
 __device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 // columns of q | k | v
 __device__ __forceinline__ int memory_columns(const Memory &a) { return 2 * a.G * a.dg + a.H * a.vg; }
-// log of the decay of channel c < dg of head h from its logit (bias not in yet)
+// a decay from its logit, in full precision (rate: of the head)
 template <MemoryRule RULE>
-__device__ __forceinline__ float log_decay(const Memory &a, int h, int c, float z) {
-  if (c >= a.dim) return 0.f;
-  z += a.dbias[(size_t)h * a.dg + c];
-  if constexpr (RULE == kMemoryDelta) return -a.rate[h] * softplus_f(z);
-  else return -a.inv_tau * softplus_f(-z);
+__device__ __forceinline__ float decay_of(const Memory &a, float rate, float z) {
+  if constexpr (RULE == kMemoryDelta) return expf(-rate * softplus_f(z));
+  else return expf(-a.inv_tau * softplus_f(-z));
+}
+// bf16 model: its log, base 2, by the base-2 instructions; what the logarithm loses of
+// small values (6e-8) is what a decay next to 1 has no bits for
+constexpr float kLog2e = 1.4426950408889634f;
+__device__ __forceinline__ float ex2(float v) { return __builtin_amdgcn_exp2f(v); }
+__device__ __forceinline__ float softplus2(float z) {
+  z *= kLog2e;
+  return fmaxf(z, 0.f) + __builtin_amdgcn_logf(1.f + ex2(-fabsf(z)));
+}
+template <MemoryRule RULE>
+__device__ __forceinline__ float log2_decay(const Memory &a, float rate, float z) {
+  if constexpr (RULE == kMemoryDelta) return -rate * softplus2(z);
+  else return -a.inv_tau * softplus2(-z);
 }
 // a head's log input and forget gates of one token
 __device__ __forceinline__ void memory_gates(const Memory &a, int t, int h, float &i, float &f) {

@@ -49,11 +49,9 @@ struct AttnPrep {
   const double *freq = nullptr, *vfreq = nullptr;
   int rot = 0;
   float rot_mult = 1.f;
-  // rotary kind: taps > 0: a causal convolution of every product column over time,
-  // before norm and rotation; conv [taps][columns] (columns (H + G) dg + G vg), the
-  // last row the current token's.  The last taps - 1 product rows of a request are
-  // carried: carry [slots][2 banks][taps - 1][columns], the latest first.  off_tokens:
-  // the step's tokens in its metadata
+  // rotary kind, made in the attention's launch: taps > 0: a causal convolution of the
+  // product's columns over time first (conv_rows.h; a launch of its own otherwise);
+  // off_tokens: the step's tokens in its metadata
   const float *conv = nullptr;
   int taps = 0;
   float *carry = nullptr;

@@ -115,14 +115,14 @@ __device__ __forceinline__ void load_head(const AttnPrep &a, int T, int t, int h
     }
   }
 }
-// (rotary kind) The convolution over time of one head's columns: v, a token's product,
-// becomes the sum over its taps, and the rows that later steps need go to the other bank.
-// Up to TAPS taps (none in wide heads) their weights and the earlier rows are kept in
-// registers: load(), then the tokens of a run in turn.
+// (rotary kind, few rows) The convolution over time of one head's columns: v, a token's
+// product, becomes the sum over its taps, and the rows that later steps need go to the
+// other bank.  Up to TAPS taps: their weights and the earlier rows are asked for with the
+// product (load).
 template <int NE>
 struct HeadConv {
-  static constexpr int TAPS = NE <= 4 ? 4 : 1, PAST = TAPS - 1;
-  float w[TAPS][NE], x[PAST > 0 ? PAST : 1][NE];  // of the token d back, and its row
+  static constexpr int TAPS = 4, PAST = TAPS - 1;
+  float w[TAPS][NE], x[PAST][NE];  // of the token d back, and its row
   static __device__ __forceinline__ size_t columns(const AttnPrep &a) {
     return (size_t)(a.H + a.G) * a.dg + (size_t)a.G * a.vg;
   }
@@ -133,7 +133,7 @@ struct HeadConv {
   static __device__ __forceinline__ float before(const AttnPrep &a, int T, int t, const PagedToken &tk, int d,
                                                  size_t col) {
     if (d > tk.pos) return 0.f;
-    if (tk.back >= d) return slab_sum(a.y, (size_t)T * a.y.NP, (size_t)(t - d) * a.y.NP + col);
+    if (tk.back >= d) return sum_at(a.y, (size_t)T * a.y.NP, (size_t)(t - d) * a.y.NP + col);
     return bank(a, tk, 0)[(d - tk.back - 1) * columns(a) + col];
   }
   __device__ __forceinline__ void load(const AttnPrep &a, int T, int t, const PagedToken &tk, int hd) {
@@ -150,8 +150,6 @@ struct HeadConv {
       }
     }
   }
-  // NT > 1: the next token of the run follows
-  template <int NT>
   __device__ __forceinline__ void apply(const AttnPrep &a, int T, int t, const PagedToken &tk, int hd,
                                         float (&v)[NE]) {
     const int wd = head_width(a, hd), c0 = head_start(a, hd), past = a.taps - 1;
@@ -173,11 +171,6 @@ struct HeadConv {
 #pragma unroll
         for (int d = 1; d <= PAST; ++d) sum = fmaf(x[d - 1][i], w[d][i], sum);
         v[i] = sum;
-        if constexpr (NT > 1 && PAST > 0) {
-#pragma unroll
-          for (int d = PAST; d > 1; --d) x[d - 1][i] = x[d - 2][i];
-          x[0][i] = u;
-        }
       } else {
         if (tk.back == 0)
           for (int d = 1; tk.ahead + d < past; ++d) now[(tk.ahead + d) * C + col] = before(a, T, t, tk, d, col);
@@ -405,15 +398,6 @@ __global__ __launch_bounds__(512) void rotary_prep_kernel(const PagedToken *__re
     load_bias<NE>(a, hd, bias);
 #pragma unroll
     for (int k = 0; k < NT; ++k) load_head<NE>(a, T, min(t0 + k, T - 1), hd, bias, v[k]);
-    if (a.taps > 0) {
-      HeadConv<NE> cv;
-#pragma unroll
-      for (int k = 0; k < NT; ++k)
-        if (t0 + k < T) {
-          if (k == 0 || tk[k].back == 0) cv.load(a, T, t0 + k, tk[k], hd);
-          cv.template apply<NT>(a, T, t0 + k, tk[k], hd, v[k]);
-        }
-    }
     if (isv) {
       if (a.vfreq)
 #pragma unroll
@@ -639,7 +623,7 @@ __device__ __forceinline__ void attn_few_rows(const char *__restrict__ blob, con
       const int tk = token_of(it), pos = bk.pos0 + tk, tile = pos / kPageTokens;
       if constexpr (KIND == kRotary)  // (split blocks carry the same rows)
         if (pr.taps > 0)
-          cv.template apply<1>(pr, T, t0 + tk, ptok[tk], head_of(it), x);
+          cv.apply(pr, T, t0 + tk, ptok[tk], head_of(it), x);
       if (it < nq) {
         make(it, pos, x);
         store_head<uint16_t, NE>([&](int c) { return sQ + it * LDQ + c; }, DP, x);
@@ -1038,6 +1022,8 @@ static hipError_t launch_attn_kind(const char *blob, const PagedLists &pl, AttnA
                                    float *ml, hipStream_t s, const AttnPrep *pr, int T) {
   if (pl.num_blocks <= 0) return hipSuccess;
   if (!a.ldo) a.ldo = a.H * a.vg;
+  if (pr && pr->taps > 0 && (KIND != kRotary || !pr->conv || (pr->taps > 1 && !pr->carry)))
+    return hipErrorInvalidValue;
   if (pr && (pl.row_tiles != 1 || pr->H != a.H || pr->G != a.G || pr->dp != a.dp || pr->vp != a.vp ||
              pr->vg != a.vg || pr->y.S < 1 || pr->y.S > 8 || pr->every < 1))
     return hipErrorInvalidValue;

@@ -217,7 +217,7 @@ hipError_t launch_row_norm(const char *blob, int off_rows, const float *x, const
 }
 
 // One workgroup per row, a thread's chunks of 8 columns; all loads before the
-// reduction.
+// reduction, of slabs MAXS at a time.
 template <int NT, int MAXC, int MAXS>
 __global__ __launch_bounds__(NT) void sum_norm_kernel(SumNorm a) {
   constexpr int U = 4;  // expert rows in flight
@@ -232,11 +232,14 @@ __global__ __launch_bounds__(NT) void sum_norm_kernel(SumNorm a) {
   for (int c = 0; c < MAXC; ++c) {
     const int ch = min((int)threadIdx.x + c * NT, nchunk - 1);
     f4 p[MAXS ? MAXS : 1][2];
+    auto slabs = [&](int s0) {
 #pragma unroll
-    for (int sl = 0; sl < MAXS; ++sl) {
-      const float *q = a.y.p + (size_t)row * a.y.NP + ch * 8 + (size_t)min(sl, a.y.S - 1) * a.T * a.y.NP;
-      p[sl][0] = *reinterpret_cast<const f4 *>(q), p[sl][1] = *reinterpret_cast<const f4 *>(q + 4);
-    }
+      for (int sl = 0; sl < MAXS; ++sl) {
+        const float *q = a.y.p + (size_t)row * a.y.NP + ch * 8 + (size_t)min(s0 + sl, a.y.S - 1) * a.T * a.y.NP;
+        p[sl][0] = *reinterpret_cast<const f4 *>(q), p[sl][1] = *reinterpret_cast<const f4 *>(q + 4);
+      }
+    };
+    slabs(0);
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
       x[c][h] = *reinterpret_cast<const f4 *>(a.x + (size_t)row * H + ch * 8 + 4 * h) * alpha;
@@ -263,9 +266,12 @@ __global__ __launch_bounds__(NT) void sum_norm_kernel(SumNorm a) {
       for (int k = 0; k < U; ++k)
         if (w[k] != 0.f) y[0] += r[k][0] * w[k], y[1] += r[k][1] * w[k];
     }
+    for (int s0 = 0; MAXS > 0 && s0 < a.y.S; s0 += MAXS ? MAXS : 1) {
+      if (s0 > 0) slabs(s0);
 #pragma unroll
-    for (int sl = 0; sl < MAXS; ++sl)
-      if (sl < a.y.S) y[0] += p[sl][0], y[1] += p[sl][1];
+      for (int sl = 0; sl < MAXS; ++sl)
+        if (s0 + sl < a.y.S) y[0] += p[sl][0], y[1] += p[sl][1];
+    }
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
       x[c][h] += y[h];
@@ -301,8 +307,7 @@ hipError_t launch_sum_norm(const SumNorm &a, hipStream_t s) {
   do {                                   \
     if (a.y.S == 0) FFMI_SM(NT, MC, 0);  \
     else if (a.y.S == 1) FFMI_SM(NT, MC, 1); \
-    else if (a.y.S <= 4) FFMI_SM(NT, MC, 4); \
-    else FFMI_SM(NT, MC, 8);             \
+    else FFMI_SM(NT, MC, 4);             \
   } while (0)
   if (nchunk <= 128) FFMI_SMS(128, 1);
   else if (nchunk <= 256) FFMI_SMS(256, 1);

@@ -9,7 +9,7 @@ hipError_t launch_rotary_prep(const char *blob, int off_tokens, int T, const Att
   if (T <= 0) return hipSuccess;
   const int wide = std::max(std::max(a.dp, a.vp), std::max(a.dg, a.vg));
   if (wide > 1024 || a.y.S < 1 || a.y.S > 8 || a.rot < 0 || a.rot > a.dim || a.rot % 2 || (a.rot && !a.freq) ||
-      a.taps < 0 || (a.taps > 0 && !a.conv) || (a.taps > 1 && !a.carry))
+      a.taps > 0)
     return hipErrorInvalidValue;
   const PagedToken *tok = reinterpret_cast<const PagedToken *>(blob + off_tokens);
   const int runs = (a.H + 2 * a.G + 7) / 8;  // of eight heads

@@ -25,6 +25,7 @@
 
 #include <algorithm>
 
+#include "../kernels/conv_rows.h"
 #include "../kernels/memory.h"
 #include "../kernels/moe.h"
 #include "../kernels/paged_attn.h"
@@ -72,6 +73,7 @@ struct Pekarax : public PagedDecoder {
   int max_slots = 0;
   void *q = nullptr, *cat = nullptr;
   uint16_t *hrow = nullptr, *low = nullptr;
+  float *crows = nullptr;  // an attention's convolved product
   float *zs = nullptr, *slabs = nullptr, *ml = nullptr;
   size_t zs_bytes = 0;
   MemoryScratch scratch;
@@ -206,7 +208,7 @@ struct Pekarax : public PagedDecoder {
     return FFMI_OK;
   }
   ffmi_status init_layers() override {
-    size_t qw = 32, cw = 32, lw = 0;
+    size_t qw = 32, cw = 32, lw = 0, rw = 0;
     double wbytes = 0;
     int min_groups = 1 << 30;
     std::vector<RowShape> shapes;
@@ -217,7 +219,7 @@ struct Pekarax : public PagedDecoder {
       if (L.attention) {
         shapes.push_back(RowShape{L.att.heads / L.att.groups, L.att.groups, kAttnTiles, true});
         min_groups = std::min(min_groups, L.att.groups);
-        qw = std::max(qw, (size_t)L.att.heads * L.att.dp);
+        qw = std::max(qw, (size_t)L.att.heads * L.att.dp), rw = std::max(rw, (size_t)L.att.cols);
       }
       cw = std::max(cw, (size_t)L.no);
       gemms.insert(gemms.end(), {{L.nq, Wp}, {Wp, L.no}});
@@ -236,6 +238,7 @@ struct Pekarax : public PagedDecoder {
     FFMI_TRY(init_step(shapes, max_slots, gemms, wbytes));
     FFMI_TRY(alloc_zero(&q, (size_t)Tm * qw * es()));
     FFMI_TRY(alloc_zero(&cat, (size_t)Tm * cw * es()));
+    if (rw) FFMI_TRY(alloc(&crows, (size_t)Tm * rw * 4));
     if (lw) {
       FFMI_TRY(alloc_zero(&low, (size_t)Tm * lw * 2));
       FFMI_TRY(alloc(&zs, zs_bytes));
@@ -448,6 +451,13 @@ struct Pekarax : public PagedDecoder {
     const bool rows = !mfma_form(A);
     // decoding and short portions: in the attention's launch
     const bool fused = !rows && pl.row_tiles == 1;
+    if (!fused) {
+      ConvRows c;
+      c.u = y, c.T = step.T, c.cols = A.cols, c.taps = A.taps, c.conv = A.conv, c.carry = A.carry, c.hf = crows;
+      c.off_tokens = step.off_tokens;
+      FFMI_HIP(launch_conv_rows(step.dev, c, stream));
+      p.y.p = crows, p.y.S = 1, p.y.NP = A.cols, p.taps = 0;
+    }
     if (!fused) FFMI_HIP(launch_rotary_prep(step.dev, step.off_tokens, step.T, p, f32, stream));
     AttnArgs a;
     a.q = q, a.kc = A.kc, a.vc = A.vc, a.o = cat, a.ldo = L.no;

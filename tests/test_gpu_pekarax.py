@@ -499,6 +499,51 @@ def test_memory_widths(tmp_path, dim, vdim):
             close(run(eng, toks, cuts), want, full)
 
 
+def together(rm, m, seqs, steps):
+    """requests side by side: steps of (portion of each)"""
+    ids = [9000 + _next[0] * 10 + i for i in range(len(seqs))]
+    _next[0] += 1
+    at, got = [0] * len(seqs), [[] for _ in seqs]
+    for step in steps:
+        entries = [(ids[i], seqs[i][at[i]:at[i] + n], range(n)) for i, n in enumerate(step) if n]
+        out, r = rm.replay_step(m, entries), 0
+        for i, n in enumerate(step):
+            if n:
+                got[i].append(out[r:r + n])
+                at[i], r = at[i] + n, r + n
+    for i in ids:
+        rm.replay_end(m, i)
+    return [np.concatenate(g) for g in got]
+
+
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("dim", [24, 64, 128, 200])
+def test_many_heads_and_portions(tmp_path, dim, full):
+    """Long portions of several requests in one step, in heads enough that a workgroup
+    of the pass over the chunks takes more columns; then single tokens beside portions."""
+    cfg = PM.model_config(50, 48, [PM.delta(12, 6, dim, 180, low=(9, 9)), PM.gla(12, dim, 192),
+                                   PM.parallel((1, 1, 16, 16, 1.0), (12, dim, 180, 10.0), 0.3, 1.0)])
+    w = PM.random_weights(cfg, 8)
+    rm, m = make_engine(PM.write_checkpoint(tmp_path / "m", cfg, w), full, batch=512)
+    steps = [(70, 17, 130, 64), (1, 66, 1, 20), (1, 1, 1, 1), (2, 1, 18, 0), (1, 1, 1, 19)]
+    seqs = [tokens(cfg, sum(s[i] for s in steps), 40 + i) for i in range(4)]
+    for got, seq in zip(together(rm, m, seqs, steps), seqs):
+        close(got, R.forward(cfg, w, seq), full)
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_many_wide_heads_at_decode(tmp_path, full):
+    """Few wide heads' columns are split over workgroups, a slice each or several; with
+    one, two and four requests."""
+    cfg = PM.model_config(50, 48, [PM.gla(90, 136, 160), PM.parallel((1, 1, 16, 16, 1.0), (90, 136, 160, 10.0), 0.3, 1.0)])
+    w = PM.random_weights(cfg, 8)
+    rm, m = make_engine(PM.write_checkpoint(tmp_path / "m", cfg, w), full)
+    steps = [(3, 0, 0, 0), (1, 2, 0, 0), (1, 1, 1, 0), (1, 3, 1, 0), (1, 1, 1, 1), (2, 1, 1, 16), (1, 1, 1, 0)]
+    seqs = [tokens(cfg, sum(s[i] for s in steps), 40 + i) for i in range(4)]
+    for got, seq in zip(together(rm, m, seqs, steps), seqs):
+        close(got, R.forward(cfg, w, seq), full)
+
+
 @pytest.mark.parametrize("full", [True, False])
 @pytest.mark.parametrize("strength", ["mixed", "far apart", "none", "at once"])
 @pytest.mark.parametrize("kind", ["delta", "gla", "normed"])
