@@ -483,7 +483,8 @@ __global__ __launch_bounds__(256, KS <= 4 ? 2 : 1) void memory_chunk_kernel(cons
   }
 }
 
-// The pass over the chunks: a workgroup per (VS state columns, head, span).  Wave w: rows
+// The pass over the chunks: a workgroup per (head, VS state columns, span); a head's are
+// mostly on one XCD, which then reads the chunk's operands once.  Wave w: rows
 // 16 w .. of u and o, and of the state 16 columns and an even share of the rows, in
 // registers (lane: 4 rows of one column); the state goes to LDS once a chunk as the
 // operand [column][row], u as rows.  What the next chunk needs is fetched a chunk ahead.
@@ -498,7 +499,7 @@ __global__ __launch_bounds__(256, KS * VS <= (RULE == kMemoryDelta ? 64 : 128) ?
   if (sp.n <= limit) return;
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l15 = lane & 15;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int h = blockIdx.y, c0 = blockIdx.x * VS, vw = min(VS, a.vs - c0);
+  const int h = blockIdx.x, c0 = blockIdx.y * VS, vw = min(VS, a.vs - c0);
   const int ri = wave * 16 + l15, vcol = wave % VT * 16 + l15, d0 = wave / VT * ND;
   const size_t id0 = (size_t)sp.chunk0 * a.H + h;
 
@@ -719,7 +720,7 @@ hipError_t run_chunks(const char *blob, int off_spans, int num_spans, int num_ch
   // narrow workgroups where the spans and heads alone do not fill the chip
   const bool wide = (long)a.H * num_spans * (a.vs / 16) > 512;
 #define FFMI_MS(KS, VS)                                                                                             \
-  hipLaunchKernelGGL((memory_scan_kernel<RULE, KS, VS>), dim3((a.vs + VS - 1) / VS, a.H, num_spans), dim3(256), 0, s, \
+  hipLaunchKernelGGL((memory_scan_kernel<RULE, KS, VS>), dim3(a.H, (a.vs + VS - 1) / VS, num_spans), dim3(256), 0, s, \
                      blob, off_spans, a, w, limit)
 #define FFMI_MC(KS)                                                                                              \
   do {                                                                                                           \
